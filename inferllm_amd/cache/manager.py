@@ -6,7 +6,8 @@ names it).  Lines with the same needs form a *group* with storage of its own:
 
 * kind "full": every key and value of a sequence is kept;
 * kind "window": only the last `window` keys are ever read, so a sequence keeps a
-  ring of pages and its storage stops growing.
+  ring of pages and its storage stops growing; with `keep_first` the sequence's first tokens
+  are read too, however far back, and the pages that hold them stay ahead of the ring.
 
 What a line keeps per token is a list of named tensors (`TokenTensor`: name, per-token shape,
 dtype), which its mixer states: attention keeps "k" and "v" of [kv heads, head_dim]; another
@@ -57,16 +58,19 @@ class TokenTensor:
 @dataclass(frozen=True)
 class KVSpec:
     """What one cache line needs: which tokens are kept ("full": all, "window": the last
-    `window`) and the tensors kept of each."""
+    `window` and the first `keep_first`) and the tensors kept of each."""
     kind: str
     tensors: Tuple[TokenTensor, ...]
     window: Optional[int] = None
+    keep_first: int = 0
 
     def __post_init__(self):
         if self.kind not in ("full", "window"):
             raise CacheError(f"unknown cache kind {self.kind!r}")
         if self.kind == "window" and not (self.window and self.window > 0):
             raise CacheError("a window cache needs a positive window")
+        if self.keep_first < 0 or (self.keep_first and self.kind != "window"):
+            raise CacheError("kept first tokens go with a window")
         names = [t.name for t in self.tensors]
         if not names or len(set(names)) != len(names):
             raise CacheError(f"a cache line needs per-token tensors with distinct names, got {names}")
@@ -104,11 +108,13 @@ class KVGroup:
             # rows: a step stores all its keys before its rows read, so the keys of a step of n
             # tokens must not reach round the ring into the window of the step's first row
             self.ring = (spec.window + max(0, step_rows - 1) + page_size - 2) // page_size + 1
-            if self.ring >= seq_pages:
-                self.ring = 0           # the window never wraps: same as "full"
+            # logical pages ahead of the ring that stay: those of the kept first tokens
+            self.kept_pages = round_up(spec.keep_first, page_size) // page_size
+            if self.kept_pages + self.ring >= seq_pages:
+                self.ring = self.kept_pages = 0    # the window never wraps: same as "full"
         else:
-            self.ring = 0
-        self.pages_per_seq = self.ring if self.ring else seq_pages
+            self.ring = self.kept_pages = 0
+        self.pages_per_seq = self.kept_pages + self.ring if self.ring else seq_pages
         self.n_pages = min(pages_full, n_slots * self.pages_per_seq)
         self.pool = FreeList(self.n_pages, "page", scatter=True)
         self.spare_page = self.n_pages
@@ -146,7 +152,7 @@ class KVGroup:
 
     def pages_needed(self, length: int) -> int:
         n = (length + self.page_size - 1) // self.page_size
-        return min(n, self.ring) if self.ring else n
+        return min(n, self.pages_per_seq) if self.ring else n
 
     def reserve(self, slot: int, length: int) -> None:
         pages = self.held.setdefault(slot, [])

@@ -28,7 +28,7 @@ class PartSpec:
 
 @dataclass
 class LayerSpec:
-    """A block: its arrangement ("pre_norm", "parallel", "hyper_connections") and the parts it
+    """A block: its arrangement ("pre_norm", "parallel", "sandwich", "post_norm", "hyper_connections") and the parts it
     is made of.  An arrangement with one norm (both parts read its rows) has no
     `feed_forward_norm`.  An arrangement with constants or tensors of its own (the weights with
     which several residual streams are mixed) takes them as `block_params` and `block_tensors`

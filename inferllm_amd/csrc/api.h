@@ -44,6 +44,18 @@ int illm_relu_squared(const void* x, void* out, int dt, size_t n, void* stream);
 // out[i] = 0.5 x (1 + tanh(sqrt(2 / pi) (x + 0.044715 x^3))).
 int illm_gelu_tanh(const void* x, void* out, int dt, size_t n, void* stream);
 
+// xIELU with par = (cp, cn), two floats on the device: out = (x > 0 ? cp x^2 : cn (e^x - 1 - x)) + x / 2.
+int illm_xielu(const void* x, const float* par, void* out, int dt, size_t n, void* stream);
+
+// ---- norms behind a sublayer (post_norm.hip)
+// One pass over the rows: x <- x + gain * post(a) (a null: nothing), then out = the row itself or a
+// norm of it.  Kinds of norm: 0 none, 1 RMS norm under w, 2 layer norm under w and b (pb, b may be null).
+// With row_idx only those rows are formed and x stays; out null: x alone is moved on.
+int illm_post_add_norm(float* x, const void* a, int a_dt, int post_kind, const void* pw, const void* pb,
+                       int pw_dt, float post_eps, float gain, int out_kind, const void* w, const void* b,
+                       int w_dt, float eps, void* out, int out_dt, const int32_t* row_idx, int rows, int E,
+                       void* stream);
+
 // Residual add and RMS norm.  in_row = row_idx ? row_idx[r] : r;
 // v = x[in_row] (+ delta[in_row]); when delta is given and row_idx is not, v is
 // written back to x.  out[r] = v * rsqrt(mean(v^2) + eps) * w.  delta may be `planes` >= 1
@@ -347,9 +359,9 @@ int illm_few_outputs_f32(const void* x, int x_dt, const float* w, float* z, int 
 
 // idx, wt [T, top]: the `top` outputs of z [T, NE] (float32) with the largest softmax(z) + corr
 // (corr may be null), in falling order, and their softmax values.  NE <= 512.
-// score_kind 0: softmax over all outputs; 1: every output's sigmoid.
+// score_kind 0: softmax over all outputs; 1: every output's sigmoid.  The weights are scale times them.
 int illm_moe_route(const float* z, const void* corr, int corr_dt, int T, int NE, int top,
-                   int32_t* idx, float* wt, int score_kind, void* stream);
+                   int32_t* idx, float* wt, int score_kind, float scale, void* stream);
 
 // order [NP]: the pairs whose choice is below NEr, grouped by choice; tiles [3 max_tiles + 1]:
 // (expert, first place in order, rows <= tile_rows) per tile and, last, their number.
@@ -362,8 +374,8 @@ int illm_moe_group(const int32_t* idx, int NP, int NEr, int32_t* order, int32_t*
 // Y[p] = X[p / x_div] . W[e_p]^T for every grouped pair p (W [experts][N][K]); gated: W
 // [experts][2 N][K] = [gate | up] rows and Y[p] = silu(X Wg^T) * (X Wu^T).  Y [NP, N] of dt.
 // act_kind (gated only) 0: silu(g) * u; 1: with g = min(g, limit), u = clamp(u, -limit, limit):
-// g * sigmoid(1.702 g) * (u + 1).  row_w (may be null; gated only): a weight per pair that
-// multiplies the pair's X row (applied to the two products, which is the same).
+// g * sigmoid(1.702 g) * (u + 1); not gated, 2: Y[p] = max(X W^T, 0)^2, 0: the product.  row_w (may be
+// null): a weight per pair that multiplies the pair's X row (applied to the products, which is the same).
 int illm_moe_rows(const void* X, int x_div, const void* W, int dt, int gated, const int32_t* order,
                   const int32_t* tiles, int max_tiles, void* Y, int N, int K, int act_kind,
                   float limit, const float* row_w, void* stream);
@@ -420,18 +432,24 @@ int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt, const int
                        const void* vcache, const int32_t* page_table, int table_stride,
                        int page_size, int ring, int n_seqs, int max_rows, int nh, int nkv, int dk,
                        int dv, float scale, float cap, int window, const float* slopes, int chunk,
-                       const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse, void* stream);
+                       const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse,
+                       int keep, int kept, int own_stride, int own_k, int own_v, void* stream);
 int illm_attn_cap_decode(const void* q, int q_stride, void* out, int dt, const void* kcache,
                          const void* vcache, const int32_t* page_table, int table_stride,
                          int page_size, int ring, const int32_t* seq_slot, const int32_t* seq_len,
                          float* partial, int nsplit, int B, int nh, int nkv, int dk, int dv,
                          float scale, float cap, int window, const float* slopes, int chunk,
-                         const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse, void* stream);
+                         const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse,
+                         int keep, int kept, void* stream);
 // The two calls above also take: `slopes` float32 [nh] (null: none), score -= slopes[h] (i - j);
 // `chunk` > 0, a row sees only the keys j with floor(j / chunk) = floor(i / chunk); `gate` (null: none),
 // rows [., gate_stride] of the queries' dtype, out *= sigmoid(gate[row, gate_off + h dv + d]) (with
 // `gate_heads` gate[row, gate_off + h]); `lse` (null: none), float32 [rows, nh]: max + log(sum) of each
-// softmax (single tokens: with nsplit >= 2).
+// softmax (single tokens: with nsplit >= 2); `keep` > 0 (with a window, without chunks): the sequence's
+// first `keep` tokens are seen beside the window; `kept`: the pages that stay in place ahead of the
+// cache line's ring.  illm_attn_cap_rows with own_stride > 0 reads keys and values not from the cache
+// but from the step's own rows, kcache and vcache then their base (row r of sequence b at (cu[b] + r)
+// own_stride, key heads from column own_k, value heads from own_v); every sequence starts in this step.
 // In place: q and k of rows [q (nh dk) | .. k at k_off | v at v_off] each divided by the root mean
 // square over all their heads and multiplied by qw, kw (null: untouched); v <- (1 - lam[0]) v +
 // lam[0] first[row, first_off ..] (lam null: untouched); k and v stored in the paged cache (null: not).
@@ -444,11 +462,12 @@ int illm_qkv_norm_mix_store(void* rows, int dt, int row_len, int k_off, int v_of
 
 // ---- what stands around the plain gated recurrence (linear_scan.hip, delta_rule.hip)
 // The scan of illm_delta_scan with a choice of rule: `correct` 1, the delta rule; 0, the plain gated
-// rule S <- diag(g) S + k (beta v)^T, o = S^T q.
+// rule S <- diag(g) S + k (beta v)^T, o = S^T q; with `removal` float32 [T, H, dk] (correct 0, G = H)
+// S <- diag(g) S - removal (u^T S) + k v^T, u = beta k, both terms from the old state.
 int illm_gated_scan(const float* qn, const float* kn, const float* vv, const float* beta,
                     const float* dec, int DW, float* state, const int32_t* cu,
                     const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int G, int H, int dk,
-                    int dv, int correct, void* stream);
+                    int dv, int correct, const float* removal, void* stream);
 // A state-space mixer's inputs from U [T, u_stride]: columns x_off.. = x (H dv) | B (G N) | C (G N)
 // through the short convolution (conv_w float32 [C, taps], conv_b [C], tail [slots, taps - 1, C] of
 // U's dtype) and SiLU into vv, kn, qn; beta = softplus(U[dt_off + h] + dt_bias[h]),
@@ -508,12 +527,16 @@ int illm_clamped_swish_mul(const void* gate_up, void* out, int dt, int T, int F,
 // turned by their positions (cos_sin float32 [n_positions, rot / 2, 2]; pairing 0: i with i + rot / 2,
 // 1: 2i with 2i + 1; null: none), then, with `unit_norm`, divided by their root mean square, query head
 // h then times q_scale[h] (float32 [nh]; null: none); k and v
-// stored in the paged cache (kcache null: not stored; nkv 0: queries alone).
+// stored in the paged cache (kcache null: not stored; nkv 0: queries alone).  Ahead of the rotation
+// `bias` float32 [q | k | v] (null: none) is added and q and k heads are RMS-normed (eps) under qw, kw
+// [dk] (null: not).  `slot_len` (int32 by slot, the lengths after the step; null: every row is stored):
+// rows that later rows of the step overwrite in the ring are not stored.  `kept` as above.
 int illm_qk_rotate_store(void* rows, int dt, int row_len, int k_off, int v_off, const float* cos_sin,
                          int rot, int pairing, int n_positions, int unit_norm, float eps,
                          const float* q_scale, const int32_t* row_pos, const int32_t* row_slot, void* kcache, void* vcache,
                          const int32_t* page_table, int table_stride, int page_size, int ring, int T,
-                         int nh, int nkv, int dk, int dv, void* stream);
+                         int nh, int nkv, int dk, int dv, const float* bias, const void* qw,
+                         const void* kw, int w_dt, const int32_t* slot_len, int kept, void* stream);
 // For every row whose position ends a block of `pool` tokens: the block's mean key and value, from
 // the cache, into row (position / pool) of the sequence in kpool, vpool (same layout and page table).
 int illm_pool_store(const int32_t* row_pos, const int32_t* row_slot, const void* kcache,
@@ -555,6 +578,43 @@ int illm_lru_gates(const float* u, const float* Wt, const float* br, const float
 int illm_lru_scan(const float* a, const float* x, float* state, const void* Y, int y_dt, int y_stride,
                   int y_off, const float* yb, void* out, int out_dt, const int32_t* cu,
                   const int32_t* seq_slot, int n_seqs, int max_rows, int C, float* scratch, void* stream);
+
+// ---- lightning attention and the delta rule with a removal vector (fixed_decay.hip)
+// Lightning attention from U [T, u_stride], q at q_off and k at k_off (H dk), v at v_off (H dv), all
+// through SiLU, one decay a head (float32 [H]).  _prepare: float32 inputs of illm_gated_scan (weight 1).
+// _step: one row a sequence, S <- decay S + k v^T in state [slots, H, dk, dv] and o = S^T q (float32
+// [rows, H, dv]) in one launch.  _chunks: any number of rows, in chunks of illm_lightning_chunk() tokens
+// on the matrix cores' float32 instruction; dk, dv <= 128 in steps of 4, offsets and u_stride in steps of
+// 4; `part`: (T / chunk + n_seqs + 1) H dk dv floats.
+int illm_lightning_prepare(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                           const float* decay, float* qn, float* kn, float* vv, float* beta, float* dec,
+                           int T, int H, int dk, int dv, void* stream);
+int illm_lightning_step(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                        const float* decay, float* state, const int32_t* row_slot, float* o, int B, int H,
+                        int dk, int dv, void* stream);
+int illm_lightning_chunk(void);
+int illm_lightning_chunks(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                          const float* decay, float* state, float* part, const int32_t* cu,
+                          const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int H, int dk, int dv,
+                          void* stream);
+// The delta rule with a removal vector from U: r, k, v and the rates' pre-activations at a_off, all H d
+// wide; u = k / sqrt(sum k^2 + 1e-6) a head, decay = exp(-rate sigmoid(Z + w0)), removal = sigmoid(a + a_bias) u.
+// _prepare: float32 inputs of illm_gated_scan (beta = 1 / |k|).  _step: one row a sequence in one launch,
+// Z = w2 tanh(U[w1_off ..]) (w2 [H d, rank] of U's dtype, rank <= 512).
+int illm_removal_prepare(const void* U, int dt, int u_stride, int r_off, int k_off, int v_off, int a_off,
+                         const float* a_bias, const void* Z, int z_dt, int z_stride, const float* w0,
+                         float rate, float* qn, float* kn, float* vv, float* beta, float* dec,
+                         float* removal, int T, int H, int d, void* stream);
+int illm_removal_step(const void* U, int dt, int u_stride, int r_off, int k_off, int v_off, int a_off,
+                      const float* a_bias, int w1_off, int rank, const void* w2, const float* w0, float rate,
+                      float* state, const int32_t* row_slot, float* o, int B, int H, int d, void* stream);
+// out[t, i] = tanh(U[t, off + i]), i < n, of U's dtype.
+int illm_tanh_columns(const void* U, int dt, int u_stride, int off, void* out, int T, int n, void* stream);
+// o float32 [T, width] RMS-normed in `groups` equal parts of the row, times w [width], times
+// silu (gate_kind 0) or sigmoid (1) of Z[:, z_off ..].
+int illm_group_norm_gate(const float* o, const void* w, int w_dt, const void* Z, int z_dt, int z_stride,
+                         int z_off, int gate_kind, void* out, int out_dt, int T, int width, int groups,
+                         float eps, void* stream);
 
 #ifdef __cplusplus
 }

@@ -1,7 +1,8 @@
 // Causal attention whose scores pass a soft cap and whose keys and values have sizes of their own:
 //     score = cap * tanh((q . k) * scale / cap)     (cap <= 0: no cap)
-// softmax over the visible keys (all j <= i, or the last `window`), context = sum p_j v_j with
-// values of width dv where queries and keys have width dk.  Three more things a caller may ask for:
+// softmax over the visible keys (all j <= i, or the last `window` and with them the sequence's first
+// `keep`), context = sum p_j v_j with values of width dv where queries and keys have width dk.  Three
+// more things a caller may ask for:
 // a bias by distance, score -= slopes[h] (i - j) (`slopes` null: none); chunks, position i sees only
 // the keys of its own chunk, floor(j / chunk) = floor(i / chunk), counted from the sequence's
 // position 0 (`chunk` <= 0: none); an output gate, out *= sigmoid(gate[row, gate_off + h dv + d])
@@ -11,7 +12,10 @@
 // Keys and values live in the paged cache, K [page][kv head][row][dk], V [page][kv head][row][dv],
 // under one page table; a step first stores its rows (`kv_store2`) and then every row attends over
 // the cache at absolute positions, so whole prompts, portions of prompts and single tokens take
-// the same path.  Float32 arithmetic over float32 or bfloat16 storage: widths of up to 128 in steps
+// the same path.  A line that keeps a window as a ring of pages (the first `kept` pages beside it)
+// does not hold a long prompt: rows of a step whose sequences all start may read the step's own rows
+// instead (`own_stride` > 0: keys at column own_k, values at own_v of the rows that q lies in).
+// Float32 arithmetic over float32 or bfloat16 storage: widths of up to 128 in steps
 // of 4 (single tokens: of 16 bytes) take the kernels on the matrix cores' float32 instruction and
 // with eight lanes a key, every other width the plain ones on the vector units.
 #include <math.h>
@@ -156,7 +160,7 @@ attn_cap_rows_kernel(const void* __restrict__ q, int q_stride, void* __restrict_
                      int table_stride, int page_size, int ring, int nh, int nkv, int dk, int dv,
                      float scale, float cap, int window, const float* __restrict__ slopes, int chunk,
                      const void* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
-                     float* __restrict__ lse) {
+                     float* __restrict__ lse, int keep, int kept, int own_stride, int own_k, int own_v) {
     extern __shared__ float smem[];
     const int kp = dk + 1, vp = dv + 1;
     float* qs = smem;               // [CQ][kp]
@@ -188,19 +192,22 @@ attn_cap_rows_kernel(const void* __restrict__ q, int q_stride, void* __restrict_
     k_lo = (k_lo / CK) * CK;
     const float slope = slopes ? slopes[h] : 0.f;
     const int c_lo = chunk > 0 ? (qpos / chunk) * chunk : 0;            // first key of this row's chunk
+    const int k_first = min(k_lo, ((keep + CK - 1) / CK) * CK);         // tiles [0, k_first): the kept tokens'
 
-    for (int k0 = k_lo; k0 < k_hi; k0 += CK) {
+    for (int k0 = k_first > 0 ? 0 : k_lo; k0 < k_hi; k0 = k0 + CK == k_first ? k_lo : k0 + CK) {
         __syncthreads();
         for (int e = tid; e < CK * dk; e += 256) {
             const int r = e / dk, d = e - r * dk;
             ks[r * kp + d] = k0 + r < total
-                ? ld_f(kcache, dt, cache_row_offset(page_table, table_stride, slot, k0 + r, page_size, ring, nkv, kvh, dk) + d)
+                ? ld_f(kcache, dt, (own_stride ? (size_t)(start + k0 + r) * own_stride + own_k + (size_t)kvh * dk
+                                               : cache_row_offset(page_table, table_stride, slot, k0 + r, page_size, ring, nkv, kvh, dk, kept)) + d)
                 : 0.f;
         }
         for (int e = tid; e < CK * dv; e += 256) {
             const int r = e / dv, d = e - r * dv;
             vs[r * vp + d] = k0 + r < total
-                ? ld_f(vcache, dt, cache_row_offset(page_table, table_stride, slot, k0 + r, page_size, ring, nkv, kvh, dv) + d)
+                ? ld_f(vcache, dt, (own_stride ? (size_t)(start + k0 + r) * own_stride + own_v + (size_t)kvh * dv
+                                               : cache_row_offset(page_table, table_stride, slot, k0 + r, page_size, ring, nkv, kvh, dv, kept)) + d)
                 : 0.f;
         }
         __syncthreads();
@@ -211,7 +218,7 @@ attn_cap_rows_kernel(const void* __restrict__ q, int q_stride, void* __restrict_
             const int j = g + 8 * c, kj = k0 + j;
             float a = 0.f;
             for (int d = 0; d < dk; ++d) a = fmaf(qs[i * kp + d], ks[j * kp + d], a);
-            const bool ok = qrow < len && kj <= qpos && kj >= c_lo && (window <= 0 || kj > qpos - window);
+            const bool ok = qrow < len && kj <= qpos && kj >= c_lo && (window <= 0 || kj > qpos - window || kj < keep);
             s[c] = ok ? soft_cap(a * scale, cap, inv_cap) - slope * (float)(qpos - kj) : NEG_INF;
             tm = fmaxf(tm, s[c]);
         }
@@ -318,7 +325,7 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
                           int table_stride, int page_size, int ring, int nh, int nkv, int dk, int dv,
                           float scale, float cap, int window, const float* __restrict__ slopes, int chunk,
                           const void* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
-                          float* __restrict__ lse) {
+                          float* __restrict__ lse, int keep, int kept, int own_stride, int own_k, int own_v) {
     constexpr int DKP = 32 * KT, DVP = 32 * VT, KLD = DKP + 1;
     __shared__ float ks[MK * KLD];
     __shared__ float vs[MK * DVP];
@@ -358,7 +365,8 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
             const int kj = min(k0 + row, total - 1);       // keys past the end: a valid row, masked below
             kreg[i].zero();
             if (d < dk)
-                kreg[i].load(kcache, cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dk) + d);
+                kreg[i].load(kcache, (own_stride ? (size_t)(start + kj) * own_stride + own_k + (size_t)kvh * dk
+                                                 : cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dk, kept)) + d);
         }
 #pragma unroll
         for (int i = 0; i < VT; ++i) {
@@ -366,7 +374,8 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
             const int kj = min(k0 + row, total - 1);
             vreg[i].zero();
             if (d < dv)
-                vreg[i].load(vcache, cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dv) + d);
+                vreg[i].load(vcache, (own_stride ? (size_t)(start + kj) * own_stride + own_v + (size_t)kvh * dv
+                                                 : cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dv, kept)) + d);
         }
     };
     auto stage = [&]() __attribute__((always_inline)) {
@@ -396,13 +405,17 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
     const int wc_lo = chunk > 0 ? (wq_lo / chunk) * chunk : 0;     // the wave's first row sees farthest back
     const int c_lo = chunk > 0 ? (qpos / chunk) * chunk : 0;
     const int k_last = k_lo + ((k_hi - 1 - k_lo) / MK) * MK;
-    fetch(k_lo);
-    for (int k0 = k_lo; k0 < k_hi; k0 += MK) {
+    const int k_first = min(k_lo, ((keep + MK - 1) / MK) * MK);    // tiles [0, k_first): the kept tokens'
+    int k_next = k_first > 0 ? 0 : k_lo;
+    fetch(k_next);
+    for (int k0 = k_next; k0 < k_hi; k0 = k_next) {
         __syncthreads();
         stage();
         __syncthreads();
-        fetch(min(k0 + MK, k_last));              // (unconditional: the last tile is asked for twice)
-        if (!wave_has_rows || k0 > wq_hi || k0 + MK - 1 < wc_lo || (window > 0 && k0 + MK - 1 <= wq_lo - window))
+        k_next = k0 + MK == k_first ? k_lo : k0 + MK;
+        fetch(min(k_next, k_last));               // (unconditional: the last tile is asked for twice)
+        if (!wave_has_rows || k0 > wq_hi || k0 + MK - 1 < wc_lo ||
+            (window > 0 && k0 >= keep && k0 + MK - 1 <= wq_lo - window))
             continue;
         cap_f32x16_t sc;
 #pragma unroll
@@ -415,7 +428,7 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
 #pragma unroll
         for (int v = 0; v < 16; ++v) {
             const int kj = k0 + 8 * (v >> 2) + 4 * half + (v & 3);
-            const bool ok = qrow < len && kj <= qpos && kj >= c_lo && (window <= 0 || kj > qpos - window);
+            const bool ok = qrow < len && kj <= qpos && kj >= c_lo && (window <= 0 || kj > qpos - window || kj < keep);
             sc[v] = ok ? soft_cap(sc[v] * scale, cap, inv_cap) - slope * (float)(qpos - kj) : NEG_INF;
             tm = fmaxf(tm, sc[v]);
         }
@@ -474,19 +487,25 @@ extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt
                                   int table_stride, int page_size, int ring, int n_seqs, int max_rows,
                                   int nh, int nkv, int dk, int dv, float scale, float cap, int window,
                                   const float* slopes, int chunk, const void* gate, int gate_stride,
-                                  int gate_off, int gate_heads, float* lse, void* stream) {
+                                  int gate_off, int gate_heads, float* lse, int keep, int kept,
+                                  int own_stride, int own_k, int own_v, void* stream) {
+    if (keep < 0 || kept < 0 || (keep > 0 && (window <= 0 || chunk > 0)) || own_stride < 0 ||
+        (own_stride && (own_k < 0 || own_v < 0 || own_k + nkv * dk > own_stride || own_v + nkv * dv > own_stride)))
+        return ILLM_ERR_ARG;
     if (gate && (gate_off < 0 || gate_off + nh * (gate_heads ? 1 : dv) > gate_stride)) return ILLM_ERR_ARG;
     if (n_seqs < 0 || max_rows < 0 || nh <= 0 || nkv <= 0 || nh % nkv || dk <= 0 || dk > 256 ||
         dv <= 0 || dv > 256 || page_size <= 0 || !illm_dtype_ok(dt) || nh > 65535 || n_seqs > 65535)
         return ILLM_ERR_ARG;
     if (n_seqs == 0 || max_rows == 0) return ILLM_OK;
-    if (g_attn_cap_mfma && dk <= 128 && dv <= 128 && dk % 4 == 0 && dv % 4 == 0 && q_stride % 4 == 0) {
+    if (g_attn_cap_mfma && dk <= 128 && dv <= 128 && dk % 4 == 0 && dv % 4 == 0 && q_stride % 4 == 0 &&
+        own_stride % 4 == 0 && own_k % 4 == 0 && own_v % 4 == 0) {
         const dim3 grid((max_rows + MQ - 1) / MQ, nh, n_seqs);
         const int kt = (dk + 31) / 32, vt = (dv + 31) / 32;
 #define GO(DT_, KT_, VT_)                                                                          \
     hipLaunchKernelGGL((attn_cap_rows_mfma_kernel<DT_, KT_, VT_>), grid, dim3(256), 0, (hipStream_t)stream, \
                        q, q_stride, out, cu, seq_slot, seq_start, kcache, vcache, page_table, table_stride, \
-                       page_size, ring, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, gate, gate_stride, gate_off, gate_heads, lse)
+                       page_size, ring, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, gate, gate_stride, gate_off, gate_heads, lse, \
+                       keep, kept, own_stride, own_k, own_v)
 #define GO_V(DT_, KT_)                                                                             \
     switch (vt) { case 1: GO(DT_, KT_, 1); break; case 2: GO(DT_, KT_, 2); break;                  \
                   case 3: GO(DT_, KT_, 3); break; default: GO(DT_, KT_, 4); break; }
@@ -507,8 +526,29 @@ extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt
     hipLaunchKernelGGL(attn_cap_rows_kernel, dim3((max_rows + CQ - 1) / CQ, nh, n_seqs), dim3(256), lds,
                        (hipStream_t)stream, q, q_stride, out, dt, cu, seq_slot, seq_start, kcache, vcache,
                        page_table, table_stride, page_size, ring, nh, nkv, dk, dv, scale, cap, window, slopes,
-                       chunk, gate, gate_stride, gate_off, gate_heads, lse);
+                       chunk, gate, gate_stride, gate_off, gate_heads, lse, keep, kept, own_stride, own_k, own_v);
     return illm_launch_status();
+}
+
+// The keys a single token sees, numbered without a gap: with `keep` first tokens before the window the
+// nk = min(keep, window's first key) kept ones are 0 .. nk - 1 and the window follows at nk (key number
+// v stands at position v + skip from there on); else numbers are positions (nk = 0, skip = 0).
+struct SeenKeys {
+    int lo, hi, nk, skip;
+    __device__ __forceinline__ int at(int v) const { return v < nk ? v : v + skip; }
+};
+__device__ __forceinline__ SeenKeys seen_keys(int len, int window, int chunk, int keep) {
+    SeenKeys s;
+    s.lo = window > 0 ? max(0, len - window) : 0;
+    if (chunk > 0) s.lo = max(s.lo, ((len - 1) / chunk) * chunk);     // the new token's own chunk
+    s.hi = len; s.nk = 0; s.skip = 0;
+    if (keep > 0 && s.lo > 0) {
+        s.nk = min(keep, s.lo);
+        s.skip = s.lo - s.nk;
+        s.lo = 0;
+        s.hi = len - s.skip;
+    }
+    return s;
 }
 
 // ---------------------------------------------------------------- single tokens
@@ -524,19 +564,18 @@ attn_cap_decode_kernel(const void* __restrict__ q, int q_stride, const void* __r
                        int table_stride, int page_size, int ring, const int32_t* __restrict__ seq_slot,
                        const int32_t* __restrict__ seq_len, float* __restrict__ partial, int nsplit,
                        int nh, int nkv, int dk, int dv, float scale, float cap, int window,
-                       const float* __restrict__ slopes, int chunk) {
+                       const float* __restrict__ slopes, int chunk, int keep, int kept) {
     __shared__ float wacc[4][256];
     __shared__ float wm[4], wl[4];
     const int h = blockIdx.x, b = blockIdx.y, sp = blockIdx.z;
     const int w = wave_index(), lane = threadIdx.x & 63;
     const int len = seq_len[b], slot = seq_slot[b];
     const int kvh = h / (nh / nkv);
-    int lo_all = window > 0 ? max(0, len - window) : 0;
-    if (chunk > 0) lo_all = max(lo_all, ((len - 1) / chunk) * chunk);   // the new token's own chunk
+    const SeenKeys seen = seen_keys(len, window, chunk, keep);
     const float slope = slopes ? slopes[h] : 0.f;
-    const int tiles = (len + 63) / 64, t0 = lo_all / 64;
+    const int tiles = (seen.hi + 63) / 64, t0 = seen.lo / 64;
     const int per = (tiles - t0 + nsplit - 1) / nsplit;
-    const int k_lo = max(lo_all, (t0 + sp * per) * 64), k_hi = min(len, (t0 + (sp + 1) * per) * 64);
+    const int k_lo = max(seen.lo, (t0 + sp * per) * 64), k_hi = min(seen.hi, (t0 + (sp + 1) * per) * 64);
     const float inv_cap = cap > 0.f ? 1.0f / cap : 0.f;
     float qv[4], acc[4];
 #pragma unroll
@@ -553,9 +592,9 @@ attn_cap_decode_kernel(const void* __restrict__ q, int q_stride, const void* __r
         size_t vat[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const int kj = min(k0 + j, k_hi - 1);
-            const size_t kat = cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dk);
-            vat[j] = cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dv);
+            const int kj = seen.at(min(k0 + j, k_hi - 1));
+            const size_t kat = cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dk, kept);
+            vat[j] = cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dv, kept);
             float a = 0.f;
 #pragma unroll
             for (int c = 0; c < 4; ++c) {
@@ -574,7 +613,7 @@ attn_cap_decode_kernel(const void* __restrict__ q, int q_stride, const void* __r
         float tm = NEG_INF;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            s[j] = k0 + j < k_hi ? soft_cap(s[j], cap, inv_cap) - slope * (float)(len - 1 - (k0 + j)) : NEG_INF;
+            s[j] = k0 + j < k_hi ? soft_cap(s[j], cap, inv_cap) - slope * (float)(len - 1 - seen.at(k0 + j)) : NEG_INF;
             tm = fmaxf(tm, s[j]);
         }
         const float m_new = fmaxf(m, tm);
@@ -650,7 +689,8 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
                              const int32_t* __restrict__ seq_len, float* __restrict__ partial, int nsplit,
                              int nh, int nkv, int dk, int dv, float scale, float cap, int window,
                              const float* __restrict__ slopes, int chunk, void* __restrict__ out,
-                             const void* __restrict__ gate, int gate_stride, int gate_off, int gate_heads) {
+                             const void* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
+                             int keep, int kept) {
     constexpr int U = DT == ILLM_BF16 ? 8 : 4;          // elements of a unit
     constexpr int NK = U * KQ, NV = U * VQ;             // dims of a key, of a value, a lane holds
     __shared__ float wacc[4][DH][8 * NV];
@@ -661,11 +701,10 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
     const int b = blockIdx.y, sp = blockIdx.z;
     const int w = wave_index(), lane = threadIdx.x & 63, grp = lane >> 3, sub = lane & 7;
     const int len = seq_len[b], slot = seq_slot[b];
-    int lo_all = window > 0 ? max(0, len - window) : 0;
-    if (chunk > 0) lo_all = max(lo_all, ((len - 1) / chunk) * chunk);
-    const int tiles = (len + 63) / 64, t0 = lo_all / 64;
+    const SeenKeys seen = seen_keys(len, window, chunk, keep);
+    const int tiles = (seen.hi + 63) / 64, t0 = seen.lo / 64;
     const int per = (tiles - t0 + nsplit - 1) / nsplit;
-    const int k_lo = max(lo_all, (t0 + sp * per) * 64), k_hi = min(len, (t0 + (sp + 1) * per) * 64);
+    const int k_lo = max(seen.lo, (t0 + sp * per) * 64), k_hi = min(seen.hi, (t0 + (sp + 1) * per) * 64);
     const float inv_cap = cap > 0.f ? 1.0f / cap : 0.f;
     float qv[DH][NK], acc[DH][NV], m[DH], l[DH], slope[DH];
 #pragma unroll
@@ -699,12 +738,12 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
     // the page of a round's key is looked up a round before its rows are asked for, so that a round
     // waits for one trip to memory, not for two in a row
     auto page_of = [&](int base) __attribute__((always_inline)) {
-        int lp = min(base + grp, k_hi - 1) / page_size;
-        if (ring > 0) lp %= ring;
+        int lp = seen.at(min(base + grp, k_hi - 1)) / page_size;
+        if (ring > 0 && lp >= kept) lp = kept + (lp - kept) % ring;
         return page_table[(size_t)slot * table_stride + lp];
     };
     auto fetch = [&](int base, int page) __attribute__((always_inline)) {
-        const int kj = min(base + grp, k_hi - 1);
+        const int kj = seen.at(min(base + grp, k_hi - 1));
         const size_t row = ((size_t)page * nkv + kvh) * page_size + (kj % page_size);
         const size_t kat = row * dk, vat = row * dv;
         const size_t esz = DT == ILLM_BF16 ? 2 : 4;
@@ -736,8 +775,8 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
             fetch(base + 32, page_next);
             page_next = page_of(base + 64);
         }
-        const int kj = base + grp;
-        const bool valid = kj < k_hi;
+        const bool valid = base + grp < k_hi;
+        const int kj = seen.at(base + grp);
 #pragma unroll
         for (int i = 0; i < DH; ++i) {
             if (i >= hb) continue;
@@ -845,7 +884,9 @@ extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int 
                                     int ring, const int32_t* seq_slot, const int32_t* seq_len,
                                     float* partial, int nsplit, int B, int nh, int nkv, int dk, int dv,
                                     float scale, float cap, int window, const float* slopes, int chunk,
-                                    const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse, void* stream) {
+                                    const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse,
+                                    int keep, int kept, void* stream) {
+    if (keep < 0 || kept < 0 || (keep > 0 && (window <= 0 || chunk > 0))) return ILLM_ERR_ARG;
     if (gate && (gate_off < 0 || gate_off + nh * (gate_heads ? 1 : dv) > gate_stride)) return ILLM_ERR_ARG;
     if (B < 0 || nh <= 0 || nkv <= 0 || nh % nkv || dk <= 0 || dk > 256 || dv <= 0 || dv > 256 ||
         page_size <= 0 || nsplit < 1 || nsplit > 65535 || B > 65535 || !illm_dtype_ok(dt) || !partial ||
@@ -864,11 +905,13 @@ extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int 
     if (dh == 2)                                                                                   \
         hipLaunchKernelGGL((attn_cap_decode_rows8_kernel<DT_, KQ_, VQ_, 2>), grid, dim3(256), 0, st, q, q_stride, \
                            kcache, vcache, page_table, table_stride, page_size, ring, seq_slot, seq_len, partial, \
-                           nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads); \
+                           nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads, \
+                           keep, kept);                                                            \
     else                                                                                           \
         hipLaunchKernelGGL((attn_cap_decode_rows8_kernel<DT_, KQ_, VQ_, 4>), grid, dim3(256), 0, st, q, q_stride, \
                            kcache, vcache, page_table, table_stride, page_size, ring, seq_slot, seq_len, partial, \
-                           nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads)
+                           nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads, \
+                           keep, kept)
 #define GO_V(DT_, KQ_)                                                                             \
     switch (vq) { case 1: { GO(DT_, KQ_, 1); } break; case 2: { GO(DT_, KQ_, 2); } break;          \
                   case 3: { GO(DT_, KQ_, 3); } break; default: { GO(DT_, KQ_, 4); } break; }
@@ -883,11 +926,11 @@ extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int 
     } else if (dt == ILLM_BF16)
         hipLaunchKernelGGL(attn_cap_decode_kernel<ILLM_BF16>, dim3(nh, B, nsplit), dim3(256), 0, st, q,
                            q_stride, kcache, vcache, page_table, table_stride, page_size, ring, seq_slot,
-                           seq_len, partial, nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk);
+                           seq_len, partial, nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, keep, kept);
     else
         hipLaunchKernelGGL(attn_cap_decode_kernel<ILLM_F32>, dim3(nh, B, nsplit), dim3(256), 0, st, q,
                            q_stride, kcache, vcache, page_table, table_stride, page_size, ring, seq_slot,
-                           seq_len, partial, nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk);
+                           seq_len, partial, nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, keep, kept);
     if (hipGetLastError() != hipSuccess) return ILLM_ERR_LAUNCH;
     hipLaunchKernelGGL(attn_cap_merge_kernel, dim3(nh, B), dim3(64), 0, st, partial, out, dt, nsplit, nh, dv,
                        gate, gate_stride, gate_off, gate_heads, lse);

@@ -13,8 +13,8 @@
 // Float32 arithmetic over float32 or bfloat16 storage; key and value widths of up to 256.
 //
 // Beside the attention: `qk_rotate_store` turns q and k of packed rows by their positions (either
-// pairing, the first `rot` dims of a head), optionally divides every head by its root mean square
-// and multiplies query head h by q_scale[h] (a scale of the scores that differs by head, taken into
+// pairing, the first `rot` dims of a head), optionally adds a bias and norms every head under a weight
+// before that, optionally divides every head by its root mean square after it and multiplies query head h by q_scale[h] (a scale of the scores that differs by head, taken into
 // the queries), and stores k and v (widths of their own) in the cache; `pool_store` forms the pooled rows of the
 // blocks that a step completes.
 #include <math.h>
@@ -29,19 +29,35 @@
 // ---------------------------------------------------------------- rotation, unit norm, store
 // grid (rows, nh + nkv); 64 threads.  Block (t, h): h < nh is query head h (columns h dk ..), else
 // key head h - nh (columns k_off ..), whose block also stores the value head (columns v_off ..).
+// `bias` float32 [q (nh dk) | k (nkv dk) | v (nkv dv)] (null: none) is added first, then every q and k
+// head is RMS-normed under qw, kw [dk] (null: not).  With `slot_len` (the sequences' lengths after the
+// step) rows that a later row of the step would overwrite in the ring of pages are not stored.
 __global__ void __launch_bounds__(64)
 qk_rotate_store_kernel(void* __restrict__ rows, int dt, int row_len, int k_off, int v_off,
                        const float* __restrict__ cos_sin, int rot, int pairing, int unit_norm, float eps,
                        const float* __restrict__ q_scale, const int32_t* __restrict__ row_pos, const int32_t* __restrict__ row_slot,
                        void* __restrict__ kcache, void* __restrict__ vcache,
                        const int32_t* __restrict__ page_table, int table_stride, int page_size, int ring,
-                       int nh, int nkv, int dk, int dv) {
+                       int nh, int nkv, int dk, int dv, const float* __restrict__ bias,
+                       const void* __restrict__ qw, const void* __restrict__ kw, int w_dt,
+                       const int32_t* __restrict__ slot_len, int kept) {
     __shared__ float x[256];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int pos = row_pos[t];
     const bool is_k = h >= nh;
     const size_t base = (size_t)t * row_len + (is_k ? k_off + (size_t)(h - nh) * dk : (size_t)h * dk);
-    for (int d = lane; d < dk; d += 64) x[d] = ld_f(rows, dt, base + d);
+    const float* hb = bias ? bias + (size_t)h * dk : nullptr;         // (k heads follow the q heads)
+    float ss0 = 0.f;
+    for (int d = lane; d < dk; d += 64) {
+        const float v = ld_f(rows, dt, base + d) + (hb ? hb[d] : 0.f);
+        x[d] = v;
+        ss0 = fmaf(v, v, ss0);
+    }
+    const void* hw = is_k ? kw : qw;
+    if (hw) {
+        const float inv0 = 1.0f / sqrtf(wave_sum(ss0) / (float)dk + eps);
+        for (int d = lane; d < dk; d += 64) x[d] = (x[d] * inv0) * ld_f(hw, w_dt, d);     // (a lane's own entries)
+    }
     __syncthreads();
     if (cos_sin && rot > 0) {
         const float* cs = cos_sin + (size_t)pos * rot;              // [rot / 2][2]
@@ -64,20 +80,24 @@ qk_rotate_store_kernel(void* __restrict__ rows, int dt, int row_len, int k_off, 
     }
     if (q_scale && !is_k) inv *= q_scale[h];
     size_t kat = 0, vat = 0;
-    const bool store = is_k && kcache != nullptr;
+    bool store = is_k && kcache != nullptr;
     if (store) {
-        const int slot = row_slot[t];
-        kat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dk);
-        vat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dv);
+        const int slot = row_slot[t], lp = pos / page_size;
+        if (ring > 0 && slot_len && lp >= kept && lp + ring <= (slot_len[slot] - 1) / page_size) store = false;
+        kat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dk, kept);
+        vat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dv, kept);
     }
     for (int d = lane; d < dk; d += 64) {
         const float y = x[d] * inv;
         st_f(rows, dt, base + d, y);
         if (store) st_f(kcache, dt, kat + d, y);
     }
-    if (store) {
+    if (is_k && (store || bias)) {
         const size_t vb = (size_t)t * row_len + v_off + (size_t)(h - nh) * dv;
         for (int d = lane; d < dv; d += 64) {
+            if (bias)
+                st_f(rows, dt, vb + d, ld_f(rows, dt, vb + d) + bias[(size_t)(nh + nkv) * dk + (size_t)(h - nh) * dv + d]);
+            if (!store) continue;
             if (dt == ILLM_BF16) ((bf16_t*)vcache)[vat + d] = ((const bf16_t*)rows)[vb + d];
             else ((float*)vcache)[vat + d] = ((const float*)rows)[vb + d];
         }
@@ -89,7 +109,9 @@ extern "C" int illm_qk_rotate_store(void* rows, int dt, int row_len, int k_off, 
                                     int unit_norm, float eps, const float* q_scale, const int32_t* row_pos,
                                     const int32_t* row_slot, void* kcache, void* vcache,
                                     const int32_t* page_table, int table_stride, int page_size, int ring,
-                                    int T, int nh, int nkv, int dk, int dv, void* stream) {
+                                    int T, int nh, int nkv, int dk, int dv, const float* bias, const void* qw,
+                                    const void* kw, int w_dt, const int32_t* slot_len, int kept, void* stream) {
+    if (kept < 0 || ((qw || kw) && !illm_dtype_ok(w_dt))) return ILLM_ERR_ARG;
     if (T < 0 || nh < 0 || nkv < 0 || nh + nkv <= 0 || nh + nkv > 65535 || dk <= 0 || dk > 256 || dv < 0 ||
         dv > 256 || !illm_dtype_ok(dt) || rot < 0 || rot % 2 || rot > dk || (pairing != 0 && pairing != 1) ||
         nh * dk > row_len || (nkv > 0 && (k_off + nkv * dk > row_len || v_off + nkv * dv > row_len)) ||
@@ -98,7 +120,8 @@ extern "C" int illm_qk_rotate_store(void* rows, int dt, int row_len, int k_off, 
     if (T == 0) return ILLM_OK;
     hipLaunchKernelGGL(qk_rotate_store_kernel, dim3(T, nh + nkv), dim3(64), 0, (hipStream_t)stream, rows,
                        dt, row_len, k_off, v_off, cos_sin, rot, pairing, unit_norm, eps, q_scale, row_pos, row_slot,
-                       kcache, vcache, page_table, table_stride, page_size, ring, nh, nkv, dk, dv);
+                       kcache, vcache, page_table, table_stride, page_size, ring, nh, nkv, dk, dv, bias, qw, kw,
+                       w_dt, slot_len, kept);
     return illm_launch_status();
 }
 

@@ -14,6 +14,11 @@
 
 #define ILLM_WAVE 64
 
+// norms of a row (post_norm.hip)
+#define ILLM_NORM_NONE 0
+#define ILLM_NORM_RMS 1
+#define ILLM_NORM_LAYER 2
+
 typedef uint16_t bf16_t;
 
 __device__ __forceinline__ float bf16_to_f32(bf16_t v) {
@@ -42,6 +47,27 @@ __device__ __forceinline__ float ld_f(const void* p, int dt, size_t i) {
 __device__ __forceinline__ void st_f(void* p, int dt, size_t i, float v) {
     if (dt == ILLM_BF16) ((bf16_t*)p)[i] = f32_to_bf16(v);
     else ((float*)p)[i] = v;
+}
+
+// four neighbouring elements (number 4 i4 .. 4 i4 + 3) as float32, and back
+__device__ __forceinline__ float4 ld_f4(const void* p, int dt, size_t i4) {
+    if (dt == ILLM_BF16) {
+        const uint2 u = ((const uint2*)p)[i4];
+        return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u),
+                           __uint_as_float(u.y << 16), __uint_as_float(u.y & 0xffff0000u));
+    }
+    return ((const float4*)p)[i4];
+}
+
+__device__ __forceinline__ void st_f4(void* p, int dt, size_t i4, float4 v) {
+    if (dt == ILLM_BF16) {
+        uint2 u;
+        u.x = pack_bf16x2(v.x, v.y);
+        u.y = pack_bf16x2(v.z, v.w);
+        ((uint2*)p)[i4] = u;
+    } else {
+        ((float4*)p)[i4] = v;
+    }
 }
 
 typedef uint32_t illm_u32x4_t __attribute__((ext_vector_type(4)));
@@ -105,13 +131,13 @@ static inline int illm_launch_status() {
 static inline bool illm_dtype_ok(int dt) { return dt == ILLM_F32 || dt == ILLM_BF16; }
 
 // Where position `pos` of the sequence in `slot` lies in a paged cache line laid
-// out as [page][kv head][row in page][head_dim].  `ring` > 0: only the last
-// `ring` logical pages of a sequence are kept (a window).
+// out as [page][kv head][row in page][head_dim].  `ring` > 0: the first `kept` logical pages of
+// a sequence stay and of the later ones only the last `ring` are kept (a window).
 __device__ __forceinline__ size_t cache_row_offset(const int32_t* page_table, int table_stride,
                                                    int slot, int pos, int page_size, int ring,
-                                                   int nkv, int kvh, int hd) {
+                                                   int nkv, int kvh, int hd, int kept = 0) {
     int lp = pos / page_size;
-    if (ring > 0) lp %= ring;
+    if (ring > 0 && lp >= kept) lp = kept + (lp - kept) % ring;
     const int phys = page_table[(size_t)slot * table_stride + lp];
     return (((size_t)phys * nkv + kvh) * page_size + (pos % page_size)) * (size_t)hd;
 }

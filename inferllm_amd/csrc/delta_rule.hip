@@ -12,7 +12,10 @@
 // The scan also runs the plain gated rule without the correction (`correct` 0),
 //     S <- diag(g) S + k (beta v)^T;   o = S^T q
 // which is the recurrence of state-space and matrix-memory mixers (linear_scan.hip prepares their
-// inputs): beta is then the weight of the token's outer product.
+// inputs): beta is then the weight of the token's outer product.  And it runs the delta rule with a
+// removal vector of its own (`removal` given, c = a u with a rate a per channel),
+//     S <- diag(g) S - c (u^T S) + k v^T,  u = beta k;   o = S^T q
+// where both terms read the old state; beta is then 1 / |k|.
 // Everything but the stored projections is float32.  A sequence's rows in a step are consecutive;
 // a step may go on from any state (single tokens, portions of a prompt) or start from the zeros a
 // fresh slot holds.  Sums run in an order fixed by the sizes alone.
@@ -199,17 +202,23 @@ __device__ __forceinline__ float group_sum(float v) {
     return v;
 }
 
+// the rules of the scan: which one a kernel runs (see the head of the file)
+#define RULE_PLAIN 0
+#define RULE_DELTA 1
+#define RULE_REMOVAL 2
+
 // Steps of few tokens a sequence (single tokens above all): what counts is the state's bytes.
 // grid (ceil(dv / 64), H, sequences); 4 waves: a lane is a column, wave w holds rows [w NS, w NS + NS)
 // of it, so a row of S is read and written 256 bytes a wave; k, q and the decays of a row are the
 // same for a whole wave.  The waves' partial sums meet in LDS, in wave order.
-template <int NS, bool CORRECT>
+template <int NS, int RULE>
 __global__ void __launch_bounds__(256)
 delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
                   const float* __restrict__ vv, const float* __restrict__ beta,
                   const float* __restrict__ dec, int DW, float* __restrict__ state,
                   const int32_t* __restrict__ cu, const int32_t* __restrict__ seq_slot,
-                  float* __restrict__ o, int G, int H, int dk, int dv) {
+                  float* __restrict__ o, int G, int H, int dk, int dv, const float* __restrict__ removal) {
+    constexpr bool CORRECT = RULE != RULE_PLAIN;
     __shared__ float red[2][4][64];
     const int b = blockIdx.z, h = blockIdx.y, lane = threadIdx.x & 63, w = wave_index();
     const int col = blockIdx.x * 64 + lane;
@@ -231,7 +240,7 @@ delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
         for (int ii = 0; ii < NS; ++ii) {
             const int i = i0 + ii;
             kc[ii] = i < dk ? kp[i] : 0.f;
-            s[ii] *= i < dk ? (DW == 1 ? dp[0] : dp[i]) : 1.f;
+            if (RULE != RULE_REMOVAL) s[ii] *= i < dk ? (DW == 1 ? dp[0] : dp[i]) : 1.f;
             pa[ii & 3] = fmaf(s[ii], kc[ii], pa[ii & 3]);
         }
         float kv = 0.f;
@@ -241,11 +250,15 @@ delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
             kv = (red[0][0][lane] + red[0][1][lane]) + (red[0][2][lane] + red[0][3][lane]);
         }
         const float v = live ? vv[((size_t)row * H + h) * dv + col] : 0.f;
-        const float u = beta[(size_t)row * H + h] * (v - kv);
+        const float bt = beta[(size_t)row * H + h];
+        const float u = RULE == RULE_REMOVAL ? v : bt * (v - kv);
+        const float read = bt * kv;                     // (the old state under the unit key)
+        const float* cp = RULE == RULE_REMOVAL ? removal + ((size_t)row * H + h) * dk : nullptr;
         pa[0] = pa[1] = pa[2] = pa[3] = 0.f;
 #pragma unroll
         for (int ii = 0; ii < NS; ++ii) {
             const int i = i0 + ii;
+            if (RULE == RULE_REMOVAL && i < dk) s[ii] = fmaf(-cp[i], read, s[ii] * (DW == 1 ? dp[0] : dp[i]));
             s[ii] = fmaf(kc[ii], u, s[ii]);
             pa[ii & 3] = fmaf(s[ii], i < dk ? qp[i] : 0.f, pa[ii & 3]);
         }
@@ -266,20 +279,22 @@ delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
 // dependent operations a token, so nothing may wait for memory inside it: the k, q and decay rows of
 // DELTA_CHUNK tokens go through LDS in two buffers, the next chunk's loads (and its v and beta, in
 // registers) are issued before this chunk's arithmetic and stored after it.  One wave a block;
-// dynamic LDS: 2 * DELTA_CHUNK * 3 * 16 NS floats.
+// dynamic LDS: 2 * DELTA_CHUNK * 3 * 16 NS floats (with a removal vector 4 in place of 3).
 #define DELTA_CHUNK 8
-template <int NS, bool CORRECT>
+template <int NS, int RULE>
 __global__ void __launch_bounds__(64)
 delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
                        const float* __restrict__ vv, const float* __restrict__ beta,
                        const float* __restrict__ dec, int DW, float* __restrict__ state,
                        const int32_t* __restrict__ cu, const int32_t* __restrict__ seq_slot,
-                       float* __restrict__ o, int G, int H, int dk, int dv) {
+                       float* __restrict__ o, int G, int H, int dk, int dv, const float* __restrict__ removal) {
+    constexpr bool CORRECT = RULE != RULE_PLAIN;
+    constexpr int NVEC = RULE == RULE_REMOVAL ? 4 : 3;  // rows a token in LDS
     constexpr int PARTS = 16, COLS = 4, TC = DELTA_CHUNK;
     constexpr int DKP = PARTS * NS;                     // a row of k, q or decays in LDS, filled up
     constexpr int JJ = (DKP + 63) / 64;                 // pieces of 64 floats in it
     constexpr int NA = NS >= 4 ? 4 : NS;
-    extern __shared__ float stage[];                    // [2][TC][k | q | decay][DKP]
+    extern __shared__ float stage[];                    // [2][TC][k | q | decay | removal?][DKP]
     const int b = blockIdx.z, h = blockIdx.y, lane = threadIdx.x;
     const int part = lane % PARTS, col = blockIdx.x * COLS + lane / PARTS;
     const int r0 = cu[b], n = cu[b + 1] - r0;
@@ -296,9 +311,12 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
     const float* dbase = dec + ((size_t)r0 * H + h) * DW;
     const float* vbase = vv + ((size_t)r0 * H + h) * dv + (live ? col : 0);
     const float* bbase = beta + (size_t)r0 * H + h;
+    const float* cbase = RULE == RULE_REMOVAL ? removal + ((size_t)r0 * H + h) * dk : nullptr;
+    const int cstep = H * dk;
     float* op = o + ((size_t)r0 * H + h) * dv + col;
     const int kstep = G * dk, dstep = H * DW, vstep = H * dv;
     float sk[TC][JJ], sq[TC][JJ], sg[TC][JJ], sv[TC], sb[TC];
+    float sr[TC][RULE == RULE_REMOVAL ? JJ : 1];
     // Rows beyond dk are filled with k = q = 0 and decay 1, and the tokens of the last chunk beyond
     // the sequence with k = q = v = beta = 0 and decay 1, which leave the state as it is: the
     // arithmetic needs no bounds and no branches.  A whole chunk is loaded through pointers that
@@ -314,6 +332,7 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
         const float* dp = dbase + (size_t)(T0) * dstep;                                           \
         const float* vp = vbase + (size_t)(T0) * vstep;                                           \
         const float* bp = bbase + (size_t)(T0) * H;                                               \
+        const float* cp = cbase + (RULE == RULE_REMOVAL ? (size_t)(T0) * cstep : 0);              \
         _Pragma("unroll") for (int tt = 0; tt < TC; ++tt) {                                       \
             _Pragma("unroll") for (int jj = 0; jj < JJ; ++jj) {                                   \
                 const int j = in_k[jj] ? lane + 64 * jj : jlast;      /* read in bounds, then choose */ \
@@ -321,10 +340,12 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
                 sk[tt][jj] = in_k[jj] ? kx : 0.f;                                                 \
                 sq[tt][jj] = in_k[jj] ? qx : 0.f;                                                 \
                 sg[tt][jj] = in_k[jj] ? gx : 1.f;                                                 \
+                if (RULE == RULE_REMOVAL) { const float cx = cp[j]; sr[tt][jj] = in_k[jj] ? cx : 0.f; } \
             }                                                                                     \
             sv[tt] = *vp;                                                                         \
             sb[tt] = *bp;                                                                         \
             kp += kstep; qp += kstep; dp += dstep; vp += vstep; bp += H;                          \
+            if (RULE == RULE_REMOVAL) cp += cstep;                                                \
         }                                                                                         \
     } else {                                                                                      \
         _Pragma("unroll") for (int tt = 0; tt < TC; ++tt) {                                       \
@@ -336,6 +357,7 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
                 sk[tt][jj] = use ? kbase[(size_t)at * kstep + j] : 0.f;                           \
                 sq[tt][jj] = use ? qbase[(size_t)at * kstep + j] : 0.f;                           \
                 sg[tt][jj] = use ? dbase[(size_t)at * dstep + (DW == 1 ? 0 : j)] : 1.f;           \
+                if (RULE == RULE_REMOVAL) sr[tt][jj] = use ? cbase[(size_t)at * cstep + j] : 0.f; \
             }                                                                                     \
             sv[tt] = ok ? vbase[(size_t)at * vstep] : 0.f;                                        \
             sb[tt] = ok ? bbase[(size_t)at * H] : 0.f;                                            \
@@ -343,10 +365,13 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
     }
 #define DELTA_STORE(BUF)                                                                          \
     _Pragma("unroll") for (int tt = 0; tt < TC; ++tt) {                                           \
-        float* dst = stage + ((size_t)(BUF) * TC + tt) * 3 * DKP;                                 \
+        float* dst = stage + ((size_t)(BUF) * TC + tt) * NVEC * DKP;                              \
         _Pragma("unroll") for (int jj = 0; jj < JJ; ++jj) {                                       \
             const int j = lane + 64 * jj;                                                         \
-            if (j < DKP) { dst[j] = sk[tt][jj]; dst[DKP + j] = sq[tt][jj]; dst[2 * DKP + j] = sg[tt][jj]; } \
+            if (j < DKP) {                                                                        \
+                dst[j] = sk[tt][jj]; dst[DKP + j] = sq[tt][jj]; dst[2 * DKP + j] = sg[tt][jj];    \
+                if (RULE == RULE_REMOVAL) dst[3 * DKP + j] = sr[tt][jj];                          \
+            }                                                                                     \
         }                                                                                         \
     }
     DELTA_LOAD(0)
@@ -359,18 +384,18 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
         for (int tt = 0; tt < TC; ++tt) { cv[tt] = sv[tt]; cb[tt] = sb[tt]; }
         const bool more = t0 + TC < n;
         if (more) { DELTA_LOAD(t0 + TC) }
-        const float* src0 = stage + (size_t)buf * TC * 3 * DKP + part;
+        const float* src0 = stage + (size_t)buf * TC * NVEC * DKP + part;
         float ovs[TC];
 #pragma unroll
         for (int tt = 0; tt < TC; ++tt) {
-            const float* src = src0 + tt * 3 * DKP;
+            const float* src = src0 + tt * NVEC * DKP;
             float kc[NS], pa[NA];
 #pragma unroll
             for (int a = 0; a < NA; ++a) pa[a] = 0.f;
 #pragma unroll
             for (int ii = 0; ii < NS; ++ii) {
                 kc[ii] = src[PARTS * ii];
-                s[ii] *= src[2 * DKP + PARTS * ii];
+                if (RULE != RULE_REMOVAL) s[ii] *= src[2 * DKP + PARTS * ii];
                 pa[ii % NA] = fmaf(s[ii], kc[ii], pa[ii % NA]);
             }
             float kv = 0.f;
@@ -380,12 +405,18 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
                 for (int a = 1; a < NA; ++a) kv += pa[a];
                 kv = group_sum<PARTS>(kv);
             }
-            const float u = cb[tt] * (cv[tt] - kv);
+            const float u = RULE == RULE_REMOVAL ? cv[tt] : cb[tt] * (cv[tt] - kv);
+            const float read = cb[tt] * kv;
 #pragma unroll
             for (int a = 0; a < NA; ++a) pa[a] = 0.f;
 #pragma unroll
             for (int ii = 0; ii < NS; ++ii) {
-                s[ii] = fmaf(kc[ii], u, s[ii]);
+                if (RULE == RULE_REMOVAL) {
+                    // (all but the last operation is off the chain that hangs on `read`)
+                    const float kept = fmaf(kc[ii], u, s[ii] * src[2 * DKP + PARTS * ii]);
+                    s[ii] = fmaf(-src[3 * DKP + PARTS * ii], read, kept);
+                } else
+                    s[ii] = fmaf(kc[ii], u, s[ii]);
                 pa[ii % NA] = fmaf(s[ii], src[DKP + PARTS * ii], pa[ii % NA]);
             }
             float ov = pa[0];
@@ -415,7 +446,8 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
 extern "C" int illm_gated_scan(const float* qn, const float* kn, const float* vv, const float* beta,
                                const float* dec, int DW, float* state, const int32_t* cu,
                                const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int G,
-                               int H, int dk, int dv, int correct, void* stream) {
+                               int H, int dk, int dv, int correct, const float* removal, void* stream) {
+    if (removal && (correct || G != H)) return ILLM_ERR_ARG;
     if (n_seqs < 0 || G <= 0 || H <= 0 || H % G || dk <= 0 || dk > 256 || dv <= 0 ||
         (DW != 1 && DW != dk) || H > 65535 || n_seqs > 65535)
         return ILLM_ERR_ARG;
@@ -423,37 +455,45 @@ extern "C" int illm_gated_scan(const float* qn, const float* kn, const float* vv
     hipStream_t st = (hipStream_t)stream;
     if (max_rows >= 16) {
         const int ns = (dk + 15) / 16;
-        const size_t lds = (size_t)2 * DELTA_CHUNK * 3 * 16 * (ns <= 1 ? 1 : ns <= 2 ? 2 : ns <= 4 ? 4 : ns <= 8 ? 8 : 16) * sizeof(float);
+        const size_t lds = (size_t)2 * DELTA_CHUNK * (removal ? 4 : 3) * 16 * (ns <= 1 ? 1 : ns <= 2 ? 2 : ns <= 4 ? 4 : ns <= 8 ? 8 : 16) * sizeof(float);
         const dim3 grid((dv + 3) / 4, H, n_seqs);
+#define GOL_R(NS_, RULE_)                                                                         \
+    do {                                                                                          \
+        if (lds > 48 * 1024 &&                                                                    \
+            hipFuncSetAttribute((const void*)delta_scan_long_kernel<NS_, RULE_>,                  \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
+            return ILLM_ERR_LAUNCH;                                                               \
+        hipLaunchKernelGGL((delta_scan_long_kernel<NS_, RULE_>), grid, dim3(64), lds, st, qn, kn, vv, beta, \
+                           dec, DW, state, cu, seq_slot, o, G, H, dk, dv, removal);               \
+    } while (0)
 #define GOL(NS_)                                                                                  \
-    if (correct)                                                                                  \
-        hipLaunchKernelGGL((delta_scan_long_kernel<NS_, true>), grid, dim3(64), lds, st, qn, kn, vv, beta, \
-                           dec, DW, state, cu, seq_slot, o, G, H, dk, dv);                        \
-    else                                                                                          \
-        hipLaunchKernelGGL((delta_scan_long_kernel<NS_, false>), grid, dim3(64), lds, st, qn, kn, vv, beta, \
-                           dec, DW, state, cu, seq_slot, o, G, H, dk, dv)
+    if (removal) GOL_R(NS_, RULE_REMOVAL);                                                        \
+    else if (correct) GOL_R(NS_, RULE_DELTA);                                                     \
+    else GOL_R(NS_, RULE_PLAIN)
         if (ns <= 1) { GOL(1); }
         else if (ns <= 2) { GOL(2); }
         else if (ns <= 4) { GOL(4); }
         else if (ns <= 8) { GOL(8); }
         else { GOL(16); }
 #undef GOL
+#undef GOL_R
     } else {
         const int ns = (dk + 3) / 4;
         const dim3 grid((dv + 63) / 64, H, n_seqs);
+#define GOS_R(NS_, RULE_)                                                                         \
+    hipLaunchKernelGGL((delta_step_kernel<NS_, RULE_>), grid, dim3(256), 0, st, qn, kn, vv, beta, dec, DW, \
+                       state, cu, seq_slot, o, G, H, dk, dv, removal)
 #define GOS(NS_)                                                                                  \
-    if (correct)                                                                                  \
-        hipLaunchKernelGGL((delta_step_kernel<NS_, true>), grid, dim3(256), 0, st, qn, kn, vv, beta, dec, \
-                           DW, state, cu, seq_slot, o, G, H, dk, dv);                             \
-    else                                                                                          \
-        hipLaunchKernelGGL((delta_step_kernel<NS_, false>), grid, dim3(256), 0, st, qn, kn, vv, beta, dec, \
-                           DW, state, cu, seq_slot, o, G, H, dk, dv)
+    if (removal) GOS_R(NS_, RULE_REMOVAL);                                                        \
+    else if (correct) GOS_R(NS_, RULE_DELTA);                                                     \
+    else GOS_R(NS_, RULE_PLAIN)
         if (ns <= 4) { GOS(4); }
         else if (ns <= 8) { GOS(8); }
         else if (ns <= 16) { GOS(16); }
         else if (ns <= 32) { GOS(32); }
         else { GOS(64); }
 #undef GOS
+#undef GOS_R
     }
     return illm_launch_status();
 }
@@ -463,7 +503,7 @@ extern "C" int illm_delta_scan(const float* qn, const float* kn, const float* vv
                                const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int G,
                                int H, int dk, int dv, void* stream) {
     return illm_gated_scan(qn, kn, vv, beta, dec, DW, state, cu, seq_slot, o, n_seqs, max_rows, G, H, dk,
-                           dv, 1, stream);
+                           dv, 1, nullptr, stream);
 }
 
 // grid (rows, H); one wave: out[r, h dv + j] = o / sqrt(mean_j o^2 + eps) * w[j] * act(z[r, h dv + j]),

@@ -149,14 +149,6 @@ __global__ void relu_squared_kernel(const void* __restrict__ x, void* __restrict
     st_f(out, dt, i, v * v);
 }
 
-extern "C" int illm_relu_squared(const void* x, void* out, int dt, size_t n, void* stream) {
-    if (!illm_dtype_ok(dt)) return ILLM_ERR_ARG;
-    if (n == 0) return ILLM_OK;
-    hipLaunchKernelGGL(relu_squared_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0,
-                       (hipStream_t)stream, x, out, dt, n);
-    return illm_launch_status();
-}
-
 // 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), the tanh form of GELU.
 __global__ void gelu_tanh_kernel(const void* __restrict__ x, void* __restrict__ out, int dt, size_t n) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -193,6 +185,64 @@ extern "C" int illm_gelu_tanh(const void* x, void* out, int dt, size_t n, void* 
     }
     hipLaunchKernelGGL(gelu_tanh_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0,
                        (hipStream_t)stream, x, out, dt, n);
+    return illm_launch_status();
+}
+
+// xIELU with two numbers on the device, par = (cp, cn): z > 0: cp z^2 + z / 2; z <= 0: cn (e^z - 1 - z) + z / 2.
+__device__ __forceinline__ float xielu_f(float z, float cp, float cn) {
+    return (z > 0.f ? cp * z * z : cn * (expm1f(z) - z)) + 0.5f * z;
+}
+
+__global__ void xielu_kernel(const void* __restrict__ x, const float* __restrict__ par, void* __restrict__ out,
+                             int dt, size_t n) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) st_f(out, dt, i, xielu_f(ld_f(x, dt, i), par[0], par[1]));
+}
+
+// bfloat16 with n % 8 == 0: 8 values (16 bytes) a thread; ACT 0: max(z, 0)^2, 1: xIELU
+template <int ACT>
+__global__ void __launch_bounds__(256)
+act_bf16x8_kernel(const bf16_t* __restrict__ x, const float* __restrict__ par, bf16_t* __restrict__ out, size_t n8) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n8) return;
+    const float cp = ACT ? par[0] : 0.f, cn = ACT ? par[1] : 0.f;
+    auto act = [&](float z) {
+        if (ACT) return xielu_f(z, cp, cn);
+        z = fmaxf(z, 0.f);
+        return z * z;
+    };
+    const uint4 v = ((const uint4*)x)[i];
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+    uint32_t o[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k)
+        o[k] = pack_bf16x2(act(__uint_as_float(w[k] << 16)), act(__uint_as_float(w[k] & 0xffff0000u)));
+    ((uint4*)out)[i] = make_uint4(o[0], o[1], o[2], o[3]);
+}
+
+extern "C" int illm_xielu(const void* x, const float* par, void* out, int dt, size_t n, void* stream) {
+    if (!illm_dtype_ok(dt) || !par) return ILLM_ERR_ARG;
+    if (n == 0) return ILLM_OK;
+    if (dt == ILLM_BF16 && n % 8 == 0 && n / 8 / 256 < 0x7fffffffu) {
+        hipLaunchKernelGGL(act_bf16x8_kernel<1>, dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0,
+                           (hipStream_t)stream, (const bf16_t*)x, par, (bf16_t*)out, n / 8);
+        return illm_launch_status();
+    }
+    hipLaunchKernelGGL(xielu_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, (hipStream_t)stream, x,
+                       par, out, dt, n);
+    return illm_launch_status();
+}
+
+extern "C" int illm_relu_squared(const void* x, void* out, int dt, size_t n, void* stream) {
+    if (!illm_dtype_ok(dt)) return ILLM_ERR_ARG;
+    if (n == 0) return ILLM_OK;
+    if (dt == ILLM_BF16 && n % 8 == 0 && n / 8 / 256 < 0x7fffffffu) {
+        hipLaunchKernelGGL(act_bf16x8_kernel<0>, dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0,
+                           (hipStream_t)stream, (const bf16_t*)x, (const float*)nullptr, (bf16_t*)out, n / 8);
+        return illm_launch_status();
+    }
+    hipLaunchKernelGGL(relu_squared_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, (hipStream_t)stream,
+                       x, out, dt, n);
     return illm_launch_status();
 }
 

@@ -1,0 +1,568 @@
+// Two linear mixers with a matrix of state S [key dim, value dim] (float32) per head and no convolution:
+//
+// Lightning attention, one fixed decay lam a head: q, k, v through SiLU,
+//     S <- lam S + k v^T;   o = S^T q
+//   lightning_prepare   the inputs of illm_gated_scan as float32 (any number of rows)
+//   lightning_step      single tokens: SiLU, the state's update and o in one launch
+//   lightning_chunks    long steps, chunks of FD_CHUNK tokens in parallel (three launches, see below)
+//
+// The delta rule with a removal vector, one decay w and one rate a per key channel, u = k / |k|:
+//     w = exp(-rate sigmoid(z + w0)),  a = sigmoid(y + a_bias),   S <- diag(w) S - (a u)(u^T S) + k v^T;   o = S^T r
+//   removal_prepare     the inputs of illm_gated_scan (with `removal`) as float32
+//   removal_step        single tokens in one launch, z = W2 tanh(y1) of the low-rank map included
+//
+// Behind either: group_norm_gate, o RMS-normed in equal parts of the row, a weight of the row's width, a
+// gate.  Everything but the stored projections is float32.  A sequence's rows in a step are consecutive.
+#include <math.h>
+
+#include "api.h"
+#include "common.h"
+
+__device__ __forceinline__ float fd_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
+__device__ __forceinline__ float fd_silu(float x) { return x / (1.0f + expf(-x)); }
+
+// ---------------------------------------------------------------- inputs of the scan
+// grid (rows); 256 threads.  U [T, u_stride]: q at q_off and k at k_off (H dk), v at v_off (H dv).
+__global__ void __launch_bounds__(256)
+lightning_prepare_kernel(const void* __restrict__ U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                         const float* __restrict__ decay, float* __restrict__ qn, float* __restrict__ kn,
+                         float* __restrict__ vv, float* __restrict__ beta, float* __restrict__ dec, int H,
+                         int dk, int dv) {
+    const size_t t = blockIdx.x, u0 = t * u_stride;
+    for (int e = threadIdx.x; e < H * dk; e += 256) {
+        qn[t * H * dk + e] = fd_silu(ld_f(U, dt, u0 + q_off + e));
+        kn[t * H * dk + e] = fd_silu(ld_f(U, dt, u0 + k_off + e));
+    }
+    for (int e = threadIdx.x; e < H * dv; e += 256) vv[t * H * dv + e] = fd_silu(ld_f(U, dt, u0 + v_off + e));
+    for (int e = threadIdx.x; e < H; e += 256) { beta[t * H + e] = 1.0f; dec[t * H + e] = decay[e]; }
+}
+
+static bool fd_columns_ok(int u_stride, int off, int n) { return off >= 0 && off + n <= u_stride; }
+
+extern "C" int illm_lightning_prepare(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                                      const float* decay, float* qn, float* kn, float* vv, float* beta,
+                                      float* dec, int T, int H, int dk, int dv, void* stream) {
+    if (T < 0 || H <= 0 || dk <= 0 || dv <= 0 || !illm_dtype_ok(dt) || !fd_columns_ok(u_stride, q_off, H * dk) ||
+        !fd_columns_ok(u_stride, k_off, H * dk) || !fd_columns_ok(u_stride, v_off, H * dv))
+        return ILLM_ERR_ARG;
+    if (T == 0) return ILLM_OK;
+    hipLaunchKernelGGL(lightning_prepare_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, U, dt, u_stride,
+                       q_off, k_off, v_off, decay, qn, kn, vv, beta, dec, H, dk, dv);
+    return illm_launch_status();
+}
+
+// grid (rows, ceil(H / 4)); a wave takes a head, lanes over its d channels (d <= 256).  U: r, k, v at
+// r_off, k_off, v_off and the rates' pre-activations at a_off, all H d wide; Z [T, z_stride] (H d wide).
+#define FD_VEC 4
+__global__ void __launch_bounds__(256)
+removal_prepare_kernel(const void* __restrict__ U, int dt, int u_stride, int r_off, int k_off, int v_off,
+                       int a_off, const float* __restrict__ a_bias, const void* __restrict__ Z, int z_dt,
+                       int z_stride, const float* __restrict__ w0, float rate, float* __restrict__ qn,
+                       float* __restrict__ kn, float* __restrict__ vv, float* __restrict__ beta,
+                       float* __restrict__ dec, float* __restrict__ removal, int H, int d) {
+    const size_t t = blockIdx.x, u0 = t * u_stride;
+    const int h = blockIdx.y * 4 + wave_index(), lane = threadIdx.x & 63;
+    if (h >= H) return;
+    float k[FD_VEC], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < FD_VEC; ++e) {
+        const int i = lane + 64 * e;
+        k[e] = i < d ? ld_f(U, dt, u0 + k_off + h * d + i) : 0.f;
+        ss = fmaf(k[e], k[e], ss);
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) + 1e-6f);
+    if (lane == 0) beta[t * H + h] = inv;
+#pragma unroll
+    for (int e = 0; e < FD_VEC; ++e) {
+        const int i = lane + 64 * e, c = h * d + i;
+        if (i >= d) continue;
+        const size_t at = t * H * d + c;
+        qn[at] = ld_f(U, dt, u0 + r_off + c);
+        kn[at] = k[e];
+        vv[at] = ld_f(U, dt, u0 + v_off + c);
+        dec[at] = expf(-rate * fd_sigmoid(ld_f(Z, z_dt, t * z_stride + c) + w0[c]));
+        removal[at] = fd_sigmoid(ld_f(U, dt, u0 + a_off + c) + a_bias[c]) * (k[e] * inv);
+    }
+}
+
+extern "C" int illm_removal_prepare(const void* U, int dt, int u_stride, int r_off, int k_off, int v_off,
+                                    int a_off, const float* a_bias, const void* Z, int z_dt, int z_stride,
+                                    const float* w0, float rate, float* qn, float* kn, float* vv, float* beta,
+                                    float* dec, float* removal, int T, int H, int d, void* stream) {
+    if (T < 0 || H <= 0 || d <= 0 || d > 64 * FD_VEC || !illm_dtype_ok(dt) || !illm_dtype_ok(z_dt) ||
+        z_stride < H * d || !fd_columns_ok(u_stride, r_off, H * d) || !fd_columns_ok(u_stride, k_off, H * d) ||
+        !fd_columns_ok(u_stride, v_off, H * d) || !fd_columns_ok(u_stride, a_off, H * d) || (H + 3) / 4 > 65535)
+        return ILLM_ERR_ARG;
+    if (T == 0) return ILLM_OK;
+    hipLaunchKernelGGL(removal_prepare_kernel, dim3(T, (H + 3) / 4), dim3(256), 0, (hipStream_t)stream, U, dt,
+                       u_stride, r_off, k_off, v_off, a_off, a_bias, Z, z_dt, z_stride, w0, rate, qn, kn, vv,
+                       beta, dec, removal, H, d);
+    return illm_launch_status();
+}
+
+// out[t, i] = tanh(U[t, off + i]), i < n.
+__global__ void __launch_bounds__(256)
+tanh_columns_kernel(const void* __restrict__ U, int dt, int u_stride, int off, void* __restrict__ out, int n) {
+    const size_t t = blockIdx.x;
+    for (int i = threadIdx.x; i < n; i += 256) st_f(out, dt, t * n + i, tanhf(ld_f(U, dt, t * u_stride + off + i)));
+}
+
+extern "C" int illm_tanh_columns(const void* U, int dt, int u_stride, int off, void* out, int T, int n,
+                                 void* stream) {
+    if (T < 0 || n <= 0 || !illm_dtype_ok(dt) || !fd_columns_ok(u_stride, off, n)) return ILLM_ERR_ARG;
+    if (T == 0) return ILLM_OK;
+    hipLaunchKernelGGL(tanh_columns_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, U, dt, u_stride, off, out, n);
+    return illm_launch_status();
+}
+
+// ---------------------------------------------------------------- single tokens
+// grid (ceil(dv / 64), H, rows); 4 waves: a lane is a column of the state, wave w holds rows [w NS, w NS +
+// NS) of it (NS >= ceil(dk / 4)).  Row b belongs to the sequence in slot row_slot[b].  The head's vectors
+// (k, q and, with a removal vector, the decays and the vector) are formed by the block into LDS while the
+// state's rows are on their way; the waves' partial sums meet in LDS, in wave order.
+#define FD_RANK_MAX 512
+struct RemovalArgs {
+    const float* a_bias;      // [H d]
+    const void* w2;           // [H d, rank], the projections' type
+    const float* w0;          // [H d]
+    int a_off, w1_off, rank;
+    float rate;
+};
+
+template <int NS, int DT, bool REMOVAL>
+__global__ void __launch_bounds__(256)
+fixed_step_kernel(const void* __restrict__ U, int u_stride, int q_off, int k_off, int v_off,
+                  const float* __restrict__ decay, RemovalArgs ra, float* __restrict__ state,
+                  const int32_t* __restrict__ row_slot, float* __restrict__ o, int H, int dk, int dv) {
+    __shared__ float sk[4 * NS], sq[4 * NS], sw[REMOVAL ? 4 * NS : 1], sc[REMOVAL ? 4 * NS : 1];
+    __shared__ float low[REMOVAL ? FD_RANK_MAX : 1];
+    __shared__ float part[REMOVAL ? 256 : 1];
+    __shared__ float red[2][4][64];
+    __shared__ float redb[16];
+    const int b = blockIdx.z, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = wave_index();
+    const int col = blockIdx.x * 64 + lane, i0 = w * NS;
+    const bool live = col < dv;
+    const size_t u0 = (size_t)b * u_stride;
+    float* sp = state + (((size_t)row_slot[b] * H + h) * dk) * dv + col;
+    float s[NS];
+#pragma unroll
+    for (int ii = 0; ii < NS; ++ii) s[ii] = (live && i0 + ii < dk) ? sp[(size_t)(i0 + ii) * dv] : 0.f;
+    float v = live ? ld_f(U, DT, u0 + v_off + (size_t)h * dv + col) : 0.f;
+    if (!REMOVAL) v = fd_silu(v);
+    const int i = tid;                                  // a thread a channel (dk <= 256)
+    const bool mine = i < dk;
+    float k = mine ? ld_f(U, DT, u0 + k_off + (size_t)h * dk + i) : 0.f;
+    float q = mine ? ld_f(U, DT, u0 + q_off + (size_t)h * dk + i) : 0.f;
+    float inv = 1.f;
+    if (REMOVAL) {
+        for (int r = tid; r < ra.rank; r += 256) low[r] = tanhf(ld_f(U, DT, u0 + ra.w1_off + r));
+        inv = 1.0f / sqrtf(block_sum(k * k, redb) + 1e-6f);      // (its barriers also publish `low`)
+        // z of the head's channels: 256 / DKP threads a channel, each a share of the rank
+        constexpr int DKP = 4 * NS, SH = 256 / DKP;
+        const int zi = tid % DKP, sh = tid / DKP;
+        float z = 0.f;
+        if (zi < dk) {
+            const size_t w2 = ((size_t)h * dk + zi) * ra.rank;
+            const int per = (ra.rank + SH - 1) / SH, r1 = min(ra.rank, (sh + 1) * per);
+#pragma unroll 8
+            for (int r = sh * per; r < r1; ++r) z = fmaf(ld_f(ra.w2, DT, w2 + r), low[r], z);
+        }
+        part[tid] = z;
+        __syncthreads();
+        if (mine) {
+            z = ra.w0[h * dk + i];
+#pragma unroll
+            for (int x = 0; x < SH; ++x) z += part[x * DKP + i];
+            sw[i] = expf(-ra.rate * fd_sigmoid(z));
+            sc[i] = fd_sigmoid(ld_f(U, DT, u0 + ra.a_off + (size_t)h * dk + i) + ra.a_bias[h * dk + i]) * (k * inv);
+        } else if (i < DKP) {
+            sw[i] = 1.f; sc[i] = 0.f;
+        }
+    } else {
+        k = fd_silu(k); q = fd_silu(q);
+    }
+    if (i < 4 * NS) { sk[i] = mine ? k : 0.f; sq[i] = mine ? q : 0.f; }
+    __syncthreads();
+    float pa[4] = {0.f, 0.f, 0.f, 0.f};
+    float read = 0.f;
+    if (REMOVAL) {
+#pragma unroll
+        for (int ii = 0; ii < NS; ++ii) pa[ii & 3] = fmaf(s[ii], sk[i0 + ii], pa[ii & 3]);
+        red[0][w][lane] = (pa[0] + pa[1]) + (pa[2] + pa[3]);
+        __syncthreads();
+        read = inv * ((red[0][0][lane] + red[0][1][lane]) + (red[0][2][lane] + red[0][3][lane]));
+        pa[0] = pa[1] = pa[2] = pa[3] = 0.f;
+    }
+    const float lam = REMOVAL ? 1.f : decay[h];
+#pragma unroll
+    for (int ii = 0; ii < NS; ++ii) {
+        if (REMOVAL) s[ii] = fmaf(-sc[i0 + ii], read, s[ii] * sw[i0 + ii]);
+        else s[ii] *= lam;
+        s[ii] = fmaf(sk[i0 + ii], v, s[ii]);
+        pa[ii & 3] = fmaf(s[ii], sq[i0 + ii], pa[ii & 3]);
+    }
+    red[1][w][lane] = (pa[0] + pa[1]) + (pa[2] + pa[3]);
+#pragma unroll
+    for (int ii = 0; ii < NS; ++ii)
+        if (live && i0 + ii < dk) sp[(size_t)(i0 + ii) * dv] = s[ii];
+    __syncthreads();
+    if (w == 0 && live)
+        o[((size_t)b * H + h) * dv + col] = (red[1][0][lane] + red[1][1][lane]) + (red[1][2][lane] + red[1][3][lane]);
+}
+
+static int fixed_step_launch(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                             const float* decay, RemovalArgs ra, bool removal, float* state,
+                             const int32_t* row_slot, float* o, int B, int H, int dk, int dv, hipStream_t st) {
+    const dim3 grid((dv + 63) / 64, H, B);
+    const int ns = (dk + 3) / 4;
+#define GO(NS_, DT_, R_)                                                                                \
+    hipLaunchKernelGGL((fixed_step_kernel<NS_, DT_, R_>), grid, dim3(256), 0, st, U, u_stride, q_off, k_off, \
+                       v_off, decay, ra, state, row_slot, o, H, dk, dv)
+#define GO_D(NS_)                                                                                       \
+    if (dt == ILLM_BF16) { if (removal) GO(NS_, ILLM_BF16, true); else GO(NS_, ILLM_BF16, false); }     \
+    else { if (removal) GO(NS_, ILLM_F32, true); else GO(NS_, ILLM_F32, false); }
+    if (ns <= 4) { GO_D(4) }
+    else if (ns <= 8) { GO_D(8) }
+    else if (ns <= 16) { GO_D(16) }
+    else if (ns <= 32) { GO_D(32) }
+    else { GO_D(64) }
+#undef GO_D
+#undef GO
+    return illm_launch_status();
+}
+
+extern "C" int illm_lightning_step(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                                   const float* decay, float* state, const int32_t* row_slot, float* o, int B,
+                                   int H, int dk, int dv, void* stream) {
+    if (B < 0 || B > 65535 || H <= 0 || H > 65535 || dk <= 0 || dk > 256 || dv <= 0 || !illm_dtype_ok(dt) ||
+        !fd_columns_ok(u_stride, q_off, H * dk) || !fd_columns_ok(u_stride, k_off, H * dk) ||
+        !fd_columns_ok(u_stride, v_off, H * dv))
+        return ILLM_ERR_ARG;
+    if (B == 0) return ILLM_OK;
+    return fixed_step_launch(U, dt, u_stride, q_off, k_off, v_off, decay, RemovalArgs{}, false, state, row_slot, o,
+                             B, H, dk, dv, (hipStream_t)stream);
+}
+
+extern "C" int illm_removal_step(const void* U, int dt, int u_stride, int r_off, int k_off, int v_off, int a_off,
+                                 const float* a_bias, int w1_off, int rank, const void* w2, const float* w0,
+                                 float rate, float* state, const int32_t* row_slot, float* o, int B, int H,
+                                 int d, void* stream) {
+    if (B < 0 || B > 65535 || H <= 0 || H > 65535 || d <= 0 || d > 256 || rank <= 0 || rank > FD_RANK_MAX ||
+        !illm_dtype_ok(dt) || !fd_columns_ok(u_stride, r_off, H * d) || !fd_columns_ok(u_stride, k_off, H * d) ||
+        !fd_columns_ok(u_stride, v_off, H * d) || !fd_columns_ok(u_stride, a_off, H * d) ||
+        !fd_columns_ok(u_stride, w1_off, rank))
+        return ILLM_ERR_ARG;
+    if (B == 0) return ILLM_OK;
+    return fixed_step_launch(U, dt, u_stride, r_off, k_off, v_off, nullptr,
+                             RemovalArgs{a_bias, w2, w0, a_off, w1_off, rank, rate}, true, state, row_slot, o, B, H,
+                             d, d, (hipStream_t)stream);
+}
+
+// ---------------------------------------------------------------- lightning attention in chunks
+// A step's rows of a sequence in chunks of FD_CHUNK tokens (the last one shorter, n_c tokens):
+//   chunk_sums    per (chunk, head): sum_i lam^(n_c - 1 - i) k_i v_i^T, the chunk's part of the state
+//   chunk_carry   per head, chunk after chunk: the state at every chunk's start (in place of the sums)
+//                 and the sequence's last state back into the slot
+//   chunk_rows    per (chunk, head): o_i = lam^(i + 1) S_start^T q_i + sum_(j <= i) lam^(i - j) (q_i . k_j) v_j
+// Products on the matrix cores' float32 instruction (32x32x2: float32 operands, products and sums).
+// Chunk c of sequence b lies at place cu[b] / FD_CHUNK + b + c of `part` [places][H][dk][dv].  Key and value
+// sizes up to 128 in steps of 4, filled up with zeros to whole tiles of 32 (KT, VT).
+#define FD_CHUNK 64
+typedef float fd_f32x16_t __attribute__((ext_vector_type(16)));
+
+template <int DT>
+__device__ __forceinline__ float4 ld4_silu(const void* p, size_t at) {
+    float4 x = ld_f4(p, DT, at / 4);
+    x.x = fd_silu(x.x); x.y = fd_silu(x.y); x.z = fd_silu(x.z); x.w = fd_silu(x.w);
+    return x;
+}
+
+// grid (chunks, H, sequences); 256 threads.  Both operands lie in LDS as [token][channel]; a wave takes
+// every fourth tile of 32 x 32 of the sum.
+template <int DT, int KT, int VT>
+__global__ void __launch_bounds__(256)
+lightning_chunk_sums_kernel(const void* __restrict__ U, int u_stride, int k_off, int v_off,
+                            const float* __restrict__ decay, float* __restrict__ part,
+                            const int32_t* __restrict__ cu, int H, int dk, int dv) {
+    constexpr int DKP = 32 * KT, DVP = 32 * VT, NT = (KT * VT + 3) / 4;
+    __shared__ float ks[FD_CHUNK * DKP];
+    __shared__ float vs[FD_CHUNK * DVP];
+    __shared__ float pw[FD_CHUNK];
+    const int b = blockIdx.z, h = blockIdx.y, c = blockIdx.x, tid = threadIdx.x;
+    const int r0 = cu[b], n = cu[b + 1] - r0, t0 = c * FD_CHUNK;
+    if (t0 >= n) return;                                // the whole block
+    const int nc = min(FD_CHUNK, n - t0);
+    if (tid < FD_CHUNK) pw[tid] = tid < nc ? powf(decay[h], (float)(nc - 1 - tid)) : 0.f;
+    __syncthreads();
+    for (int e = tid; e < FD_CHUNK * (DKP / 4); e += 256) {
+        const int row = e / (DKP / 4), d = 4 * (e % (DKP / 4));
+        float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (row < nc && d < dk) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + k_off + (size_t)h * dk + d);
+        const float f = pw[row];
+        *(float4*)(ks + row * DKP + d) = make_float4(x.x * f, x.y * f, x.z * f, x.w * f);
+    }
+    for (int e = tid; e < FD_CHUNK * (DVP / 4); e += 256) {
+        const int row = e / (DVP / 4), d = 4 * (e % (DVP / 4));
+        float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (row < nc && d < dv) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + v_off + (size_t)h * dv + d);
+        *(float4*)(vs + row * DVP + d) = x;
+    }
+    __syncthreads();
+    const int lane = tid & 63, w = wave_index(), col = lane & 31, half = lane >> 5;
+    float* dst = part + (((size_t)(r0 / FD_CHUNK + b + c)) * H + h) * dk * dv;
+#pragma unroll
+    for (int x = 0; x < NT; ++x) {
+        const int tile = w + 4 * x;
+        if (tile >= KT * VT) continue;
+        const int m0 = 32 * (tile / VT), n0 = 32 * (tile % VT);
+        fd_f32x16_t acc;
+#pragma unroll
+        for (int v = 0; v < 16; ++v) acc[v] = 0.f;
+#pragma unroll 8
+        for (int s2 = 0; s2 < FD_CHUNK / 2; ++s2)
+            acc = __builtin_amdgcn_mfma_f32_32x32x2f32(ks[(2 * s2 + half) * DKP + m0 + col],
+                                                       vs[(2 * s2 + half) * DVP + n0 + col], acc, 0, 0, 0);
+#pragma unroll
+        for (int v = 0; v < 16; ++v) {
+            const int m = m0 + 8 * (v >> 2) + 4 * half + (v & 3), nn = n0 + col;
+            if (m < dk && nn < dv) dst[(size_t)m * dv + nn] = acc[v];
+        }
+    }
+}
+
+// grid (ceil(dk dv / 1024), H, sequences); 256 threads, 4 neighbouring numbers each (dv % 4 == 0).
+#define FD_AHEAD 8
+__global__ void __launch_bounds__(256)
+lightning_chunk_carry_kernel(float* __restrict__ part, const float* __restrict__ decay,
+                             float* __restrict__ state, const int32_t* __restrict__ cu,
+                             const int32_t* __restrict__ seq_slot, int H, int dk, int dv) {
+    const int b = blockIdx.z, h = blockIdx.y, i4 = blockIdx.x * 256 + threadIdx.x;
+    const int r0 = cu[b], n = cu[b + 1] - r0, n4 = dk * dv / 4;
+    if (n <= 0 || i4 >= n4) return;
+    const int chunks = (n + FD_CHUNK - 1) / FD_CHUNK;
+    const float lam = decay[h];
+    const float full = powf(lam, (float)FD_CHUNK), last = powf(lam, (float)(n - (chunks - 1) * FD_CHUNK));
+    float4* sp = (float4*)(state + ((size_t)seq_slot[b] * H + h) * dk * dv) + i4;
+    float4* pp = (float4*)(part + ((size_t)(r0 / FD_CHUNK + b) * H + h) * dk * dv) + i4;
+    const size_t step = (size_t)H * n4;
+    float4 S = *sp;
+    for (int c0 = 0; c0 < chunks; c0 += FD_AHEAD) {
+        float4 add[FD_AHEAD];
+#pragma unroll
+        for (int x = 0; x < FD_AHEAD; ++x)
+            if (c0 + x < chunks) add[x] = pp[(size_t)(c0 + x) * step];
+#pragma unroll
+        for (int x = 0; x < FD_AHEAD; ++x) {
+            if (c0 + x >= chunks) continue;
+            pp[(size_t)(c0 + x) * step] = S;
+            const float f = c0 + x == chunks - 1 ? last : full;
+            S.x = fmaf(f, S.x, add[x].x); S.y = fmaf(f, S.y, add[x].y);
+            S.z = fmaf(f, S.z, add[x].z); S.w = fmaf(f, S.w, add[x].w);
+        }
+    }
+    *sp = S;
+}
+
+// grid (chunks, H, sequences); 256 threads: wave w takes the chunk's 32 tokens of tile w % 2 and every
+// second value tile from w / 2 on.  Both products are kept transposed, so that a lane's column is its
+// token: scores^T = K . Q^T leaves the 16 scores of token (lane % 32) in a lane and its partner 32 lanes
+// on, and in o^T = V^T . P^T they are the second operand as they stand.  k and v lie in LDS, q in
+// registers; the start state is read straight from memory (32 neighbouring values a row).
+template <int DT, int KT, int VT>
+__global__ void __launch_bounds__(256)
+lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off, int k_off, int v_off,
+                            const float* __restrict__ decay, const float* __restrict__ part,
+                            const int32_t* __restrict__ cu, float* __restrict__ o, int H, int dk, int dv) {
+    constexpr int DKP = 32 * KT, DVP = 32 * VT, KLD = DKP + 1, VW = (VT + 1) / 2;
+    __shared__ float ks[FD_CHUNK * KLD];
+    __shared__ float vs[FD_CHUNK * DVP];
+    __shared__ float pw[FD_CHUNK + 1];
+    const int b = blockIdx.z, h = blockIdx.y, c = blockIdx.x, tid = threadIdx.x;
+    const int r0 = cu[b], n = cu[b + 1] - r0, t0 = c * FD_CHUNK;
+    if (t0 >= n) return;                                // the whole block
+    const int nc = min(FD_CHUNK, n - t0);
+    const int lane = tid & 63, w = wave_index(), col = lane & 31, half = lane >> 5;
+    const int it = w & 1, i = 32 * it + col;            // the lane's token within the chunk
+    if (tid <= FD_CHUNK) pw[tid] = powf(decay[h], (float)tid);
+    float qr[DKP / 2];                                  // dims 2 s + half (zeros beyond dk)
+    {
+        const size_t at = (size_t)(r0 + t0 + min(i, nc - 1)) * u_stride + q_off + (size_t)h * dk;
+#pragma unroll
+        for (int j = 0; j < DKP / 4; ++j) {
+            float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (4 * j < dk) x = ld4_silu<DT>(U, at + 4 * j);
+            qr[2 * j] = half ? x.y : x.x;
+            qr[2 * j + 1] = half ? x.w : x.z;
+        }
+    }
+    for (int e = tid; e < FD_CHUNK * (DKP / 4); e += 256) {
+        const int row = e / (DKP / 4), d = 4 * (e % (DKP / 4));
+        float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (row < nc && d < dk) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + k_off + (size_t)h * dk + d);
+        float* to = ks + row * KLD + d;
+        to[0] = x.x; to[1] = x.y; to[2] = x.z; to[3] = x.w;
+    }
+    for (int e = tid; e < FD_CHUNK * (DVP / 4); e += 256) {
+        const int row = e / (DVP / 4), d = 4 * (e % (DVP / 4));
+        float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (row < nc && d < dv) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + v_off + (size_t)h * dv + d);
+        *(float4*)(vs + row * DVP + d) = x;
+    }
+    __syncthreads();
+    if (32 * it >= nc) return;                          // (no barrier follows)
+    const float* S = part + (((size_t)(r0 / FD_CHUNK + b + c)) * H + h) * dk * dv;
+    fd_f32x16_t acc[VW];
+#pragma unroll
+    for (int t = 0; t < VW; ++t) {
+        const int n0 = 32 * (2 * t + (w >> 1));
+#pragma unroll
+        for (int v = 0; v < 16; ++v) acc[t][v] = 0.f;
+        if (n0 >= dv) continue;
+        const bool in = n0 + col < dv;
+#pragma unroll 8
+        for (int s2 = 0; s2 < DKP / 2; ++s2) {
+            const int m = 2 * s2 + half;
+            const float a = (in && m < dk) ? S[(size_t)m * dv + n0 + col] : 0.f;
+            acc[t] = __builtin_amdgcn_mfma_f32_32x32x2f32(a, qr[s2], acc[t], 0, 0, 0);
+        }
+    }
+    const float f = pw[min(i, nc - 1) + 1];
+#pragma unroll
+    for (int t = 0; t < VW; ++t)
+#pragma unroll
+        for (int v = 0; v < 16; ++v) acc[t][v] *= f;
+    for (int jt = 0; jt <= it; ++jt) {
+        fd_f32x16_t sc;
+#pragma unroll
+        for (int v = 0; v < 16; ++v) sc[v] = 0.f;
+        const float* kr = ks + (32 * jt + col) * KLD + half;
+#pragma unroll
+        for (int s2 = 0; s2 < DKP / 2; ++s2)
+            sc = __builtin_amdgcn_mfma_f32_32x32x2f32(kr[2 * s2], qr[s2], sc, 0, 0, 0);
+#pragma unroll
+        for (int v = 0; v < 16; ++v) {
+            const int j = 32 * jt + 8 * (v >> 2) + 4 * half + (v & 3);
+            sc[v] = j <= i ? sc[v] * pw[i - j] : 0.f;
+        }
+#pragma unroll
+        for (int t = 0; t < VW; ++t) {
+            const int n0 = 32 * (2 * t + (w >> 1));
+            if (n0 >= DVP) continue;
+            const float* vr = vs + (32 * jt + 4 * half) * DVP + n0 + col;
+#pragma unroll
+            for (int v = 0; v < 16; ++v)
+                acc[t] = __builtin_amdgcn_mfma_f32_32x32x2f32(vr[(8 * (v >> 2) + (v & 3)) * DVP], sc[v], acc[t], 0, 0, 0);
+        }
+    }
+    if (i >= nc) return;
+    float* op = o + ((size_t)(r0 + t0 + i) * H + h) * dv;
+#pragma unroll
+    for (int t = 0; t < VW; ++t)
+#pragma unroll
+        for (int g = 0; g < 4; ++g) {
+            const int d = 32 * (2 * t + (w >> 1)) + 8 * g + 4 * half;
+            if (d < dv)
+                *(float4*)(op + d) = make_float4(acc[t][4 * g], acc[t][4 * g + 1], acc[t][4 * g + 2], acc[t][4 * g + 3]);
+        }
+}
+
+extern "C" int illm_lightning_chunk(void) { return FD_CHUNK; }
+
+// `part`: (T / FD_CHUNK + n_seqs + 1) H dk dv floats.
+extern "C" int illm_lightning_chunks(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                                     const float* decay, float* state, float* part, const int32_t* cu,
+                                     const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int H, int dk,
+                                     int dv, void* stream) {
+    if (n_seqs < 0 || n_seqs > 65535 || max_rows < 0 || H <= 0 || H > 65535 || dk <= 0 || dk > 128 || dk % 4 ||
+        dv <= 0 || dv > 128 || dv % 4 || !illm_dtype_ok(dt) || u_stride % 4 || q_off % 4 || k_off % 4 || v_off % 4 ||
+        !fd_columns_ok(u_stride, q_off, H * dk) || !fd_columns_ok(u_stride, k_off, H * dk) ||
+        !fd_columns_ok(u_stride, v_off, H * dv) || !part)
+        return ILLM_ERR_ARG;
+    if (n_seqs == 0 || max_rows == 0) return ILLM_OK;
+    hipStream_t st = (hipStream_t)stream;
+    const dim3 grid((max_rows + FD_CHUNK - 1) / FD_CHUNK, H, n_seqs);
+    const int kt = (dk + 31) / 32, vt = (dv + 31) / 32;
+#define GO(DT_, KT_, VT_)                                                                               \
+    do {                                                                                                \
+        hipLaunchKernelGGL((lightning_chunk_sums_kernel<DT_, KT_, VT_>), grid, dim3(256), 0, st, U, u_stride, \
+                           k_off, v_off, decay, part, cu, H, dk, dv);                                   \
+        hipLaunchKernelGGL(lightning_chunk_carry_kernel, dim3((dk * dv / 4 + 255) / 256, H, n_seqs), dim3(256), 0, \
+                           st, part, decay, state, cu, seq_slot, H, dk, dv);                            \
+        hipLaunchKernelGGL((lightning_chunk_rows_kernel<DT_, KT_, VT_>), grid, dim3(256), 0, st, U, u_stride, \
+                           q_off, k_off, v_off, decay, part, cu, o, H, dk, dv);                         \
+    } while (0)
+#define GO_V(DT_, KT_)                                                                                  \
+    switch (vt) { case 1: GO(DT_, KT_, 1); break; case 2: GO(DT_, KT_, 2); break;                       \
+                  case 3: GO(DT_, KT_, 3); break; default: GO(DT_, KT_, 4); break; }
+#define GO_K(DT_)                                                                                       \
+    switch (kt) { case 1: GO_V(DT_, 1) break; case 2: GO_V(DT_, 2) break;                               \
+                  case 3: GO_V(DT_, 3) break; default: GO_V(DT_, 4) break; }
+    if (dt == ILLM_BF16) { GO_K(ILLM_BF16) } else { GO_K(ILLM_F32) }
+#undef GO_K
+#undef GO_V
+#undef GO
+    return illm_launch_status();
+}
+
+// ---------------------------------------------------------------- behind the recurrence
+// out[r, j] = o[r, j] / sqrt(mean over j's part of o^2 + eps) * w[j] * act(Z[r, z_off + j]) with the row of
+// `width` numbers in `groups` equal parts; act = silu (gate_kind 0) or sigmoid (1).
+// Parts of up to 512 numbers: grid (rows, ceil(groups / 4)), a wave a part; longer ones: grid (rows,
+// groups), a block a part.
+__device__ __forceinline__ float fd_gate(float z, int gate_kind) { return gate_kind ? fd_sigmoid(z) : fd_silu(z); }
+
+template <bool WAVE>
+__global__ void __launch_bounds__(256)
+group_norm_gate_kernel(const float* __restrict__ o, const void* __restrict__ w, int w_dt,
+                       const void* __restrict__ Z, int z_dt, int z_stride, int z_off, int gate_kind,
+                       void* __restrict__ out, int out_dt, int width, int part, float eps) {
+    __shared__ float red[16];
+    const size_t r = blockIdx.x;
+    const int g = WAVE ? blockIdx.y * 4 + wave_index() : blockIdx.y;
+    const int j0 = g * part, t = WAVE ? threadIdx.x & 63 : threadIdx.x, step = WAVE ? 64 : 256;
+    if (WAVE && j0 >= width) return;
+    const float* op = o + r * width + j0;
+    float ss = 0.f;
+    if (part % 4 == 0 && z_stride % 4 == 0 && z_off % 4 == 0) {
+        for (int j = t; j < part / 4; j += step) {
+            const float4 x = ((const float4*)op)[j];
+            ss += x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
+        }
+        ss = WAVE ? wave_sum(ss) : block_sum(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)part + eps);
+        for (int j = t; j < part / 4; j += step) {
+            float4 x = ((const float4*)op)[j];
+            const float4 ww = ld_f4(w, w_dt, j0 / 4 + j), z = ld_f4(Z, z_dt, (r * z_stride + z_off + j0) / 4 + j);
+            x.x = (x.x * inv) * ww.x * fd_gate(z.x, gate_kind);
+            x.y = (x.y * inv) * ww.y * fd_gate(z.y, gate_kind);
+            x.z = (x.z * inv) * ww.z * fd_gate(z.z, gate_kind);
+            x.w = (x.w * inv) * ww.w * fd_gate(z.w, gate_kind);
+            st_f4(out, out_dt, (r * width + j0) / 4 + j, x);
+        }
+        return;
+    }
+    for (int j = t; j < part; j += step) ss = fmaf(op[j], op[j], ss);
+    ss = WAVE ? wave_sum(ss) : block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)part + eps);
+    for (int j = t; j < part; j += step)
+        st_f(out, out_dt, r * width + j0 + j, (op[j] * inv) * ld_f(w, w_dt, j0 + j) *
+                                                  fd_gate(ld_f(Z, z_dt, r * z_stride + z_off + j0 + j), gate_kind));
+}
+
+extern "C" int illm_group_norm_gate(const float* o, const void* w, int w_dt, const void* Z, int z_dt, int z_stride,
+                                    int z_off, int gate_kind, void* out, int out_dt, int T, int width, int groups,
+                                    float eps, void* stream) {
+    if (T < 0 || width <= 0 || groups <= 0 || groups > 65535 || width % groups || !illm_dtype_ok(w_dt) ||
+        !illm_dtype_ok(z_dt) || !illm_dtype_ok(out_dt) || !fd_columns_ok(z_stride, z_off, width) ||
+        (gate_kind != 0 && gate_kind != 1))
+        return ILLM_ERR_ARG;
+    if (T == 0) return ILLM_OK;
+    const int part = width / groups;
+    if (part <= 512)
+        hipLaunchKernelGGL(group_norm_gate_kernel<true>, dim3(T, (groups + 3) / 4), dim3(256), 0, (hipStream_t)stream,
+                           o, w, w_dt, Z, z_dt, z_stride, z_off, gate_kind, out, out_dt, width, part, eps);
+    else
+        hipLaunchKernelGGL(group_norm_gate_kernel<false>, dim3(T, groups), dim3(256), 0, (hipStream_t)stream, o, w,
+                           w_dt, Z, z_dt, z_stride, z_off, gate_kind, out, out_dt, width, part, eps);
+    return illm_launch_status();
+}

@@ -108,20 +108,33 @@ extern "C" int illm_few_outputs_f32(const void* x, int x_dt, const float* w, flo
 // (gate from above, up on both sides, at `limit`) gate * sigmoid(1.702 gate) * (up + 1).
 #define MOE_ACT_SILU 0
 #define MOE_ACT_CLAMPED 1
+// Experts without a gate: the up product alone, act(z) = max(z, 0)^2 (as `act_kind` of a product that
+// is not gated; any other kind there leaves the product as it is).
+#define MOE_ACT_RELU2 2
 __device__ __forceinline__ float moe_act(float gate, float up, int act_kind, float limit) {
     if (act_kind == MOE_ACT_SILU) return (gate / (1.0f + expf(-gate))) * up;
     gate = fminf(gate, limit);
     up = fminf(fmaxf(up, -limit), limit);
     return (gate / (1.0f + expf(-1.702f * gate))) * (up + 1.0f);
 }
+static inline bool moe_act_ok(int act_kind, int gated) {
+    return act_kind == MOE_ACT_SILU || act_kind == (gated ? MOE_ACT_CLAMPED : MOE_ACT_RELU2);
+}
+// what a product without a gate leaves of a sum (`rounded`: the activations' type is bfloat16, which
+// the product takes before the activation, as a product of its own would leave it)
+__device__ __forceinline__ float moe_plain_act(float v, int act_kind, bool rounded) {
+    if (act_kind != MOE_ACT_RELU2) return v;
+    v = fmaxf(rounded ? bf16_to_f32(f32_to_bf16(v)) : v, 0.f);
+    return v * v;
+}
 
 // One wave per token: s = the scores of all NE outputs (float32), choice score = s + correction,
-// the `top` largest choice scores (lowest index on ties) in falling order; weights are s.
+// the `top` largest choice scores (lowest index on ties) in falling order; weights are scale * s.
 #define MOE_EPL 8                                   // outputs a lane holds: up to 512 experts
 __device__ __forceinline__ void
 moe_route_row(const float* zr, const void* __restrict__ corr, int corr_dt, int NE, int top,
               int32_t* __restrict__ idx_row, float* __restrict__ wt_row, int32_t* idx_copy,
-              int score_kind) {
+              int score_kind, float scale) {
     const int lane = threadIdx.x & 63;
     float s[MOE_EPL], c[MOE_EPL];
     float mx = -INFINITY;
@@ -166,7 +179,7 @@ moe_route_row(const float* zr, const void* __restrict__ corr, int corr_dt, int N
         w = wave_sum(w);                               // only the owner's lane holds a value
         if (lane == 0) {
             idx_row[k] = be;
-            wt_row[k] = w;
+            wt_row[k] = scale * w;
             if (idx_copy) idx_copy[k] = be;
         }
     }
@@ -174,18 +187,18 @@ moe_route_row(const float* zr, const void* __restrict__ corr, int corr_dt, int N
 
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const float* __restrict__ z, const void* __restrict__ corr, int corr_dt, int NE,
-                 int top, int32_t* __restrict__ idx, float* __restrict__ wt, int score_kind) {
+                 int top, int32_t* __restrict__ idx, float* __restrict__ wt, int score_kind, float scale) {
     const size_t t = blockIdx.x;
-    moe_route_row(z + t * NE, corr, corr_dt, NE, top, idx + t * top, wt + t * top, nullptr, score_kind);
+    moe_route_row(z + t * NE, corr, corr_dt, NE, top, idx + t * top, wt + t * top, nullptr, score_kind, scale);
 }
 
 extern "C" int illm_moe_route(const float* z, const void* corr, int corr_dt, int T, int NE, int top,
-                              int32_t* idx, float* wt, int score_kind, void* stream) {
+                              int32_t* idx, float* wt, int score_kind, float scale, void* stream) {
     if ((score_kind != MOE_SCORE_SOFTMAX && score_kind != MOE_SCORE_SIGMOID) || T < 0 || NE <= 0 || NE > 64 * MOE_EPL || top <= 0 || top > NE || (corr && !illm_dtype_ok(corr_dt)))
         return ILLM_ERR_ARG;
     if (T == 0) return ILLM_OK;
     hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(64), 0, (hipStream_t)stream, z, corr, corr_dt,
-                       NE, top, idx, wt, score_kind);
+                       NE, top, idx, wt, score_kind, scale);
     return illm_launch_status();
 }
 
@@ -336,7 +349,8 @@ moe_rows_kernel(const void* __restrict__ X, int x_div, const void* __restrict__ 
                         if (row_w) { gate *= row_w[pair[r]]; upv *= row_w[pair[r]]; }   // W (w x) = w (W x)
                         if (DT == ILLM_BF16) { gate = bf16_to_f32(f32_to_bf16(gate)); upv = bf16_to_f32(f32_to_bf16(upv)); }
                         v = moe_act(gate, upv, act_kind, limit);
-                    }
+                    } else
+                        v = moe_plain_act(row_w ? v * row_w[pair[r]] : v, act_kind, DT == ILLM_BF16);
                     if (DT == ILLM_BF16) ((bf16_t*)Y)[(size_t)pair[r] * N + col + lane] = f32_to_bf16(v);
                     else ((float*)Y)[(size_t)pair[r] * N + col + lane] = v;
                 }
@@ -349,7 +363,7 @@ extern "C" int illm_moe_rows(const void* X, int x_div, const void* W, int dt, in
                              const int32_t* order, const int32_t* tiles, int max_tiles, void* Y,
                              int N, int K, int act_kind, float limit, const float* row_w,
                              void* stream) {
-    if ((act_kind != MOE_ACT_SILU && act_kind != MOE_ACT_CLAMPED) || x_div <= 0 || N <= 0 || K <= 0 || max_tiles < 0 || max_tiles > 2147483647 / 3 ||
+    if (!moe_act_ok(act_kind, gated) || x_div <= 0 || N <= 0 || K <= 0 || max_tiles < 0 || max_tiles > 2147483647 / 3 ||
         !illm_dtype_ok(dt))
         return ILLM_ERR_ARG;
     if (max_tiles == 0) return ILLM_OK;
@@ -511,7 +525,8 @@ moe_rows_mfma_kernel(const bf16_t* __restrict__ X, int x_div, const bf16_t* __re
                     const float gate = bf16_to_f32(f32_to_bf16(a[nt][mt][i] * rw));
                     const float upv = bf16_to_f32(f32_to_bf16(g[nt][mt][i] * rw));
                     v = moe_act(gate, upv, act_kind, limit);
-                }
+                } else
+                    v = moe_plain_act(row_w ? v * row_w[pair[mt]] : v, act_kind, true);
                 Y[(size_t)pair[mt] * N + col] = f32_to_bf16(v);
             }
     }
@@ -631,7 +646,8 @@ moe_rows_mfma_lds_kernel(const bf16_t* __restrict__ X, int x_div, const bf16_t* 
                     const float gate = bf16_to_f32(f32_to_bf16(a[nt][mt][i] * rw));
                     const float upv = bf16_to_f32(f32_to_bf16(g[nt][mt][i] * rw));
                     v = moe_act(gate, upv, act_kind, limit);
-                }
+                } else
+                    v = moe_plain_act(row_w ? v * row_w[pair[mt]] : v, act_kind, true);
                 Y[(size_t)pair[mt] * N + col] = f32_to_bf16(v);
             }
     }
@@ -641,7 +657,7 @@ extern "C" int illm_moe_rows_mfma(const void* X, int x_div, const void* W, int g
                                   const int32_t* order, const int32_t* tiles, int max_tiles,
                                   void* Y, int N, int K, int act_kind, float limit,
                                   const float* row_w, void* stream) {
-    if ((act_kind != MOE_ACT_SILU && act_kind != MOE_ACT_CLAMPED) || x_div <= 0 || N <= 0 || K <= 0 || K % 32 || max_tiles < 0 || max_tiles > 2147483647 / 3 ||
+    if (!moe_act_ok(act_kind, gated) || x_div <= 0 || N <= 0 || K <= 0 || K % 32 || max_tiles < 0 || max_tiles > 2147483647 / 3 ||
         (tile_rows != 16 && tile_rows != 32 && tile_rows != 64))
         return ILLM_ERR_ARG;
     if (max_tiles == 0) return ILLM_OK;

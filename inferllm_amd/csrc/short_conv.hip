@@ -20,26 +20,6 @@ __device__ __forceinline__ float conv_round(float v, int dt) {
     return dt == ILLM_BF16 ? bf16_to_f32(f32_to_bf16(v)) : v;
 }
 
-__device__ __forceinline__ float4 sc_ld4(const void* p, int dt, size_t i4) {
-    if (dt == ILLM_BF16) {
-        const uint2 u = ((const uint2*)p)[i4];
-        return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u),
-                           __uint_as_float(u.y << 16), __uint_as_float(u.y & 0xffff0000u));
-    }
-    return ((const float4*)p)[i4];
-}
-
-__device__ __forceinline__ void sc_st4(void* p, int dt, size_t i4, float4 v) {
-    if (dt == ILLM_BF16) {
-        uint2 u;
-        u.x = pack_bf16x2(v.x, v.y);
-        u.y = pack_bf16x2(v.z, v.w);
-        ((uint2*)p)[i4] = u;
-    } else {
-        ((float4*)p)[i4] = v;
-    }
-}
-
 // Four channels a thread where the rows allow (C, the offset and the strides multiples of 4): grid
 // (rows, ceil(C / 1024)).
 __global__ void __launch_bounds__(256)
@@ -64,7 +44,7 @@ short_conv_vec4_kernel(const void* __restrict__ X, int x_dt, int x_stride, int x
     for (int j = 0; j < CONV_MAX_TAPS; ++j) {
         if (j >= taps) continue;
         const int rr = max(r - (K - j), 0);
-        in[j] = sc_ld4(X, x_dt, ((size_t)rr * x_stride + x_off) / 4 + c4);
+        in[j] = ld_f4(X, x_dt, ((size_t)rr * x_stride + x_off) / 4 + c4);
     }
     int n = 0;
 #pragma unroll
@@ -84,7 +64,7 @@ short_conv_vec4_kernel(const void* __restrict__ X, int x_dt, int x_stride, int x
             }
             in[j] = v;
         } else {
-            in[j] = sc_ld4(tail, tail_dt, ((size_t)slot * K + (K - (back - n))) * (C / 4) + c4);
+            in[j] = ld_f4(tail, tail_dt, ((size_t)slot * K + (K - (back - n))) * (C / 4) + c4);
         }
         if (back == 0) cur = in[j];
     }
@@ -99,11 +79,11 @@ short_conv_vec4_kernel(const void* __restrict__ X, int x_dt, int x_stride, int x
             if (j < taps) y[e] = fmaf(cw[j], ((const float*)&in[j])[e], y[e]);
         if (add_input) y[e] += ((const float*)&cur)[e];
     }
-    sc_st4(out, out_dt, ((size_t)r * out_stride) / 4 + c4, make_float4(y[0], y[1], y[2], y[3]));
+    st_f4(out, out_dt, ((size_t)r * out_stride) / 4 + c4, make_float4(y[0], y[1], y[2], y[3]));
     if (update_tail) {
 #pragma unroll
         for (int j = 1; j < CONV_MAX_TAPS; ++j)
-            if (j < taps) sc_st4(tail, tail_dt, ((size_t)slot * K + (j - 1)) * (C / 4) + c4, in[j]);
+            if (j < taps) st_f4(tail, tail_dt, ((size_t)slot * K + (j - 1)) * (C / 4) + c4, in[j]);
     }
 }
 
@@ -328,9 +308,9 @@ post_add_rmsnorm_kernel(float* __restrict__ x, const void* __restrict__ a, int a
         for (int k = 0; k < NV; ++k) {
             const int i4 = threadIdx.x + 256 * k;
             xv[k] = i4 < n4 ? ((const float4*)(x + ib))[i4] : zero4;
-            av[k] = (a && i4 < n4) ? sc_ld4(a, a_dt, ib / 4 + i4) : zero4;
-            pwv[k] = (a && i4 < n4) ? sc_ld4(post_w, post_w_dt, i4) : zero4;
-            wv4[k] = i4 < n4 ? sc_ld4(w, w_dt, i4) : zero4;
+            av[k] = (a && i4 < n4) ? ld_f4(a, a_dt, ib / 4 + i4) : zero4;
+            pwv[k] = (a && i4 < n4) ? ld_f4(post_w, post_w_dt, i4) : zero4;
+            wv4[k] = i4 < n4 ? ld_f4(w, w_dt, i4) : zero4;
         }
         if (a) {
             float sa = 0.f;
@@ -366,7 +346,7 @@ post_add_rmsnorm_kernel(float* __restrict__ x, const void* __restrict__ a, int a
                 float4 old[CONV_MAX_TAPS - 1];
 #pragma unroll
                 for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
-                    if (j < K) old[j] = sc_ld4(tail, tail_dt, ((size_t)slot * K + j) * n4 + i4);
+                    if (j < K) old[j] = ld_f4(tail, tail_dt, ((size_t)slot * K + j) * n4 + i4);
                 float hq[4];
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
@@ -382,10 +362,10 @@ post_add_rmsnorm_kernel(float* __restrict__ x, const void* __restrict__ a, int a
                 // the tail moves on by the new input
 #pragma unroll
                 for (int j = 1; j < CONV_MAX_TAPS - 1; ++j)
-                    if (j < K) sc_st4(tail, tail_dt, ((size_t)slot * K + (j - 1)) * n4 + i4, old[j]);
-                sc_st4(tail, tail_dt, ((size_t)slot * K + (K - 1)) * n4 + i4, make_float4(hq[0], hq[1], hq[2], hq[3]));
+                    if (j < K) st_f4(tail, tail_dt, ((size_t)slot * K + (j - 1)) * n4 + i4, old[j]);
+                st_f4(tail, tail_dt, ((size_t)slot * K + (K - 1)) * n4 + i4, make_float4(hq[0], hq[1], hq[2], hq[3]));
             }
-            sc_st4(out, out_dt, ob / 4 + i4, make_float4(h[0], h[1], h[2], h[3]));
+            st_f4(out, out_dt, ob / 4 + i4, make_float4(h[0], h[1], h[2], h[3]));
         }
         return;
     }

@@ -198,6 +198,15 @@ def gelu_tanh(x: torch.Tensor) -> torch.Tensor:
     return out
 
 
+def xielu(x: torch.Tensor, par: torch.Tensor) -> torch.Tensor:
+    """(par[0] x^2 if x > 0 else par[1] (e^x - 1 - x)) + x / 2, element by element; par float32 [2]."""
+    _gpu(x, par)
+    _need(par.dtype == torch.float32 and par.shape == (2,), "xielu: par float32 [2]")
+    out = torch.empty_like(x)
+    _check(_lib().illm_xielu(_p(x), _p(par), _p(out), _code(x), ctypes.c_size_t(x.numel()), _stream()), "xielu")
+    return out
+
+
 def add_rmsnorm(x: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Tensor, eps: float,
                 out_dtype: torch.dtype, row_idx: Optional[torch.Tensor] = None,
                 weight2: Optional[torch.Tensor] = None):
@@ -1366,13 +1375,15 @@ def few_outputs_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 
 
 MOE_SCORES = {"softmax": 0, "sigmoid": 1}            # a router's scores: over all outputs, or each its own
-MOE_ACTIVATIONS = {"silu": 0, "clamped_swish": 1}    # see `moe_experts`
+MOE_ACTIVATIONS = {"silu": 0, "clamped_swish": 1, "relu_squared": 2}    # see `moe_experts`
+MOE_PLAIN_ACTIVATIONS = ("relu_squared",)            # of experts without a gate
 
 
-def moe_route(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, score: str = "softmax"):
+def moe_route(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, score: str = "softmax",
+              scale: float = 1.0):
     """(idx int32 [T, top], weight float32 [T, top]): per row of the router's float32 outputs z
-    the `top` largest score(z) + correction, and their scores (`score`: "softmax" over all
-    outputs, or "sigmoid" of each)."""
+    the `top` largest score(z) + correction, and `scale` times their scores (`score`: "softmax" over
+    all outputs, or "sigmoid" of each)."""
     _need(score in MOE_SCORES, f"moe_route: score {score!r}; known: {sorted(MOE_SCORES)}")
     _gpu(z, correction)
     _need(z.dtype == torch.float32 and z.dim() == 2, "moe_route: float32 [T, outputs]")
@@ -1382,7 +1393,7 @@ def moe_route(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, sco
     wt = torch.empty((T, top), dtype=torch.float32, device=z.device)
     _check(_lib().illm_moe_route(_p(z), _p(correction),
                                  _code(correction) if correction is not None else 0, T, NE, top,
-                                 _p(idx), _p(wt), MOE_SCORES[score], _stream()), "moe_route")
+                                 _p(idx), _p(wt), MOE_SCORES[score], ctypes.c_float(scale), _stream()), "moe_route")
     return idx, wt
 
 
@@ -1413,14 +1424,17 @@ def _moe_group(idx: torch.Tensor, n_exp: int, dtype: torch.dtype, E: int, F: int
 
 
 def moe_plan(h: torch.Tensor, w_router: torch.Tensor, correction: Optional[torch.Tensor], top: int,
-             w_gate_up: Optional[torch.Tensor], score: str = "softmax"):
+             w_gate_up: Optional[torch.Tensor], score: str = "softmax", scale: float = 1.0,
+             gated: bool = True):
     """A routed layer's plan for the rows h: (idx, weight, grouped).  idx, weight [T, top] as
     `moe_route` gives them for the router's float32 outputs h . w_router^T; grouped: the pairs
-    grouped by expert for `moe_experts` (None without stacked experts)."""
+    grouped by expert for `moe_experts` (None without stacked experts).  `gated` False: the stacked
+    experts have an up matrix [F, E] alone."""
     E = h.shape[1]
     n_exp = w_gate_up.shape[0] if w_gate_up is not None else 0
-    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score)
-    grouped = _moe_group(idx, n_exp, h.dtype, E, w_gate_up.shape[1] // 2) if n_exp else None
+    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score, scale)
+    grouped = (_moe_group(idx, n_exp, h.dtype, E, w_gate_up.shape[1] // (2 if gated else 1))
+               if n_exp else None)
     return idx, wt, grouped
 
 
@@ -1432,7 +1446,8 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, w_gate_up: torch.Tensor, w_d
     down(act(gate h, up h)); rows of other pairs are not written.  `activation` "silu":
     silu(g) * u; "clamped_swish": with g = min(g, limit) and u = clamp(u, -limit, limit),
     g * sigmoid(1.702 g) * (u + 1).  `input_weight` float32 [T, top]: the pair's expert sees
-    weight * h instead of h.  `grouped`: the pairs by expert as `moe_plan` left them (else they
+    weight * h instead of h.  "relu_squared": experts without a gate, w_gate_up [experts, F, E] the up
+    matrices alone, down(max(up h, 0)^2).  `grouped`: the pairs by expert as `moe_plan` left them (else they
     are grouped here)."""
     _need(activation in MOE_ACTIVATIONS, f"moe_experts: activation {activation!r}; known: {sorted(MOE_ACTIVATIONS)}")
     act_kind, lim = MOE_ACTIVATIONS[activation], ctypes.c_float(limit)
@@ -1444,23 +1459,24 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, w_gate_up: torch.Tensor, w_d
     T, E = h.shape
     top = idx.shape[1]
     n_exp, F2, _ = w_gate_up.shape
-    _need(w_gate_up.shape[2] == E and w_down.shape == (n_exp, E, F2 // 2) and F2 % 2 == 0
+    gated = activation not in MOE_PLAIN_ACTIVATIONS
+    F = F2 // 2 if gated else F2
+    _need(w_gate_up.shape[2] == E and w_down.shape == (n_exp, E, F) and (not gated or F2 % 2 == 0)
           and w_gate_up.dtype == h.dtype and w_down.dtype == h.dtype and idx.shape[0] == T,
           "moe_experts: shapes or dtypes")
     NP = T * top
-    F = F2 // 2
     order, tiles, max_tiles, rows, mfma = grouped if grouped is not None else _moe_group(idx, n_exp, h.dtype, E, F)
     act = torch.empty((NP, F), dtype=h.dtype, device=h.device)
     y = torch.empty((NP, E), dtype=h.dtype, device=h.device)
     if mfma:
-        _check(_lib().illm_moe_rows_mfma(_p(h), top, _p(w_gate_up), 1, rows, _p(order), _p(tiles),
+        _check(_lib().illm_moe_rows_mfma(_p(h), top, _p(w_gate_up), 1 if gated else 0, rows, _p(order), _p(tiles),
                                          max_tiles, _p(act), F, E, act_kind, lim, _p(input_weight),
                                          _stream()), "moe_rows_mfma (gate|up)")
         _check(_lib().illm_moe_rows_mfma(_p(act), 1, _p(w_down), 0, rows, _p(order), _p(tiles),
                                          max_tiles, _p(y), E, F, 0, ctypes.c_float(0.0), _p(None),
                                          _stream()), "moe_rows_mfma (down)")
         return y
-    _check(_lib().illm_moe_rows(_p(h), top, _p(w_gate_up), _code(h), 1, _p(order), _p(tiles),
+    _check(_lib().illm_moe_rows(_p(h), top, _p(w_gate_up), _code(h), 1 if gated else 0, _p(order), _p(tiles),
                                 max_tiles, _p(act), F, E, act_kind, lim, _p(input_weight), _stream()),
            "moe_rows (gate|up)")
     _check(_lib().illm_moe_rows(_p(act), 1, _p(w_down), _code(h), 0, _p(order), _p(tiles),
@@ -1574,14 +1590,22 @@ def attn_cap_rows(q: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Ten
                   nh: int, nkv: int, dk: int, dv: int, scale: float, cap: float,
                   window: int, slopes: Optional[torch.Tensor] = None, chunk: int = 0,
                   gate: Optional[torch.Tensor] = None, gate_off: int = 0,
-                  gate_heads: bool = False, lse: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  gate_heads: bool = False, lse: Optional[torch.Tensor] = None, keep: int = 0,
+                  kept: int = 0, own=None) -> torch.Tensor:
     """Causal attention of a step's packed rows over the paged cache (which holds the step's own
     keys and values by now): row r of sequence b stands at position seq_start[b] + r; scores
     cap tanh(q . k scale / cap) (cap 0: none); queries and keys of width dk, values of dv.
     `slopes` float32 [nh]: score -= slopes[h] (i - j).  `chunk` > 0: a row sees only the keys of its
     own chunk of positions.  `gate` [T, n] (columns gate_off ..): out *= sigmoid(gate), one
     number a head and value dim, or with `gate_heads` one a head.  `lse` float32 [T, nh] takes
-    max + log(sum) of every row's and head's softmax.  Returns [T, nh dv]."""
+    max + log(sum) of every row's and head's softmax.  `keep` (with a window): the sequence's first
+    `keep` tokens are seen beside the window; `kept`: pages that stay ahead of the line's ring.
+    `own` = (k_off, v_off): keys and values are read from those columns of q's own rows and not from
+    the cache (steps whose sequences all start).  Returns [T, nh dv]."""
+    _need(0 <= keep and (keep == 0 or (window > 0 and chunk == 0)), "attn_cap_rows: kept tokens go with a window, without chunks")
+    own_stride, own_k, own_v = (q.shape[1], int(own[0]), int(own[1])) if own is not None else (0, 0, 0)
+    _need(own is None or (own_k + nkv * dk <= own_stride and own_v + nkv * dv <= own_stride),
+          "attn_cap_rows: own keys and values lie within the rows")
     _cap_extras_ok(q, slopes, gate, gate_off, nh, dv, "attn_cap_rows", gate_heads)
     _lse_ok(lse, q.shape[0], nh, "attn_cap_rows")
     _gpu(q, cu_seqlens, seq_slot, seq_start, kcache, vcache, page_table)
@@ -1589,10 +1613,12 @@ def attn_cap_rows(q: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Ten
     _cap_cache_ok(q, kcache, vcache, page_table, page_size, nh, nkv, dk, dv, "attn_cap_rows")
     out = torch.empty((q.shape[0], nh * dv), dtype=q.dtype, device=q.device)
     _check(_lib().illm_attn_cap_rows(
-        _p(q), q.shape[1], _p(out), _code(q), _p(cu_seqlens), _p(seq_slot), _p(seq_start), _p(kcache),
-        _p(vcache), _p(page_table), page_table.shape[1], page_size, ring, n_seqs, max_rows, nh, nkv,
+        _p(q), q.shape[1], _p(out), _code(q), _p(cu_seqlens), _p(seq_slot), _p(seq_start),
+        _p(q if own is not None else kcache), _p(q if own is not None else vcache), _p(page_table),
+        page_table.shape[1], page_size, ring, n_seqs, max_rows, nh, nkv,
         dk, dv, ctypes.c_float(scale), ctypes.c_float(cap), window, _p(slopes), int(chunk), _p(gate),
-        gate.shape[1] if gate is not None else 0, gate_off, 1 if gate_heads else 0, _p(lse), _stream()),
+        gate.shape[1] if gate is not None else 0, gate_off, 1 if gate_heads else 0, _p(lse), int(keep),
+        int(kept), own_stride, own_k, own_v, _stream()),
         f"attn_cap_rows (sizes {dk}, {dv})")
     return out
 
@@ -1602,9 +1628,11 @@ def attn_cap_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
                     seq_len: torch.Tensor, nh: int, nkv: int, dk: int, dv: int, scale: float,
                     cap: float, window: int, nsplit: int, slopes: Optional[torch.Tensor] = None,
                     chunk: int = 0, gate: Optional[torch.Tensor] = None, gate_off: int = 0,
-                    gate_heads: bool = False, lse: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    gate_heads: bool = False, lse: Optional[torch.Tensor] = None, keep: int = 0,
+                    kept: int = 0) -> torch.Tensor:
     """The same attention for one new token per sequence: row b of q against the seq_len[b] keys
     (the new one included) of its slot, the keys cut into `nsplit` ranges.  Returns [B, nh dv]."""
+    _need(0 <= keep and (keep == 0 or (window > 0 and chunk == 0)), "attn_cap_decode: kept tokens go with a window, without chunks")
     _cap_extras_ok(q, slopes, gate, gate_off, nh, dv, "attn_cap_decode", gate_heads)
     _lse_ok(lse, q.shape[0], nh, "attn_cap_decode")
     _need(lse is None or nsplit >= 2, "attn_cap_decode: lse comes from the merge of two or more ranges")
@@ -1619,7 +1647,7 @@ def attn_cap_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
         page_table.shape[1], page_size, ring, _p(seq_slot), _p(seq_len), _p(partial), nsplit, B, nh,
         nkv, dk, dv, ctypes.c_float(scale), ctypes.c_float(cap), window, _p(slopes), int(chunk),
         _p(gate), gate.shape[1] if gate is not None else 0, gate_off, 1 if gate_heads else 0, _p(lse),
-        _stream()), f"attn_cap_decode (sizes {dk}, {dv})")
+        int(keep), int(kept), _stream()), f"attn_cap_decode (sizes {dk}, {dv})")
     return out
 
 
@@ -1679,10 +1707,13 @@ def delta_conv_tail(P: torch.Tensor, tail: torch.Tensor, cu_seqlens: torch.Tenso
 
 
 def delta_scan(qn, kn, vv, beta, dec, state: torch.Tensor, cu_seqlens: torch.Tensor,
-               seq_slot: torch.Tensor, n_seqs: int, max_rows: int, correct: bool = True) -> torch.Tensor:
+               seq_slot: torch.Tensor, n_seqs: int, max_rows: int, correct: bool = True,
+               removal: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The recurrence S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q over every
     sequence's rows in order, from `state` float32 [slots, H, dk, dv] and back into it.  With
-    `correct` False the plain gated rule, u = beta v: S <- diag(g) S + k (beta v)^T.
+    `correct` False the plain gated rule, u = beta v: S <- diag(g) S + k (beta v)^T; with `removal`
+    float32 [T, H, dk] too, S <- diag(g) S - removal (u^T S) + k v^T with u = beta k, both terms from
+    the old S.
     `max_rows`: the most rows a sequence brings (long sequences are laid out for their chain of
     tokens, short steps for the state's bytes).  Returns o float32 [T, H, dv]."""
     _gpu(qn, kn, vv, beta, dec, state, cu_seqlens, seq_slot)
@@ -1692,10 +1723,13 @@ def delta_scan(qn, kn, vv, beta, dec, state: torch.Tensor, cu_seqlens: torch.Ten
     _need(all(t.dtype == torch.float32 for t in (qn, kn, vv, beta, dec, state)), "delta_scan: float32")
     _need(kn.shape == qn.shape and beta.shape == (T, H) and dec.shape[:2] == (T, H)
           and dec.shape[2] in (1, dk) and state.shape[1:] == (H, dk, dv), "delta_scan: shapes")
+    _gpu(removal)
+    _need(removal is None or (not correct and G == H and removal.dtype == torch.float32
+                              and removal.shape == (T, H, dk)), "delta_scan: removal float32 [T, H, dk], without `correct`")
     o = torch.empty((T, H, dv), dtype=torch.float32, device=qn.device)
     _check(_lib().illm_gated_scan(_p(qn), _p(kn), _p(vv), _p(beta), _p(dec), dec.shape[2], _p(state),
                                   _p(cu_seqlens), _p(seq_slot), _p(o), n_seqs, max_rows, G, H, dk, dv,
-                                  1 if correct else 0, _stream()),
+                                  1 if correct else 0, _p(removal), _stream()),
            "delta_scan")
     return o
 
@@ -1877,15 +1911,65 @@ def rms_rows_gain(a: torch.Tensor, weight: torch.Tensor, eps: float, gain: float
 
 
 class PostNormed:
-    """gain * a / sqrt(mean(a^2) + eps) * weight, not yet formed: what a sublayer with a norm of its
-    own behind it leaves to be added to the residual stream.  A norm that adds it in its own kernel
-    (`post_add_rmsnorm`) takes the pieces, any other asks for `tensor()` (float32)."""
+    """gain * norm(a), not yet formed: what a sublayer with a norm of its own behind it leaves to be
+    added to the residual stream.  `kind` "rms": a / sqrt(mean(a^2) + eps) * weight; "layer": the
+    layer norm with `weight` and, if given, `bias`.  A norm that adds it in its own kernel
+    (`post_add_rmsnorm`, `post_add_norm`) takes the pieces, any other asks for `tensor()` (float32)."""
 
-    def __init__(self, a: torch.Tensor, weight: torch.Tensor, eps: float, gain: float):
+    def __init__(self, a: torch.Tensor, weight: torch.Tensor, eps: float, gain: float, kind: str = "rms",
+                 bias: Optional[torch.Tensor] = None):
+        _need(kind in ("rms", "layer") and (bias is None or kind == "layer"), f"PostNormed: kind {kind!r}")
         self.a, self.weight, self.eps, self.gain = a, weight, float(eps), float(gain)
+        self.kind, self.bias = kind, bias
 
     def tensor(self) -> torch.Tensor:
-        return rms_rows_gain(self.a, self.weight, self.eps, self.gain)
+        if self.kind == "rms":
+            return rms_rows_gain(self.a, self.weight, self.eps, self.gain)
+        out = torch.zeros(self.a.shape, dtype=torch.float32, device=self.a.device)
+        post_add_norm(out, self, None, None, None, 0.0, None)
+        return out
+
+
+NORM_KINDS = {None: 0, "rms": 1, "layer": 2}
+POST_NORM_MAX_WIDTH = 16000
+
+
+def post_add_norm(x: torch.Tensor, post, kind: Optional[str], weight: Optional[torch.Tensor],
+                  bias: Optional[torch.Tensor], eps: float, out_dtype: Optional[torch.dtype],
+                  row_idx: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """One pass over float32 rows x [T, E]: x += `post` (a `PostNormed` whose norm is formed here, a
+    tensor of x's shape that is added as it is, or None), then the rows themselves (`kind` None) or
+    their norm under `weight` (`kind` "rms", or "layer" with `bias`) in `out_dtype` (None: x alone is
+    moved on and nothing returned).  With `row_idx` only those rows, and x stays.  Rows that are
+    asked for as float32 themselves are x."""
+    _gpu(x, weight, bias, row_idx)
+    _i32(row_idx)
+    _need(x.dtype == torch.float32 and x.dim() == 2, "post_add_norm: x must be float32 [T, E]")
+    _need(kind in NORM_KINDS and (kind is None) == (weight is None), "post_add_norm: a kind of norm and its weight")
+    T, E = x.shape
+    _need(E <= POST_NORM_MAX_WIDTH or E % 4 == 0 and E <= 8192, f"post_add_norm: width {E} is beyond the kernel's {POST_NORM_MAX_WIDTH}")
+    for t in (weight, bias):
+        _need(t is None or (t.shape == (E,) and t.dtype == weight.dtype), "post_add_norm: weight and bias [E] of one dtype")
+    a = pw = pb = None
+    post_kind, post_eps, gain = None, 0.0, 1.0
+    if isinstance(post, PostNormed):
+        a, pw, pb, post_kind, post_eps, gain = post.a, post.weight, post.bias, post.kind, post.eps, post.gain
+        _need(pw.shape == (E,) and (pb is None or (pb.shape == (E,) and pb.dtype == pw.dtype)),
+              "post_add_norm: the sublayer's norm has x's width")
+    elif post is not None:
+        a = post
+    _gpu(a, pw, pb)
+    _need(a is None or a.shape == x.shape, "post_add_norm: what is added has x's shape")
+    rows = T if row_idx is None else row_idx.numel()
+    out = None
+    if out_dtype is not None and not (kind is None and row_idx is None and out_dtype == torch.float32):
+        out = torch.empty((rows, E), dtype=out_dtype, device=x.device)
+    _check(_lib().illm_post_add_norm(
+        _p(x), _p(a), _code(a) if a is not None else 0, NORM_KINDS[post_kind], _p(pw), _p(pb),
+        _code(pw) if pw is not None else 0, ctypes.c_float(post_eps), ctypes.c_float(gain), NORM_KINDS[kind],
+        _p(weight), _p(bias), _code(weight) if weight is not None else 0, ctypes.c_float(eps), _p(out),
+        _code(out) if out is not None else 0, _p(row_idx), rows, E, _stream()), "post_add_norm")
+    return x if out is None and out_dtype is not None else out
 
 
 POST_ADD_MAX_WIDTH = 16384
@@ -1906,6 +1990,7 @@ def post_add_rmsnorm(x: torch.Tensor, post: Optional[PostNormed], weight: torch.
     if post is not None:
         a, pw = post.a, post.weight
         _gpu(a, pw)
+        _need(post.kind == "rms", "post_add_rmsnorm: the sublayer's own norm is an RMS norm")
         _need(a.shape == x.shape and pw.shape == (E,), "post_add_rmsnorm: the sublayer's output has x's shape")
     rows = T if row_idx is None else row_idx.numel()
     cw = tail = slots = None
@@ -1947,15 +2032,27 @@ def qk_rotate_store(rows: torch.Tensor, k_off: int, v_off: int, cos_sin: Optiona
                     row_slot: torch.Tensor, kcache: Optional[torch.Tensor],
                     vcache: Optional[torch.Tensor], page_table: Optional[torch.Tensor], page_size: int,
                     ring: int, nh: int, nkv: int, dk: int, dv: int,
-                    q_scale: Optional[torch.Tensor] = None) -> None:
+                    q_scale: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None,
+                    q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None,
+                    slot_len: Optional[torch.Tensor] = None, kept: int = 0) -> None:
     """In place on packed rows [q (nh dk) | .. k at k_off (nkv dk) | v at v_off (nkv dv)], in float32:
     the first `rot` dims of every q and k head turned by the row's position (cos_sin float32
     [positions, rot / 2, 2]; pairing 0: i with i + rot / 2, 1: 2i with 2i + 1), then with `unit_norm`
     every head divided by its root mean square, then query head h times `q_scale`[h] (float32 [nh]:
     a scale of the scores that differs by head, taken into the queries); k and v stored in the paged
     cache K [pages, nkv, page_size, dk], V [pages, nkv, page_size, dv] (None: not stored; nkv 0: rows
-    of queries alone)."""
-    _gpu(rows, cos_sin, row_pos, row_slot, kcache, vcache, page_table, q_scale)
+    of queries alone).  Before all that `bias` float32 [q | k | v] is added and every q and k head is
+    RMS-normed (`eps`) under `q_weight`, `k_weight` [dk].  `kept`: pages that stay ahead of the cache
+    line's ring; `slot_len` (the slots' lengths after the step): rows that a later row of the step
+    overwrites in the ring are not stored."""
+    _gpu(rows, cos_sin, row_pos, row_slot, kcache, vcache, page_table, q_scale, bias, q_weight, k_weight, slot_len)
+    _i32(slot_len)
+    _need(bias is None or (bias.dtype == torch.float32 and bias.shape == (nh * dk + nkv * (dk + dv),)
+                           and k_off == nh * dk and v_off == k_off + nkv * dk),
+          "qk_rotate_store: bias float32 for rows [q | k | v]")
+    _need((q_weight is None) == (k_weight is None) and (q_weight is None or (
+        q_weight.shape == (dk,) and k_weight.shape == (dk,) and q_weight.dtype == k_weight.dtype)),
+          "qk_rotate_store: both norm weights [dk] or none")
     _need(q_scale is None or (q_scale.dtype == torch.float32 and q_scale.shape == (nh,)),
           f"qk_rotate_store: q_scale float32 [{nh}]")
     T = rows.shape[0]
@@ -1972,7 +2069,8 @@ def qk_rotate_store(rows: torch.Tensor, k_off: int, v_off: int, cos_sin: Optiona
         _p(rows), _code(rows), rows.shape[1], k_off, v_off, _p(cos_sin), rot if cos_sin is not None else 0,
         pairing, cos_sin.shape[0] if cos_sin is not None else 0, 1 if unit_norm else 0, ctypes.c_float(eps),
         _p(q_scale), _p(row_pos), _p(row_slot), _p(kcache), _p(vcache), _p(page_table),
-        page_table.shape[1] if page_table is not None else 0, page_size, ring, T, nh, nkv, dk, dv,
+        page_table.shape[1] if page_table is not None else 0, page_size, ring, T, nh, nkv, dk, dv, _p(bias),
+        _p(q_weight), _p(k_weight), _code(q_weight) if q_weight is not None else 0, _p(slot_len), int(kept),
         _stream()), "qk_rotate_store")
 
 
@@ -2130,6 +2228,149 @@ def lru_scan(a: torch.Tensor, x: torch.Tensor, state: torch.Tensor, Y: torch.Ten
     _check(_lib().illm_lru_scan(_p(a), _p(x), _p(state), _p(Y), _code(Y), Y.shape[1], y_off, _p(y_bias),
                                 _p(out), _code(out), _p(cu_seqlens), _p(seq_slot), n_seqs, int(max_rows), C,
                                 _p(scratch), _stream()), "lru_scan")
+    return out
+
+
+# ------------------------------------------------------------------ lightning attention, the delta rule with a removal vector
+def _columns_ok(U: torch.Tensor, what: str, *spans) -> None:
+    _need(U.dim() == 2 and all(0 <= off and off + n <= U.shape[1] for off, n in spans),
+          f"{what}: the projections' columns lie within the rows")
+
+
+def _decay_ok(decay: torch.Tensor, state: torch.Tensor, H: int, dk: int, dv: int, what: str) -> None:
+    _need(decay.dtype == torch.float32 and decay.shape == (H,) and state.dtype == torch.float32
+          and state.dim() == 4 and state.shape[1:] == (H, dk, dv), f"{what}: decay float32 [H], state float32 [slots, H, dk, dv]")
+
+
+def lightning_prepare(U: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor, H: int,
+                      dk: int, dv: int):
+    """Lightning attention's float32 inputs for the plain gated rule (`delta_scan`): silu of U's q and k
+    columns (H dk) and v columns (H dv), weight 1, the heads' fixed decays (float32 [H]).
+    Returns (q [T, H, dk], k, v [T, H, dv], weight [T, H], decay [T, H, 1])."""
+    _gpu(U, decay)
+    _columns_ok(U, "lightning_prepare", (q_off, H * dk), (k_off, H * dk), (v_off, H * dv))
+    _need(decay.dtype == torch.float32 and decay.shape == (H,), "lightning_prepare: decay float32 [H]")
+    T = U.shape[0]
+    new = lambda *shape: torch.empty(shape, dtype=torch.float32, device=U.device)
+    qn, kn, vv, beta, dec = new(T, H, dk), new(T, H, dk), new(T, H, dv), new(T, H), new(T, H, 1)
+    _check(_lib().illm_lightning_prepare(_p(U), _code(U), U.shape[1], q_off, k_off, v_off, _p(decay), _p(qn), _p(kn),
+                                         _p(vv), _p(beta), _p(dec), T, H, dk, dv, _stream()), "lightning_prepare")
+    return qn, kn, vv, beta, dec
+
+
+def lightning_step(U: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor,
+                   state: torch.Tensor, row_slot: torch.Tensor, H: int, dk: int, dv: int) -> torch.Tensor:
+    """One row a sequence: S <- decay S + k v^T, o = S^T q with q, k, v = silu of U's columns, in one
+    launch.  Returns o float32 [rows, H, dv]."""
+    _gpu(U, decay, state, row_slot)
+    _columns_ok(U, "lightning_step", (q_off, H * dk), (k_off, H * dk), (v_off, H * dv))
+    _decay_ok(decay, state, H, dk, dv, "lightning_step")
+    B = U.shape[0]
+    _i32(row_slot, B)
+    o = torch.empty((B, H, dv), dtype=torch.float32, device=U.device)
+    _check(_lib().illm_lightning_step(_p(U), _code(U), U.shape[1], q_off, k_off, v_off, _p(decay), _p(state),
+                                      _p(row_slot), _p(o), B, H, dk, dv, _stream()), "lightning_step")
+    return o
+
+
+LIGHTNING_CHUNKS_FROM = 64     # rows a sequence from which the chunks run in parallel
+
+
+def lightning_chunks_fits(U: torch.Tensor, q_off: int, k_off: int, v_off: int, dk: int, dv: int) -> bool:
+    return (dk <= 128 and dv <= 128
+            and all(n % 4 == 0 for n in (dk, dv, q_off, k_off, v_off, U.shape[1])))
+
+
+def lightning_chunks(U: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor,
+                     state: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Tensor, n_seqs: int,
+                     max_rows: int, H: int, dk: int, dv: int) -> torch.Tensor:
+    """The same recurrence over every sequence's rows, chunk by chunk in parallel (csrc/fixed_decay.hip):
+    a row's sums run in another order than token by token.  Returns o float32 [T, H, dv]."""
+    _gpu(U, decay, state, cu_seqlens, seq_slot)
+    _i32(cu_seqlens, n_seqs + 1); _i32(seq_slot, n_seqs)
+    _columns_ok(U, "lightning_chunks", (q_off, H * dk), (k_off, H * dk), (v_off, H * dv))
+    _decay_ok(decay, state, H, dk, dv, "lightning_chunks")
+    _need(lightning_chunks_fits(U, q_off, k_off, v_off, dk, dv), "lightning_chunks: sizes not taken")
+    T = U.shape[0]
+    places = T // _lib().illm_lightning_chunk() + n_seqs + 1
+    part = torch.empty((places, H, dk, dv), dtype=torch.float32, device=U.device)
+    o = torch.empty((T, H, dv), dtype=torch.float32, device=U.device)
+    _check(_lib().illm_lightning_chunks(_p(U), _code(U), U.shape[1], q_off, k_off, v_off, _p(decay), _p(state),
+                                        _p(part), _p(cu_seqlens), _p(seq_slot), _p(o), n_seqs, int(max_rows), H,
+                                        dk, dv, _stream()), "lightning_chunks")
+    return o
+
+
+def tanh_columns(U: torch.Tensor, off: int, n: int) -> torch.Tensor:
+    """[T, n]: tanh of U's columns off .. off + n, in U's dtype."""
+    _gpu(U)
+    _columns_ok(U, "tanh_columns", (off, n))
+    out = torch.empty((U.shape[0], n), dtype=U.dtype, device=U.device)
+    _check(_lib().illm_tanh_columns(_p(U), _code(U), U.shape[1], off, _p(out), U.shape[0], n, _stream()), "tanh_columns")
+    return out
+
+
+def _removal_ok(H, d, a_bias, w0, what):
+    _need(all(t.dtype == torch.float32 and t.shape == (H * d,) for t in (a_bias, w0)),
+          f"{what}: a_bias, w0 float32 [H d]")
+
+
+def removal_prepare(U: torch.Tensor, r_off: int, k_off: int, v_off: int, a_off: int, a_bias: torch.Tensor,
+                    Z: torch.Tensor, w0: torch.Tensor, rate: float, H: int, d: int):
+    """Float32 inputs of `delta_scan` with `removal` from U's columns r, k, v and a (H d each) and the
+    decays' pre-activations Z [T, H d]: decay = exp(-rate sigmoid(Z + w0)), beta = 1 / sqrt(sum k^2 +
+    1e-6) a head, removal = sigmoid(a + a_bias) beta k.
+    Returns (r [T, H, d], k, v, beta [T, H], decay [T, H, d], removal [T, H, d])."""
+    _gpu(U, a_bias, Z, w0)
+    _columns_ok(U, "removal_prepare", *((off, H * d) for off in (r_off, k_off, v_off, a_off)))
+    _removal_ok(H, d, a_bias, w0, "removal_prepare")
+    T = U.shape[0]
+    _need(Z.shape == (T, H * d), "removal_prepare: Z [T, H d]")
+    new = lambda *shape: torch.empty(shape, dtype=torch.float32, device=U.device)
+    qn, kn, vv, dec, rem, beta = new(T, H, d), new(T, H, d), new(T, H, d), new(T, H, d), new(T, H, d), new(T, H)
+    _check(_lib().illm_removal_prepare(_p(U), _code(U), U.shape[1], r_off, k_off, v_off, a_off, _p(a_bias), _p(Z),
+                                       _code(Z), Z.shape[1], _p(w0), ctypes.c_float(rate), _p(qn), _p(kn), _p(vv),
+                                       _p(beta), _p(dec), _p(rem), T, H, d, _stream()), "removal_prepare")
+    return qn, kn, vv, beta, dec, rem
+
+
+REMOVAL_STEP_MAX_RANK = 512
+
+
+def removal_step(U: torch.Tensor, r_off: int, k_off: int, v_off: int, a_off: int, a_bias: torch.Tensor,
+                 w1_off: int, w2: torch.Tensor, w0: torch.Tensor, rate: float, state: torch.Tensor,
+                 row_slot: torch.Tensor, H: int, d: int) -> torch.Tensor:
+    """One row a sequence: preparation (Z = w2 tanh(U[:, w1_off ..]), w2 [H d, rank] of U's dtype), the
+    state's update and o = S^T r in one launch.  Returns o float32 [rows, H, d]."""
+    _gpu(U, a_bias, w2, w0, state, row_slot)
+    rank = w2.shape[1]
+    _columns_ok(U, "removal_step", (w1_off, rank), *((off, H * d) for off in (r_off, k_off, v_off, a_off)))
+    _removal_ok(H, d, a_bias, w0, "removal_step")
+    _need(w2.dtype == U.dtype and w2.shape[0] == H * d and 0 < rank <= REMOVAL_STEP_MAX_RANK
+          and state.dtype == torch.float32 and state.dim() == 4 and state.shape[1:] == (H, d, d),
+          "removal_step: w2 [H d, rank] of U's dtype, state float32 [slots, H, d, d]")
+    B = U.shape[0]
+    _i32(row_slot, B)
+    o = torch.empty((B, H, d), dtype=torch.float32, device=U.device)
+    _check(_lib().illm_removal_step(_p(U), _code(U), U.shape[1], r_off, k_off, v_off, a_off, _p(a_bias), w1_off, rank,
+                                    _p(w2), _p(w0), ctypes.c_float(rate), _p(state), _p(row_slot), _p(o), B, H, d,
+                                    _stream()), "removal_step")
+    return o
+
+
+def group_norm_gate(o: torch.Tensor, groups: int, weight: torch.Tensor, Z: torch.Tensor, z_off: int, gate: str,
+                    eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """[T, width] rows o (float32 [T, ..], width numbers each) RMS-normed in `groups` equal parts of the
+    row, times weight [width], times act(Z[:, z_off ..]), act "silu" or "sigmoid"."""
+    _gpu(o, weight, Z)
+    T = o.shape[0]
+    width = weight.numel()
+    _need(o.dtype == torch.float32 and o.numel() == T * width and width % groups == 0 and gate in DELTA_GATES
+          and Z.dim() == 2 and Z.shape[0] == T and z_off + width <= Z.shape[1], "group_norm_gate: shapes or gate")
+    out = torch.empty((T, width), dtype=out_dtype, device=o.device)
+    _check(_lib().illm_group_norm_gate(_p(o), _p(weight), _code(weight), _p(Z), _code(Z), Z.shape[1], z_off,
+                                       DELTA_GATES[gate], _p(out), _code(out), T, width, int(groups),
+                                       ctypes.c_float(eps), _stream()), "group_norm_gate")
     return out
 
 

@@ -1,3 +1,3 @@
-from . import dotorax, kukupel, llama, rabapel, sabipel  # registers Dotorax, Kukupel, LlamaForCausalLM, Rabapel and Sabipel
+from . import dotorax, febivik, kukupel, llama, rabapel, sabipel  # registers Dotorax, Febivik, Kukupel, LlamaForCausalLM, Rabapel and Sabipel
 
-__all__ = ["dotorax", "kukupel", "llama", "rabapel", "sabipel"]
+__all__ = ["dotorax", "febivik", "kukupel", "llama", "rabapel", "sabipel"]

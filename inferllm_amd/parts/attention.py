@@ -255,12 +255,18 @@ class GatedAttention(Mixer):
       b P + P - 1 <= i - window): the means of the block's keys and values as the cache holds them,
       kept beside the keys and values ("kp", "vp": block b in row b of the sequence's pages);
       tokens and blocks share one softmax;
+    * `keep_first` n > 0 (with `window`): a row also sees the sequence's first n tokens, at their true
+      positions; the cache keeps their pages ahead of the window's ring;
+    * `bias`: stored biases of the q, k and v projections;
+    * `qk_norm` "head_weighted": every q and k head passes an RMS norm over its dims (`eps`) with a
+      plain weight [key_dim] that the heads share, before the rotation;
     * `own_kv` False: the layer has no key and value projections and reads the cache line of an
       earlier layer of the step (the schedule names it with `writes_cache` False).
 
     Scores, softmax, norms and the mixing are float32.  A step stores its keys and values in the
     paged cache first and every row attends over the cache at its position, so prompts, portions
-    of prompts and single tokens run the same way.
+    of prompts and single tokens run the same way.  Where the line is a ring of pages, which a long
+    prompt would write round, a step whose sequences all start attends over its own rows instead.
     """
 
     graph_safe_prompts = True
@@ -270,10 +276,17 @@ class GatedAttention(Mixer):
                  value_dim: int, softmax_scale: Optional[float] = None, softcap: float = 0.0,
                  window: Optional[int] = None, chunk: int = 0, slope_power: float = 0.0,
                  qk_norm=False, eps: float = 1e-6, value_mix: Optional[str] = None,
-                 gate=False, head_scale: bool = False, pool: int = 0, own_kv: bool = True, tensors=None):
+                 gate=False, head_scale: bool = False, pool: int = 0, own_kv: bool = True, keep_first: int = 0,
+                 bias: bool = False, tensors=None):
         super().__init__(tensors)
-        if qk_norm not in (False, True, "head") or gate not in (False, True, "head"):
-            raise ValueError(f"gated attention: qk_norm {qk_norm!r} or gate {gate!r}: False, True or 'head'")
+        if qk_norm not in (False, True, "head", "head_weighted") or gate not in (False, True, "head"):
+            raise ValueError(f"gated attention: qk_norm {qk_norm!r} or gate {gate!r}: False, True or 'head' "
+                             "(qk_norm also 'head_weighted')")
+        if int(keep_first or 0) and (not window or pool or chunk):
+            raise ValueError("gated attention: kept first tokens go with a window, without pooled blocks or chunks")
+        if (bias or qk_norm == "head_weighted") and (value_mix or not own_kv):
+            raise ValueError("gated attention: biases and weighted norms a head go with keys and values of the "
+                             "layer's own, not mixed ones")
         if int(pool or 0) and not window:
             raise ValueError("gated attention: pooled blocks lie before a window; `pool` needs `window`")
         if int(pool or 0) and (gate or chunk or softcap or slope_power):
@@ -298,11 +311,12 @@ class GatedAttention(Mixer):
         self.softcap, self.slope_power = float(softcap or 0.0), float(slope_power or 0.0)
         self.qk_norm, self.eps, self.value_mix, self.gate = qk_norm, float(eps), value_mix, gate
         self.has_head_scale, self.pool, self.own_kv = bool(head_scale), int(pool or 0), bool(own_kv)
+        self.keep_first, self.has_bias = int(keep_first or 0), bool(bias)
         self.gate_width = self.nh * (1 if gate == "head" else self.dv)
         self.k_off = self.nh * self.dk
         self.v_off = self.k_off + (self.nkv * self.dk if self.own_kv else 0)
         self.g_off = self.v_off + (self.nkv * self.dv if self.own_kv else 0)
-        self.slopes = self.lam = self.q_norm = self.k_norm = self.head_scale = None
+        self.slopes = self.lam = self.q_norm = self.k_norm = self.head_scale = self.bias = None
 
     def shapes(self) -> Dict[str, TensorWant]:
         keep = dict(keep_stored=True)
@@ -314,6 +328,12 @@ class GatedAttention(Mixer):
         if self.qk_norm is True:
             out["q_norm"] = TensorWant((self.nh * self.dk,), init="ones_normal", **keep)
             out["k_norm"] = TensorWant((self.nkv * self.dk,), init="ones_normal", **keep)
+        if self.qk_norm == "head_weighted":
+            out["q_norm"] = TensorWant((self.dk,), init="ones_normal", **keep)
+            out["k_norm"] = TensorWant((self.dk,), init="ones_normal", **keep)
+        if self.has_bias:
+            out.update(q_bias=TensorWant((self.nh * self.dk,), **keep), k_bias=TensorWant((self.nkv * self.dk,), **keep),
+                       v_bias=TensorWant((self.nkv * self.dv,), **keep))
         if self.value_mix == "mixed":
             out["value_mix"] = TensorWant((), **keep)
         if self.gate:
@@ -329,7 +349,7 @@ class GatedAttention(Mixer):
             return KVSpec("full", (TokenTensor("k", k), TokenTensor("v", v), TokenTensor("kp", k),
                                    TokenTensor("vp", v)))
         return KVSpec("window" if self.window else "full", (TokenTensor("k", k), TokenTensor("v", v)),
-                      self.window)
+                      self.window, self.keep_first)
 
     def load(self, tensors) -> None:
         take = lambda n: self._take(tensors, n)
@@ -337,7 +357,9 @@ class GatedAttention(Mixer):
         self.w_in = ops.decode_weight(_fuse(rows), "plain", self.decode_copies)     # [q | k | v | g]
         self.w_o = ops.decode_weight(take("o").contiguous(), "plain", self.decode_copies)
         dev = take("q").device
-        if self.qk_norm is True:
+        if self.has_bias:
+            self.bias = torch.cat([take(n).to(torch.float32) for n in ("q_bias", "k_bias", "v_bias")]).contiguous()
+        if self.qk_norm in (True, "head_weighted"):
             self.q_norm, self.k_norm = take("q_norm").contiguous(), take("k_norm").contiguous()
         if self.has_head_scale:
             self.head_scale = take("head_scale").to(torch.float32).contiguous()
@@ -359,16 +381,24 @@ class GatedAttention(Mixer):
                              "one without reads a line that an earlier layer of the step stored")
         rows = ops.linear(h, self.w_in)
         store = writes_cache
-        if position is not None or self.qk_norm == "head":
-            # rotation, the norm a head and the store in one pass over the rows
+        weighted = self.qk_norm == "head_weighted"
+        if position is not None or self.qk_norm == "head" or weighted or self.has_bias:
+            # biases, norms a head, rotation and the store in one pass over the rows
             table = position.table(ctx.device) if position is not None else None
             ops.qk_rotate_store(rows, self.k_off, self.v_off, table,
                                 position.rotary_dim if position is not None else 0,
                                 0 if position is None or position.pairing == "half" else 1,
                                 self.qk_norm == "head", self.eps, ctx.row_pos, ctx.row_slot,
                                 kc if store else None, vc if store else None, group.table, group.page_size,
-                                group.ring, nh, nkv if self.own_kv else 0, dk, dv, q_scale=self.head_scale)
+                                group.ring, nh, nkv if self.own_kv else 0, dk, dv, q_scale=self.head_scale,
+                                bias=self.bias, q_weight=self.q_norm if weighted else None,
+                                k_weight=self.k_norm if weighted else None,
+                                slot_len=ctx.cache.slot_len if ctx.prefill and group.ring else None,
+                                kept=group.kept_pages)
         else:
+            if group.ring:
+                raise ValueError("gated attention: a window whose line is a ring of pages needs the store that "
+                                 "rotates, norms a head or adds biases")
             first, first_off = None, 0
             if self.value_mix == "mixed":
                 first, first_off, width = ctx.exchange["value_mix_source"]
@@ -398,14 +428,15 @@ class GatedAttention(Mixer):
             o = ops.attn_cap_rows(rows, ctx.cu_seqlens, ctx.seq_slot, ctx.seq_start, kc, vc, group.table,
                                   group.page_size, group.ring, ctx.n_seqs, ctx.max_rows, nh, nkv, dk, dv,
                                   self.scale, self.softcap, window, self.slopes, self.chunk, gate, self.g_off,
-                                  by_head, lse)
+                                  by_head, lse, keep=self.keep_first, kept=group.kept_pages,
+                                  own=(self.k_off, self.v_off) if group.ring and not ctx.continues else None)
             if lse is not None:
                 ops.attn_pooled_rows(rows, ctx.cu_seqlens, ctx.seq_slot, ctx.seq_start, kc, vc, kp, vp,
                                      group.table, group.page_size, ctx.n_seqs, ctx.max_rows, nh, nkv, dk, dv,
                                      self.scale, None, window, self.pool, out=o, lse=lse)
         else:
             longest = ctx.max_len
-            for bound in (window, self.chunk):
+            for bound in (window + self.keep_first if window else 0, self.chunk):
                 longest = min(longest, bound) if bound else longest
             tiles = max(1, (longest + 63) // 64)
             # a block takes up to four query heads of a kv head; enough blocks for two a compute unit
@@ -416,7 +447,8 @@ class GatedAttention(Mixer):
                 nsplit = max(nsplit, 2)              # the kernel that merges the ranges writes `lse`
             o = ops.attn_cap_decode(rows, kc, vc, group.table, group.page_size, group.ring, ctx.seq_slot,
                                     ctx.seq_len, nh, nkv, dk, dv, self.scale, self.softcap, window,
-                                    nsplit, self.slopes, self.chunk, gate, self.g_off, by_head, lse)
+                                    nsplit, self.slopes, self.chunk, gate, self.g_off, by_head, lse,
+                                    keep=self.keep_first, kept=group.kept_pages)
             if lse is not None:
                 ops.attn_pooled_decode(rows, kc, vc, kp, vp, group.table, group.page_size, ctx.seq_slot,
                                        ctx.seq_len, nh, nkv, dk, dv, self.scale, None, window, self.pool,

@@ -165,7 +165,7 @@ class SandwichBlock(Block):
         if isinstance(pending, ops.NormedRows):
             pending = None                       # its sum is in x already
         params = norm.rms_params()
-        plain = pending is None or isinstance(pending, ops.PostNormed)
+        plain = pending is None or (isinstance(pending, ops.PostNormed) and pending.kind == "rms")
         if (params is not None and plain and not ctx.prefill and self.taps > 1
                 and self.size <= ops.POST_ADD_MAX_WIDTH):
             return ops.post_add_rmsnorm(x, pending, params[0], params[1], ctx.act_dtype,
@@ -187,6 +187,40 @@ class SandwichBlock(Block):
             return self._leave(a, 1, next_norm)
         h2 = self._enter(self.feed_forward_norm, 2, x, self._leave(a, 1, self.feed_forward_norm), ctx)
         return self._leave(self.feed_forward.forward(h2, ctx), 2, next_norm)
+
+
+@register_part("block", "post_norm")
+class PostNormBlock(Block):
+    """x <- x + norm1(mixer(x)); x <- x + norm2(feed_forward(x)): a norm behind each sublayer and none
+    in front; the sublayers read the stream itself (rounded to the engine's dtype).
+
+    The norms are parts that give the norm of a sublayer's output as pieces (`post(y)`: `rms_norm`,
+    `layer_norm`).  Between two sublayers there is one pass over the rows: the norm of the first one's
+    output, the sum, the rows for the second one (`ops.post_add_norm`).  A layer whose feed-forward is
+    "none" has no second norm.
+    """
+
+    graph_safe_prompts = True
+
+    takes_next_norm = True           # to hand a norm that forms a sublayer's own norm the pieces
+    takes_prepared_rows = True       # (prepared rows mean: the sum is in x already)
+
+    @staticmethod
+    def _read(x, pending, ctx: StepContext):
+        """The stream with `pending` added, as the next sublayer reads it."""
+        if isinstance(pending, ops.NormedRows):
+            pending = None                       # its sum is in x already
+        if isinstance(pending, tuple):
+            pending = ops.sum_rows(*pending)
+        return ops.post_add_norm(x, pending, None, None, None, 0.0, ctx.act_dtype)
+
+    def forward(self, x, pending, ctx: StepContext, line, writes_cache, next_norm=None):
+        h = self._read(x, pending, ctx)
+        post = self.mixer_norm.post(self.mixer.forward(h, ctx, line, writes_cache, self.position))
+        if self.feed_forward_norm is not None:
+            h = self._read(x, post, ctx)
+            post = self.feed_forward_norm.post(self.feed_forward.forward(h, ctx))
+        return post if next_norm is not None and getattr(next_norm, "adds_post_normed", False) else post.tensor()
 
 
 @register_part("block", "hyper_connections")

@@ -70,13 +70,14 @@ class NoFeedForward(FeedForward):
 
 
 # activation -> the op that computes it
-_ACTIVATIONS = {"relu_squared": "relu_squared", "gelu_tanh": "gelu_tanh"}
+_ACTIVATIONS = {"relu_squared": "relu_squared", "gelu_tanh": "gelu_tanh", "xielu": "xielu"}
 
 
 @register_part("feed_forward", "dense_activation")
 class DenseActivation(FeedForward):
-    """down(act(up h)) without a gate; `activation` "relu_squared": max(z, 0)^2, or "gelu_tanh":
-    0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))."""
+    """down(act(up h)) without a gate; `activation` "relu_squared": max(z, 0)^2, "gelu_tanh":
+    0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), or "xielu" with two stored numbers `act` =
+    (p, q): softplus(p) z^2 + z / 2 for z > 0, (1/2 + softplus(q)) (e^z - 1 - z) + z / 2 else."""
 
     graph_safe_prompts = True
 
@@ -86,21 +87,28 @@ class DenseActivation(FeedForward):
         if activation not in _ACTIVATIONS:
             raise ValueError(f"unknown activation {activation!r}; known: {sorted(_ACTIVATIONS)}")
         self.E, self.F, self.activation = int(hidden_size), int(intermediate_size), activation
-        self.w_up = self.w_down = None
+        self.w_up = self.w_down = self.act = None
 
     def shapes(self) -> Dict[str, TensorWant]:
-        return {"up": TensorWant((self.F, self.E)), "down": TensorWant((self.E, self.F))}
+        out = {"up": TensorWant((self.F, self.E)), "down": TensorWant((self.E, self.F))}
+        if self.activation == "xielu":
+            out["act"] = TensorWant((2,), init="normal", keep_stored=True)
+        return out
 
     def load(self, tensors) -> None:
         self.w_up = ops.decode_weight(self._take(tensors, "up").contiguous(), "plain", self.decode_copies)
         self.w_down = ops.decode_weight(self._take(tensors, "down").contiguous(), "plain", self.decode_copies)
+        if self.activation == "xielu":
+            pq = torch.nn.functional.softplus(self._take(tensors, "act").to(torch.float64))
+            self.act = (pq + torch.tensor([0.0, 0.5], dtype=torch.float64, device=pq.device)).to(torch.float32)
 
     def tunables(self):
         return (("plain", self.w_down, {}),)
 
     def forward(self, h, ctx: StepContext):
         act = getattr(ops, _ACTIVATIONS[self.activation])
-        return ops.linear(act(ops.linear(h, self.w_up)), self.w_down)
+        z = ops.linear(h, self.w_up)
+        return ops.linear(act(z) if self.act is None else act(z, self.act), self.w_down)
 
 
 @register_part("feed_forward", "clamped_gated")
@@ -136,7 +144,7 @@ class ClampedGated(FeedForward):
 
 @register_part("feed_forward", "routed_experts")
 class RoutedExperts(FeedForward):
-    """A mixture of gated experts, of which every token uses `top`.
+    """A mixture of experts, of which every token uses `top`.
 
         s = softmax(W_router h) over `num_experts` real experts followed by `num_identity`
             identity experts (float32)
@@ -152,6 +160,9 @@ class RoutedExperts(FeedForward):
     all.  `activation` "clamped_swish" with `limit`: g = min(W_gate h, limit), u = clamp(W_up h,
     -limit, limit), expert(h) = W_down (g sigmoid(1.702 g) (u + 1)).  `weight_on` "input": the
     weight multiplies what the expert reads, out = sum over chosen e of expert_e(s_e h).
+    `activation` "relu_squared": experts (and the shared one) without a gate, expert(h) =
+    W_down max(W_up h, 0)^2, and no ".gate" tensors.  `router_scale`: the weights are that times the
+    chosen scores.
     Tensor parameters: "router", "correction", "e<i>.gate" / ".up" / ".down", "shared.gate" /
     ".up" / ".down", "shared.sg".  The result is float32.
     """
@@ -161,7 +172,7 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int,
                  num_identity: int = 0, correction: bool = True, shared_size: int = 0,
                  shared_gate: bool = True, score: str = "softmax", activation: str = "silu",
-                 limit: float = 0.0, weight_on: str = "output", tensors=None):
+                 limit: float = 0.0, weight_on: str = "output", router_scale: float = 1.0, tensors=None):
         super().__init__(tensors)
         if score not in ops.MOE_SCORES or activation not in ops.MOE_ACTIVATIONS:
             raise ValueError(f"routed experts: score {score!r} or activation {activation!r} is unknown; "
@@ -173,6 +184,7 @@ class RoutedExperts(FeedForward):
         if weight_on == "input" and int(num_identity):
             raise ValueError("routed experts: identity experts take their weight on the output")
         self.score, self.activation, self.limit, self.weight_on = score, activation, float(limit), weight_on
+        self.gated, self.router_scale = activation not in ops.MOE_PLAIN_ACTIVATIONS, float(router_scale)
         self.E, self.F = int(hidden_size), int(expert_size)
         self.n_real, self.n_id, self.top = int(num_experts), int(num_identity), int(top)
         self.has_correction, self.Fs = bool(correction), int(shared_size)
@@ -192,11 +204,13 @@ class RoutedExperts(FeedForward):
         if self.has_correction:
             out["correction"] = TensorWant((self.n_real + self.n_id,), keep_stored=True)
         for i in range(self.n_real):
-            out[f"e{i}.gate"] = TensorWant((self.F, self.E))
+            if self.gated:
+                out[f"e{i}.gate"] = TensorWant((self.F, self.E))
             out[f"e{i}.up"] = TensorWant((self.F, self.E))
             out[f"e{i}.down"] = TensorWant((self.E, self.F))
         if self.Fs:
-            out["shared.gate"] = TensorWant((self.Fs, self.E))
+            if self.gated:
+                out["shared.gate"] = TensorWant((self.Fs, self.E))
             out["shared.up"] = TensorWant((self.Fs, self.E))
             out["shared.down"] = TensorWant((self.E, self.Fs))
             if self.has_shared_gate:
@@ -208,12 +222,14 @@ class RoutedExperts(FeedForward):
         self.w_router = take("router").to(torch.float32).contiguous()      # the router runs in float32
         self.correction = take("correction").contiguous() if self.has_correction else None
         if self.n_real:
-            self.w_gate_up = torch.stack([torch.cat([take(f"e{i}.gate"), take(f"e{i}.up")], dim=0)
+            parts = ("gate", "up") if self.gated else ("up",)
+            self.w_gate_up = torch.stack([torch.cat([take(f"e{i}.{t}") for t in parts], dim=0)
                                           for i in range(self.n_real)]).contiguous()
             self.w_down = torch.stack([take(f"e{i}.down") for i in range(self.n_real)]).contiguous()
         if self.Fs:
-            self.w_shared_gate_up = ops.decode_weight(_fuse([take("shared.gate"), take("shared.up")]),
-                                                      "gate_up", self.decode_copies)
+            self.w_shared_gate_up = (
+                ops.decode_weight(_fuse([take("shared.gate"), take("shared.up")]), "gate_up", self.decode_copies)
+                if self.gated else ops.decode_weight(take("shared.up").contiguous(), "plain", self.decode_copies))
             self.w_shared_down = ops.decode_weight(take("shared.down").contiguous(), "plain",
                                                    self.decode_copies)
             if self.has_shared_gate:
@@ -221,7 +237,7 @@ class RoutedExperts(FeedForward):
 
     def forward(self, h, ctx: StepContext):
         idx, weight, grouped = ops.moe_plan(h, self.w_router, self.correction, self.top,
-                                            self.w_gate_up, self.score)
+                                            self.w_gate_up, self.score, self.router_scale, self.gated)
         on_input = self.weight_on == "input"
         y = (ops.moe_experts(h, idx, self.w_gate_up, self.w_down, grouped, self.activation, self.limit,
                              weight if on_input else None) if self.n_real else None)
@@ -229,5 +245,7 @@ class RoutedExperts(FeedForward):
             weight = None                        # the experts' rows are summed as they are
         shared = None
         if self.Fs:
-            shared = ops.linear(ops.gate_up_silu(h, self.w_shared_gate_up), self.w_shared_down)
+            inner = (ops.gate_up_silu(h, self.w_shared_gate_up) if self.gated
+                     else ops.relu_squared(ops.linear(h, self.w_shared_gate_up)))
+            shared = ops.linear(inner, self.w_shared_down)
         return ops.moe_combine(h, idx, weight, y, self.n_real, shared, self.w_sg)

@@ -1,4 +1,4 @@
-"""RMS norm fused with the residual add that precedes it."""
+"""Norms fused with the residual add that precedes them."""
 from __future__ import annotations
 
 from typing import Dict, Optional
@@ -50,10 +50,16 @@ class RMSNorm(Norm):
 
     def forward(self, x, delta, ctx: StepContext, row_idx=None):
         if isinstance(delta, ops.PostNormed):
+            if delta.kind != "rms":
+                return ops.post_add_norm(x, delta, "rms", self.weight, None, self.eps, ctx.act_dtype, row_idx)
             if self.size <= ops.POST_ADD_MAX_WIDTH:
                 return ops.post_add_rmsnorm(x, delta, self.weight, self.eps, ctx.act_dtype, row_idx)
             delta = delta.tensor()
         return ops.add_rmsnorm(x, delta, self.weight, self.eps, ctx.act_dtype, row_idx)
+
+    def post(self, y) -> ops.PostNormed:
+        """The norm of a sublayer's output `y`, as pieces that whoever adds it to the stream forms."""
+        return ops.PostNormed(y, self.weight, self.eps, 1.0)
 
     def forward_with(self, other: "RMSNorm", x, delta, ctx: StepContext):
         """(this norm's rows, `other`'s rows) of the same x (+ delta) in one pass, or None if the two
@@ -62,6 +68,38 @@ class RMSNorm(Norm):
                 or other.weight.dtype != self.weight.dtype):
             return None
         return ops.add_rmsnorm(x, delta, self.weight, self.eps, ctx.act_dtype, weight2=other.weight)
+
+
+@register_part("norm", "layer_norm")
+class LayerNorm(Norm):
+    """y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight + bias, statistics in float32.
+    `bias` False: no bias."""
+
+    graph_safe_prompts = True
+    adds_post_normed = True          # (see RMSNorm)
+
+    def __init__(self, size: int, eps: float, bias: bool = True, tensors=None):
+        super().__init__(tensors)
+        self.size, self.eps, self.has_bias = int(size), float(eps), bool(bias)
+        self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
+
+    def shapes(self) -> Dict[str, TensorWant]:
+        out = {"weight": TensorWant((self.size,), init="ones_normal", keep_stored=True)}
+        if self.has_bias:
+            out["bias"] = TensorWant((self.size,), init="normal", keep_stored=True)
+        return out
+
+    def load(self, tensors) -> None:
+        self.weight = self._take(tensors, "weight").contiguous()
+        if self.has_bias:
+            self.bias = self._take(tensors, "bias").to(self.weight.dtype).contiguous()
+
+    def post(self, y) -> ops.PostNormed:
+        return ops.PostNormed(y, self.weight, self.eps, 1.0, "layer", self.bias)
+
+    def forward(self, x, delta, ctx: StepContext, row_idx=None):
+        return ops.post_add_norm(x, delta, "layer", self.weight, self.bias, self.eps, ctx.act_dtype, row_idx)
 
 
 @register_part("norm", "stream_rms_norm")

@@ -19,11 +19,14 @@ def scaled_frequencies(theta: float, rotary_dim: int, scaling: Optional[dict]):
     slow}.  d(n) = rotary_dim * ln(original / (2 pi n)) / (2 ln theta) is the (fractional) pair
     count at which a wave makes n turns over `original` positions; between lo = floor(d(fast)) and
     hi = ceil(d(slow)) the frequency goes linearly from f to f / factor, and cos and sin are
-    multiplied by 0.1 ln(factor) + 1."""
+    multiplied by 0.1 ln(factor) + 1.  `scaling` = {factor} alone: linear scaling, every frequency
+    divided by it and the gain 1."""
     i = torch.arange(rotary_dim // 2, dtype=torch.float64)
     f = torch.pow(torch.tensor(float(theta), dtype=torch.float64), -2.0 * i / rotary_dim)
     if not scaling:
         return f, 1.0
+    if set(scaling) == {"factor"}:
+        return f / float(scaling["factor"]), 1.0
     factor, original = float(scaling["factor"]), float(scaling["original"])
 
     def pairs_at(turns: float) -> float:
@@ -63,7 +66,7 @@ class Rotary(PositionEncoding):
     LLaMA-2 graph's RotMode::ModelRotHalf); "interleaved": pairs (2i, 2i+1)
     (naive.cpp:415-440).  theta, rotary_dim and max_positions are parameters; `scaling`
     ({factor, original, fast, slow}, see `scaled_frequencies`) stretches the slow pairs for
-    contexts longer than `original`.
+    contexts longer than `original`, or ({factor} alone) all pairs alike.
     """
 
     graph_safe_prompts = True
@@ -77,7 +80,10 @@ class Rotary(PositionEncoding):
             raise ValueError(f"rotary_dim {rotary_dim} must be even and within head_dim {head_dim}")
         self.head_dim, self.rotary_dim = int(head_dim), int(rotary_dim)
         self.theta, self.pairing, self.max_positions = float(theta), pairing, int(max_positions)
-        if scaling:
+        if scaling and set(scaling) == {"factor"}:
+            if not float(scaling["factor"]) > 0:
+                raise ValueError(f"rotary scaling needs a positive factor: {scaling!r}")
+        elif scaling:
             lacking = [k for k in ("factor", "original", "fast", "slow") if k not in scaling]
             if lacking or not float(scaling["factor"]) > 0 or not float(scaling["original"]) > 0:
                 raise ValueError(f"rotary scaling needs positive factor and original, and fast and slow: {scaling!r}")

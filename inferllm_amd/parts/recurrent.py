@@ -1,10 +1,12 @@
 """Mixers that keep a matrix of state per head and update it by the plain gated rule
 S <- g S + k (w v)^T, o = S^T q: a state-space mixer with a scalar decay a head, and a matrix
 memory with exponential gates; gated linear attention, which is that rule with a decay per key
-channel; and a gated linear recurrent unit, whose state is one number a channel."""
+channel; lightning attention, with one fixed decay a head; the delta rule with a removal vector of
+its own; and a gated linear recurrent unit, whose state is one number a channel."""
 from __future__ import annotations
 
-from typing import Dict
+import math
+from typing import Dict, Sequence
 
 import torch
 
@@ -230,6 +232,148 @@ class GatedLinearAttention(Mixer):
         o = ops.delta_scan(qn, kn, vv, weight, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
                            ctx.max_rows if ctx.prefill else 1, correct=False)
         y = ops.delta_finish(o, self.norm_w, U, self.g_off, "silu", self.eps, ctx.act_dtype)
+        return ops.linear(y, self.w_o)
+
+
+@register_part("mixer", "lightning_attention")
+class LightningAttention(Mixer):
+    """Per head a matrix of state S [key_dim, value_dim] with one fixed decay:
+
+        q = silu(W_q h),  k = silu(W_k h),  v = silu(W_v h)
+        S <- decay_h S + k v^T;   o = S^T q
+        out = W_o (o / rms(o) * norm * sigmoid(W_g h))
+
+    rms over all heads' outputs side by side (`eps`), `norm` of that width.  Kept per sequence: S
+    (float32).  A step goes on from whatever the slot holds: single tokens in one launch, many rows
+    a sequence in chunks.  The recurrence is float32; the projections take the engine's dtype.
+    """
+
+    graph_safe_prompts = True
+    takes_continuations = True
+
+    def __init__(self, hidden_size: int, num_heads: int, key_dim: int, value_dim: int, decay: Sequence[float],
+                 eps: float, tensors=None):
+        super().__init__(tensors)
+        if key_dim > 256:
+            raise ValueError(f"lightning attention: a key size of {key_dim} is beyond the kernels' limit of 256")
+        if len(decay) != int(num_heads) or any(not 0.0 <= float(g) <= 1.0 for g in decay):
+            raise ValueError(f"lightning attention: one decay in [0, 1] for each of {num_heads} heads, got {decay!r}")
+        self.E, self.H, self.dk, self.dv = int(hidden_size), int(num_heads), int(key_dim), int(value_dim)
+        self.eps, self.decay_values, self.decay = float(eps), [float(g) for g in decay], None
+
+    def shapes(self) -> Dict[str, TensorWant]:
+        E, H, dk, dv = self.E, self.H, self.dk, self.dv
+        return {"q": TensorWant((H * dk, E)), "k": TensorWant((H * dk, E)), "v": TensorWant((H * dv, E)),
+                "g": TensorWant((H * dv, E)), "o": TensorWant((E, H * dv)),
+                "norm": TensorWant((H * dv,), init="ones_normal", keep_stored=True)}
+
+    def state_spec(self):
+        return {"S": StateSpec((self.H, self.dk, self.dv), torch.float32)}
+
+    def load(self, tensors) -> None:
+        take = lambda n: self._take(tensors, n)
+        H, dk, dv = self.H, self.dk, self.dv
+        # one product for everything that reads h: [q | k | v | g]
+        self.w_in = ops.decode_weight(_fuse([take(n) for n in ("q", "k", "v", "g")]), "plain", self.decode_copies)
+        self.k_off, self.v_off = H * dk, 2 * H * dk
+        self.g_off = self.v_off + H * dv
+        self.norm_w = take("norm").contiguous()
+        self.decay = torch.tensor(self.decay_values, dtype=torch.float32, device=self.norm_w.device)
+        self.w_o = ops.decode_weight(take("o").contiguous(), "plain", self.decode_copies)
+
+    def tunables(self):
+        return (("plain", self.w_o, {}),)
+
+    def forward(self, h, ctx: StepContext, line, writes_cache, position):
+        H, dk, dv = self.H, self.dk, self.dv
+        U = ops.linear(h, self.w_in)
+        S = ctx.cache.state_line(line)["S"]
+        cols = (0, self.k_off, self.v_off)
+        if not ctx.prefill:
+            o = ops.lightning_step(U, *cols, self.decay, S, ctx.row_slot, H, dk, dv)
+        elif ctx.max_rows >= ops.LIGHTNING_CHUNKS_FROM and ops.lightning_chunks_fits(U, *cols, dk, dv):
+            o = ops.lightning_chunks(U, *cols, self.decay, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
+                                     ctx.max_rows, H, dk, dv)
+        else:
+            qn, kn, vv, weight, dec = ops.lightning_prepare(U, *cols, self.decay, H, dk, dv)
+            o = ops.delta_scan(qn, kn, vv, weight, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
+                               ctx.max_rows, correct=False)
+        y = ops.group_norm_gate(o, 1, self.norm_w, U, self.g_off, "sigmoid", self.eps, ctx.act_dtype)
+        return ops.linear(y, self.w_o)
+
+
+# decay = exp(-rate sigmoid(z)): the rule fixes the rate, so a channel keeps at least exp(-rate) a token
+REMOVAL_DECAY_RATE = math.exp(-0.5)
+
+
+@register_part("mixer", "removal_delta_rule")
+class RemovalDeltaRule(Mixer):
+    """A generalized delta rule: per head a matrix of state S [dim, dim] whose decay, removal and
+    writing each have a vector of their own:
+
+        r = W_r h,  k = W_k h,  v = W_v h,   u = k / sqrt(sum k^2 + 1e-6) a head
+        w = exp(-exp(-1/2) sigmoid(W_w2 tanh(W_w1 h) + w0)),   a = sigmoid(W_a h + b_a)     a head and channel
+        S <- diag(w) S - (a u) (u^T S) + k v^T   (both terms from the old S);   o = S^T r
+        out = W_o (o / rms(o) * norm * sigmoid(W_g h))
+
+    rms over each head's outputs (`eps`), `norm` of all heads' width.  Kept per sequence: S (float32).
+    A step goes on from whatever the slot holds, single tokens in one launch.  Decays, rates, unit
+    keys and the state are float32; the projections take the engine's dtype.
+    """
+
+    graph_safe_prompts = True
+    takes_continuations = True
+
+    def __init__(self, hidden_size: int, num_heads: int, dim: int, decay_rank: int, eps: float, tensors=None):
+        super().__init__(tensors)
+        if dim > 256:
+            raise ValueError(f"removal delta rule: a head size of {dim} is beyond the kernels' limit of 256")
+        if int(decay_rank) <= 0:
+            raise ValueError("removal delta rule: the decays' rank must be positive")
+        self.E, self.H, self.d, self.rank, self.eps = int(hidden_size), int(num_heads), int(dim), int(decay_rank), float(eps)
+
+    def shapes(self) -> Dict[str, TensorWant]:
+        E, n, R = self.E, self.H * self.d, self.rank
+        keep = dict(keep_stored=True)
+        return {"r": TensorWant((n, E)), "k": TensorWant((n, E)), "v": TensorWant((n, E)), "g": TensorWant((n, E)),
+                "a": TensorWant((n, E)), "a_bias": TensorWant((n,), **keep), "w1": TensorWant((R, E)),
+                "w2": TensorWant((n, R)), "w0": TensorWant((n,), **keep),
+                "norm": TensorWant((n,), init="ones_normal", **keep), "o": TensorWant((E, n))}
+
+    def state_spec(self):
+        return {"S": StateSpec((self.H, self.d, self.d), torch.float32)}
+
+    def load(self, tensors) -> None:
+        take = lambda n: self._take(tensors, n)
+        f32 = lambda n: take(n).to(torch.float32).contiguous()
+        n = self.H * self.d
+        # one product for everything that reads h: [r | k | v | a | g | w1]
+        self.w_in = ops.decode_weight(_fuse([take(t) for t in ("r", "k", "v", "a", "g", "w1")]), "plain",
+                                      self.decode_copies)
+        self.k_off, self.v_off, self.a_off, self.g_off, self.w1_off = n, 2 * n, 3 * n, 4 * n, 5 * n
+        self.w2_rows = take("w2").to(ops.plain_weight(self.w_in).dtype).contiguous()
+        self.w_w2 = ops.decode_weight(self.w2_rows, "plain", self.decode_copies)
+        self.a_bias, self.w0, self.norm_w = f32("a_bias"), f32("w0"), take("norm").contiguous()
+        self.w_o = ops.decode_weight(take("o").contiguous(), "plain", self.decode_copies)
+
+    def tunables(self):
+        return (("plain", self.w_o, {}),)
+
+    def forward(self, h, ctx: StepContext, line, writes_cache, position):
+        H, d = self.H, self.d
+        U = ops.linear(h, self.w_in)
+        S = ctx.cache.state_line(line)["S"]
+        cols = (0, self.k_off, self.v_off, self.a_off)
+        if not ctx.prefill and self.rank <= ops.REMOVAL_STEP_MAX_RANK and self.w2_rows.dtype == U.dtype:
+            o = ops.removal_step(U, *cols, self.a_bias, self.w1_off, self.w2_rows, self.w0, REMOVAL_DECAY_RATE, S,
+                                 ctx.row_slot, H, d)
+        else:
+            Z = ops.linear(ops.tanh_columns(U, self.w1_off, self.rank), self.w_w2)
+            rn, kn, vv, beta, dec, removal = ops.removal_prepare(U, *cols, self.a_bias, Z, self.w0, REMOVAL_DECAY_RATE,
+                                                                 H, d)
+            o = ops.delta_scan(rn, kn, vv, beta, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
+                               ctx.max_rows if ctx.prefill else 1, correct=False, removal=removal)
+        y = ops.group_norm_gate(o, H, self.norm_w, U, self.g_off, "sigmoid", self.eps, ctx.act_dtype)
         return ops.linear(y, self.w_o)
 
 

@@ -51,10 +51,10 @@ def silu_mul(gate_up):
     return (g / (1.0 + torch.exp(-g)) * u).to(gate_up.dtype)
 
 
-def cache_offsets(page_table, slot, pos, page_size, ring):
+def cache_offsets(page_table, slot, pos, page_size, ring, kept=0):
     lp = pos // page_size
-    if ring > 0:
-        lp = lp % ring
+    if ring > 0 and lp >= kept:
+        lp = kept + (lp - kept) % ring
     return int(page_table[slot, lp]), pos % page_size
 
 
@@ -376,15 +376,15 @@ def few_outputs_f32(x, w):
     return (x.to(F64) @ w.to(F64).t()).to(torch.float32)
 
 
-def moe_route(z, correction, top, score="softmax"):
+def moe_route(z, correction, top, score="softmax", scale=1.0):
     s = torch.softmax(z.to(F64), dim=-1) if score == "softmax" else torch.sigmoid(z.to(F64))
     pick = s + correction.to(F64) if correction is not None else s
     idx = torch.topk(pick, top, dim=-1).indices
-    return idx.to(torch.int32), torch.gather(s, 1, idx).to(torch.float32)
+    return idx.to(torch.int32), (scale * torch.gather(s, 1, idx)).to(torch.float32)
 
 
-def moe_plan(h, w_router, correction, top, w_gate_up, score="softmax"):
-    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score)
+def moe_plan(h, w_router, correction, top, w_gate_up, score="softmax", scale=1.0, gated=True):
+    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score, scale)
     return idx, wt, None
 
 
@@ -398,7 +398,9 @@ def moe_experts(h, idx, w_gate_up, w_down, grouped=None, activation="silu", limi
             if e < w_gate_up.shape[0]:
                 x = h[t].to(F64) * (input_weight[t, k].to(F64) if input_weight is not None else 1.0)
                 gu = w_gate_up[e].to(F64) @ x
-                if activation == "silu":
+                if activation == "relu_squared":
+                    a = torch.clamp(gu, min=0) ** 2          # an up matrix alone
+                elif activation == "silu":
                     a = torch.nn.functional.silu(gu[:F]) * gu[F:]
                 else:
                     g, u = torch.clamp(gu[:F], max=limit), torch.clamp(gu[F:], -limit, limit)
@@ -441,9 +443,11 @@ def scaled_sum_tensor(self):
 
 
 # ---------------------------------------------------------------- attention with a soft cap
-def kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv):
+def kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv,
+              kept=0):
+    # (rows in order: of two that land on one place of a ring the later one stays)
     for r in range(rows.shape[0]):
-        page, at = cache_offsets(page_table, int(row_slot[r]), int(row_pos[r]), page_size, ring)
+        page, at = cache_offsets(page_table, int(row_slot[r]), int(row_pos[r]), page_size, ring, kept)
         kcache[page, :, at, :] = rows[r, k_off:k_off + nkv * dk].view(nkv, dk)
         vcache[page, :, at, :] = rows[r, v_off:v_off + nkv * dv].view(nkv, dv)
 
@@ -495,21 +499,27 @@ def qkv_norm_mix_store(rows, k_off, v_off, q_weight, k_weight, eps, lam, first, 
         kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv)
 
 
-def _cached(kcache, vcache, page_table, slot, first, total, page_size, ring):
-    at = [cache_offsets(page_table, slot, pos, page_size, ring) for pos in range(first, total)]
+def _cached(kcache, vcache, page_table, slot, first, total, page_size, ring, keep=0, kept=0):
+    seen = list(range(min(keep, first))) + list(range(first, total))
+    at = [cache_offsets(page_table, slot, pos, page_size, ring, kept) for pos in seen]
     return (torch.stack([kcache[p, :, r, :] for p, r in at]), torch.stack([vcache[p, :, r, :] for p, r in at]))
 
 
 def attn_cap_rows(q, cu_seqlens, seq_slot, seq_start, kcache, vcache, page_table, page_size, ring,
                   n_seqs, max_rows, nh, nkv, dk, dv, scale, cap, window, slopes=None, chunk=0, gate=None,
-                  gate_off=0, gate_heads=False, lse=None):
+                  gate_off=0, gate_heads=False, lse=None, keep=0, kept=0, own=None):
     out = torch.zeros(q.shape[0], nh * dv, dtype=q.dtype)
     for b in range(n_seqs):
         s0, s1 = int(cu_seqlens[b]), int(cu_seqlens[b + 1])
         for a in range(s1 - s0):
             pos = int(seq_start[b]) + a
             first = _first_seen(pos, window, chunk)
-            k, v = _cached(kcache, vcache, page_table, int(seq_slot[b]), first, pos + 1, page_size, ring)
+            if own is None:
+                k, v = _cached(kcache, vcache, page_table, int(seq_slot[b]), first, pos + 1, page_size, ring, keep, kept)
+            else:
+                seen = [s0 + j for j in list(range(min(keep, first))) + list(range(first, pos + 1))]
+                k = q[seen, own[0]:own[0] + nkv * dk].view(-1, nkv, dk)
+                v = q[seen, own[1]:own[1] + nkv * dv].view(-1, nkv, dv)
             row = _attend_capped(q[s0 + a, :nh * dk].view(nh, dk), k, v, scale, cap, slopes,
                                  lse[s0 + a] if lse is not None else None).reshape(-1)
             out[s0 + a] = _gated(row, gate, s0 + a, gate_off, nh if gate_heads else 0).to(q.dtype)
@@ -518,12 +528,12 @@ def attn_cap_rows(q, cu_seqlens, seq_slot, seq_start, kcache, vcache, page_table
 
 def attn_cap_decode(q, kcache, vcache, page_table, page_size, ring, seq_slot, seq_len, nh, nkv, dk, dv,
                     scale, cap, window, nsplit, slopes=None, chunk=0, gate=None, gate_off=0, gate_heads=False,
-                    lse=None):
+                    lse=None, keep=0, kept=0):
     out = torch.zeros(q.shape[0], nh * dv, dtype=q.dtype)
     for b in range(q.shape[0]):
         n = int(seq_len[b])
         first = _first_seen(n - 1, window, chunk)
-        k, v = _cached(kcache, vcache, page_table, int(seq_slot[b]), first, n, page_size, ring)
+        k, v = _cached(kcache, vcache, page_table, int(seq_slot[b]), first, n, page_size, ring, keep, kept)
         row = _attend_capped(q[b, :nh * dk].view(nh, dk), k, v, scale, cap, slopes,
                              lse[b] if lse is not None else None).reshape(-1)
         out[b] = _gated(row, gate, b, gate_off, nh if gate_heads else 0).to(q.dtype)
@@ -573,7 +583,7 @@ def delta_conv_tail(P, tail, cu_seqlens, seq_slot, n_seqs, taps, col_off=0):
             tail[slot, j] = P[r0 + at, :C].to(tail.dtype) if at >= 0 else old[j + n]
 
 
-def delta_scan(qn, kn, vv, beta, dec, state, cu_seqlens, seq_slot, n_seqs, max_rows, correct=True):
+def delta_scan(qn, kn, vv, beta, dec, state, cu_seqlens, seq_slot, n_seqs, max_rows, correct=True, removal=None):
     T, G, dk = qn.shape
     H, dv = vv.shape[1], vv.shape[2]
     o = torch.zeros(T, H, dv, dtype=torch.float32)
@@ -583,6 +593,13 @@ def delta_scan(qn, kn, vv, beta, dec, state, cu_seqlens, seq_slot, n_seqs, max_r
             for h in range(H):
                 g = h // (H // G)
                 S = state[slot, h].to(F64) * dec[r, h].to(F64).expand(dk)[:, None]
+                if removal is not None:
+                    unit = beta[r, h].to(F64) * kn[r, g].to(F64)
+                    S = (S - torch.outer(removal[r, h].to(F64), unit @ state[slot, h].to(F64))
+                         + torch.outer(kn[r, g].to(F64), vv[r, h].to(F64)))
+                    o[r, h] = (S.t() @ qn[r, g].to(F64)).to(torch.float32)
+                    state[slot, h] = S.to(torch.float32)
+                    continue
                 u = beta[r, h].to(F64) * (vv[r, h].to(F64) - (S.t() @ kn[r, g].to(F64) if correct else 0.0))
                 S = S + torch.outer(kn[r, g].to(F64), u)
                 o[r, h] = (S.t() @ qn[r, g].to(F64)).to(torch.float32)
@@ -769,13 +786,21 @@ def clamped_swish_mul(gate_up, limit):
 
 # ---------------------------------------------------------------- attention over a window and pooled blocks
 def qk_rotate_store(rows, k_off, v_off, cos_sin, rot, pairing, unit_norm, eps, row_pos, row_slot, kcache,
-                    vcache, page_table, page_size, ring, nh, nkv, dk, dv, q_scale=None):
+                    vcache, page_table, page_size, ring, nh, nkv, dk, dv, q_scale=None, bias=None, q_weight=None,
+                    k_weight=None, slot_len=None, kept=0):
     half = rot // 2
     for r in range(rows.shape[0]):
-        for off, heads in ((0, nh), (k_off, nkv)):
+        if bias is not None:
+            at = (nh + nkv) * dk
+            rows[r, v_off:v_off + nkv * dv] = (rows[r, v_off:v_off + nkv * dv].to(F64) + bias[at:].to(F64)).to(rows.dtype)
+        for off, heads, nw in ((0, nh, q_weight), (k_off, nkv, k_weight)):
             if not heads:
                 continue
             x = rows[r, off:off + heads * dk].to(F64).view(heads, dk).clone()
+            if bias is not None:
+                x = x + bias[off:off + heads * dk].to(F64).view(heads, dk)
+            if nw is not None:
+                x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * nw.to(F64)
             if cos_sin is not None and rot:
                 c, s = cos_sin[int(row_pos[r]), :, 0].to(F64), cos_sin[int(row_pos[r]), :, 1].to(F64)
                 ia = torch.arange(half) if pairing == 0 else 2 * torch.arange(half)
@@ -788,7 +813,8 @@ def qk_rotate_store(rows, k_off, v_off, cos_sin, rot, pairing, unit_norm, eps, r
                 x = x * q_scale.to(F64)[:, None]
             rows[r, off:off + heads * dk] = x.reshape(-1).to(rows.dtype)
     if kcache is not None:
-        kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv)
+        kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv,
+                  kept)
 
 
 def pool_store(row_pos, row_slot, kcache, vcache, kpool, vpool, page_table, page_size, nkv, dk, dv, pool):
@@ -882,6 +908,89 @@ def lru_scan(a, x, state, Y, y_off, y_bias, cu_seqlens, seq_slot, n_seqs, max_ro
     return out.to(out_dtype)
 
 
+# ---------------------------------------------------------------- norms behind a sublayer
+def _norm_rows(v, kind, weight, bias, eps):
+    if kind == "layer":
+        v = v - v.mean(-1, keepdim=True)
+    v = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * weight.to(F64)
+    return v if bias is None else v + bias.to(F64)
+
+
+def post_add_norm(x, post, kind, weight, bias, eps, out_dtype, row_idx=None):
+    v = x.to(F64)
+    if post is not None and hasattr(post, "kind"):
+        v = v + post.gain * _norm_rows(post.a.to(F64), post.kind, post.weight, post.bias, post.eps)
+    elif post is not None:
+        v = v + post.to(F64)
+    if row_idx is None:
+        x.copy_(v.to(torch.float32))
+    else:
+        v = v[row_idx.long()]
+    if out_dtype is None:
+        return None
+    if kind is None:
+        return x if row_idx is None and out_dtype == torch.float32 else v.to(out_dtype)
+    return _norm_rows(v, kind, weight, bias, eps).to(out_dtype)
+
+
+def xielu(x, par):
+    z = x.to(F64)
+    below = par[1].to(F64) * (torch.exp(torch.clamp(z, max=0)) - 1 - z)
+    return (torch.where(z > 0, par[0].to(F64) * z * z, below) + z / 2).to(x.dtype)
+
+
+# ---------------------------------------------------------------- lightning attention, the delta rule with a removal vector
+def _silu(x):
+    return x * torch.sigmoid(x)
+
+
+def lightning_prepare(U, q_off, k_off, v_off, decay, H, dk, dv):
+    T = U.shape[0]
+    u = _silu(U.to(F64))
+    take = lambda off, d: u[:, off:off + H * d].reshape(T, H, d).to(torch.float32).contiguous()
+    dec = decay.to(torch.float32).expand(T, H).reshape(T, H, 1).contiguous()
+    return take(q_off, dk), take(k_off, dk), take(v_off, dv), torch.ones(T, H), dec
+
+
+def lightning_chunks(U, q_off, k_off, v_off, decay, state, cu_seqlens, seq_slot, n_seqs, max_rows, H, dk, dv):
+    q, k, v, one, dec = lightning_prepare(U, q_off, k_off, v_off, decay, H, dk, dv)
+    return delta_scan(q, k, v, one, dec, state, cu_seqlens, seq_slot, n_seqs, max_rows, correct=False)
+
+
+def lightning_step(U, q_off, k_off, v_off, decay, state, row_slot, H, dk, dv):
+    B = U.shape[0]
+    return lightning_chunks(U, q_off, k_off, v_off, decay, state, torch.arange(B + 1), row_slot, B, 1, H, dk, dv)
+
+
+def tanh_columns(U, off, n):
+    return torch.tanh(U[:, off:off + n].to(F64)).to(U.dtype)
+
+
+def removal_prepare(U, r_off, k_off, v_off, a_off, a_bias, Z, w0, rate, H, d):
+    T = U.shape[0]
+    cols = lambda off: U[:, off:off + H * d].to(F64).view(T, H, d)
+    r, k, v = cols(r_off), cols(k_off), cols(v_off)
+    beta = 1.0 / torch.sqrt((k * k).sum(-1) + 1e-6)
+    a = torch.sigmoid(cols(a_off) + a_bias.to(F64).view(H, d))
+    dec = torch.exp(-rate * torch.sigmoid(Z.to(F64).view(T, H, d) + w0.to(F64).view(H, d)))
+    return tuple(t.to(torch.float32).contiguous() for t in (r, k, v, beta, dec, a * k * beta[..., None]))
+
+
+def removal_step(U, r_off, k_off, v_off, a_off, a_bias, w1_off, w2, w0, rate, state, row_slot, H, d):
+    B = U.shape[0]
+    Z = torch.tanh(U[:, w1_off:w1_off + w2.shape[1]].to(F64)) @ w2.to(F64).t()
+    r, k, v, beta, dec, rem = removal_prepare(U, r_off, k_off, v_off, a_off, a_bias, Z, w0, rate, H, d)
+    return delta_scan(r, k, v, beta, dec, state, torch.arange(B + 1), row_slot, B, 1, correct=False, removal=rem)
+
+
+def group_norm_gate(o, groups, weight, Z, z_off, gate, eps, out_dtype):
+    T, width = o.shape[0], weight.numel()
+    x = o.to(F64).reshape(T, groups, -1)
+    x = (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)).reshape(T, width) * weight.to(F64)
+    z = Z[:, z_off:z_off + width].to(F64)
+    return (x * (torch.sigmoid(z) if gate == "sigmoid" else _silu(z))).to(out_dtype)
+
+
 def patch(monkeypatch):
     """Put these functions in place of the GPU ops (CPU tests only)."""
     from inferllm_amd.kernels import ops
@@ -896,6 +1005,8 @@ def patch(monkeypatch):
                  "delta_conv_tail", "delta_scan", "delta_finish", "qkv_norm_mix_store", "ssm_prepare",
                  "ssm_finish", "memory_prepare", "memory_finish", "embed_pairs", "remember_last", "gelu_tanh",
                  "short_conv", "short_conv_tail", "rms_rows_gain", "post_add_rmsnorm", "gate_up_act", "clamped_swish_mul", "qk_rotate_store",
-                 "pool_store", "attn_pooled_rows", "attn_pooled_decode", "gla_prepare", "lru_gates", "lru_scan"):
+                 "pool_store", "attn_pooled_rows", "attn_pooled_decode", "gla_prepare", "lru_gates", "lru_scan",
+                 "post_add_norm", "xielu", "lightning_prepare", "lightning_chunks", "lightning_step", "tanh_columns",
+                 "removal_prepare", "removal_step", "group_norm_gate"):
         monkeypatch.setattr(ops, name, globals()[name])
     monkeypatch.setattr(ops.ScaledSum, "tensor", scaled_sum_tensor)
