@@ -22,7 +22,7 @@ of MI355X (HBM 8 TB/s, dense bf16 MFMA 2.5 PFLOP/s, float32 157.3 TFLOP/s).
 The run fails (non-zero) if any timed run produced a non-finite logit or the same
 greedy token everywhere.
 
-`--design rabapel`, `--design kukupel`, `--design sabipel` and `--design dotorax` are other workloads with a line of their own (the
+`--design rabapel`, `kukupel`, `sabipel`, `dotorax` and `febivik` are other workloads with a line of their own (the
 default's stays as it is):
 Rabapel (latent attention, layers that alternate a dense and a routed feed-forward) at two
 sizes beside LLaMA at the same width, heads and layer count: prefill of 2,048 tokens and decoding
@@ -30,7 +30,9 @@ at batch 1, 8 and 64, each with its fraction of the matrix or HBM peak.
 Kukupel likewise beside Rabapel, and Sabipel (state-space, matrix-memory and chunked-attention
 layers with dense feed-forwards) beside Kukupel, and Dotorax (rotated attention with shared keys,
 gated linear attention, a window with pooled blocks beside a recurrent unit, gated feed-forwards,
-sublayers between two norms behind a short convolution) beside Sabipel.
+sublayers between two norms behind a short convolution) beside Sabipel, and Febivik (lightning
+attention, a delta rule with a removal vector, a window that keeps the first tokens, squared-ReLU
+experts, norms behind the sublayers) beside Kukupel.
 """
 import argparse
 import json
@@ -644,6 +646,116 @@ def dotorax_main(args) -> int:
     return 0
 
 
+# ---------------------------------------------------------------- Febivik beside Kukupel
+def febivik_config(width, heads, kv_heads, layers, experts, expert_ff, top, window=1024, keep=4, vocab=32000):
+    """Layers in the order attention, lightning, general_delta, lightning ...: attention heads of 128
+    query and 128 value dims, half of each rotated, over a window that keeps the first tokens, and a
+    dense feed-forward of 4 times the width; lightning and delta-rule heads of 128 x 128 (decays' rank
+    64) with routed feed-forwards beside a shared expert of twice an expert's size."""
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+           "mask": {"size": window, "keep_first": keep},
+           "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0}}}
+    light = {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** -(1 + 9 * h / heads) for h in range(heads)]}
+    delta = {"heads": heads, "dim": 128, "rank": 64}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top, "scale": 2.5},
+           "shared": {"ff": 2 * expert_ff}}
+    kinds = (("attention", att, {"kind": "dense", "ff": 4 * width}), ("lightning", light, moe),
+             ("general_delta", delta, moe), ("lightning", light, moe))
+    return {"architecture": "Febivik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": 8192,
+            "layers": [dict(zip(("type", "mixer", "mlp"), json.loads(json.dumps(kinds[i % 4])))) for i in range(layers)]}
+
+
+def febivik_counts(cfg, esz):
+    """(step_bytes(batch, mean_ctx), flops(tokens, lens)) of a Febivik configuration, counted as
+    Kukupel's: the weights a decode step reads (of a routed layer the router, the shared expert and
+    the experts that `batch` tokens are expected to choose), attention's cache rows (a window's and
+    the kept first tokens'), the float32 states (read and written); the multiply-adds of a prompt step
+    (recurrences as 2 key x value products a token and head, the delta rule as 3)."""
+    E, V = cfg["width"], cfg["vocab"]
+
+    def mixer_parts(layer):
+        """(weights, float32 state, state products a token, cache columns a token, score columns a pair, keys seen at most)"""
+        m, kind = layer["mixer"], layer["type"]
+        if kind == "lightning":
+            H, dk, dv = m["heads"], m["dim"], m["vdim"]
+            return E * H * (2 * dk + 3 * dv), H * dk * dv, 2 * H * dk * dv, 0, 0, 0
+        if kind == "general_delta":
+            n = m["heads"] * m["dim"]
+            return 6 * E * n + m["rank"] * (E + n), n * m["dim"], 3 * n * m["dim"], 0, 0, 0
+        H, G, dk, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        mask = m.get("mask")
+        most = mask["size"] + mask.get("keep_first", 0) if mask else 0
+        return E * (H * dk + G * (dk + dv)) + H * dv * E, 0, 0, G * (dk + dv), H * (dk + dv), most
+
+    def ff_parts(mlp, batch):
+        """(weights read by `batch` tokens together, multiply-adds a token, router entries)"""
+        if mlp["kind"] == "dense":
+            return 2 * E * mlp["ff"], 2 * E * mlp["ff"], 0
+        r, ff, sh = mlp["router"], mlp["expert"]["ff"], (mlp.get("shared") or {}).get("ff", 0)
+        used = r["experts"] * (1.0 - (1.0 - r["top"] / r["experts"]) ** batch)
+        return 2 * E * (used * ff + sh), 2 * E * (r["top"] * ff + sh) + E * r["experts"], E * r["experts"]
+
+    seen = lambda n, most: min(n, most) if most else n
+
+    def step_bytes(batch, mean_ctx):
+        total = V * E * esz
+        for layer in cfg["layers"]:
+            w, state, _, kv_row, _, most = mixer_parts(layer)
+            f, _, router = ff_parts(layer["mlp"], batch)
+            total += (w + f + batch * seen(mean_ctx, most) * kv_row) * esz + router * 4 + batch * state * 4 * 2
+        return total
+
+    def flops(tokens, lens):
+        total = 2.0 * len(lens) * V * E
+        for layer in cfg["layers"]:
+            w, _, products, _, qk, most = mixer_parts(layer)
+            pairs = sum(sum(seen(p + 1, most) for p in range(n)) for n in lens) if qk else 0
+            total += 2.0 * tokens * (w + ff_parts(layer["mlp"], 1)[1] + products) + 2.0 * qk * pairs
+        return total
+
+    return step_bytes, flops
+
+
+def febivik_main(args) -> int:
+    """Febivik at two sizes beside Kukupel, the library's closest design (a delta rule, attention and
+    routed feed-forwards), at the same width, heads, experts and number of layers (four): tokens/s of
+    these four-layer models, with the fraction of the matrix peak for prompts and of the HBM peak for
+    decode steps."""
+    import torch
+    from inferllm_amd import Engine
+    layers = args.layers or 4
+    esz = 2 if args.dtype == "bfloat16" else 4
+    sizes = {"2048": dict(width=2048, heads=16, kv_heads=4, experts=64, expert_ff=1408, top=6),
+             "4096": dict(width=4096, heads=32, kv_heads=8, experts=32, expert_ff=2048, top=4)}
+    few = min(args.steps, 128)
+    out = {"metric": "Febivik beside Kukupel at equal width, heads, experts and layers: prefill tok/s at 2,048 tokens, decode tok/s at batch 1/8/64",
+           "unit": "tokens/s", "n_gpus": 1, "steps": few, "warmup": 4, "dtype": "bf16" if esz == 2 else "fp32",
+           "data": "synthetic: seeded random weights, uniform random token ids", "layers": layers, "sizes": {}}
+    for name, sz in sizes.items():
+        if args.size and args.size != name:
+            continue
+        row = {}
+        fcfg, kcfg = febivik_config(layers=layers, **sz), kukupel_config(layers=layers, **sz)
+        for design, cfg, counts in (("febivik", fcfg, febivik_counts), ("kukupel", kcfg, kukupel_counts)):
+            if args.only and args.only != design:
+                continue
+            eng = Engine.from_random(cfg, seed=0, dtype=args.dtype, device="cuda:0", max_batch=64,
+                                     max_seq_len=4096, max_tokens=64 * 1024)
+            b = Bench.around(eng, cfg["vocab"], layers, args.dtype, *counts(cfg, esz))
+            torch.cuda.synchronize()
+            r = {"prefill_2048": b.prefill_run(2048, reps=4)}
+            if not args.prefill_only:
+                for batch in ((int(b_) for b_ in args.batches.split(",")) if args.batches else (1, 8, 64)):
+                    v, ms, f = b.decode_run(batch, few, 4, args.prompt)
+                    r[f"decode_b{batch}"] = {"value": round(v, 1), "ms": round(ms, 4), "hbm_frac": round(f, 4)}
+            row[design] = r
+            b.close()
+            del b, eng
+        out["sizes"][name] = row
+    print(json.dumps(out), flush=True)
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -661,13 +773,15 @@ def main() -> int:
     ap.add_argument("--no-70b", action="store_true",
                     help="leave the LLaMA-2-70B shape out of `points` (138 GB of weights: half a minute)")
     ap.add_argument("--with-70b", action="store_true", help="(the default now; kept for old command lines)")
-    ap.add_argument("--design", default="llama", choices=["llama", "rabapel", "kukupel", "sabipel", "dotorax"],
+    ap.add_argument("--design", default="llama", choices=["llama", "rabapel", "kukupel", "sabipel", "dotorax", "febivik"],
                     help="rabapel: that design at two sizes beside LLaMA at equal size (a line of its own); "
                          "kukupel: that design at two sizes beside Rabapel at equal size (likewise); "
                          "sabipel: that design at two sizes beside Kukupel at equal size (likewise); "
-                         "dotorax: that design at two sizes beside Sabipel at equal size (likewise)")
-    ap.add_argument("--size", default="", help="with --design rabapel, kukupel, sabipel or dotorax: only this width (2048 or 4096)")
-    ap.add_argument("--only", default="", help="with --design kukupel, sabipel or dotorax: only this one of the two designs")
+                         "dotorax: that design at two sizes beside Sabipel at equal size (likewise); "
+                         "febivik: that design at two sizes beside Kukupel at equal size (likewise)")
+    ap.add_argument("--size", default="", help="with another --design than llama: only this width (2048 or 4096)")
+    ap.add_argument("--only", default="", help="with --design kukupel, sabipel, dotorax or febivik: only this one of the two designs")
+    ap.add_argument("--batches", default="", help="with --design febivik: decode batches in place of 1,8,64")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU only (this library has no multi-GPU path); --gpus must be 1")
@@ -681,6 +795,8 @@ def main() -> int:
         return sabipel_main(args)
     if args.design == "dotorax":
         return dotorax_main(args)
+    if args.design == "febivik":
+        return febivik_main(args)
 
     shape_name, shape_cfg = SHAPES[args.shape]
     ctx_len = shape_cfg["max_position_embeddings"]

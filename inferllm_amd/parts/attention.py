@@ -90,7 +90,7 @@ class Attention(Mixer):
             else:
                 qkv = ops.linear(h, self.w_qkv)
                 ops.rope_store(qkv, None, 0, 0, ctx.row_pos, ctx.row_slot,
-                               ctx.cache.slot_len if ctx.prefill else None, kc, vc, group.table,
+                               ctx.overwritten_lengths, kc, vc, group.table,
                                group.page_size, group.ring, nh, nkv, hd)
             if ctx.prefill:
                 ctx.exchange[("kv_rows", line)] = qkv      # for runs that read this cache line
@@ -393,7 +393,7 @@ class GatedAttention(Mixer):
                                 group.ring, nh, nkv if self.own_kv else 0, dk, dv, q_scale=self.head_scale,
                                 bias=self.bias, q_weight=self.q_norm if weighted else None,
                                 k_weight=self.k_norm if weighted else None,
-                                slot_len=ctx.cache.slot_len if ctx.prefill and group.ring else None,
+                                slot_len=ctx.overwritten_lengths if group.ring else None,
                                 kept=group.kept_pages)
         else:
             if group.ring:

@@ -56,6 +56,14 @@ class StepContext:
     exchange: Dict[Any, Any] = field(default_factory=dict)   # between runs of layers in one step
     run: int = 0                      # which entry of the model's schedule is running (set by the model)
 
+    @property
+    def overwritten_lengths(self) -> Optional[torch.Tensor]:
+        """For the stores of whole prompts: the slots' lengths after the step, with which a row that a
+        later row of the same step would overwrite in a ring of pages is left out.  None for every
+        other step: its rows read the cache, and the step function keeps it from writing round the
+        ring, so that every row is stored."""
+        return self.cache.slot_len if self.prefill and not self.continues else None
+
 
 class Part:
     """Base of all parts: parameter names -> checkpoint names in `self.tensors`.

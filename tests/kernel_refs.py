@@ -444,9 +444,12 @@ def scaled_sum_tensor(self):
 
 # ---------------------------------------------------------------- attention with a soft cap
 def kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv,
-              kept=0):
+              kept=0, slot_len=None):
     # (rows in order: of two that land on one place of a ring the later one stays)
     for r in range(rows.shape[0]):
+        lp = int(row_pos[r]) // page_size
+        if ring > 0 and slot_len is not None and kept <= lp <= (int(slot_len[int(row_slot[r])]) - 1) // page_size - ring:
+            continue                                     # a later row's page lies in its place
         page, at = cache_offsets(page_table, int(row_slot[r]), int(row_pos[r]), page_size, ring, kept)
         kcache[page, :, at, :] = rows[r, k_off:k_off + nkv * dk].view(nkv, dk)
         vcache[page, :, at, :] = rows[r, v_off:v_off + nkv * dv].view(nkv, dv)
@@ -814,7 +817,7 @@ def qk_rotate_store(rows, k_off, v_off, cos_sin, rot, pairing, unit_norm, eps, r
             rows[r, off:off + heads * dk] = x.reshape(-1).to(rows.dtype)
     if kcache is not None:
         kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv,
-                  kept)
+                  kept, slot_len)
 
 
 def pool_store(row_pos, row_slot, kcache, vcache, kpool, vpool, page_table, page_size, nkv, dk, dv, pool):
