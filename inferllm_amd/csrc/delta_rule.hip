@@ -290,7 +290,8 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
                        float* __restrict__ o, int G, int H, int dk, int dv, const float* __restrict__ removal) {
     constexpr bool CORRECT = RULE != RULE_PLAIN;
     constexpr int NVEC = RULE == RULE_REMOVAL ? 4 : 3;  // rows a token in LDS
-    constexpr int PARTS = 16, COLS = 4, TC = DELTA_CHUNK;
+    constexpr int PARTS = 16, COLS = 4;
+    constexpr int TC = RULE == RULE_REMOVAL ? DELTA_CHUNK / 2 : DELTA_CHUNK;    // (a fourth row a token: fewer tokens, or registers run out)
     constexpr int DKP = PARTS * NS;                     // a row of k, q or decays in LDS, filled up
     constexpr int JJ = (DKP + 63) / 64;                 // pieces of 64 floats in it
     constexpr int NA = NS >= 4 ? 4 : NS;

@@ -369,7 +369,7 @@ lightning_chunk_carry_kernel(float* __restrict__ part, const float* __restrict__
 // on, and in o^T = V^T . P^T they are the second operand as they stand.  k and v lie in LDS, q in
 // registers; the start state is read straight from memory (32 neighbouring values a row).
 template <int DT, int KT, int VT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, 2)
 lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off, int k_off, int v_off,
                             const float* __restrict__ decay, const float* __restrict__ part,
                             const int32_t* __restrict__ cu, float* __restrict__ o, int H, int dk, int dv) {
@@ -419,7 +419,7 @@ lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off,
         for (int v = 0; v < 16; ++v) acc[t][v] = 0.f;
         if (n0 >= dv) continue;
         const bool in = n0 + col < dv;
-#pragma unroll 8
+#pragma unroll
         for (int s2 = 0; s2 < DKP / 2; ++s2) {
             const int m = 2 * s2 + half;
             const float a = (in && m < dk) ? S[(size_t)m * dv + n0 + col] : 0.f;

@@ -2334,6 +2334,33 @@ def removal_prepare(U: torch.Tensor, r_off: int, k_off: int, v_off: int, a_off: 
     return qn, kn, vv, beta, dec, rem
 
 
+REMOVAL_CHUNKS_FROM = 32       # rows a sequence from which the chunks run in parallel
+REMOVAL_CHUNKS_MAX_DIM = 128
+
+
+def removal_chunks(U: torch.Tensor, r_off: int, k_off: int, v_off: int, a_off: int, a_bias: torch.Tensor,
+                   Z: torch.Tensor, w0: torch.Tensor, rate: float, state: torch.Tensor, cu_seqlens: torch.Tensor,
+                   seq_slot: torch.Tensor, n_seqs: int, max_rows: int, H: int, d: int) -> torch.Tensor:
+    """`removal_prepare` and `delta_scan` with `removal` for many rows a sequence, chunk by chunk
+    (csrc/removal_chunks.hip): a row's sums run in another order than token by token.
+    Returns o float32 [T, H, d]."""
+    _gpu(U, a_bias, Z, w0, state, cu_seqlens, seq_slot)
+    _i32(cu_seqlens, n_seqs + 1); _i32(seq_slot, n_seqs)
+    _columns_ok(U, "removal_chunks", *((off, H * d) for off in (r_off, k_off, v_off, a_off)))
+    _removal_ok(H, d, a_bias, w0, "removal_chunks")
+    T = U.shape[0]
+    _need(d <= REMOVAL_CHUNKS_MAX_DIM and Z.shape == (T, H * d) and Z.dtype == U.dtype and state.dtype == torch.float32
+          and state.dim() == 4 and state.shape[1:] == (H, d, d),
+          "removal_chunks: Z [T, H d] of U's dtype, state float32 [slots, H, d, d], d <= 128")
+    places = T // _lib().illm_removal_chunk() + n_seqs + 1
+    part = torch.empty((places * H * _lib().illm_removal_chunk_floats(d),), dtype=torch.float32, device=U.device)
+    o = torch.empty((T, H, d), dtype=torch.float32, device=U.device)
+    _check(_lib().illm_removal_chunks(_p(U), _code(U), U.shape[1], r_off, k_off, v_off, a_off, _p(a_bias), _p(Z),
+                                      Z.shape[1], _p(w0), ctypes.c_float(rate), _p(state), _p(part), _p(cu_seqlens),
+                                      _p(seq_slot), _p(o), n_seqs, int(max_rows), H, d, _stream()), "removal_chunks")
+    return o
+
+
 REMOVAL_STEP_MAX_RANK = 512
 
 

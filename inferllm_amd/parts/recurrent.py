@@ -317,7 +317,8 @@ class RemovalDeltaRule(Mixer):
         out = W_o (o / rms(o) * norm * sigmoid(W_g h))
 
     rms over each head's outputs (`eps`), `norm` of all heads' width.  Kept per sequence: S (float32).
-    A step goes on from whatever the slot holds, single tokens in one launch.  Decays, rates, unit
+    A step goes on from whatever the slot holds: single tokens in one launch, many rows a sequence in
+    chunks.  Decays, rates, unit
     keys and the state are float32; the projections take the engine's dtype.
     """
 
@@ -369,11 +370,18 @@ class RemovalDeltaRule(Mixer):
                                  ctx.row_slot, H, d)
         else:
             Z = ops.linear(ops.tanh_columns(U, self.w1_off, self.rank), self.w_w2)
+            if ctx.prefill and ctx.max_rows >= ops.REMOVAL_CHUNKS_FROM and d <= ops.REMOVAL_CHUNKS_MAX_DIM:
+                o = ops.removal_chunks(U, *cols, self.a_bias, Z, self.w0, REMOVAL_DECAY_RATE, S, ctx.cu_seqlens,
+                                       ctx.seq_slot, ctx.n_seqs, ctx.max_rows, H, d)
+                return self._finish(o, U, ctx)
             rn, kn, vv, beta, dec, removal = ops.removal_prepare(U, *cols, self.a_bias, Z, self.w0, REMOVAL_DECAY_RATE,
                                                                  H, d)
             o = ops.delta_scan(rn, kn, vv, beta, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
                                ctx.max_rows if ctx.prefill else 1, correct=False, removal=removal)
-        y = ops.group_norm_gate(o, H, self.norm_w, U, self.g_off, "sigmoid", self.eps, ctx.act_dtype)
+        return self._finish(o, U, ctx)
+
+    def _finish(self, o, U, ctx: StepContext):
+        y = ops.group_norm_gate(o, self.H, self.norm_w, U, self.g_off, "sigmoid", self.eps, ctx.act_dtype)
         return ops.linear(y, self.w_o)
 
 

@@ -979,6 +979,12 @@ def removal_prepare(U, r_off, k_off, v_off, a_off, a_bias, Z, w0, rate, H, d):
     return tuple(t.to(torch.float32).contiguous() for t in (r, k, v, beta, dec, a * k * beta[..., None]))
 
 
+def removal_chunks(U, r_off, k_off, v_off, a_off, a_bias, Z, w0, rate, state, cu_seqlens, seq_slot, n_seqs, max_rows,
+                   H, d):
+    r, k, v, beta, dec, rem = removal_prepare(U, r_off, k_off, v_off, a_off, a_bias, Z, w0, rate, H, d)
+    return delta_scan(r, k, v, beta, dec, state, cu_seqlens, seq_slot, n_seqs, max_rows, correct=False, removal=rem)
+
+
 def removal_step(U, r_off, k_off, v_off, a_off, a_bias, w1_off, w2, w0, rate, state, row_slot, H, d):
     B = U.shape[0]
     Z = torch.tanh(U[:, w1_off:w1_off + w2.shape[1]].to(F64)) @ w2.to(F64).t()
@@ -1010,6 +1016,6 @@ def patch(monkeypatch):
                  "short_conv", "short_conv_tail", "rms_rows_gain", "post_add_rmsnorm", "gate_up_act", "clamped_swish_mul", "qk_rotate_store",
                  "pool_store", "attn_pooled_rows", "attn_pooled_decode", "gla_prepare", "lru_gates", "lru_scan",
                  "post_add_norm", "xielu", "lightning_prepare", "lightning_chunks", "lightning_step", "tanh_columns",
-                 "removal_prepare", "removal_step", "group_norm_gate"):
+                 "removal_prepare", "removal_chunks", "removal_step", "group_norm_gate"):
         monkeypatch.setattr(ops, name, globals()[name])
     monkeypatch.setattr(ops.ScaledSum, "tensor", scaled_sum_tensor)

@@ -593,18 +593,20 @@ def test_lightning_kernels_against_plain_torch(dtype):
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_delta_rule_with_a_removal_vector_against_plain_torch(dtype):
-    """Preparation and scan (short and long steps) and the single-token kernel with its low-rank map,
-    from states that are not zero."""
+    """Preparation and scan (short and long steps), the chunks and the single-token kernel with its
+    low-rank map, from states that are not zero; lengths on both sides of a chunk's edge, decays as
+    strong and as weak as they get."""
     from inferllm_amd.kernels import ops
     g = torch.Generator().manual_seed(12)
     rate = 0.6
-    for H, d, rank in ((3, 24, 5), (2, 128, 64), (4, 10, 3), (1, 200, 16), (2, 64, 130)):
+    for H, d, rank in ((3, 24, 5), (2, 128, 64), (4, 10, 3), (1, 200, 16), (2, 64, 130), (8, 96, 7)):
         n = H * d
         offs = (2, 2 + n, 2 + 2 * n, 2 + 3 * n)
         w1_off = 2 + 4 * n
         a_bias, w0 = torch.randn(n, generator=g), torch.randn(n, generator=g) * 2 - 1
+        w0[::5], w0[1::5] = 12.0, -12.0
         w2 = (torch.randn(n, rank, generator=g) / rank ** 0.5).to(dtype)
-        for lens in ([70, 3, 16, 1], [1, 1, 1], [5, 2]):
+        for lens in ([70, 3, 16, 1], [1, 1, 1], [5, 2], [64, 31, 33, 32], [257]):
             T = sum(lens)
             cu, seq_slot, row_slot = _packed(lens, [4, 0, 2, 5][:len(lens)])
             U = torch.randn(T, w1_off + rank + 1, generator=g).to(dtype)
@@ -619,6 +621,11 @@ def test_delta_rule_with_a_removal_vector_against_plain_torch(dtype):
             o = ops.delta_scan(*got_in[:5], s_got, cu.cuda(), seq_slot.cuda(), len(lens), max(lens), correct=False,
                                removal=got_in[5])
             _near(o, want, 2e-5); _near(s_got, s_want, 2e-5)
+            if d <= 128:
+                s_got = state.cuda()
+                o = ops.removal_chunks(U.cuda(), *offs, a_bias.cuda(), Z.cuda(), w0.cuda(), rate, s_got, cu.cuda(),
+                                       seq_slot.cuda(), len(lens), max(lens), H, d)
+                _near(o, want, 2e-5); _near(s_got, s_want, 2e-5)
             if max(lens) == 1:
                 s_want, s_got = state.clone(), state.cuda()
                 want = R.removal_step(U, *offs, a_bias, w1_off, w2, w0, rate, s_want, row_slot, H, d)
