@@ -15,9 +15,10 @@
 // the same path.  A line that keeps a window as a ring of pages (the first `kept` pages beside it)
 // does not hold a long prompt: rows of a step whose sequences all start may read the step's own rows
 // instead (`own_stride` > 0: keys at column own_k, values at own_v of the rows that q lies in).
-// Float32 arithmetic over float32 or bfloat16 storage: widths of up to 128 in steps
+// Float32 sums, scores and weights over float32 or bfloat16 storage: widths of up to 128 in steps
 // of 4 (single tokens: of 16 bytes) take the kernels on the matrix cores' float32 instruction and
-// with eight lanes a key, every other width the plain ones on the vector units.
+// with eight lanes a key (rows of bfloat16 in steps of 8 the bfloat16 instruction), every other width the
+// plain ones on the vector units.
 #include <math.h>
 
 #include "api.h"
@@ -476,8 +477,216 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
     }
 }
 
+// ---------------------------------------------------------------- the same rows from bfloat16 storage
+// Key and value widths of up to 128 in steps of 8.  The layout of the kernel above with the bfloat16
+// instruction (MFMA 32x32x16, float32 sums): keys, queries and values are bfloat16 as they are stored, so
+// the scores are float32 sums of exact products as above; a weight, which is float32, enters its product
+// as two bfloat16 terms, p = hi + lo (what is left out is below 2^-17 of it), two products for one.
+// Keys lie in LDS as rows, values transposed ([value dim][key]), the keys of a row in the order in which
+// a lane holds its weights: key 16 s + 8 b + 4 h + i at place 16 s + 8 h + 4 b + i.
+typedef __bf16 cap_bf16x8_t __attribute__((ext_vector_type(8)));
+
+template <int KT, int VT>
+__global__ void __launch_bounds__(256, 2)
+attn_cap_rows_bf16_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
+                          const int32_t* __restrict__ cu, const int32_t* __restrict__ seq_slot,
+                          const int32_t* __restrict__ seq_start, const bf16_t* __restrict__ kcache,
+                          const bf16_t* __restrict__ vcache, const int32_t* __restrict__ page_table,
+                          int table_stride, int page_size, int ring, int nh, int nkv, int dk, int dv,
+                          float scale, float cap, int window, const float* __restrict__ slopes, int chunk,
+                          const bf16_t* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
+                          float* __restrict__ lse, int keep, int kept, int own_stride, int own_k, int own_v) {
+    constexpr int DKP = 32 * KT, DVP = 32 * VT, KLD = DKP + 8, VLD = MK + 8;
+    constexpr int KP = (MK * DKP / 8 + 255) / 256;             // 16-byte pieces of a key tile a thread brings
+    constexpr int VP = ((MK / 2) * (DVP / 8) + 255) / 256;     // pairs of keys x 8 value dims a thread brings
+    __shared__ __attribute__((aligned(16))) bf16_t ks[MK * KLD];
+    __shared__ __attribute__((aligned(16))) bf16_t vs[DVP * VLD];
+    const int b = blockIdx.z, h = blockIdx.y;
+    const int start = cu[b], len = cu[b + 1] - start;
+    const int q0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * MQ;
+    if (q0 >= len) return;
+    const int pos0 = seq_start[b], slot = seq_slot[b];
+    const int total = pos0 + len;
+    const int kvh = h / (nh / nkv);
+    const int tid = threadIdx.x, lane = tid & 63, wave = wave_index();
+    const int col = lane & 31, half = lane >> 5;
+    const int qrow = q0 + 32 * wave + col;
+    const int qpos = pos0 + qrow;
+    const bool wave_has_rows = q0 + 32 * wave < len;
+    const float inv_cap = cap > 0.f ? 1.0f / cap : 0.f;
+    const float slope = slopes ? slopes[h] : 0.f;
+    const illm_u32x4_t zero4 = {0u, 0u, 0u, 0u};
+
+    illm_u32x4_t qr[2 * KT];                                   // dims 16 s + 8 half .. + 7
+    {
+        const bf16_t* qp = q + (size_t)(start + min(qrow, len - 1)) * q_stride + (size_t)h * dk;
+#pragma unroll
+        for (int s = 0; s < 2 * KT; ++s) {
+            const int d = 16 * s + 8 * half;
+            qr[s] = d < dk ? *(const illm_u32x4_t*)(qp + d) : zero4;
+        }
+    }
+    illm_u32x4_t kreg[KP], vreg[VP][2];
+    auto key_at = [&](int kj) __attribute__((always_inline)) {
+        kj = min(kj, total - 1);                               // keys past the end: a valid row, masked below
+        return own_stride ? (size_t)(start + kj) * own_stride + own_k + (size_t)kvh * dk
+                          : cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dk, kept);
+    };
+    auto value_at = [&](int kj) __attribute__((always_inline)) {
+        kj = min(kj, total - 1);
+        return own_stride ? (size_t)(start + kj) * own_stride + own_v + (size_t)kvh * dv
+                          : cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dv, kept);
+    };
+    auto fetch = [&](int k0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < KP; ++i) {
+            const int e = tid + 256 * i, row = e / (DKP / 8), d = 8 * (e % (DKP / 8));
+            kreg[i] = zero4;
+            if (row < MK && d < dk) kreg[i] = *(const illm_u32x4_t*)(kcache + key_at(k0 + row) + d);
+        }
+#pragma unroll
+        for (int i = 0; i < VP; ++i) {
+            const int e = tid + 256 * i, row = 2 * (e % (MK / 2)), d = 8 * (e / (MK / 2));
+            vreg[i][0] = vreg[i][1] = zero4;
+            if (d < dv) {
+                vreg[i][0] = *(const illm_u32x4_t*)(vcache + value_at(k0 + row) + d);
+                vreg[i][1] = *(const illm_u32x4_t*)(vcache + value_at(k0 + row + 1) + d);
+            }
+        }
+    };
+    auto stage = [&]() __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < KP; ++i) {
+            const int e = tid + 256 * i, row = e / (DKP / 8), d = 8 * (e % (DKP / 8));
+            if (row < MK) *(illm_u32x4_t*)(ks + row * KLD + d) = kreg[i];
+        }
+#pragma unroll
+        for (int i = 0; i < VP; ++i) {
+            const int e = tid + 256 * i, row = 2 * (e % (MK / 2)), d = 8 * (e / (MK / 2));
+            if (d < DVP) {
+                const int at = 16 * (row >> 4) + 8 * ((row >> 2) & 1) + 4 * ((row >> 3) & 1) + (row & 3);
+                const uint32_t* x = (const uint32_t*)&vreg[i][0];
+                const uint32_t* y = (const uint32_t*)&vreg[i][1];
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    *(uint32_t*)(vs + (d + 2 * j) * VLD + at) = (x[j] & 0xffffu) | (y[j] << 16);
+                    *(uint32_t*)(vs + (d + 2 * j + 1) * VLD + at) = (x[j] >> 16) | (y[j] & 0xffff0000u);
+                }
+            }
+        }
+    };
+    cap_f32x16_t o[VT];
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+#pragma unroll
+        for (int v = 0; v < 16; ++v) o[t][v] = 0.f;
+    float m_i = NEG_INF, l_i = 0.f;
+
+    const int k_hi = min(total, pos0 + q0 + MQ);
+    int k_lo = window > 0 ? max(0, pos0 + q0 - window + 1) : 0;
+    if (chunk > 0) k_lo = max(k_lo, ((pos0 + q0) / chunk) * chunk);
+    k_lo = (k_lo / MK) * MK;
+    const int wq_lo = pos0 + q0 + 32 * wave, wq_hi = wq_lo + 31;
+    const int wc_lo = chunk > 0 ? (wq_lo / chunk) * chunk : 0;
+    const int c_lo = chunk > 0 ? (qpos / chunk) * chunk : 0;
+    const int k_last = k_lo + ((k_hi - 1 - k_lo) / MK) * MK;
+    const int k_first = min(k_lo, ((keep + MK - 1) / MK) * MK);    // tiles [0, k_first): the kept tokens'
+    int k_next = k_first > 0 ? 0 : k_lo;
+    fetch(k_next);
+    for (int k0 = k_next; k0 < k_hi; k0 = k_next) {
+        __syncthreads();
+        stage();
+        __syncthreads();
+        k_next = k0 + MK == k_first ? k_lo : k0 + MK;
+        fetch(min(k_next, k_last));               // (unconditional: the last tile is asked for twice)
+        if (!wave_has_rows || k0 > wq_hi || k0 + MK - 1 < wc_lo ||
+            (window > 0 && k0 >= keep && k0 + MK - 1 <= wq_lo - window))
+            continue;
+        cap_f32x16_t sc;
+#pragma unroll
+        for (int v = 0; v < 16; ++v) sc[v] = 0.f;
+#pragma unroll
+        for (int s = 0; s < 2 * KT; ++s)
+            sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const cap_bf16x8_t*)(ks + col * KLD + 16 * s + 8 * half),
+                                                         *(const cap_bf16x8_t*)&qr[s], sc, 0, 0, 0);
+        // a tile that all of the wave's rows see whole needs no masks
+        const bool whole = k0 + MK - 1 <= wq_lo && q0 + 32 * wave + 31 < len && chunk <= 0 &&
+                           (window <= 0 || k0 > wq_hi - window);
+        float tm = NEG_INF;
+        if (whole && cap <= 0.f && !slopes) {
+#pragma unroll
+            for (int v = 0; v < 16; ++v) { sc[v] *= scale; tm = fmaxf(tm, sc[v]); }
+        } else {
+#pragma unroll
+            for (int v = 0; v < 16; ++v) {
+                const int kj = k0 + 8 * (v >> 2) + 4 * half + (v & 3);
+                const bool ok = qrow < len && kj <= qpos && kj >= c_lo && (window <= 0 || kj > qpos - window || kj < keep);
+                sc[v] = ok ? soft_cap(sc[v] * scale, cap, inv_cap) - slope * (float)(qpos - kj) : NEG_INF;
+                tm = fmaxf(tm, sc[v]);
+            }
+        }
+        tm = fmaxf(tm, __shfl_xor(tm, 32, ILLM_WAVE));
+        const float m_new = fmaxf(m_i, tm);
+        const float alpha = (m_new == NEG_INF) ? 1.f : __expf(m_i - m_new);
+        float psum = 0.f;
+#pragma unroll
+        for (int v = 0; v < 16; ++v) {
+            sc[v] = (sc[v] == NEG_INF) ? 0.f : __expf(sc[v] - m_new);
+            psum += sc[v];
+        }
+        psum += __shfl_xor(psum, 32, ILLM_WAVE);
+        l_i = l_i * alpha + psum;
+        m_i = m_new;
+#pragma unroll
+        for (int t = 0; t < VT; ++t)
+#pragma unroll
+            for (int v = 0; v < 16; ++v) o[t][v] *= alpha;
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+            uint32_t hi[4], lo[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const float p0 = sc[8 * s + 2 * j], p1 = sc[8 * s + 2 * j + 1];
+                hi[j] = pack_bf16x2(p0, p1);
+                lo[j] = pack_bf16x2(p0 - __uint_as_float(hi[j] << 16), p1 - __uint_as_float(hi[j] & 0xffff0000u));
+            }
+#pragma unroll
+            for (int t = 0; t < VT; ++t) {
+                const cap_bf16x8_t vt = *(const cap_bf16x8_t*)(vs + (32 * t + col) * VLD + 16 * s + 8 * half);
+                o[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vt, *(const cap_bf16x8_t*)hi, o[t], 0, 0, 0);
+                o[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vt, *(const cap_bf16x8_t*)lo, o[t], 0, 0, 0);
+            }
+        }
+    }
+    if (qrow < len) {
+        const float inv = 1.0f / l_i;
+        if (lse && half == 0) lse[(size_t)(start + qrow) * nh + h] = m_i + logf(l_i);
+        const size_t ob = (size_t)(start + qrow) * nh * dv + (size_t)h * dv;
+        const size_t gb = (size_t)(start + qrow) * gate_stride + gate_off + (size_t)h * (gate_heads ? 1 : dv);
+#pragma unroll
+        for (int t = 0; t < VT; ++t)
+#pragma unroll
+            for (int g = 0; g < 4; ++g) {
+                const int d = 32 * t + 8 * g + 4 * half;       // (dv is a multiple of 8: four at once)
+                if (d >= dv) continue;
+                float y[4];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    y[i] = o[t][4 * g + i] * inv;
+                    if (gate) y[i] *= 1.0f / (1.0f + expf(-bf16_to_f32(gate[gb + (gate_heads ? 0 : d + i)])));
+                }
+                uint2 w;
+                w.x = pack_bf16x2(y[0], y[1]);
+                w.y = pack_bf16x2(y[2], y[3]);
+                *(uint2*)(out + ob + d) = w;
+            }
+    }
+}
+
+// 0: every size to the kernels on the vector units; 1: the matrix cores where the sizes allow; 2: the matrix
+// cores' float32 instruction also for bfloat16 storage.
 static int g_attn_cap_mfma = 1;
-extern "C" void illm_set_attn_cap_mfma(int on) { g_attn_cap_mfma = on ? 1 : 0; }
+extern "C" void illm_set_attn_cap_mfma(int on) { g_attn_cap_mfma = on < 0 || on > 2 ? 1 : on; }
 static int g_attn_cap_heads = 4;
 extern "C" void illm_set_attn_cap_heads(int n) { g_attn_cap_heads = n == 2 ? 2 : 4; }
 
@@ -512,7 +721,23 @@ extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt
 #define GO_K(DT_)                                                                                  \
     switch (kt) { case 1: GO_V(DT_, 1) break; case 2: GO_V(DT_, 2) break;                          \
                   case 3: GO_V(DT_, 3) break; default: GO_V(DT_, 4) break; }
-        if (dt == ILLM_BF16) { GO_K(ILLM_BF16) } else { GO_K(ILLM_F32) }
+        const bool bf16_rows = dt == ILLM_BF16 && g_attn_cap_mfma == 1 && dk % 8 == 0 && dv % 8 == 0 && q_stride % 8 == 0 &&
+                               own_stride % 8 == 0 && own_k % 8 == 0 && own_v % 8 == 0;
+        if (bf16_rows) {
+#define GOB(KT_, VT_)                                                                              \
+    hipLaunchKernelGGL((attn_cap_rows_bf16_kernel<KT_, VT_>), grid, dim3(256), 0, (hipStream_t)stream, \
+                       (const bf16_t*)q, q_stride, (bf16_t*)out, cu, seq_slot, seq_start, (const bf16_t*)kcache, \
+                       (const bf16_t*)vcache, page_table, table_stride, page_size, ring, nh, nkv, dk, dv, scale, cap, \
+                       window, slopes, chunk, (const bf16_t*)gate, gate_stride, gate_off, gate_heads, lse, keep, kept, \
+                       own_stride, own_k, own_v)
+#define GOB_V(KT_)                                                                                 \
+    switch (vt) { case 1: GOB(KT_, 1); break; case 2: GOB(KT_, 2); break;                          \
+                  case 3: GOB(KT_, 3); break; default: GOB(KT_, 4); break; }
+            switch (kt) { case 1: GOB_V(1) break; case 2: GOB_V(2) break;
+                          case 3: GOB_V(3) break; default: GOB_V(4) break; }
+#undef GOB_V
+#undef GOB
+        } else if (dt == ILLM_BF16) { GO_K(ILLM_BF16) } else { GO_K(ILLM_F32) }
 #undef GO_K
 #undef GO_V
 #undef GO
@@ -851,31 +1076,49 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
     }
 }
 
-// grid (heads, sequences): combine the splits' partial results in split order.
+// grid (heads, sequences): combine the splits' partial results in split order.  CAP_MERGE splits' maxima,
+// sums and values are asked for together before the first is used.
+#define CAP_MERGE 16
 __global__ void attn_cap_merge_kernel(const float* __restrict__ partial, void* __restrict__ out,
                                       int dt, int nsplit, int nh, int dv, const void* __restrict__ gate,
                                       int gate_stride, int gate_off, int gate_heads, float* __restrict__ lse) {
     const int h = blockIdx.x, b = blockIdx.y;
     const float* pp = partial + ((size_t)b * nh + h) * nsplit * (dv + 2);
+    const size_t step = dv + 2;
     float mm = NEG_INF;
-    for (int s = 0; s < nsplit; ++s) mm = fmaxf(mm, pp[(size_t)s * (dv + 2) + dv]);
+    for (int s0 = 0; s0 < nsplit; s0 += CAP_MERGE) {
+        float ms[CAP_MERGE];
+#pragma unroll
+        for (int x = 0; x < CAP_MERGE; ++x) ms[x] = pp[(size_t)min(s0 + x, nsplit - 1) * step + dv];
+#pragma unroll
+        for (int x = 0; x < CAP_MERGE; ++x) mm = fmaxf(mm, ms[x]);
+    }
     float lt = 0.f;
-    for (int s = 0; s < nsplit; ++s) {
-        const float ms = pp[(size_t)s * (dv + 2) + dv];
-        lt += (ms == NEG_INF ? 0.f : expf(ms - mm)) * pp[(size_t)s * (dv + 2) + dv + 1];
-    }
-    const float inv = 1.0f / lt;
-    if (lse && threadIdx.x == 0) lse[(size_t)b * nh + h] = mm + logf(lt);
-    for (int d = threadIdx.x; d < dv; d += blockDim.x) {
+    for (int d0 = 0; d0 < dv || d0 == 0; d0 += blockDim.x) {
+        const int d = min(d0 + (int)threadIdx.x, dv - 1);
         float a = 0.f;
-        for (int s = 0; s < nsplit; ++s) {
-            const float ms = pp[(size_t)s * (dv + 2) + dv];
-            a += (ms == NEG_INF ? 0.f : expf(ms - mm)) * pp[(size_t)s * (dv + 2) + d];
+        lt = 0.f;
+        for (int s0 = 0; s0 < nsplit; s0 += CAP_MERGE) {
+            float ms[CAP_MERGE], ls[CAP_MERGE], v[CAP_MERGE];
+#pragma unroll
+            for (int x = 0; x < CAP_MERGE; ++x) {
+                const float* p = pp + (size_t)min(s0 + x, nsplit - 1) * step;
+                ms[x] = p[dv]; ls[x] = p[dv + 1]; v[x] = p[d];
+            }
+#pragma unroll
+            for (int x = 0; x < CAP_MERGE; ++x) {
+                const float f = (s0 + x >= nsplit || ms[x] == NEG_INF) ? 0.f : expf(ms[x] - mm);
+                lt += f * ls[x];
+                a += f * v[x];
+            }
         }
-        float y = a * inv;
-        if (gate) y *= 1.0f / (1.0f + expf(-ld_f(gate, dt, (size_t)b * gate_stride + gate_off + (gate_heads ? (size_t)h : (size_t)h * dv + d))));
-        st_f(out, dt, ((size_t)b * nh + h) * dv + d, y);
+        if (d0 + (int)threadIdx.x < dv) {
+            float y = a * (1.0f / lt);
+            if (gate) y *= 1.0f / (1.0f + expf(-ld_f(gate, dt, (size_t)b * gate_stride + gate_off + (gate_heads ? (size_t)h : (size_t)h * dv + d))));
+            st_f(out, dt, ((size_t)b * nh + h) * dv + d, y);
+        }
     }
+    if (lse && threadIdx.x == 0) lse[(size_t)b * nh + h] = mm + logf(lt);
 }
 
 extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int dt,

@@ -418,12 +418,16 @@ lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off,
 #pragma unroll
         for (int v = 0; v < 16; ++v) acc[t][v] = 0.f;
         if (n0 >= dv) continue;
-        const bool in = n0 + col < dv;
+        // (rows beyond dk meet zeros of q and columns beyond dv are not stored: read a valid place, no branch)
+        const float* Sc = S + min(n0 + col, dv - 1);
 #pragma unroll
-        for (int s2 = 0; s2 < DKP / 2; ++s2) {
-            const int m = 2 * s2 + half;
-            const float a = (in && m < dk) ? S[(size_t)m * dv + n0 + col] : 0.f;
-            acc[t] = __builtin_amdgcn_mfma_f32_32x32x2f32(a, qr[s2], acc[t], 0, 0, 0);
+        for (int s0 = 0; s0 < DKP / 2; s0 += 16) {
+            float a[16];
+#pragma unroll
+            for (int x = 0; x < 16; ++x) a[x] = Sc[(size_t)min(2 * (s0 + x) + half, dk - 1) * dv];
+#pragma unroll
+            for (int x = 0; x < 16; ++x)
+                acc[t] = __builtin_amdgcn_mfma_f32_32x32x2f32(a[x], qr[s0 + x], acc[t], 0, 0, 0);
         }
     }
     const float f = pw[min(i, nc - 1) + 1];

@@ -592,7 +592,7 @@ def test_pooled_window_attention_against_plain_torch(dtype):
                 _near(o1, want[last], 2 * tol)
 
 
-@pytest.mark.parametrize("matrix_cores", [1, 0])
+@pytest.mark.parametrize("matrix_cores", [1, 2, 0])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_attention_with_one_gate_a_head_against_plain_torch(dtype, matrix_cores):
     """The capped attention's kernels (rows on the matrix cores and on the vector units, single

@@ -487,7 +487,7 @@ def test_activations_without_a_gate_against_plain_torch(dtype):
     _near(ops.xielu(small.cuda(), par.cuda()), R.xielu(small, par), tol)
 
 
-@pytest.mark.parametrize("matrix_cores", [1, 0])
+@pytest.mark.parametrize("matrix_cores", [1, 2, 0])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_windows_with_kept_tokens_against_plain_torch(dtype, matrix_cores):
     """Biases, weighted norms a head, rotation and the store into a line with kept pages and a ring

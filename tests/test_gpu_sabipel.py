@@ -452,7 +452,7 @@ def test_matrix_memory_kernels_against_plain_torch(dtype):
         _near(got, want, 1e-5)
 
 
-@pytest.mark.parametrize("matrix_cores", [1, 0])
+@pytest.mark.parametrize("matrix_cores", [1, 2, 0])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_attention_with_bias_chunks_and_gate_against_plain_torch(dtype, matrix_cores):
     """Norms over whole q and k, value mixing and the store; then rows over the cache and single
