@@ -609,16 +609,16 @@ int illm_removal_step(const void* U, int dt, int u_stride, int r_off, int k_off,
                       const float* a_bias, int w1_off, int rank, const void* w2, const float* w0, float rate,
                       float* state, const int32_t* row_slot, float* o, int B, int H, int d, void* stream);
 // _chunks (removal_chunks.hip): any number of rows, in chunks of illm_removal_chunk() tokens on the matrix
-// cores' float32 instructions; d <= 128, Z of U's dtype; `part`: (T / chunk + n_seqs + 1) H
+// cores' float32 instructions; d <= 128, Z float32; `part`: (T / chunk + n_seqs + 1) H
 // illm_removal_chunk_floats(d) floats.
 int illm_removal_chunk(void);
 int illm_removal_chunk_floats(int d);
 int illm_removal_chunks(const void* U, int dt, int u_stride, int r_off, int k_off, int v_off, int a_off,
-                        const float* a_bias, const void* Z, int z_stride, const float* w0, float rate,
+                        const float* a_bias, const float* Z, int z_stride, const float* w0, float rate,
                         float* state, float* part, const int32_t* cu, const int32_t* seq_slot, float* o,
                         int n_seqs, int max_rows, int H, int d, void* stream);
-// out[t, i] = tanh(U[t, off + i]), i < n, of U's dtype.
-int illm_tanh_columns(const void* U, int dt, int u_stride, int off, void* out, int T, int n, void* stream);
+// out[t, i] = tanh(U[t, off + i]), i < n, float32.
+int illm_tanh_columns(const void* U, int dt, int u_stride, int off, float* out, int T, int n, void* stream);
 // o float32 [T, width] RMS-normed in `groups` equal parts of the row, times w [width], times
 // silu (gate_kind 0) or sigmoid (1) of Z[:, z_off ..].
 int illm_group_norm_gate(const float* o, const void* w, int w_dt, const void* Z, int z_dt, int z_stride,

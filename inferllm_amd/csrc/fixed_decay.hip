@@ -100,14 +100,14 @@ extern "C" int illm_removal_prepare(const void* U, int dt, int u_stride, int r_o
     return illm_launch_status();
 }
 
-// out[t, i] = tanh(U[t, off + i]), i < n.
+// out[t, i] = tanh(U[t, off + i]), i < n, as float32.
 __global__ void __launch_bounds__(256)
-tanh_columns_kernel(const void* __restrict__ U, int dt, int u_stride, int off, void* __restrict__ out, int n) {
+tanh_columns_kernel(const void* __restrict__ U, int dt, int u_stride, int off, float* __restrict__ out, int n) {
     const size_t t = blockIdx.x;
-    for (int i = threadIdx.x; i < n; i += 256) st_f(out, dt, t * n + i, tanhf(ld_f(U, dt, t * u_stride + off + i)));
+    for (int i = threadIdx.x; i < n; i += 256) out[t * n + i] = tanhf(ld_f(U, dt, t * u_stride + off + i));
 }
 
-extern "C" int illm_tanh_columns(const void* U, int dt, int u_stride, int off, void* out, int T, int n,
+extern "C" int illm_tanh_columns(const void* U, int dt, int u_stride, int off, float* out, int T, int n,
                                  void* stream) {
     if (T < 0 || n <= 0 || !illm_dtype_ok(dt) || !fd_columns_ok(u_stride, off, n)) return ILLM_ERR_ARG;
     if (T == 0) return ILLM_OK;

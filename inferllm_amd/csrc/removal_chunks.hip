@@ -35,7 +35,7 @@ __device__ __forceinline__ float rc_sigmoid(float x) { return 1.0f / (1.0f + exp
 template <int DT, int KT>
 __global__ void __launch_bounds__(256)
 removal_chunk_prepare_kernel(const void* __restrict__ U, int u_stride, int r_off, int k_off, int v_off,
-                             int a_off, const float* __restrict__ a_bias, const void* __restrict__ Z,
+                             int a_off, const float* __restrict__ a_bias, const float* __restrict__ Z,
                              int z_stride, const float* __restrict__ w0, float rate, float* __restrict__ part,
                              const int32_t* __restrict__ cu, int H, int d) {
     constexpr int DP = 32 * KT, LD = DP + 1, GA = RC + 4, GL = RC + 1;
@@ -80,7 +80,7 @@ removal_chunk_prepare_kernel(const void* __restrict__ U, int u_stride, int r_off
             const int hc = h * d + (in ? ch : 0);
             const float bias0 = w0[hc], abias = a_bias[hc];
             auto log_decay = [&](int t) {
-                return (in && t < nc) ? -rate * rc_sigmoid(ld_f(Z, DT, (row0 + t) * z_stride + hc) + bias0) : 0.f;
+                return (in && t < nc) ? -rate * rc_sigmoid(Z[(row0 + t) * z_stride + hc] + bias0) : 0.f;
             };
             float L = 0.f;
 #pragma unroll 4
@@ -327,7 +327,7 @@ extern "C" int illm_removal_chunk(void) { return RC; }
 extern "C" int illm_removal_chunk_floats(int d) { return d > 0 && d <= 128 ? (int)rc_floats((d + 31) / 32 * 32) : 0; }
 
 extern "C" int illm_removal_chunks(const void* U, int dt, int u_stride, int r_off, int k_off, int v_off, int a_off,
-                                   const float* a_bias, const void* Z, int z_stride, const float* w0, float rate,
+                                   const float* a_bias, const float* Z, int z_stride, const float* w0, float rate,
                                    float* state, float* part, const int32_t* cu, const int32_t* seq_slot, float* o,
                                    int n_seqs, int max_rows, int H, int d, void* stream) {
     auto cols = [&](int off) { return off >= 0 && off + H * d <= u_stride; };

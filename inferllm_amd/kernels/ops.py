@@ -2302,10 +2302,10 @@ def lightning_chunks(U: torch.Tensor, q_off: int, k_off: int, v_off: int, decay:
 
 
 def tanh_columns(U: torch.Tensor, off: int, n: int) -> torch.Tensor:
-    """[T, n]: tanh of U's columns off .. off + n, in U's dtype."""
+    """float32 [T, n]: tanh of U's columns off .. off + n."""
     _gpu(U)
     _columns_ok(U, "tanh_columns", (off, n))
-    out = torch.empty((U.shape[0], n), dtype=U.dtype, device=U.device)
+    out = torch.empty((U.shape[0], n), dtype=torch.float32, device=U.device)
     _check(_lib().illm_tanh_columns(_p(U), _code(U), U.shape[1], off, _p(out), U.shape[0], n, _stream()), "tanh_columns")
     return out
 
@@ -2349,9 +2349,9 @@ def removal_chunks(U: torch.Tensor, r_off: int, k_off: int, v_off: int, a_off: i
     _columns_ok(U, "removal_chunks", *((off, H * d) for off in (r_off, k_off, v_off, a_off)))
     _removal_ok(H, d, a_bias, w0, "removal_chunks")
     T = U.shape[0]
-    _need(d <= REMOVAL_CHUNKS_MAX_DIM and Z.shape == (T, H * d) and Z.dtype == U.dtype and state.dtype == torch.float32
+    _need(d <= REMOVAL_CHUNKS_MAX_DIM and Z.shape == (T, H * d) and Z.dtype == torch.float32 and state.dtype == torch.float32
           and state.dim() == 4 and state.shape[1:] == (H, d, d),
-          "removal_chunks: Z [T, H d] of U's dtype, state float32 [slots, H, d, d], d <= 128")
+          "removal_chunks: Z float32 [T, H d], state float32 [slots, H, d, d], d <= 128")
     places = T // _lib().illm_removal_chunk() + n_seqs + 1
     part = torch.empty((places * H * _lib().illm_removal_chunk_floats(d),), dtype=torch.float32, device=U.device)
     o = torch.empty((T, H, d), dtype=torch.float32, device=U.device)

@@ -352,8 +352,10 @@ class RemovalDeltaRule(Mixer):
         self.w_in = ops.decode_weight(_fuse([take(t) for t in ("r", "k", "v", "a", "g", "w1")]), "plain",
                                       self.decode_copies)
         self.k_off, self.v_off, self.a_off, self.g_off, self.w1_off = n, 2 * n, 3 * n, 4 * n, 5 * n
+        # (the decays' map from the tanh on is float32 arithmetic: single tokens read the stored rows,
+        # steps of several tokens a float32 copy)
         self.w2_rows = take("w2").to(ops.plain_weight(self.w_in).dtype).contiguous()
-        self.w_w2 = ops.decode_weight(self.w2_rows, "plain", self.decode_copies)
+        self.w_w2 = self.w2_rows.to(torch.float32).contiguous()
         self.a_bias, self.w0, self.norm_w = f32("a_bias"), f32("w0"), take("norm").contiguous()
         self.w_o = ops.decode_weight(take("o").contiguous(), "plain", self.decode_copies)
 

@@ -966,7 +966,7 @@ def lightning_step(U, q_off, k_off, v_off, decay, state, row_slot, H, dk, dv):
 
 
 def tanh_columns(U, off, n):
-    return torch.tanh(U[:, off:off + n].to(F64)).to(U.dtype)
+    return torch.tanh(U[:, off:off + n].to(F64)).to(torch.float32)
 
 
 def removal_prepare(U, r_off, k_off, v_off, a_off, a_bias, Z, w0, rate, H, d):

@@ -482,7 +482,7 @@ def test_activations_without_a_gate_against_plain_torch(dtype):
         _near(ops.xielu(x.cuda(), par.cuda()), R.xielu(x, par), tol)
         _near(ops.relu_squared(x.cuda()), R.relu_squared(x), tol)
         _near(ops.tanh_columns(x.cuda(), shape[1] // 2, shape[1] - shape[1] // 2),
-              R.tanh_columns(x, shape[1] // 2, shape[1] - shape[1] // 2), tol)
+              R.tanh_columns(x, shape[1] // 2, shape[1] - shape[1] // 2), 1e-5)
     small = torch.tensor([[-1e-3, 1e-4, -30.0, -100.0, 0.0, 50.0]]).to(dtype)
     _near(ops.xielu(small.cuda(), par.cuda()), R.xielu(small, par), tol)
 
@@ -610,7 +610,7 @@ def test_delta_rule_with_a_removal_vector_against_plain_torch(dtype):
             T = sum(lens)
             cu, seq_slot, row_slot = _packed(lens, [4, 0, 2, 5][:len(lens)])
             U = torch.randn(T, w1_off + rank + 1, generator=g).to(dtype)
-            Z = torch.randn(T, n, generator=g).to(dtype)
+            Z = torch.randn(T, n, generator=g)
             state = torch.randn(6, H, d, d, generator=g)
             want_in = R.removal_prepare(U, *offs, a_bias, Z, w0, rate, H, d)
             got_in = ops.removal_prepare(U.cuda(), *offs, a_bias.cuda(), Z.cuda(), w0.cuda(), rate, H, d)
