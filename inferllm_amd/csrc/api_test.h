@@ -46,7 +46,8 @@ void illm_set_rows_a_launch(int rows);
 // or not in steps of 4 use, instead of the matrix cores; 2 also bfloat16 rows to the one on their
 // float32 instruction (default 1: bfloat16 rows in steps of 8 the bfloat16 instruction).
 void illm_set_attn_cap_mfma(int on);
-// illm_attn_cap_decode, eight lanes a key: query heads of a kv head that a block takes, 4 (default) or 2.
+// illm_attn_cap_decode, eight lanes a key: query heads of a kv head that a block takes, 4, 2 or 1 (0,
+// the default: 4, or fewer while there are fewer than 256 blocks).
 void illm_set_attn_cap_heads(int n);
 
 #ifdef __cplusplus

@@ -687,8 +687,8 @@ attn_cap_rows_bf16_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __
 // cores' float32 instruction also for bfloat16 storage.
 static int g_attn_cap_mfma = 1;
 extern "C" void illm_set_attn_cap_mfma(int on) { g_attn_cap_mfma = on < 0 || on > 2 ? 1 : on; }
-static int g_attn_cap_heads = 4;
-extern "C" void illm_set_attn_cap_heads(int n) { g_attn_cap_heads = n == 2 ? 2 : 4; }
+static int g_attn_cap_heads = 0;
+extern "C" void illm_set_attn_cap_heads(int n) { g_attn_cap_heads = (n == 1 || n == 2 || n == 4) ? n : 0; }
 
 extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt, const int32_t* cu,
                                   const int32_t* seq_slot, const int32_t* seq_start,
@@ -1019,8 +1019,9 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
             d += cap_dpp<0x141>(d);
             const float sc = valid ? soft_cap(d * scale, cap, inv_cap) - slope[i] * (float)(len - 1 - kj) : NEG_INF;
             const float m_new = fmaxf(m[i], sc);
-            const float alpha = m_new == NEG_INF ? 1.f : expf(m[i] - m_new);
-            const float p = valid ? expf(sc - m_new) : 0.f;
+            // (bfloat16 keys and values: the hardware's exponential, float32 with an error of |x| 2^-24)
+            const float alpha = m_new == NEG_INF ? 1.f : DT == ILLM_BF16 ? __expf(m[i] - m_new) : expf(m[i] - m_new);
+            const float p = !valid ? 0.f : DT == ILLM_BF16 ? __expf(sc - m_new) : expf(sc - m_new);
             l[i] = l[i] * alpha + p;
             m[i] = m_new;
 #pragma unroll
@@ -1051,28 +1052,28 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
         if (lane == 0) { wm[w][i] = mm; wl[w][i] = lt; }
     }
     __syncthreads();
-    for (int i = 0; i < hb; ++i) {
+    // the four waves into one: the block's threads over all (head, value dim) pairs
+    for (int e = threadIdx.x; e < hb * dv; e += 256) {
+        const int i = e / dv, d = e - i * dv;
         float mm = wm[0][i];
         for (int x = 1; x < 4; ++x) mm = fmaxf(mm, wm[x][i]);
-        float f[4], lt = 0.f;
+        float lt = 0.f, y = 0.f;
+#pragma unroll
         for (int x = 0; x < 4; ++x) {
-            f[x] = wm[x][i] == NEG_INF ? 0.f : expf(wm[x][i] - mm);
-            lt += f[x] * wl[x][i];
+            const float f = wm[x][i] == NEG_INF ? 0.f : expf(wm[x][i] - mm);
+            lt += f * wl[x][i];
+            y += f * wacc[x][i][d];
         }
         if (nsplit == 1) {                              // the one range is the whole result: no merge
-            const float inv = 1.0f / lt;
-            for (int d = threadIdx.x; d < dv; d += 256) {
-                float y = (f[0] * wacc[0][i][d] + f[1] * wacc[1][i][d] + f[2] * wacc[2][i][d] + f[3] * wacc[3][i][d]) * inv;
-                if (gate)
-                    y *= 1.0f / (1.0f + expf(-ld_f(gate, DT, (size_t)b * gate_stride + gate_off + (gate_heads ? (size_t)(h0 + i) : (size_t)(h0 + i) * dv + d))));
-                st_f(out, DT, ((size_t)b * nh + h0 + i) * dv + d, y);
-            }
+            y *= 1.0f / lt;
+            if (gate)
+                y *= 1.0f / (1.0f + expf(-ld_f(gate, DT, (size_t)b * gate_stride + gate_off + (gate_heads ? (size_t)(h0 + i) : (size_t)(h0 + i) * dv + d))));
+            st_f(out, DT, ((size_t)b * nh + h0 + i) * dv + d, y);
             continue;
         }
         float* pp = partial + (((size_t)b * nh + h0 + i) * nsplit + sp) * (dv + 2);
-        for (int d = threadIdx.x; d < dv; d += 256)
-            pp[d] = f[0] * wacc[0][i][d] + f[1] * wacc[1][i][d] + f[2] * wacc[2][i][d] + f[3] * wacc[3][i][d];
-        if (threadIdx.x == 0) { pp[dv] = mm; pp[dv + 1] = lt; }
+        pp[d] = y;
+        if (d == 0) { pp[dv] = mm; pp[dv + 1] = lt; }
     }
 }
 
@@ -1139,13 +1140,21 @@ extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int 
     hipStream_t st = (hipStream_t)stream;
     const int unit = dt == ILLM_BF16 ? 8 : 4;
     if (g_attn_cap_mfma && dk <= 128 && dv <= 128 && dk % unit == 0 && dv % unit == 0 && q_stride % unit == 0) {
-        // four query heads of a kv head a block (their keys and values are read once), or two where
-        // that is asked for: half the registers, twice the waves a SIMD, the rows read twice
-        const int rep = nh / nkv, dh = g_attn_cap_heads == 2 ? 2 : 4;
+        // four query heads of a kv head a block (their keys and values are read once), or fewer while that
+        // leaves compute units without a block: the heads of a block are gone through one after the other
+        const int rep = nh / nkv;
+        int dh = g_attn_cap_heads;
+        if (dh == 0)
+            for (dh = 4; dh > 1 && (long)nkv * ((rep + dh - 1) / dh) * B * nsplit < 256;) dh /= 2;
         const dim3 grid(nkv * ((rep + dh - 1) / dh), B, nsplit);
         const int kq = (dk + 8 * unit - 1) / (8 * unit), vq = (dv + 8 * unit - 1) / (8 * unit);
 #define GO(DT_, KQ_, VQ_)                                                                          \
-    if (dh == 2)                                                                                   \
+    if (dh == 1)                                                                                   \
+        hipLaunchKernelGGL((attn_cap_decode_rows8_kernel<DT_, KQ_, VQ_, 1>), grid, dim3(256), 0, st, q, q_stride, \
+                           kcache, vcache, page_table, table_stride, page_size, ring, seq_slot, seq_len, partial, \
+                           nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads, \
+                           keep, kept);                                                            \
+    else if (dh == 2)                                                                              \
         hipLaunchKernelGGL((attn_cap_decode_rows8_kernel<DT_, KQ_, VQ_, 2>), grid, dim3(256), 0, st, q, q_stride, \
                            kcache, vcache, page_table, table_stride, page_size, ring, seq_slot, seq_len, partial, \
                            nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads, \
