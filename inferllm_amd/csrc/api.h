@@ -463,7 +463,7 @@ int illm_qkv_norm_mix_store(void* rows, int dt, int row_len, int k_off, int v_of
 // ---- what stands around the plain gated recurrence (linear_scan.hip, delta_rule.hip)
 // The scan of illm_delta_scan with a choice of rule: `correct` 1, the delta rule; 0, the plain gated
 // rule S <- diag(g) S + k (beta v)^T, o = S^T q; with `removal` float32 [T, H, dk] (correct 0, G = H)
-// S <- diag(g) S - removal (u^T S) + k v^T, u = beta k, both terms from the old state.
+// S_new = diag(g) S - removal (u^T S) + k v^T, u = beta k, o = S_new^T q.
 int illm_gated_scan(const float* qn, const float* kn, const float* vv, const float* beta,
                     const float* dec, int DW, float* state, const int32_t* cu,
                     const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int G, int H, int dk,

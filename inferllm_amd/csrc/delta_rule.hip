@@ -14,8 +14,8 @@
 // which is the recurrence of state-space and matrix-memory mixers (linear_scan.hip prepares their
 // inputs): beta is then the weight of the token's outer product.  And it runs the delta rule with a
 // removal vector of its own (`removal` given, c = a u with a rate a per channel),
-//     S <- diag(g) S - c (u^T S) + k v^T,  u = beta k;   o = S^T q
-// where both terms read the old state; beta is then 1 / |k|.
+//     S_new = diag(g) S - c (u^T S) + k v^T,  u = beta k;   o = S_new^T q
+// (decay and removal act side by side on what the token found); beta is then 1 / |k|.
 // Everything but the stored projections is float32.  A sequence's rows in a step are consecutive;
 // a step may go on from any state (single tokens, portions of a prompt) or start from the zeros a
 // fresh slot holds.  Sums run in an order fixed by the sizes alone.

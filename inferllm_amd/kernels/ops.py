@@ -1712,8 +1712,7 @@ def delta_scan(qn, kn, vv, beta, dec, state: torch.Tensor, cu_seqlens: torch.Ten
     """The recurrence S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q over every
     sequence's rows in order, from `state` float32 [slots, H, dk, dv] and back into it.  With
     `correct` False the plain gated rule, u = beta v: S <- diag(g) S + k (beta v)^T; with `removal`
-    float32 [T, H, dk] too, S <- diag(g) S - removal (u^T S) + k v^T with u = beta k, both terms from
-    the old S.
+    float32 [T, H, dk] too, S_new = diag(g) S - removal (u^T S) + k v^T with u = beta k.
     `max_rows`: the most rows a sequence brings (long sequences are laid out for their chain of
     tokens, short steps for the state's bytes).  Returns o float32 [T, H, dv]."""
     _gpu(qn, kn, vv, beta, dec, state, cu_seqlens, seq_slot)

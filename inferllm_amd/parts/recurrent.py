@@ -313,7 +313,7 @@ class RemovalDeltaRule(Mixer):
 
         r = W_r h,  k = W_k h,  v = W_v h,   u = k / sqrt(sum k^2 + 1e-6) a head
         w = exp(-exp(-1/2) sigmoid(W_w2 tanh(W_w1 h) + w0)),   a = sigmoid(W_a h + b_a)     a head and channel
-        S <- diag(w) S - (a u) (u^T S) + k v^T   (both terms from the old S);   o = S^T r
+        S_new = diag(w) S - (a u) (u^T S) + k v^T;   o = S_new^T r
         out = W_o (o / rms(o) * norm * sigmoid(W_g h))
 
     rms over each head's outputs (`eps`), `norm` of all heads' width.  Kept per sequence: S (float32).

@@ -97,7 +97,7 @@ def lightning(h, w, p, m, eps):
 
 
 def general_delta(h, w, p, m, eps):
-    """S <- diag(w) S - (a u) (u^T S) + k v^T, both terms from the old S, with the unit key u."""
+    """S_new = diag(w) S - (a u) (u^T S) + k v^T with the unit key u; o = S_new^T r."""
     H, d = m["heads"], m["dim"]
     T = h.shape[0]
     heads = lambda n: (h @ w[p + n].T).view(T, H, d)
