@@ -50,11 +50,13 @@ class ScheduleEntry:
     `layer` indexes `ModelSpec.layers` (the weights).  `cache_line` names the
     cache storage this run uses; runs that share a number share keys and values.
     `writes_cache` False makes the run read what an earlier run of the same step
-    stored on that line instead of storing its own.
+    stored on that line instead of storing its own.  `adds_embedding`: the embedding's output
+    is added to the residual stream ahead of this run.
     """
     layer: int
     cache_line: int
     writes_cache: bool = True
+    adds_embedding: bool = False
 
 
 @dataclass

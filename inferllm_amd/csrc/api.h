@@ -19,6 +19,11 @@ int illm_embed(const int32_t* tokens, const void* table, int table_dt, float* ou
 int illm_embed_scaled(const int32_t* tokens, const void* table, int table_dt, float* out,
                       int T, int E, int V, float scale, void* stream);
 
+// out[t, :] = v / sqrt(mean(v^2) + eps) * w, v = table[tokens[t]] * scale; `copy` (null: none) takes it too.
+int illm_embed_norm(const int32_t* tokens, const void* table, int table_dt, const void* w, int w_dt, float* out,
+                    float* copy, int T, int E, int V, float scale, float eps, void* stream);
+int illm_copy_rows(const float* x, float* out, size_t n, void* stream);
+
 // out[t, :] = table[tokens[t]] * scale + pairs[(prev * mul_prev + tokens[t] * mul_cur) mod buckets]
 // + places[row_pos[t]]: prev is the token above in the step if it belongs to the same slot, else
 // last_token[slot]; a row at position 0 takes pairs[buckets].  pairs, places may be null.  `remember`
@@ -226,6 +231,12 @@ int illm_gemm_mid_splits(int N, int K);
 // only): as for illm_gemm_skinny_bf16.
 int illm_gemm_rows_bf16(const void* X, const void* Wt, void* Y, int y_dt, int M, int N, int K,
                         const float* ssq, int parts, float eps, void* stream);
+// Products whose parts of W read rows of X of their own, X [planes][M][K] (planes <= 8): W's rows ends[p - 1] ..
+// ends[p] - 1 times plane p.  _skinny (see above): M <= 16, parts but the last multiples of 16 rows; _rows: of 32.
+int illm_gemm_skinny_planes(const void* X, const void* W, const void* Wt, void* Y, int y_dt, int M, int N, int K,
+                            int planes, const int* ends, void* stream);
+int illm_gemm_rows_planes(const void* X, const void* Wt, void* Y, int y_dt, int M, int N, int K, int planes,
+                          const int* ends, void* stream);
 int illm_gemm_rows_gateup_silu(const void* X, const void* Wt, void* Y, int y_dt, int M, int F,
                                int K, const float* ssq, int parts, float eps, void* stream);
 // The same with the clamped gate in place of SiLU where limit > 0: Y = g sigmoid(alpha g) (u + 1),
@@ -361,7 +372,9 @@ int illm_few_outputs_f32(const void* x, int x_dt, const float* w, float* z, int 
 // (corr may be null), in falling order, and their softmax values.  NE <= 512.
 // score_kind 0: softmax over all outputs; 1: every output's sigmoid.  The weights are scale times them.
 int illm_moe_route(const float* z, const void* corr, int corr_dt, int T, int NE, int top,
-                   int32_t* idx, float* wt, int score_kind, float scale, void* stream);
+                   int32_t* idx, float* wt, int score_kind, float scale, int groups, int keep, void* stream);
+// (`groups` > 0: equal groups of neighbouring outputs, of which only the `keep` with the largest sums of
+// their two largest choice scores can be chosen from; top <= keep NE / groups)
 
 // order [NP]: the pairs whose choice is below NEr, grouped by choice; tiles [3 max_tiles + 1]:
 // (expert, first place in order, rows <= tile_rows) per tile and, last, their number.
@@ -433,14 +446,15 @@ int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt, const int
                        int page_size, int ring, int n_seqs, int max_rows, int nh, int nkv, int dk,
                        int dv, float scale, float cap, int window, const float* slopes, int chunk,
                        const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse,
-                       int keep, int kept, int own_stride, int own_k, int own_v, void* stream);
+                       int keep, int kept, int own_stride, int own_k, int own_v_stride, int own_v,
+                       const float* sink, void* stream);
 int illm_attn_cap_decode(const void* q, int q_stride, void* out, int dt, const void* kcache,
                          const void* vcache, const int32_t* page_table, int table_stride,
                          int page_size, int ring, const int32_t* seq_slot, const int32_t* seq_len,
                          float* partial, int nsplit, int B, int nh, int nkv, int dk, int dv,
                          float scale, float cap, int window, const float* slopes, int chunk,
                          const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse,
-                         int keep, int kept, void* stream);
+                         int keep, int kept, const float* sink, void* stream);
 // The two calls above also take: `slopes` float32 [nh] (null: none), score -= slopes[h] (i - j);
 // `chunk` > 0, a row sees only the keys j with floor(j / chunk) = floor(i / chunk); `gate` (null: none),
 // rows [., gate_stride] of the queries' dtype, out *= sigmoid(gate[row, gate_off + h dv + d]) (with
@@ -449,7 +463,8 @@ int illm_attn_cap_decode(const void* q, int q_stride, void* out, int dt, const v
 // first `keep` tokens are seen beside the window; `kept`: the pages that stay in place ahead of the
 // cache line's ring.  illm_attn_cap_rows with own_stride > 0 reads keys and values not from the cache
 // but from the step's own rows, kcache and vcache then their base (row r of sequence b at (cu[b] + r)
-// own_stride, key heads from column own_k, value heads from own_v); every sequence starts in this step.
+// own_stride + own_k and (cu[b] + r) own_v_stride + own_v); every sequence starts in this step.  `sink`
+// (float32 [nh], null: none): exp(sink[h]) is in the softmax's denominator beside the keys'.
 // In place: q and k of rows [q (nh dk) | .. k at k_off | v at v_off] each divided by the root mean
 // square over all their heads and multiplied by qw, kw (null: untouched); v <- (1 - lam[0]) v +
 // lam[0] first[row, first_off ..] (lam null: untouched); k and v stored in the paged cache (null: not).
@@ -463,7 +478,8 @@ int illm_qkv_norm_mix_store(void* rows, int dt, int row_len, int k_off, int v_of
 // ---- what stands around the plain gated recurrence (linear_scan.hip, delta_rule.hip)
 // The scan of illm_delta_scan with a choice of rule: `correct` 1, the delta rule; 0, the plain gated
 // rule S <- diag(g) S + k (beta v)^T, o = S^T q; with `removal` float32 [T, H, dk] (correct 0, G = H)
-// S_new = diag(g) S - removal (u^T S) + k v^T, u = beta k, o = S_new^T q.
+// S_new = diag(g) S - removal (u^T S) + k v^T, u = beta k, o = S_new^T q; `correct` 2, o = S^T q + beta v from
+// the state before the token, then S <- diag(g) S + k v^T.
 int illm_gated_scan(const float* qn, const float* kn, const float* vv, const float* beta,
                     const float* dec, int DW, float* state, const int32_t* cu,
                     const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int G, int H, int dk,
@@ -530,13 +546,16 @@ int illm_clamped_swish_mul(const void* gate_up, void* out, int dt, int T, int F,
 // stored in the paged cache (kcache null: not stored; nkv 0: queries alone).  Ahead of the rotation
 // `bias` float32 [q | k | v] (null: none) is added and q and k heads are RMS-normed (eps) under qw, kw
 // [dk] (null: not).  `slot_len` (int32 by slot, the lengths after the step; null: every row is stored):
-// rows that later rows of the step overwrite in the ring are not stored.  `kept` as above.
+// rows that later rows of the step overwrite in the ring are not stored.  `kept` as above.  `v_from_k`
+// (dv = dk): the values are the keys ahead of norm and rotation, and rows have no value columns; `v_rows`
+// [T, nkv dv] (null: not) takes them.
 int illm_qk_rotate_store(void* rows, int dt, int row_len, int k_off, int v_off, const float* cos_sin,
                          int rot, int pairing, int n_positions, int unit_norm, float eps,
                          const float* q_scale, const int32_t* row_pos, const int32_t* row_slot, void* kcache, void* vcache,
                          const int32_t* page_table, int table_stride, int page_size, int ring, int T,
                          int nh, int nkv, int dk, int dv, const float* bias, const void* qw,
-                         const void* kw, int w_dt, const int32_t* slot_len, int kept, void* stream);
+                         const void* kw, int w_dt, const int32_t* slot_len, int kept, int v_from_k,
+                         void* v_rows, void* stream);
 // For every row whose position ends a block of `pool` tokens: the block's mean key and value, from
 // the cache, into row (position / pool) of the sequence in kpool, vpool (same layout and page table).
 int illm_pool_store(const int32_t* row_pos, const int32_t* row_slot, const void* kcache,
@@ -619,7 +638,51 @@ int illm_removal_chunks(const void* U, int dt, int u_stride, int r_off, int k_of
                         int n_seqs, int max_rows, int H, int d, void* stream);
 // out[t, i] = tanh(U[t, off + i]), i < n, float32.
 int illm_tanh_columns(const void* U, int dt, int u_stride, int off, float* out, int T, int n, void* stream);
-// o float32 [T, width] RMS-normed in `groups` equal parts of the row, times w [width], times
+// Retention from U likewise, q and k turned by the row's position (pairs i, i + rot / 2; cos_sin float32
+// [n_positions, rot / 2, 2]) and k times k_scale, no activations.  _prepare: qn, kn float32 [T, H, dk] and,
+// where given, vv, beta (1) and dec for illm_gated_scan.  _step: one row a sequence in one launch.  _chunks:
+// from qn, kn and v in U's columns, sizes and `part` as for illm_lightning_chunks.
+int illm_retention_prepare(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off, const float* decay,
+                           const float* cos_sin, int n_positions, int rot, float k_scale, const int32_t* row_pos,
+                           float* qn, float* kn, float* vv, float* beta, float* dec, int T, int H, int dk, int dv,
+                           void* stream);
+int illm_retention_step(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off, const float* decay,
+                        const float* cos_sin, int n_positions, int rot, float k_scale, const int32_t* row_pos,
+                        float* state, const int32_t* row_slot, float* o, int B, int H, int dk, int dv, void* stream);
+int illm_retention_chunks(const float* qn, const float* kn, const void* U, int dt, int u_stride, int v_off,
+                          const float* decay, float* state, float* part, const int32_t* cu, const int32_t* seq_slot,
+                          float* o, int n_seqs, int max_rows, int H, int dk, int dv, void* stream);
+// Time mixing (fixed_decay.hip, time_mix.hip): w = exp(-exp(z + w0)) a head and channel, o = (S + diag(bonus) k
+// v^T)^T r, S <- diag(w) S + k v^T; r, k, v rows of `stride` numbers (H d used), all heads d x d.
+// illm_token_mix: out[s] = h + (h_before - h) mu[s] for S mixes of X's rows, h_before of a step's first row from
+// tail [slots, E], which `update_tail` (one row a sequence) moves on.  _step: one row a sequence in one launch, z
+// = w2 tanh(low) (w2 [H d, rank] of the rows' dtype, rank <= 512).  _prepare: inputs of illm_gated_scan with
+// `correct` 2.  _chunks: any number of rows, in chunks of illm_time_mix_chunk() tokens on the matrix cores'
+// float32 instructions; d <= 128 in steps of 4; scratch: L T H d floats, part (T / chunk + n_seqs + 1) H d d,
+// whole as many H d.
+int illm_token_mix(const void* X, int dt, const float* mu, int S, void* tail, const int32_t* row_slot, void* out,
+                   int out_dt, int T, int E, int update_tail, void* stream);
+int illm_time_mix_step(const void* r, const void* k, const void* v, int dt, int stride, const void* low,
+                       int low_stride, int rank, const void* w2, const float* w0, const float* bonus, float* state,
+                       const int32_t* row_slot, float* o, int B, int H, int d, void* stream);
+int illm_time_mix_prepare(const void* R, const void* K, const void* V, int dt, int stride, const float* Z,
+                          const float* w0, const float* bonus, float* qn, float* kn, float* vv, float* beta,
+                          float* dec, int T, int H, int d, void* stream);
+int illm_time_mix_chunk(void);
+int illm_time_mix_chunks(const void* R, const void* K, const void* V, int dt, int stride, const float* Z,
+                         const float* w0, const float* bonus, float* state, float* L, float* part, float* whole,
+                         const int32_t* cu, const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int H, int d,
+                         void* stream);
+// One pass between two sublayers (post_norm.hip): y = a, or with b y = pair_scale (rms(a) aw + rms(b) bw);
+// x <- x + gain rms(y) pw + plus (a, plus may be null); h = rms(x) w in the output's type; out = h, or with mu
+// out[s] = h + (tail[slot] - h) mu[s] for S mixes, and tail takes h (one row a sequence).  With row_idx only those
+// rows are formed and x stays.  E <= 6144 or a multiple of 4 up to 8192.
+int illm_post_mix_norm(float* x, const void* a, int a_dt, const void* b, int b_dt, const void* aw, const void* bw,
+                       int pair_dt, float pair_eps, float pair_scale, const void* pw, int pw_dt, float post_eps,
+                       float gain, const float* plus, const void* w, int w_dt, float eps, void* out, int out_dt,
+                       const float* mu, int S, void* tail, int tail_dt, const int32_t* row_slot,
+                       const int32_t* row_idx, int rows, int E, void* stream);
+// o float32 [T, width] RMS-normed in `groups` equal parts of the row, times w [width] (null: 1), times
 // silu (gate_kind 0) or sigmoid (1) of Z[:, z_off ..].
 int illm_group_norm_gate(const float* o, const void* w, int w_dt, const void* Z, int z_dt, int z_stride,
                          int z_off, int gate_kind, void* out, int out_dt, int T, int width, int groups,

@@ -8,13 +8,15 @@
 // position 0 (`chunk` <= 0: none); an output gate, out *= sigmoid(gate[row, gate_off + h dv + d])
 // (`gate` null: none; with `gate_heads` one number a head, gate[row, gate_off + h]).  Positions enter
 // through the bias and the chunks alone.  `lse` (null: none) takes max + log(sum) of every row's and
-// head's softmax, [rows][heads], for whoever goes on with further keys.
+// head's softmax, [rows][heads], for whoever goes on with further keys.  `sink` (null: none): one number a
+// head whose exponential the denominator contains too, without a key or a value.
 // Keys and values live in the paged cache, K [page][kv head][row][dk], V [page][kv head][row][dv],
 // under one page table; a step first stores its rows (`kv_store2`) and then every row attends over
 // the cache at absolute positions, so whole prompts, portions of prompts and single tokens take
 // the same path.  A line that keeps a window as a ring of pages (the first `kept` pages beside it)
 // does not hold a long prompt: rows of a step whose sequences all start may read the step's own rows
-// instead (`own_stride` > 0: keys at column own_k, values at own_v of the rows that q lies in).
+// instead (`own_stride` > 0: keys at column own_k of the rows that q lies in, values at own_v of rows of
+// own_v_stride numbers).
 // Float32 sums, scores and weights over float32 or bfloat16 storage: widths of up to 128 in steps
 // of 4 (single tokens: of 16 bytes) take the kernels on the matrix cores' float32 instruction and
 // with eight lanes a key (rows of bfloat16 in steps of 8 the bfloat16 instruction), every other width the
@@ -27,6 +29,11 @@
 #define CQ 32  // query rows of a block
 #define CK 32  // keys of a tile
 #define NEG_INF (-INFINITY)
+
+// A sink in the softmax's denominator: l, the sum of exp(score - m), gets exp(sink - m) more.  The exponent
+// is held below the overflow of float32: a sink that far above every score leaves nothing of the values
+// either way.
+__device__ __forceinline__ void add_sink(float sink, float m, float& l) { l += expf(fminf(sink - m, 80.f)); }
 
 __device__ __forceinline__ float soft_cap(float s, float cap, float inv_cap) {
     return cap > 0.f ? cap * tanhf(s * inv_cap) : s;
@@ -161,7 +168,8 @@ attn_cap_rows_kernel(const void* __restrict__ q, int q_stride, void* __restrict_
                      int table_stride, int page_size, int ring, int nh, int nkv, int dk, int dv,
                      float scale, float cap, int window, const float* __restrict__ slopes, int chunk,
                      const void* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
-                     float* __restrict__ lse, int keep, int kept, int own_stride, int own_k, int own_v) {
+                     float* __restrict__ lse, int keep, int kept, int own_stride, int own_k,
+                          int own_v_stride, int own_v, const float* __restrict__ sink) {
     extern __shared__ float smem[];
     const int kp = dk + 1, vp = dv + 1;
     float* qs = smem;               // [CQ][kp]
@@ -207,7 +215,7 @@ attn_cap_rows_kernel(const void* __restrict__ q, int q_stride, void* __restrict_
         for (int e = tid; e < CK * dv; e += 256) {
             const int r = e / dv, d = e - r * dv;
             vs[r * vp + d] = k0 + r < total
-                ? ld_f(vcache, dt, (own_stride ? (size_t)(start + k0 + r) * own_stride + own_v + (size_t)kvh * dv
+                ? ld_f(vcache, dt, (own_stride ? (size_t)(start + k0 + r) * own_v_stride + own_v + (size_t)kvh * dv
                                                : cache_row_offset(page_table, table_stride, slot, k0 + r, page_size, ring, nkv, kvh, dv, kept)) + d)
                 : 0.f;
         }
@@ -252,6 +260,7 @@ attn_cap_rows_kernel(const void* __restrict__ q, int q_stride, void* __restrict_
         }
     }
     if (qrow < len) {
+        if (sink) add_sink(sink[h], m_i, l_i);
         const float inv = 1.0f / l_i;
         if (lse && g == 0) lse[(size_t)(start + qrow) * nh + h] = m_i + logf(l_i);
         const size_t ob = (size_t)(start + qrow) * nh * dv + (size_t)h * dv;
@@ -326,7 +335,8 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
                           int table_stride, int page_size, int ring, int nh, int nkv, int dk, int dv,
                           float scale, float cap, int window, const float* __restrict__ slopes, int chunk,
                           const void* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
-                          float* __restrict__ lse, int keep, int kept, int own_stride, int own_k, int own_v) {
+                          float* __restrict__ lse, int keep, int kept, int own_stride, int own_k,
+                          int own_v_stride, int own_v, const float* __restrict__ sink) {
     constexpr int DKP = 32 * KT, DVP = 32 * VT, KLD = DKP + 1;
     __shared__ float ks[MK * KLD];
     __shared__ float vs[MK * DVP];
@@ -375,7 +385,7 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
             const int kj = min(k0 + row, total - 1);
             vreg[i].zero();
             if (d < dv)
-                vreg[i].load(vcache, (own_stride ? (size_t)(start + kj) * own_stride + own_v + (size_t)kvh * dv
+                vreg[i].load(vcache, (own_stride ? (size_t)(start + kj) * own_v_stride + own_v + (size_t)kvh * dv
                                                  : cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dv, kept)) + d);
         }
     };
@@ -459,6 +469,7 @@ attn_cap_rows_mfma_kernel(const void* __restrict__ q, int q_stride, void* __rest
         }
     }
     if (qrow < len) {
+        if (sink) add_sink(sink[h], m_i, l_i);
         const float inv = 1.0f / l_i;
         if (lse && half == 0) lse[(size_t)(start + qrow) * nh + h] = m_i + logf(l_i);
         const size_t ob = (size_t)(start + qrow) * nh * dv + (size_t)h * dv;
@@ -495,7 +506,8 @@ attn_cap_rows_bf16_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __
                           int table_stride, int page_size, int ring, int nh, int nkv, int dk, int dv,
                           float scale, float cap, int window, const float* __restrict__ slopes, int chunk,
                           const bf16_t* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
-                          float* __restrict__ lse, int keep, int kept, int own_stride, int own_k, int own_v) {
+                          float* __restrict__ lse, int keep, int kept, int own_stride, int own_k,
+                          int own_v_stride, int own_v, const float* __restrict__ sink) {
     constexpr int DKP = 32 * KT, DVP = 32 * VT, KLD = DKP + 8, VLD = MK + 8;
     constexpr int KP = (MK * DKP / 8 + 255) / 256;             // 16-byte pieces of a key tile a thread brings
     constexpr int VP = ((MK / 2) * (DVP / 8) + 255) / 256;     // pairs of keys x 8 value dims a thread brings
@@ -534,7 +546,7 @@ attn_cap_rows_bf16_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __
     };
     auto value_at = [&](int kj) __attribute__((always_inline)) {
         kj = min(kj, total - 1);
-        return own_stride ? (size_t)(start + kj) * own_stride + own_v + (size_t)kvh * dv
+        return own_stride ? (size_t)(start + kj) * own_v_stride + own_v + (size_t)kvh * dv
                           : cache_row_offset(page_table, table_stride, slot, kj, page_size, ring, nkv, kvh, dv, kept);
     };
     auto fetch = [&](int k0) __attribute__((always_inline)) {
@@ -659,6 +671,7 @@ attn_cap_rows_bf16_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __
         }
     }
     if (qrow < len) {
+        if (sink) add_sink(sink[h], m_i, l_i);
         const float inv = 1.0f / l_i;
         if (lse && half == 0) lse[(size_t)(start + qrow) * nh + h] = m_i + logf(l_i);
         const size_t ob = (size_t)(start + qrow) * nh * dv + (size_t)h * dv;
@@ -697,9 +710,10 @@ extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt
                                   int nh, int nkv, int dk, int dv, float scale, float cap, int window,
                                   const float* slopes, int chunk, const void* gate, int gate_stride,
                                   int gate_off, int gate_heads, float* lse, int keep, int kept,
-                                  int own_stride, int own_k, int own_v, void* stream) {
+                                  int own_stride, int own_k, int own_v_stride, int own_v, const float* sink,
+                                  void* stream) {
     if (keep < 0 || kept < 0 || (keep > 0 && (window <= 0 || chunk > 0)) || own_stride < 0 ||
-        (own_stride && (own_k < 0 || own_v < 0 || own_k + nkv * dk > own_stride || own_v + nkv * dv > own_stride)))
+        (own_stride && (own_k < 0 || own_v < 0 || own_k + nkv * dk > own_stride || own_v + nkv * dv > own_v_stride)))
         return ILLM_ERR_ARG;
     if (gate && (gate_off < 0 || gate_off + nh * (gate_heads ? 1 : dv) > gate_stride)) return ILLM_ERR_ARG;
     if (n_seqs < 0 || max_rows < 0 || nh <= 0 || nkv <= 0 || nh % nkv || dk <= 0 || dk > 256 ||
@@ -707,14 +721,14 @@ extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt
         return ILLM_ERR_ARG;
     if (n_seqs == 0 || max_rows == 0) return ILLM_OK;
     if (g_attn_cap_mfma && dk <= 128 && dv <= 128 && dk % 4 == 0 && dv % 4 == 0 && q_stride % 4 == 0 &&
-        own_stride % 4 == 0 && own_k % 4 == 0 && own_v % 4 == 0) {
+        own_stride % 4 == 0 && own_k % 4 == 0 && own_v_stride % 4 == 0 && own_v % 4 == 0) {
         const dim3 grid((max_rows + MQ - 1) / MQ, nh, n_seqs);
         const int kt = (dk + 31) / 32, vt = (dv + 31) / 32;
 #define GO(DT_, KT_, VT_)                                                                          \
     hipLaunchKernelGGL((attn_cap_rows_mfma_kernel<DT_, KT_, VT_>), grid, dim3(256), 0, (hipStream_t)stream, \
                        q, q_stride, out, cu, seq_slot, seq_start, kcache, vcache, page_table, table_stride, \
                        page_size, ring, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, gate, gate_stride, gate_off, gate_heads, lse, \
-                       keep, kept, own_stride, own_k, own_v)
+                       keep, kept, own_stride, own_k, own_v_stride, own_v, sink)
 #define GO_V(DT_, KT_)                                                                             \
     switch (vt) { case 1: GO(DT_, KT_, 1); break; case 2: GO(DT_, KT_, 2); break;                  \
                   case 3: GO(DT_, KT_, 3); break; default: GO(DT_, KT_, 4); break; }
@@ -722,14 +736,14 @@ extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt
     switch (kt) { case 1: GO_V(DT_, 1) break; case 2: GO_V(DT_, 2) break;                          \
                   case 3: GO_V(DT_, 3) break; default: GO_V(DT_, 4) break; }
         const bool bf16_rows = dt == ILLM_BF16 && g_attn_cap_mfma == 1 && dk % 8 == 0 && dv % 8 == 0 && q_stride % 8 == 0 &&
-                               own_stride % 8 == 0 && own_k % 8 == 0 && own_v % 8 == 0;
+                               own_stride % 8 == 0 && own_k % 8 == 0 && own_v_stride % 8 == 0 && own_v % 8 == 0;
         if (bf16_rows) {
 #define GOB(KT_, VT_)                                                                              \
     hipLaunchKernelGGL((attn_cap_rows_bf16_kernel<KT_, VT_>), grid, dim3(256), 0, (hipStream_t)stream, \
                        (const bf16_t*)q, q_stride, (bf16_t*)out, cu, seq_slot, seq_start, (const bf16_t*)kcache, \
                        (const bf16_t*)vcache, page_table, table_stride, page_size, ring, nh, nkv, dk, dv, scale, cap, \
                        window, slopes, chunk, (const bf16_t*)gate, gate_stride, gate_off, gate_heads, lse, keep, kept, \
-                       own_stride, own_k, own_v)
+                       own_stride, own_k, own_v_stride, own_v, sink)
 #define GOB_V(KT_)                                                                                 \
     switch (vt) { case 1: GOB(KT_, 1); break; case 2: GOB(KT_, 2); break;                          \
                   case 3: GOB(KT_, 3); break; default: GOB(KT_, 4); break; }
@@ -751,7 +765,7 @@ extern "C" int illm_attn_cap_rows(const void* q, int q_stride, void* out, int dt
     hipLaunchKernelGGL(attn_cap_rows_kernel, dim3((max_rows + CQ - 1) / CQ, nh, n_seqs), dim3(256), lds,
                        (hipStream_t)stream, q, q_stride, out, dt, cu, seq_slot, seq_start, kcache, vcache,
                        page_table, table_stride, page_size, ring, nh, nkv, dk, dv, scale, cap, window, slopes,
-                       chunk, gate, gate_stride, gate_off, gate_heads, lse, keep, kept, own_stride, own_k, own_v);
+                       chunk, gate, gate_stride, gate_off, gate_heads, lse, keep, kept, own_stride, own_k, own_v_stride, own_v, sink);
     return illm_launch_status();
 }
 
@@ -915,7 +929,7 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
                              int nh, int nkv, int dk, int dv, float scale, float cap, int window,
                              const float* __restrict__ slopes, int chunk, void* __restrict__ out,
                              const void* __restrict__ gate, int gate_stride, int gate_off, int gate_heads,
-                             int keep, int kept) {
+                             int keep, int kept, const float* __restrict__ sink) {
     constexpr int U = DT == ILLM_BF16 ? 8 : 4;          // elements of a unit
     constexpr int NK = U * KQ, NV = U * VQ;             // dims of a key, of a value, a lane holds
     __shared__ float wacc[4][DH][8 * NV];
@@ -1065,6 +1079,7 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
             y += f * wacc[x][i][d];
         }
         if (nsplit == 1) {                              // the one range is the whole result: no merge
+            if (sink) add_sink(sink[h0 + i], mm, lt);
             y *= 1.0f / lt;
             if (gate)
                 y *= 1.0f / (1.0f + expf(-ld_f(gate, DT, (size_t)b * gate_stride + gate_off + (gate_heads ? (size_t)(h0 + i) : (size_t)(h0 + i) * dv + d))));
@@ -1082,7 +1097,8 @@ attn_cap_decode_rows8_kernel(const void* __restrict__ q, int q_stride, const voi
 #define CAP_MERGE 16
 __global__ void attn_cap_merge_kernel(const float* __restrict__ partial, void* __restrict__ out,
                                       int dt, int nsplit, int nh, int dv, const void* __restrict__ gate,
-                                      int gate_stride, int gate_off, int gate_heads, float* __restrict__ lse) {
+                                      int gate_stride, int gate_off, int gate_heads, float* __restrict__ lse,
+                                      const float* __restrict__ sink) {
     const int h = blockIdx.x, b = blockIdx.y;
     const float* pp = partial + ((size_t)b * nh + h) * nsplit * (dv + 2);
     const size_t step = dv + 2;
@@ -1113,6 +1129,7 @@ __global__ void attn_cap_merge_kernel(const float* __restrict__ partial, void* _
                 a += f * v[x];
             }
         }
+        if (sink) add_sink(sink[h], mm, lt);
         if (d0 + (int)threadIdx.x < dv) {
             float y = a * (1.0f / lt);
             if (gate) y *= 1.0f / (1.0f + expf(-ld_f(gate, dt, (size_t)b * gate_stride + gate_off + (gate_heads ? (size_t)h : (size_t)h * dv + d))));
@@ -1129,7 +1146,7 @@ extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int 
                                     float* partial, int nsplit, int B, int nh, int nkv, int dk, int dv,
                                     float scale, float cap, int window, const float* slopes, int chunk,
                                     const void* gate, int gate_stride, int gate_off, int gate_heads, float* lse,
-                                    int keep, int kept, void* stream) {
+                                    int keep, int kept, const float* sink, void* stream) {
     if (keep < 0 || kept < 0 || (keep > 0 && (window <= 0 || chunk > 0))) return ILLM_ERR_ARG;
     if (gate && (gate_off < 0 || gate_off + nh * (gate_heads ? 1 : dv) > gate_stride)) return ILLM_ERR_ARG;
     if (B < 0 || nh <= 0 || nkv <= 0 || nh % nkv || dk <= 0 || dk > 256 || dv <= 0 || dv > 256 ||
@@ -1153,17 +1170,17 @@ extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int 
         hipLaunchKernelGGL((attn_cap_decode_rows8_kernel<DT_, KQ_, VQ_, 1>), grid, dim3(256), 0, st, q, q_stride, \
                            kcache, vcache, page_table, table_stride, page_size, ring, seq_slot, seq_len, partial, \
                            nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads, \
-                           keep, kept);                                                            \
+                           keep, kept, sink);                                                      \
     else if (dh == 2)                                                                              \
         hipLaunchKernelGGL((attn_cap_decode_rows8_kernel<DT_, KQ_, VQ_, 2>), grid, dim3(256), 0, st, q, q_stride, \
                            kcache, vcache, page_table, table_stride, page_size, ring, seq_slot, seq_len, partial, \
                            nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads, \
-                           keep, kept);                                                            \
+                           keep, kept, sink);                                                      \
     else                                                                                           \
         hipLaunchKernelGGL((attn_cap_decode_rows8_kernel<DT_, KQ_, VQ_, 4>), grid, dim3(256), 0, st, q, q_stride, \
                            kcache, vcache, page_table, table_stride, page_size, ring, seq_slot, seq_len, partial, \
                            nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, out, gate, gate_stride, gate_off, gate_heads, \
-                           keep, kept)
+                           keep, kept, sink)
 #define GO_V(DT_, KQ_)                                                                             \
     switch (vq) { case 1: { GO(DT_, KQ_, 1); } break; case 2: { GO(DT_, KQ_, 2); } break;          \
                   case 3: { GO(DT_, KQ_, 3); } break; default: { GO(DT_, KQ_, 4); } break; }
@@ -1185,6 +1202,6 @@ extern "C" int illm_attn_cap_decode(const void* q, int q_stride, void* out, int 
                            seq_len, partial, nsplit, nh, nkv, dk, dv, scale, cap, window, slopes, chunk, keep, kept);
     if (hipGetLastError() != hipSuccess) return ILLM_ERR_LAUNCH;
     hipLaunchKernelGGL(attn_cap_merge_kernel, dim3(nh, B), dim3(64), 0, st, partial, out, dt, nsplit, nh, dv,
-                       gate, gate_stride, gate_off, gate_heads, lse);
+                       gate, gate_stride, gate_off, gate_heads, lse, sink);
     return illm_launch_status();
 }

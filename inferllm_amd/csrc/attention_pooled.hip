@@ -32,6 +32,8 @@
 // `bias` float32 [q (nh dk) | k (nkv dk) | v (nkv dv)] (null: none) is added first, then every q and k
 // head is RMS-normed under qw, kw [dk] (null: not).  With `slot_len` (the sequences' lengths after the
 // step) rows that a later row of the step would overwrite in the ring of pages are not stored.
+// `v_from_k` (dv = dk): a value head is its key head as projected (with its bias, before norm and
+// rotation); it is stored, and if `v_rows` [T, nkv dv] is given left there too.
 __global__ void __launch_bounds__(64)
 qk_rotate_store_kernel(void* __restrict__ rows, int dt, int row_len, int k_off, int v_off,
                        const float* __restrict__ cos_sin, int rot, int pairing, int unit_norm, float eps,
@@ -40,7 +42,7 @@ qk_rotate_store_kernel(void* __restrict__ rows, int dt, int row_len, int k_off, 
                        const int32_t* __restrict__ page_table, int table_stride, int page_size, int ring,
                        int nh, int nkv, int dk, int dv, const float* __restrict__ bias,
                        const void* __restrict__ qw, const void* __restrict__ kw, int w_dt,
-                       const int32_t* __restrict__ slot_len, int kept) {
+                       const int32_t* __restrict__ slot_len, int kept, int v_from_k, void* __restrict__ v_rows) {
     __shared__ float x[256];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int pos = row_pos[t];
@@ -52,6 +54,21 @@ qk_rotate_store_kernel(void* __restrict__ rows, int dt, int row_len, int k_off, 
         const float v = ld_f(rows, dt, base + d) + (hb ? hb[d] : 0.f);
         x[d] = v;
         ss0 = fmaf(v, v, ss0);
+    }
+    size_t kat = 0, vat = 0;
+    bool store = is_k && kcache != nullptr;
+    if (store) {
+        const int slot = row_slot[t], lp = pos / page_size;
+        if (ring > 0 && slot_len && lp >= kept && lp + ring <= (slot_len[slot] - 1) / page_size) store = false;
+        kat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dk, kept);
+        vat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dv, kept);
+    }
+    if (v_from_k && is_k) {                                  // the values are the keys as they are by now
+        const size_t vb = ((size_t)t * nkv + (h - nh)) * dv;
+        for (int d = lane; d < dk; d += 64) {                // (a lane's own entries)
+            if (v_rows) st_f(v_rows, dt, vb + d, x[d]);
+            if (store) st_f(vcache, dt, vat + d, x[d]);
+        }
     }
     const void* hw = is_k ? kw : qw;
     if (hw) {
@@ -79,20 +96,12 @@ qk_rotate_store_kernel(void* __restrict__ rows, int dt, int row_len, int k_off, 
         inv = 1.0f / sqrtf(ss / (float)dk + eps);
     }
     if (q_scale && !is_k) inv *= q_scale[h];
-    size_t kat = 0, vat = 0;
-    bool store = is_k && kcache != nullptr;
-    if (store) {
-        const int slot = row_slot[t], lp = pos / page_size;
-        if (ring > 0 && slot_len && lp >= kept && lp + ring <= (slot_len[slot] - 1) / page_size) store = false;
-        kat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dk, kept);
-        vat = cache_row_offset(page_table, table_stride, slot, pos, page_size, ring, nkv, h - nh, dv, kept);
-    }
     for (int d = lane; d < dk; d += 64) {
         const float y = x[d] * inv;
         st_f(rows, dt, base + d, y);
         if (store) st_f(kcache, dt, kat + d, y);
     }
-    if (is_k && (store || bias)) {
+    if (is_k && !v_from_k && (store || bias)) {
         const size_t vb = (size_t)t * row_len + v_off + (size_t)(h - nh) * dv;
         for (int d = lane; d < dv; d += 64) {
             if (bias)
@@ -110,18 +119,20 @@ extern "C" int illm_qk_rotate_store(void* rows, int dt, int row_len, int k_off, 
                                     const int32_t* row_slot, void* kcache, void* vcache,
                                     const int32_t* page_table, int table_stride, int page_size, int ring,
                                     int T, int nh, int nkv, int dk, int dv, const float* bias, const void* qw,
-                                    const void* kw, int w_dt, const int32_t* slot_len, int kept, void* stream) {
+                                    const void* kw, int w_dt, const int32_t* slot_len, int kept, int v_from_k,
+                                    void* v_rows, void* stream) {
+    if ((v_from_k && dk != dv) || (v_rows && !v_from_k)) return ILLM_ERR_ARG;
     if (kept < 0 || ((qw || kw) && !illm_dtype_ok(w_dt))) return ILLM_ERR_ARG;
     if (T < 0 || nh < 0 || nkv < 0 || nh + nkv <= 0 || nh + nkv > 65535 || dk <= 0 || dk > 256 || dv < 0 ||
         dv > 256 || !illm_dtype_ok(dt) || rot < 0 || rot % 2 || rot > dk || (pairing != 0 && pairing != 1) ||
-        nh * dk > row_len || (nkv > 0 && (k_off + nkv * dk > row_len || v_off + nkv * dv > row_len)) ||
+        nh * dk > row_len || (nkv > 0 && (k_off + nkv * dk > row_len || (!v_from_k && v_off + nkv * dv > row_len))) ||
         (cos_sin && rot > 0 && n_positions <= 0) || (kcache && (!vcache || !page_table || page_size <= 0)))
         return ILLM_ERR_ARG;
     if (T == 0) return ILLM_OK;
     hipLaunchKernelGGL(qk_rotate_store_kernel, dim3(T, nh + nkv), dim3(64), 0, (hipStream_t)stream, rows,
                        dt, row_len, k_off, v_off, cos_sin, rot, pairing, unit_norm, eps, q_scale, row_pos, row_slot,
                        kcache, vcache, page_table, table_stride, page_size, ring, nh, nkv, dk, dv, bias, qw, kw,
-                       w_dt, slot_len, kept);
+                       w_dt, slot_len, kept, v_from_k, v_rows);
     return illm_launch_status();
 }
 

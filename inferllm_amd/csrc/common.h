@@ -14,6 +14,8 @@
 
 #define ILLM_WAVE 64
 
+#define ILLM_MAX_PLANES 8   // rows of X a product's parts may have of their own (gemm_skinny.hip, gemm_rows.hip)
+
 // norms of a row (post_norm.hip)
 #define ILLM_NORM_NONE 0
 #define ILLM_NORM_RMS 1

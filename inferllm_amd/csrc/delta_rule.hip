@@ -206,6 +206,7 @@ __device__ __forceinline__ float group_sum(float v) {
 #define RULE_PLAIN 0
 #define RULE_DELTA 1
 #define RULE_REMOVAL 2
+#define RULE_BONUS 3      // o = S^T q + beta v from the state before the token; then S <- diag(g) S + k v^T
 
 // Steps of few tokens a sequence (single tokens above all): what counts is the state's bytes.
 // grid (ceil(dv / 64), H, sequences); 4 waves: a lane is a column, wave w holds rows [w NS, w NS + NS)
@@ -218,7 +219,7 @@ delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
                   const float* __restrict__ dec, int DW, float* __restrict__ state,
                   const int32_t* __restrict__ cu, const int32_t* __restrict__ seq_slot,
                   float* __restrict__ o, int G, int H, int dk, int dv, const float* __restrict__ removal) {
-    constexpr bool CORRECT = RULE != RULE_PLAIN;
+    constexpr bool CORRECT = RULE == RULE_DELTA || RULE == RULE_REMOVAL;
     __shared__ float red[2][4][64];
     const int b = blockIdx.z, h = blockIdx.y, lane = threadIdx.x & 63, w = wave_index();
     const int col = blockIdx.x * 64 + lane;
@@ -240,6 +241,7 @@ delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
         for (int ii = 0; ii < NS; ++ii) {
             const int i = i0 + ii;
             kc[ii] = i < dk ? kp[i] : 0.f;
+            if (RULE == RULE_BONUS) continue;
             if (RULE != RULE_REMOVAL) s[ii] *= i < dk ? (DW == 1 ? dp[0] : dp[i]) : 1.f;
             pa[ii & 3] = fmaf(s[ii], kc[ii], pa[ii & 3]);
         }
@@ -258,6 +260,11 @@ delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
 #pragma unroll
         for (int ii = 0; ii < NS; ++ii) {
             const int i = i0 + ii;
+            if (RULE == RULE_BONUS) {
+                pa[ii & 3] = fmaf(s[ii], i < dk ? qp[i] : 0.f, pa[ii & 3]);
+                s[ii] = fmaf(kc[ii], v, s[ii] * (i < dk ? (DW == 1 ? dp[0] : dp[i]) : 1.f));
+                continue;
+            }
             if (RULE == RULE_REMOVAL && i < dk) s[ii] = fmaf(-cp[i], read, s[ii] * (DW == 1 ? dp[0] : dp[i]));
             s[ii] = fmaf(kc[ii], u, s[ii]);
             pa[ii & 3] = fmaf(s[ii], i < dk ? qp[i] : 0.f, pa[ii & 3]);
@@ -268,7 +275,8 @@ delta_step_kernel(const float* __restrict__ qn, const float* __restrict__ kn,
         rd[w][lane] = (pa[0] + pa[1]) + (pa[2] + pa[3]);
         __syncthreads();
         if (w == 0 && live)
-            o[((size_t)row * H + h) * dv + col] = (rd[0][lane] + rd[1][lane]) + (rd[2][lane] + rd[3][lane]);
+            o[((size_t)row * H + h) * dv + col] =
+                (rd[0][lane] + rd[1][lane]) + (rd[2][lane] + rd[3][lane]) + (RULE == RULE_BONUS ? bt * v : 0.f);
     }
 #pragma unroll
     for (int ii = 0; ii < NS; ++ii)
@@ -288,7 +296,7 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
                        const float* __restrict__ dec, int DW, float* __restrict__ state,
                        const int32_t* __restrict__ cu, const int32_t* __restrict__ seq_slot,
                        float* __restrict__ o, int G, int H, int dk, int dv, const float* __restrict__ removal) {
-    constexpr bool CORRECT = RULE != RULE_PLAIN;
+    constexpr bool CORRECT = RULE == RULE_DELTA || RULE == RULE_REMOVAL;
     constexpr int NVEC = RULE == RULE_REMOVAL ? 4 : 3;  // rows a token in LDS
     constexpr int PARTS = 16, COLS = 4;
     constexpr int TC = RULE == RULE_REMOVAL ? DELTA_CHUNK / 2 : DELTA_CHUNK;    // (a fourth row a token: fewer tokens, or registers run out)
@@ -396,6 +404,7 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
 #pragma unroll
             for (int ii = 0; ii < NS; ++ii) {
                 kc[ii] = src[PARTS * ii];
+                if (RULE == RULE_BONUS) continue;
                 if (RULE != RULE_REMOVAL) s[ii] *= src[2 * DKP + PARTS * ii];
                 pa[ii % NA] = fmaf(s[ii], kc[ii], pa[ii % NA]);
             }
@@ -412,6 +421,11 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
             for (int a = 0; a < NA; ++a) pa[a] = 0.f;
 #pragma unroll
             for (int ii = 0; ii < NS; ++ii) {
+                if (RULE == RULE_BONUS) {
+                    pa[ii % NA] = fmaf(s[ii], src[DKP + PARTS * ii], pa[ii % NA]);
+                    s[ii] = fmaf(kc[ii], cv[tt], s[ii] * src[2 * DKP + PARTS * ii]);
+                    continue;
+                }
                 if (RULE == RULE_REMOVAL) {
                     // (all but the last operation is off the chain that hangs on `read`)
                     const float kept = fmaf(kc[ii], u, s[ii] * src[2 * DKP + PARTS * ii]);
@@ -424,6 +438,7 @@ delta_scan_long_kernel(const float* __restrict__ qn, const float* __restrict__ k
 #pragma unroll
             for (int a = 1; a < NA; ++a) ov += pa[a];
             ovs[tt] = group_sum<PARTS>(ov);
+            if (RULE == RULE_BONUS) ovs[tt] = fmaf(cb[tt], cv[tt], ovs[tt]);
         }
         if (writes) {
 #pragma unroll
@@ -449,6 +464,7 @@ extern "C" int illm_gated_scan(const float* qn, const float* kn, const float* vv
                                const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int G,
                                int H, int dk, int dv, int correct, const float* removal, void* stream) {
     if (removal && (correct || G != H)) return ILLM_ERR_ARG;
+    if (correct < 0 || correct > 2) return ILLM_ERR_ARG;
     if (n_seqs < 0 || G <= 0 || H <= 0 || H % G || dk <= 0 || dk > 256 || dv <= 0 ||
         (DW != 1 && DW != dk) || H > 65535 || n_seqs > 65535)
         return ILLM_ERR_ARG;
@@ -469,6 +485,7 @@ extern "C" int illm_gated_scan(const float* qn, const float* kn, const float* vv
     } while (0)
 #define GOL(NS_)                                                                                  \
     if (removal) GOL_R(NS_, RULE_REMOVAL);                                                        \
+    else if (correct == 2) GOL_R(NS_, RULE_BONUS);                                                \
     else if (correct) GOL_R(NS_, RULE_DELTA);                                                     \
     else GOL_R(NS_, RULE_PLAIN)
         if (ns <= 1) { GOL(1); }
@@ -486,6 +503,7 @@ extern "C" int illm_gated_scan(const float* qn, const float* kn, const float* vv
                        state, cu, seq_slot, o, G, H, dk, dv, removal)
 #define GOS(NS_)                                                                                  \
     if (removal) GOS_R(NS_, RULE_REMOVAL);                                                        \
+    else if (correct == 2) GOS_R(NS_, RULE_BONUS);                                                \
     else if (correct) GOS_R(NS_, RULE_DELTA);                                                     \
     else GOS_R(NS_, RULE_PLAIN)
         if (ns <= 4) { GOS(4); }

@@ -37,6 +37,55 @@ extern "C" int illm_embed(const int32_t* tokens, const void* table, int table_dt
     return illm_embed_scaled(tokens, table, table_dt, out, T, E, V, 1.0f, stream);
 }
 
+// The token's row under an RMS norm: out = v / sqrt(mean(v^2) + eps) * w with v = table[id] * scale.  `copy`
+// (null: none) takes the rows a second time.  grid (rows); 256 threads.
+__global__ void __launch_bounds__(256)
+embed_norm_kernel(const int32_t* __restrict__ tokens, const void* __restrict__ table, int table_dt,
+                  const void* __restrict__ w, int w_dt, float* __restrict__ out, float* __restrict__ copy, int E,
+                  int V, float scale, float eps) {
+    __shared__ float red[16];
+    const int t = blockIdx.x;
+    int id = tokens[t];
+    id = id < 0 ? 0 : (id >= V ? V - 1 : id);
+    const size_t src = (size_t)id * E, dst = (size_t)t * E;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < E; i += 256) {
+        const float v = ld_f(table, table_dt, src + i) * scale;
+        ss = fmaf(v, v, ss);
+    }
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)E + eps);
+    for (int i = threadIdx.x; i < E; i += 256) {
+        const float y = (ld_f(table, table_dt, src + i) * scale * inv) * ld_f(w, w_dt, i);
+        out[dst + i] = y;
+        if (copy) copy[dst + i] = y;
+    }
+}
+
+extern "C" int illm_embed_norm(const int32_t* tokens, const void* table, int table_dt, const void* w, int w_dt,
+                               float* out, float* copy, int T, int E, int V, float scale, float eps, void* stream) {
+    if (T < 0 || E <= 0 || V <= 0 || !illm_dtype_ok(table_dt) || !illm_dtype_ok(w_dt)) return ILLM_ERR_ARG;
+    if (T == 0) return ILLM_OK;
+    hipLaunchKernelGGL(embed_norm_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, tokens, table, table_dt, w, w_dt,
+                       out, copy, E, V, scale, eps);
+    return illm_launch_status();
+}
+
+// A copy of float32 rows (a kernel and no memory-copy command, for code under graph capture).
+__global__ void __launch_bounds__(256)
+copy_rows_kernel(const float* __restrict__ x, float* __restrict__ out, size_t n) {
+    const size_t step = (size_t)gridDim.x * 256;
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += step) out[i] = x[i];
+}
+
+extern "C" int illm_copy_rows(const float* x, float* out, size_t n, void* stream) {
+    if (!x || !out) return ILLM_ERR_ARG;
+    if (n == 0) return ILLM_OK;
+    const size_t blocks = (n + 255) / 256;
+    hipLaunchKernelGGL(copy_rows_kernel, dim3(blocks < 4096 ? blocks : 4096), dim3(256), 0, (hipStream_t)stream, x, out, n);
+    return illm_launch_status();
+}
+
 // Token row times a scale, plus a row of a table hashed by the pair (previous token, token), plus a
 // learned row of the position:
 //     out = table[id] * scale + pairs[(prev * mul_prev + id * mul_cur) mod buckets] + places[pos]

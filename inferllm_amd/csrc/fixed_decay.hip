@@ -1,4 +1,4 @@
-// Two linear mixers with a matrix of state S [key dim, value dim] (float32) per head and no convolution:
+// Four linear mixers with a matrix of state S [key dim, value dim] (float32) per head and no convolution:
 //
 // Lightning attention, one fixed decay lam a head: q, k, v through SiLU,
 //     S <- lam S + k v^T;   o = S^T q
@@ -11,7 +11,17 @@
 //   removal_prepare     the inputs of illm_gated_scan (with `removal`) as float32
 //   removal_step        single tokens in one launch, z = W2 tanh(y1) of the low-rank map included
 //
-// Behind either: group_norm_gate, o RMS-normed in equal parts of the row, a weight of the row's width, a
+// Retention, one fixed decay lam a head, q and k turned by their positions (pairs i, i + rot / 2) and k
+// times dk^-1/2, neither activated:  S <- lam S + k v^T;   o = S^T q
+//   retention_prepare   q, k (and, for illm_gated_scan, the rest of its inputs) as float32
+//   retention_step      single tokens: rotation, the state's update and o in one launch
+//   retention_chunks    long steps, as lightning_chunks
+//
+// Time mixing with a decay w a key channel and a bonus u for the current token, w = exp(-exp(z + w0)):
+//     o = (S + diag(u) k v^T)^T r;   S <- diag(w) S + k v^T
+//   time_mix_step       single tokens in one launch, z = W2 tanh(y1) included (long steps: time_mix.hip)
+//
+// Behind any: group_norm_gate, o RMS-normed in equal parts of the row, a weight of the row's width, a
 // gate.  Everything but the stored projections is float32.  A sequence's rows in a step are consecutive.
 #include <math.h>
 
@@ -48,6 +58,49 @@ extern "C" int illm_lightning_prepare(const void* U, int dt, int u_stride, int q
     if (T == 0) return ILLM_OK;
     hipLaunchKernelGGL(lightning_prepare_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, U, dt, u_stride,
                        q_off, k_off, v_off, decay, qn, kn, vv, beta, dec, H, dk, dv);
+    return illm_launch_status();
+}
+
+// grid (rows); 256 threads.  q and k heads turned by the row's position and k times k_scale; vv, beta and
+// dec may be null (the chunks take v and the decays as they are).
+__global__ void __launch_bounds__(256)
+retention_prepare_kernel(const void* __restrict__ U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                         const float* __restrict__ decay, const float* __restrict__ cos_sin, int rot, float k_scale,
+                         const int32_t* __restrict__ row_pos, float* __restrict__ qn, float* __restrict__ kn,
+                         float* __restrict__ vv, float* __restrict__ beta, float* __restrict__ dec, int H,
+                         int dk, int dv) {
+    const size_t t = blockIdx.x, u0 = t * u_stride;
+    const float* cs = rot > 0 ? cos_sin + (size_t)row_pos[t] * rot : nullptr;
+    const int half = rot / 2;
+    for (int e = threadIdx.x; e < H * dk; e += 256) {
+        const int i = e % dk;
+        float q = ld_f(U, dt, u0 + q_off + e), k = ld_f(U, dt, u0 + k_off + e);
+        if (i < rot) {
+            const int j = i < half ? i : i - half, other = e + (i < half ? half : -half);
+            const float c = cs[2 * j], sn = i < half ? -cs[2 * j + 1] : cs[2 * j + 1];
+            q = q * c + ld_f(U, dt, u0 + q_off + other) * sn;
+            k = k * c + ld_f(U, dt, u0 + k_off + other) * sn;
+        }
+        qn[t * H * dk + e] = q;
+        kn[t * H * dk + e] = k * k_scale;
+    }
+    if (vv)
+        for (int e = threadIdx.x; e < H * dv; e += 256) vv[t * H * dv + e] = ld_f(U, dt, u0 + v_off + e);
+    if (beta)
+        for (int e = threadIdx.x; e < H; e += 256) { beta[t * H + e] = 1.0f; dec[t * H + e] = decay[e]; }
+}
+
+extern "C" int illm_retention_prepare(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                                      const float* decay, const float* cos_sin, int n_positions, int rot, float k_scale,
+                                      const int32_t* row_pos, float* qn, float* kn, float* vv, float* beta,
+                                      float* dec, int T, int H, int dk, int dv, void* stream) {
+    if (T < 0 || H <= 0 || dk <= 0 || dv <= 0 || !illm_dtype_ok(dt) || rot < 0 || rot % 2 || rot > dk ||
+        (rot > 0 && (!cos_sin || n_positions <= 0 || !row_pos)) || !fd_columns_ok(u_stride, q_off, H * dk) ||
+        !fd_columns_ok(u_stride, k_off, H * dk) || !fd_columns_ok(u_stride, v_off, H * dv) || (!beta) != (!dec))
+        return ILLM_ERR_ARG;
+    if (T == 0) return ILLM_OK;
+    hipLaunchKernelGGL(retention_prepare_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, U, dt, u_stride, q_off,
+                       k_off, v_off, decay, cos_sin, rot, k_scale, row_pos, qn, kn, vv, beta, dec, H, dk, dv);
     return illm_launch_status();
 }
 
@@ -121,63 +174,92 @@ extern "C" int illm_tanh_columns(const void* U, int dt, int u_stride, int off, f
 // (k, q and, with a removal vector, the decays and the vector) are formed by the block into LDS while the
 // state's rows are on their way; the waves' partial sums meet in LDS, in wave order.
 #define FD_RANK_MAX 512
-struct RemovalArgs {
-    const float* a_bias;      // [H d]
+enum { FD_LIGHTNING = 0, FD_REMOVAL = 1, FD_RETENTION = 2, FD_TIME_MIX = 3 };
+struct StepArgs {
+    const float* decay;       // FD_LIGHTNING, FD_RETENTION: [H]
+    const void* rates;        // FD_REMOVAL: the rates' pre-activations, rows like q's
+    const float* rate_bias;   // FD_REMOVAL: [H d]
+    const void* low;          // FD_REMOVAL, FD_TIME_MIX: y1 of the low-rank map, [rows, low_stride]
+    int low_stride, rank;
     const void* w2;           // [H d, rank], the projections' type
     const float* w0;          // [H d]
-    int a_off, w1_off, rank;
-    float rate;
+    float rate;               // FD_REMOVAL
+    const float* bonus;       // FD_TIME_MIX: [H d]
+    const float* cos_sin;     // FD_RETENTION: [positions, rot / 2, 2]
+    const int32_t* row_pos;
+    int rot;
+    float k_scale;
 };
 
-template <int NS, int DT, bool REMOVAL>
+template <int NS, int DT, int MODE>
 __global__ void __launch_bounds__(256)
-fixed_step_kernel(const void* __restrict__ U, int u_stride, int q_off, int k_off, int v_off,
-                  const float* __restrict__ decay, RemovalArgs ra, float* __restrict__ state,
+fixed_step_kernel(const void* __restrict__ q_rows, const void* __restrict__ k_rows,
+                  const void* __restrict__ v_rows, int stride, StepArgs sa, float* __restrict__ state,
                   const int32_t* __restrict__ row_slot, float* __restrict__ o, int H, int dk, int dv) {
-    __shared__ float sk[4 * NS], sq[4 * NS], sw[REMOVAL ? 4 * NS : 1], sc[REMOVAL ? 4 * NS : 1];
-    __shared__ float low[REMOVAL ? FD_RANK_MAX : 1];
-    __shared__ float part[REMOVAL ? 256 : 1];
+    constexpr bool REMOVAL = MODE == FD_REMOVAL, MIX = MODE == FD_TIME_MIX, LOW = REMOVAL || MIX;
+    __shared__ float sk[4 * NS], sq[4 * NS], sw[LOW ? 4 * NS : 1], sc[REMOVAL ? 4 * NS : 1];
+    __shared__ float low[LOW ? FD_RANK_MAX : 1];
+    __shared__ float part[LOW ? 256 : 1];
     __shared__ float red[2][4][64];
     __shared__ float redb[16];
     const int b = blockIdx.z, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = wave_index();
     const int col = blockIdx.x * 64 + lane, i0 = w * NS;
     const bool live = col < dv;
-    const size_t u0 = (size_t)b * u_stride;
+    const size_t u0 = (size_t)b * stride;
     float* sp = state + (((size_t)row_slot[b] * H + h) * dk) * dv + col;
     float s[NS];
 #pragma unroll
     for (int ii = 0; ii < NS; ++ii) s[ii] = (live && i0 + ii < dk) ? sp[(size_t)(i0 + ii) * dv] : 0.f;
-    float v = live ? ld_f(U, DT, u0 + v_off + (size_t)h * dv + col) : 0.f;
-    if (!REMOVAL) v = fd_silu(v);
+    float v = live ? ld_f(v_rows, DT, u0 + (size_t)h * dv + col) : 0.f;
+    if (MODE == FD_LIGHTNING) v = fd_silu(v);
     const int i = tid;                                  // a thread a channel (dk <= 256)
     const bool mine = i < dk;
-    float k = mine ? ld_f(U, DT, u0 + k_off + (size_t)h * dk + i) : 0.f;
-    float q = mine ? ld_f(U, DT, u0 + q_off + (size_t)h * dk + i) : 0.f;
-    float inv = 1.f;
-    if (REMOVAL) {
-        for (int r = tid; r < ra.rank; r += 256) low[r] = tanhf(ld_f(U, DT, u0 + ra.w1_off + r));
-        inv = 1.0f / sqrtf(block_sum(k * k, redb) + 1e-6f);      // (its barriers also publish `low`)
+    float k = mine ? ld_f(k_rows, DT, u0 + (size_t)h * dk + i) : 0.f;
+    float q = mine ? ld_f(q_rows, DT, u0 + (size_t)h * dk + i) : 0.f;
+    float inv = 1.f, bonus = 0.f;
+    if (LOW) {
+        for (int r = tid; r < sa.rank; r += 256) low[r] = tanhf(ld_f(sa.low, DT, (size_t)b * sa.low_stride + r));
+        // (the sum's barriers also publish `low`)
+        if (REMOVAL) inv = 1.0f / sqrtf(block_sum(k * k, redb) + 1e-6f);
+        else bonus = block_sum(mine ? q * sa.bonus[h * dk + i] * k : 0.f, redb);
         // z of the head's channels: 256 / DKP threads a channel, each a share of the rank
         constexpr int DKP = 4 * NS, SH = 256 / DKP;
         const int zi = tid % DKP, sh = tid / DKP;
         float z = 0.f;
         if (zi < dk) {
-            const size_t w2 = ((size_t)h * dk + zi) * ra.rank;
-            const int per = (ra.rank + SH - 1) / SH, r1 = min(ra.rank, (sh + 1) * per);
+            const size_t w2 = ((size_t)h * dk + zi) * sa.rank;
+            const int per = (sa.rank + SH - 1) / SH, r1 = min(sa.rank, (sh + 1) * per);
 #pragma unroll 8
-            for (int r = sh * per; r < r1; ++r) z = fmaf(ld_f(ra.w2, DT, w2 + r), low[r], z);
+            for (int r = sh * per; r < r1; ++r) z = fmaf(ld_f(sa.w2, DT, w2 + r), low[r], z);
         }
         part[tid] = z;
         __syncthreads();
         if (mine) {
-            z = ra.w0[h * dk + i];
+            z = sa.w0[h * dk + i];
 #pragma unroll
             for (int x = 0; x < SH; ++x) z += part[x * DKP + i];
-            sw[i] = expf(-ra.rate * fd_sigmoid(z));
-            sc[i] = fd_sigmoid(ld_f(U, DT, u0 + ra.a_off + (size_t)h * dk + i) + ra.a_bias[h * dk + i]) * (k * inv);
+            if (REMOVAL) {
+                sw[i] = expf(-sa.rate * fd_sigmoid(z));
+                sc[i] = fd_sigmoid(ld_f(sa.rates, DT, u0 + (size_t)h * dk + i) + sa.rate_bias[h * dk + i]) * (k * inv);
+            } else {
+                sw[i] = expf(-expf(z));
+            }
         } else if (i < DKP) {
-            sw[i] = 1.f; sc[i] = 0.f;
+            sw[i] = 1.f;
+            if (REMOVAL) sc[i] = 0.f;
         }
+    } else if (MODE == FD_RETENTION) {
+        if (i < 4 * NS) { sk[i] = k; sq[i] = q; }
+        __syncthreads();
+        if (i < sa.rot) {
+            const int half = sa.rot / 2, j = i < half ? i : i - half, other = i < half ? i + half : j;
+            const float* cs = sa.cos_sin + (size_t)sa.row_pos[b] * sa.rot + 2 * j;
+            const float c = cs[0], sn = i < half ? -cs[1] : cs[1];
+            k = k * c + sk[other] * sn;
+            q = q * c + sq[other] * sn;
+        }
+        k *= sa.k_scale;
+        __syncthreads();
     } else {
         k = fd_silu(k); q = fd_silu(q);
     }
@@ -193,9 +275,14 @@ fixed_step_kernel(const void* __restrict__ U, int u_stride, int q_off, int k_off
         read = inv * ((red[0][0][lane] + red[0][1][lane]) + (red[0][2][lane] + red[0][3][lane]));
         pa[0] = pa[1] = pa[2] = pa[3] = 0.f;
     }
-    const float lam = REMOVAL ? 1.f : decay[h];
+    const float lam = LOW ? 1.f : sa.decay[h];
 #pragma unroll
     for (int ii = 0; ii < NS; ++ii) {
+        if (MIX) {                                       // o from the state before the token
+            pa[ii & 3] = fmaf(s[ii], sq[i0 + ii], pa[ii & 3]);
+            s[ii] = fmaf(sk[i0 + ii], v, s[ii] * sw[i0 + ii]);
+            continue;
+        }
         if (REMOVAL) s[ii] = fmaf(-sc[i0 + ii], read, s[ii] * sw[i0 + ii]);
         else s[ii] *= lam;
         s[ii] = fmaf(sk[i0 + ii], v, s[ii]);
@@ -206,21 +293,28 @@ fixed_step_kernel(const void* __restrict__ U, int u_stride, int q_off, int k_off
     for (int ii = 0; ii < NS; ++ii)
         if (live && i0 + ii < dk) sp[(size_t)(i0 + ii) * dv] = s[ii];
     __syncthreads();
-    if (w == 0 && live)
-        o[((size_t)b * H + h) * dv + col] = (red[1][0][lane] + red[1][1][lane]) + (red[1][2][lane] + red[1][3][lane]);
+    if (w == 0 && live) {
+        float y = (red[1][0][lane] + red[1][1][lane]) + (red[1][2][lane] + red[1][3][lane]);
+        if (MIX) y = fmaf(bonus, v, y);
+        o[((size_t)b * H + h) * dv + col] = y;
+    }
 }
 
-static int fixed_step_launch(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
-                             const float* decay, RemovalArgs ra, bool removal, float* state,
-                             const int32_t* row_slot, float* o, int B, int H, int dk, int dv, hipStream_t st) {
+static const void* fd_at(const void* base, int dt, size_t column) {
+    return (const char*)base + column * (dt == ILLM_BF16 ? 2 : 4);
+}
+
+template <int MODE>
+static int fixed_step_launch(const void* q, const void* k, const void* v, int dt, int stride, StepArgs sa,
+                             float* state, const int32_t* row_slot, float* o, int B, int H, int dk, int dv,
+                             hipStream_t st) {
     const dim3 grid((dv + 63) / 64, H, B);
     const int ns = (dk + 3) / 4;
-#define GO(NS_, DT_, R_)                                                                                \
-    hipLaunchKernelGGL((fixed_step_kernel<NS_, DT_, R_>), grid, dim3(256), 0, st, U, u_stride, q_off, k_off, \
-                       v_off, decay, ra, state, row_slot, o, H, dk, dv)
+#define GO(NS_, DT_)                                                                                    \
+    hipLaunchKernelGGL((fixed_step_kernel<NS_, DT_, MODE>), grid, dim3(256), 0, st, q, k, v, stride, sa, state, \
+                       row_slot, o, H, dk, dv)
 #define GO_D(NS_)                                                                                       \
-    if (dt == ILLM_BF16) { if (removal) GO(NS_, ILLM_BF16, true); else GO(NS_, ILLM_BF16, false); }     \
-    else { if (removal) GO(NS_, ILLM_F32, true); else GO(NS_, ILLM_F32, false); }
+    if (dt == ILLM_BF16) GO(NS_, ILLM_BF16); else GO(NS_, ILLM_F32);
     if (ns <= 4) { GO_D(4) }
     else if (ns <= 8) { GO_D(8) }
     else if (ns <= 16) { GO_D(16) }
@@ -239,8 +333,10 @@ extern "C" int illm_lightning_step(const void* U, int dt, int u_stride, int q_of
         !fd_columns_ok(u_stride, v_off, H * dv))
         return ILLM_ERR_ARG;
     if (B == 0) return ILLM_OK;
-    return fixed_step_launch(U, dt, u_stride, q_off, k_off, v_off, decay, RemovalArgs{}, false, state, row_slot, o,
-                             B, H, dk, dv, (hipStream_t)stream);
+    StepArgs sa = {};
+    sa.decay = decay;
+    return fixed_step_launch<FD_LIGHTNING>(fd_at(U, dt, q_off), fd_at(U, dt, k_off), fd_at(U, dt, v_off), dt, u_stride,
+                                           sa, state, row_slot, o, B, H, dk, dv, (hipStream_t)stream);
 }
 
 extern "C" int illm_removal_step(const void* U, int dt, int u_stride, int r_off, int k_off, int v_off, int a_off,
@@ -253,9 +349,40 @@ extern "C" int illm_removal_step(const void* U, int dt, int u_stride, int r_off,
         !fd_columns_ok(u_stride, w1_off, rank))
         return ILLM_ERR_ARG;
     if (B == 0) return ILLM_OK;
-    return fixed_step_launch(U, dt, u_stride, r_off, k_off, v_off, nullptr,
-                             RemovalArgs{a_bias, w2, w0, a_off, w1_off, rank, rate}, true, state, row_slot, o, B, H,
-                             d, d, (hipStream_t)stream);
+    StepArgs sa = {};
+    sa.rates = fd_at(U, dt, a_off); sa.rate_bias = a_bias; sa.rate = rate;
+    sa.low = fd_at(U, dt, w1_off); sa.low_stride = u_stride; sa.rank = rank; sa.w2 = w2; sa.w0 = w0;
+    return fixed_step_launch<FD_REMOVAL>(fd_at(U, dt, r_off), fd_at(U, dt, k_off), fd_at(U, dt, v_off), dt, u_stride,
+                                         sa, state, row_slot, o, B, H, d, d, (hipStream_t)stream);
+}
+
+extern "C" int illm_retention_step(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                                   const float* decay, const float* cos_sin, int n_positions, int rot, float k_scale,
+                                   const int32_t* row_pos, float* state, const int32_t* row_slot, float* o, int B,
+                                   int H, int dk, int dv, void* stream) {
+    if (B < 0 || B > 65535 || H <= 0 || H > 65535 || dk <= 0 || dk > 256 || dv <= 0 || !illm_dtype_ok(dt) ||
+        rot < 0 || rot % 2 || rot > dk || (rot > 0 && (!cos_sin || n_positions <= 0 || !row_pos)) ||
+        !fd_columns_ok(u_stride, q_off, H * dk) || !fd_columns_ok(u_stride, k_off, H * dk) ||
+        !fd_columns_ok(u_stride, v_off, H * dv))
+        return ILLM_ERR_ARG;
+    if (B == 0) return ILLM_OK;
+    StepArgs sa = {};
+    sa.decay = decay; sa.cos_sin = cos_sin; sa.row_pos = row_pos; sa.rot = rot; sa.k_scale = k_scale;
+    return fixed_step_launch<FD_RETENTION>(fd_at(U, dt, q_off), fd_at(U, dt, k_off), fd_at(U, dt, v_off), dt, u_stride,
+                                           sa, state, row_slot, o, B, H, dk, dv, (hipStream_t)stream);
+}
+
+extern "C" int illm_time_mix_step(const void* r, const void* k, const void* v, int dt, int stride, const void* low,
+                                  int low_stride, int rank, const void* w2, const float* w0, const float* bonus,
+                                  float* state, const int32_t* row_slot, float* o, int B, int H, int d, void* stream) {
+    if (B < 0 || B > 65535 || H <= 0 || H > 65535 || d <= 0 || d > 256 || rank <= 0 || rank > FD_RANK_MAX ||
+        !illm_dtype_ok(dt) || stride < H * d || low_stride < rank)
+        return ILLM_ERR_ARG;
+    if (B == 0) return ILLM_OK;
+    StepArgs sa = {};
+    sa.low = low; sa.low_stride = low_stride; sa.rank = rank; sa.w2 = w2; sa.w0 = w0; sa.bonus = bonus;
+    return fixed_step_launch<FD_TIME_MIX>(r, k, v, dt, stride, sa, state, row_slot, o, B, H, d, d,
+                                          (hipStream_t)stream);
 }
 
 // ---------------------------------------------------------------- lightning attention in chunks
@@ -270,18 +397,19 @@ extern "C" int illm_removal_step(const void* U, int dt, int u_stride, int r_off,
 #define FD_CHUNK 64
 typedef float fd_f32x16_t __attribute__((ext_vector_type(16)));
 
-template <int DT>
-__device__ __forceinline__ float4 ld4_silu(const void* p, size_t at) {
+template <int DT, bool SILU>
+__device__ __forceinline__ float4 ld4_act(const void* p, size_t at) {
     float4 x = ld_f4(p, DT, at / 4);
+    if (!SILU) return x;
     x.x = fd_silu(x.x); x.y = fd_silu(x.y); x.z = fd_silu(x.z); x.w = fd_silu(x.w);
     return x;
 }
 
 // grid (chunks, H, sequences); 256 threads.  Both operands lie in LDS as [token][channel]; a wave takes
 // every fourth tile of 32 x 32 of the sum.
-template <int DT, int KT, int VT>
+template <int KDT, int DT, bool SILU, int KT, int VT>
 __global__ void __launch_bounds__(256)
-lightning_chunk_sums_kernel(const void* __restrict__ U, int u_stride, int k_off, int v_off,
+lightning_chunk_sums_kernel(const void* __restrict__ K, int k_stride, const void* __restrict__ V, int v_stride,
                             const float* __restrict__ decay, float* __restrict__ part,
                             const int32_t* __restrict__ cu, int H, int dk, int dv) {
     constexpr int DKP = 32 * KT, DVP = 32 * VT, NT = (KT * VT + 3) / 4;
@@ -297,14 +425,14 @@ lightning_chunk_sums_kernel(const void* __restrict__ U, int u_stride, int k_off,
     for (int e = tid; e < FD_CHUNK * (DKP / 4); e += 256) {
         const int row = e / (DKP / 4), d = 4 * (e % (DKP / 4));
         float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (row < nc && d < dk) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + k_off + (size_t)h * dk + d);
+        if (row < nc && d < dk) x = ld4_act<KDT, SILU>(K, (size_t)(r0 + t0 + row) * k_stride + (size_t)h * dk + d);
         const float f = pw[row];
         *(float4*)(ks + row * DKP + d) = make_float4(x.x * f, x.y * f, x.z * f, x.w * f);
     }
     for (int e = tid; e < FD_CHUNK * (DVP / 4); e += 256) {
         const int row = e / (DVP / 4), d = 4 * (e % (DVP / 4));
         float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (row < nc && d < dv) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + v_off + (size_t)h * dv + d);
+        if (row < nc && d < dv) x = ld4_act<DT, SILU>(V, (size_t)(r0 + t0 + row) * v_stride + (size_t)h * dv + d);
         *(float4*)(vs + row * DVP + d) = x;
     }
     __syncthreads();
@@ -368,9 +496,10 @@ lightning_chunk_carry_kernel(float* __restrict__ part, const float* __restrict__
 // token: scores^T = K . Q^T leaves the 16 scores of token (lane % 32) in a lane and its partner 32 lanes
 // on, and in o^T = V^T . P^T they are the second operand as they stand.  k and v lie in LDS, q in
 // registers; the start state is read straight from memory (32 neighbouring values a row).
-template <int DT, int KT, int VT>
+template <int KDT, int DT, bool SILU, int KT, int VT>
 __global__ void __launch_bounds__(256, 2)
-lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off, int k_off, int v_off,
+lightning_chunk_rows_kernel(const void* __restrict__ Q, const void* __restrict__ K, int k_stride,
+                            const void* __restrict__ V, int v_stride,
                             const float* __restrict__ decay, const float* __restrict__ part,
                             const int32_t* __restrict__ cu, float* __restrict__ o, int H, int dk, int dv) {
     constexpr int DKP = 32 * KT, DVP = 32 * VT, KLD = DKP + 1, VW = (VT + 1) / 2;
@@ -386,11 +515,11 @@ lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off,
     if (tid <= FD_CHUNK) pw[tid] = powf(decay[h], (float)tid);
     float qr[DKP / 2];                                  // dims 2 s + half (zeros beyond dk)
     {
-        const size_t at = (size_t)(r0 + t0 + min(i, nc - 1)) * u_stride + q_off + (size_t)h * dk;
+        const size_t at = (size_t)(r0 + t0 + min(i, nc - 1)) * k_stride + (size_t)h * dk;
 #pragma unroll
         for (int j = 0; j < DKP / 4; ++j) {
             float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (4 * j < dk) x = ld4_silu<DT>(U, at + 4 * j);
+            if (4 * j < dk) x = ld4_act<KDT, SILU>(Q, at + 4 * j);
             qr[2 * j] = half ? x.y : x.x;
             qr[2 * j + 1] = half ? x.w : x.z;
         }
@@ -398,14 +527,14 @@ lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off,
     for (int e = tid; e < FD_CHUNK * (DKP / 4); e += 256) {
         const int row = e / (DKP / 4), d = 4 * (e % (DKP / 4));
         float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (row < nc && d < dk) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + k_off + (size_t)h * dk + d);
+        if (row < nc && d < dk) x = ld4_act<KDT, SILU>(K, (size_t)(r0 + t0 + row) * k_stride + (size_t)h * dk + d);
         float* to = ks + row * KLD + d;
         to[0] = x.x; to[1] = x.y; to[2] = x.z; to[3] = x.w;
     }
     for (int e = tid; e < FD_CHUNK * (DVP / 4); e += 256) {
         const int row = e / (DVP / 4), d = 4 * (e % (DVP / 4));
         float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (row < nc && d < dv) x = ld4_silu<DT>(U, (size_t)(r0 + t0 + row) * u_stride + v_off + (size_t)h * dv + d);
+        if (row < nc && d < dv) x = ld4_act<DT, SILU>(V, (size_t)(r0 + t0 + row) * v_stride + (size_t)h * dv + d);
         *(float4*)(vs + row * DVP + d) = x;
     }
     __syncthreads();
@@ -472,45 +601,75 @@ lightning_chunk_rows_kernel(const void* __restrict__ U, int u_stride, int q_off,
 
 extern "C" int illm_lightning_chunk(void) { return FD_CHUNK; }
 
-// `part`: (T / FD_CHUNK + n_seqs + 1) H dk dv floats.
-extern "C" int illm_lightning_chunks(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
-                                     const float* decay, float* state, float* part, const int32_t* cu,
-                                     const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int H, int dk,
-                                     int dv, void* stream) {
-    if (n_seqs < 0 || n_seqs > 65535 || max_rows < 0 || H <= 0 || H > 65535 || dk <= 0 || dk > 128 || dk % 4 ||
-        dv <= 0 || dv > 128 || dv % 4 || !illm_dtype_ok(dt) || u_stride % 4 || q_off % 4 || k_off % 4 || v_off % 4 ||
-        !fd_columns_ok(u_stride, q_off, H * dk) || !fd_columns_ok(u_stride, k_off, H * dk) ||
-        !fd_columns_ok(u_stride, v_off, H * dv) || !part)
-        return ILLM_ERR_ARG;
-    if (n_seqs == 0 || max_rows == 0) return ILLM_OK;
-    hipStream_t st = (hipStream_t)stream;
+// q and k rows of type KDT and k_stride numbers, v rows of type DT and v_stride.
+template <int KDT, int DT, bool SILU>
+static int chunks_launch(const void* Q, const void* K, int k_stride, const void* V, int v_stride, const float* decay,
+                         float* state, float* part, const int32_t* cu, const int32_t* seq_slot, float* o,
+                         int n_seqs, int max_rows, int H, int dk, int dv, hipStream_t st) {
     const dim3 grid((max_rows + FD_CHUNK - 1) / FD_CHUNK, H, n_seqs);
     const int kt = (dk + 31) / 32, vt = (dv + 31) / 32;
-#define GO(DT_, KT_, VT_)                                                                               \
+#define GO(KT_, VT_)                                                                                    \
     do {                                                                                                \
-        hipLaunchKernelGGL((lightning_chunk_sums_kernel<DT_, KT_, VT_>), grid, dim3(256), 0, st, U, u_stride, \
-                           k_off, v_off, decay, part, cu, H, dk, dv);                                   \
+        hipLaunchKernelGGL((lightning_chunk_sums_kernel<KDT, DT, SILU, KT_, VT_>), grid, dim3(256), 0, st, K, \
+                           k_stride, V, v_stride, decay, part, cu, H, dk, dv);                          \
         hipLaunchKernelGGL(lightning_chunk_carry_kernel, dim3((dk * dv / 4 + 255) / 256, H, n_seqs), dim3(256), 0, \
                            st, part, decay, state, cu, seq_slot, H, dk, dv);                            \
-        hipLaunchKernelGGL((lightning_chunk_rows_kernel<DT_, KT_, VT_>), grid, dim3(256), 0, st, U, u_stride, \
-                           q_off, k_off, v_off, decay, part, cu, o, H, dk, dv);                         \
+        hipLaunchKernelGGL((lightning_chunk_rows_kernel<KDT, DT, SILU, KT_, VT_>), grid, dim3(256), 0, st, Q, K, \
+                           k_stride, V, v_stride, decay, part, cu, o, H, dk, dv);                       \
     } while (0)
-#define GO_V(DT_, KT_)                                                                                  \
-    switch (vt) { case 1: GO(DT_, KT_, 1); break; case 2: GO(DT_, KT_, 2); break;                       \
-                  case 3: GO(DT_, KT_, 3); break; default: GO(DT_, KT_, 4); break; }
-#define GO_K(DT_)                                                                                       \
-    switch (kt) { case 1: GO_V(DT_, 1) break; case 2: GO_V(DT_, 2) break;                               \
-                  case 3: GO_V(DT_, 3) break; default: GO_V(DT_, 4) break; }
-    if (dt == ILLM_BF16) { GO_K(ILLM_BF16) } else { GO_K(ILLM_F32) }
-#undef GO_K
+#define GO_V(KT_)                                                                                       \
+    switch (vt) { case 1: GO(KT_, 1); break; case 2: GO(KT_, 2); break;                                 \
+                  case 3: GO(KT_, 3); break; default: GO(KT_, 4); break; }
+    switch (kt) { case 1: GO_V(1) break; case 2: GO_V(2) break; case 3: GO_V(3) break; default: GO_V(4) break; }
 #undef GO_V
 #undef GO
     return illm_launch_status();
 }
 
+static bool chunks_sizes_ok(int n_seqs, int max_rows, int H, int dk, int dv) {
+    return n_seqs >= 0 && n_seqs <= 65535 && max_rows >= 0 && H > 0 && H <= 65535 && dk > 0 && dk <= 128 &&
+           dk % 4 == 0 && dv > 0 && dv <= 128 && dv % 4 == 0;
+}
+
+// `part`: (T / FD_CHUNK + n_seqs + 1) H dk dv floats.
+extern "C" int illm_lightning_chunks(const void* U, int dt, int u_stride, int q_off, int k_off, int v_off,
+                                     const float* decay, float* state, float* part, const int32_t* cu,
+                                     const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int H, int dk,
+                                     int dv, void* stream) {
+    if (!chunks_sizes_ok(n_seqs, max_rows, H, dk, dv) || !illm_dtype_ok(dt) || u_stride % 4 || q_off % 4 ||
+        k_off % 4 || v_off % 4 || !fd_columns_ok(u_stride, q_off, H * dk) || !fd_columns_ok(u_stride, k_off, H * dk) ||
+        !fd_columns_ok(u_stride, v_off, H * dv) || !part)
+        return ILLM_ERR_ARG;
+    if (n_seqs == 0 || max_rows == 0) return ILLM_OK;
+    const void *q = fd_at(U, dt, q_off), *k = fd_at(U, dt, k_off), *v = fd_at(U, dt, v_off);
+    if (dt == ILLM_BF16)
+        return chunks_launch<ILLM_BF16, ILLM_BF16, true>(q, k, u_stride, v, u_stride, decay, state, part, cu, seq_slot,
+                                                         o, n_seqs, max_rows, H, dk, dv, (hipStream_t)stream);
+    return chunks_launch<ILLM_F32, ILLM_F32, true>(q, k, u_stride, v, u_stride, decay, state, part, cu, seq_slot, o,
+                                                   n_seqs, max_rows, H, dk, dv, (hipStream_t)stream);
+}
+
+// The same chunks without activations: qn, kn float32 [T, H, dk] (illm_retention_prepare), v in U's columns
+// v_off .. as stored.
+extern "C" int illm_retention_chunks(const float* qn, const float* kn, const void* U, int dt, int u_stride, int v_off,
+                                     const float* decay, float* state, float* part, const int32_t* cu,
+                                     const int32_t* seq_slot, float* o, int n_seqs, int max_rows, int H, int dk,
+                                     int dv, void* stream) {
+    if (!chunks_sizes_ok(n_seqs, max_rows, H, dk, dv) || !illm_dtype_ok(dt) || u_stride % 4 || v_off % 4 ||
+        !fd_columns_ok(u_stride, v_off, H * dv) || !part)
+        return ILLM_ERR_ARG;
+    if (n_seqs == 0 || max_rows == 0) return ILLM_OK;
+    const void* v = fd_at(U, dt, v_off);
+    if (dt == ILLM_BF16)
+        return chunks_launch<ILLM_F32, ILLM_BF16, false>(qn, kn, H * dk, v, u_stride, decay, state, part, cu, seq_slot,
+                                                         o, n_seqs, max_rows, H, dk, dv, (hipStream_t)stream);
+    return chunks_launch<ILLM_F32, ILLM_F32, false>(qn, kn, H * dk, v, u_stride, decay, state, part, cu, seq_slot, o,
+                                                    n_seqs, max_rows, H, dk, dv, (hipStream_t)stream);
+}
+
 // ---------------------------------------------------------------- behind the recurrence
 // out[r, j] = o[r, j] / sqrt(mean over j's part of o^2 + eps) * w[j] * act(Z[r, z_off + j]) with the row of
-// `width` numbers in `groups` equal parts; act = silu (gate_kind 0) or sigmoid (1).
+// `width` numbers in `groups` equal parts (w null: no weight); act = silu (gate_kind 0) or sigmoid (1).
 // Parts of up to 512 numbers: grid (rows, ceil(groups / 4)), a wave a part; longer ones: grid (rows,
 // groups), a block a part.
 __device__ __forceinline__ float fd_gate(float z, int gate_kind) { return gate_kind ? fd_sigmoid(z) : fd_silu(z); }
@@ -536,7 +695,7 @@ group_norm_gate_kernel(const float* __restrict__ o, const void* __restrict__ w, 
         const float inv = 1.0f / sqrtf(ss / (float)part + eps);
         for (int j = t; j < part / 4; j += step) {
             float4 x = ((const float4*)op)[j];
-            const float4 ww = ld_f4(w, w_dt, j0 / 4 + j), z = ld_f4(Z, z_dt, (r * z_stride + z_off + j0) / 4 + j);
+            const float4 ww = w ? ld_f4(w, w_dt, j0 / 4 + j) : make_float4(1.f, 1.f, 1.f, 1.f), z = ld_f4(Z, z_dt, (r * z_stride + z_off + j0) / 4 + j);
             x.x = (x.x * inv) * ww.x * fd_gate(z.x, gate_kind);
             x.y = (x.y * inv) * ww.y * fd_gate(z.y, gate_kind);
             x.z = (x.z * inv) * ww.z * fd_gate(z.z, gate_kind);
@@ -549,14 +708,14 @@ group_norm_gate_kernel(const float* __restrict__ o, const void* __restrict__ w, 
     ss = WAVE ? wave_sum(ss) : block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)part + eps);
     for (int j = t; j < part; j += step)
-        st_f(out, out_dt, r * width + j0 + j, (op[j] * inv) * ld_f(w, w_dt, j0 + j) *
+        st_f(out, out_dt, r * width + j0 + j, (op[j] * inv) * (w ? ld_f(w, w_dt, j0 + j) : 1.f) *
                                                   fd_gate(ld_f(Z, z_dt, r * z_stride + z_off + j0 + j), gate_kind));
 }
 
 extern "C" int illm_group_norm_gate(const float* o, const void* w, int w_dt, const void* Z, int z_dt, int z_stride,
                                     int z_off, int gate_kind, void* out, int out_dt, int T, int width, int groups,
                                     float eps, void* stream) {
-    if (T < 0 || width <= 0 || groups <= 0 || groups > 65535 || width % groups || !illm_dtype_ok(w_dt) ||
+    if (T < 0 || width <= 0 || groups <= 0 || groups > 65535 || width % groups || (w && !illm_dtype_ok(w_dt)) ||
         !illm_dtype_ok(z_dt) || !illm_dtype_ok(out_dt) || !fd_columns_ok(z_stride, z_off, width) ||
         (gate_kind != 0 && gate_kind != 1))
         return ILLM_ERR_ARG;

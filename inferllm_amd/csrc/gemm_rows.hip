@@ -55,6 +55,9 @@ struct GrScale {
     float eps;
     float act_limit;             // gate|up: > 0, the clamped gate g sigmoid(act_alpha g) (u + 1) with
     float act_alpha;             // g = min(gate, limit), u = clamp(up, -limit, limit); else silu(gate) up
+    int planes;                  // GR_PLAIN: > 1, W's tiles are that many parts and part p, whose tiles end at
+    int ends[ILLM_MAX_PLANES];   // ends[p], reads plane p of X (plane_stride numbers apart); a block's tiles
+    size_t plane_stride;         // are of one part
 };
 
 // GR_PIECE: k-steps of 32 in a piece.  A block of four or more tiles has at most two parts of K,
@@ -72,6 +75,11 @@ gemm_rows_kernel(const bf16_t* __restrict__ X, const bf16_t* __restrict__ Wt, vo
     const int tl = wave % TB, part = wave / TB;
     const int tile = blockIdx.x * TB + tl;
     const bool tile_ok = tile < tiles;
+    if (MODE == GR_PLAIN && scale.planes > 1) {
+        int plane = 0;
+        for (int p = 0; p + 1 < scale.planes; ++p) plane += (int)(blockIdx.x * TB) >= scale.ends[p] ? 1 : 0;
+        X += (size_t)plane * scale.plane_stride;
+    }
     const int ksteps = K / 32;
     const int pieces = (ksteps + GR_PIECE - 1) / GR_PIECE;
     const int per = (pieces + kp - 1) / kp;                  // pieces a part takes
@@ -349,11 +357,19 @@ extern "C" void illm_set_rows_shape(int tb, int kp) {
 #define GR_PIECE_STEPS 2      // k-steps of 32 in a piece (pieces of 128 k measured no better at 16
                               // rows and worse at 64)
 
-static void rows_shape(int tiles, int K, int mt, int* tb, int* kp) {
+// whether blocks of t tiles are each of one part of W (see GrScale)
+static bool tiles_of_one_part(const GrScale& scale, int t) {
+    for (int p = 0; p + 1 < scale.planes; ++p)
+        if (scale.ends[p] % t) return false;
+    return true;
+}
+
+static void rows_shape(int tiles, int K, int mt, const GrScale& scale, int* tb, int* kp) {
     const int cus = 256;
     int best_tb = 2;
     long long best = -1;
     for (int t = 2; t <= 8; ++t) {
+        if (!tiles_of_one_part(scale, t)) continue;
         const int blocks = (tiles + t - 1) / t;
         const long long cost = (long long)((blocks + cus - 1) / cus) * t;
         if (best < 0 || cost < best || (cost == best && mt > 1)) {
@@ -361,7 +377,7 @@ static void rows_shape(int tiles, int K, int mt, int* tb, int* kp) {
             best_tb = t;
         }
     }
-    *tb = GR_TB ? GR_TB : best_tb;
+    *tb = GR_TB && tiles_of_one_part(scale, GR_TB) ? GR_TB : best_tb;
     *kp = GR_KP ? GR_KP : (*tb <= 3 ? 2 : 1);
     const int kp_max = (*tb >= 4 ? 2 : 4) / (mt > 4 ? 2 : 1);   // the kernel's launch bounds
     if (*kp > kp_max) *kp = kp_max;
@@ -373,7 +389,7 @@ template <int MT, int MODE>
 static int launch_rows(const bf16_t* x, const bf16_t* wt, void* y, int y_dt, int rows, int N, int K,
                        int tiles, const GrRope& rope, const GrScale& scale, hipStream_t st) {
     int tb, kp;
-    rows_shape(tiles, K, MT, &tb, &kp);
+    rows_shape(tiles, K, MT, scale, &tb, &kp);
     constexpr int ps = GR_PIECE_STEPS;
     const size_t x_bytes = (size_t)kp * 2 * MT * 16 * ps * 4 * 16 + (MT == 1 ? 64 : 0);
     const size_t red_bytes = (size_t)(kp - 1) * tb * MT * 64 * 16;
@@ -442,6 +458,23 @@ extern "C" int illm_gemm_rows_bf16(const void* X, const void* Wt, void* Y, int y
     const GrScale scale = {ssq, parts, eps};
     return rows_product<GR_PLAIN>(X, Wt, Y, y_dt, M, N, K, (N + 15) / 16, GrRope(), scale,
                                   (hipStream_t)stream);
+}
+
+// The product whose parts of W read rows of X of their own: X [planes][M][K], W's rows ends[p - 1] .. ends[p] - 1
+// times plane p; every part but the last a multiple of 32 rows.
+extern "C" int illm_gemm_rows_planes(const void* X, const void* Wt, void* Y, int y_dt, int M, int N, int K,
+                                     int planes, const int* ends, void* stream) {
+    if (!rows_args_ok(X, Wt, Y, M, N, K, nullptr, 0) || !illm_dtype_ok(y_dt) || planes < 1 ||
+        planes > ILLM_MAX_PLANES || ends[planes - 1] != N)
+        return ILLM_ERR_ARG;
+    GrScale scale = {};
+    scale.planes = planes;
+    scale.plane_stride = (size_t)M * K;
+    for (int p = 0; p < planes; ++p) {
+        if (ends[p] <= (p ? ends[p - 1] : 0) || (p + 1 < planes && ends[p] % 32)) return ILLM_ERR_ARG;
+        scale.ends[p] = ends[p] / 16;
+    }
+    return rows_product<GR_PLAIN>(X, Wt, Y, y_dt, M, N, K, (N + 15) / 16, GrRope(), scale, (hipStream_t)stream);
 }
 
 // With limit > 0 the clamped gate in place of SiLU: Y = g sigmoid(alpha g) (u + 1), g = min(gate, limit),

@@ -60,7 +60,9 @@ struct SkResidual {
     float eps;
     float act_limit;             // gate|up: > 0, the clamped gate g sigmoid(act_alpha g) (u + 1) with
     float act_alpha;             // g = min(gate, limit), u = clamp(up, -limit, limit); else silu(gate) up
-};
+    int planes;                  // SK_PLAIN: > 1, W's rows are that many parts and part p, whose rows end at
+    int ends[ILLM_MAX_PLANES];   // ends[p] (multiples of a block's rows but for the last), reads plane p of
+};                               // X [planes][M][K]
 
 // TILED (NTB == 1, K % 32 == 0): W is a copy laid out for this kernel, [tile][k-step][16 rows][32 k]
 // with tile = blockIdx.x holding the 16 rows that block works on (in its mode's order): a load
@@ -129,6 +131,11 @@ gemm_skinny_kernel(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,
         if (lane < 16) row_rs[lane] = 1.0f / sqrtf(tot / (float)K + res.eps);
     }
     const int n_base = blockIdx.x * (DUAL ? 8 * NTB : 16 * NTB);
+    if (MODE == SK_PLAIN && res.planes > 1) {
+        int plane = 0;
+        for (int p = 0; p + 1 < res.planes; ++p) plane += n_base >= res.ends[p] ? 1 : 0;
+        X += (size_t)plane * M * K;
+    }
     int tile_row[NTB];           // SK_PLAIN: first W row of each of the block's tiles
 #pragma unroll
     for (int nt = 0; nt < NTB; ++nt) tile_row[nt] = n_base + nt * 16;
@@ -450,7 +457,7 @@ gemm_skinny_kernel(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,
     }
 }
 
-static const SkResidual SK_NO_RESIDUAL = {0, nullptr, ILLM_BF16, nullptr, nullptr, nullptr, 0, 0.f, 0.f, 0.f};
+static const SkResidual SK_NO_RESIDUAL = {0, nullptr, ILLM_BF16, nullptr, nullptr, nullptr, 0, 0.f, 0.f, 0.f, 0, {}};
 
 template <int MT, int NTB, int U, int MODE = SK_PLAIN, bool TILED = false, bool ONE_SHOT = false>
 static int launch_skinny(const void* X, const void* W, void* Y, int y_dt, int M, int N, int K,
@@ -543,6 +550,27 @@ extern "C" int illm_gemm_skinny_bf16(const void* X, const void* W, const void* W
         return launch_skinny<1, 1, 4, SK_PLAIN, true>(X, Wt, Y, y_dt, M, N, K, waves,
                                                       (hipStream_t)stream, SkRope(), res);
     }
+    return launch_skinny<1, 1, 4>(X, W, Y, y_dt, M, N, K, waves, (hipStream_t)stream, SkRope(), res);
+}
+
+// The product whose parts of W read rows of X of their own: X [planes][M][K], W's rows ends[p - 1] .. ends[p] - 1
+// times plane p; M <= 16, every part but the last a multiple of 16 rows.
+extern "C" int illm_gemm_skinny_planes(const void* X, const void* W, const void* Wt, void* Y, int y_dt, int M,
+                                       int N, int K, int planes, const int* ends, void* stream) {
+    if (M <= 0 || M > 16 || N <= 0 || K <= 0 || (K % 8) || !illm_dtype_ok(y_dt) || planes < 1 ||
+        planes > ILLM_MAX_PLANES || ends[planes - 1] != N)
+        return ILLM_ERR_ARG;
+    SkResidual res = SK_NO_RESIDUAL;
+    res.planes = planes;
+    for (int p = 0; p < planes; ++p) {
+        if (ends[p] <= (p ? ends[p - 1] : 0) || (p + 1 < planes && ends[p] % 16)) return ILLM_ERR_ARG;
+        res.ends[p] = ends[p];
+    }
+    const int blocks = (N + 15) / 16;
+    int waves = ((use_tiled(Wt, M, K) ? SK_WAVES_ON_CHIP_TILED : SK_WAVES_ON_CHIP) + blocks / 2) / blocks;
+    waves = clamp_waves(waves < 1 ? 1 : waves, 1, 1, 4, K);
+    if (use_tiled(Wt, M, K))
+        return launch_skinny<1, 1, 4, SK_PLAIN, true>(X, Wt, Y, y_dt, M, N, K, waves, (hipStream_t)stream, SkRope(), res);
     return launch_skinny<1, 1, 4>(X, W, Y, y_dt, M, N, K, waves, (hipStream_t)stream, SkRope(), res);
 }
 

@@ -130,11 +130,14 @@ __device__ __forceinline__ float moe_plain_act(float v, int act_kind, bool round
 
 // One wave per token: s = the scores of all NE outputs (float32), choice score = s + correction,
 // the `top` largest choice scores (lowest index on ties) in falling order; weights are scale * s.
+// `groups` > 0: the outputs are that many equal groups of neighbours, of which only the `keep` with the
+// largest sums of their two largest choice scores (lowest index on ties) can be chosen from.
 #define MOE_EPL 8                                   // outputs a lane holds: up to 512 experts
 __device__ __forceinline__ void
 moe_route_row(const float* zr, const void* __restrict__ corr, int corr_dt, int NE, int top,
               int32_t* __restrict__ idx_row, float* __restrict__ wt_row, int32_t* idx_copy,
-              int score_kind, float scale) {
+              int score_kind, float scale, int groups, int keep) {
+    __shared__ float choice[64 * MOE_EPL], group_score[64 * MOE_EPL];
     const int lane = threadIdx.x & 63;
     float s[MOE_EPL], c[MOE_EPL];
     float mx = -INFINITY;
@@ -158,6 +161,36 @@ moe_route_row(const float* zr, const void* __restrict__ corr, int corr_dt, int N
         // softmax over all outputs, or every output's own sigmoid
         s[i] = score_kind == MOE_SCORE_SIGMOID ? (e < NE ? 1.0f / (1.0f + expf(-zr[e])) : 0.f) : s[i] / sum;
         c[i] = e < NE ? s[i] + (corr ? ld_f(corr, corr_dt, e) : 0.f) : -INFINITY;
+    }
+    if (groups > 0) {                                  // (the block is this one wave)
+        const int size = NE / groups;
+#pragma unroll
+        for (int i = 0; i < MOE_EPL; ++i)
+            if (lane + 64 * i < NE) choice[lane + 64 * i] = c[i];
+        __syncthreads();
+        for (int g = lane; g < groups; g += 64) {
+            float a = -INFINITY, b = -INFINITY;        // the two largest
+            for (int j = 0; j < size; ++j) {
+                const float v = choice[g * size + j];
+                if (v > a) { b = a; a = v; }
+                else if (v > b) b = v;
+            }
+            group_score[g] = size > 1 ? a + b : a;
+        }
+        __syncthreads();
+        for (int g = lane; g < groups; g += 64) {
+            const float mine = group_score[g];
+            int before = 0;
+            for (int j = 0; j < groups; ++j)
+                if (group_score[j] > mine || (group_score[j] == mine && j < g)) ++before;
+            choice[g] = before < keep ? 1.f : 0.f;     // (the choice scores have been read)
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < MOE_EPL; ++i) {
+            const int e = lane + 64 * i;
+            if (e < NE && choice[e / size] == 0.f) c[i] = -INFINITY;
+        }
     }
     for (int k = 0; k < top; ++k) {
         float best = -INFINITY;
@@ -187,18 +220,23 @@ moe_route_row(const float* zr, const void* __restrict__ corr, int corr_dt, int N
 
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const float* __restrict__ z, const void* __restrict__ corr, int corr_dt, int NE,
-                 int top, int32_t* __restrict__ idx, float* __restrict__ wt, int score_kind, float scale) {
+                 int top, int32_t* __restrict__ idx, float* __restrict__ wt, int score_kind, float scale,
+                 int groups, int keep) {
     const size_t t = blockIdx.x;
-    moe_route_row(z + t * NE, corr, corr_dt, NE, top, idx + t * top, wt + t * top, nullptr, score_kind, scale);
+    moe_route_row(z + t * NE, corr, corr_dt, NE, top, idx + t * top, wt + t * top, nullptr, score_kind, scale, groups,
+                  keep);
 }
 
 extern "C" int illm_moe_route(const float* z, const void* corr, int corr_dt, int T, int NE, int top,
-                              int32_t* idx, float* wt, int score_kind, float scale, void* stream) {
+                              int32_t* idx, float* wt, int score_kind, float scale, int groups, int keep,
+                              void* stream) {
+    if (groups < 0 || (groups > 0 && (NE % groups || keep <= 0 || keep > groups || top > keep * (NE / groups))))
+        return ILLM_ERR_ARG;
     if ((score_kind != MOE_SCORE_SOFTMAX && score_kind != MOE_SCORE_SIGMOID) || T < 0 || NE <= 0 || NE > 64 * MOE_EPL || top <= 0 || top > NE || (corr && !illm_dtype_ok(corr_dt)))
         return ILLM_ERR_ARG;
     if (T == 0) return ILLM_OK;
     hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(64), 0, (hipStream_t)stream, z, corr, corr_dt,
-                       NE, top, idx, wt, score_kind, scale);
+                       NE, top, idx, wt, score_kind, scale, groups, keep);
     return illm_launch_status();
 }
 

@@ -129,10 +129,14 @@ class DecoderModel:
         x = self.embedding.forward(ctx)
         for position in self.embedding_hooks:
             position.on_embedding(x, ctx)
+        # (x is updated in place: runs that add the embedding's output again need a copy of it)
+        embedded = ops.copy_rows(x) if any(e.adds_embedding for e in self.schedule) else None
         pending = None
         for i, e in enumerate(self.schedule):
             layer = self.layers[e.layer]
             ctx.run = i
+            if e.adds_embedding:
+                pending = ops.plus_rows(pending, embedded)
             if getattr(layer, "takes_next_norm", False):
                 # the norm that will meet this block's output, for kernels that prepare it; none if
                 # the block that follows does not say that it takes rows prepared for its norm

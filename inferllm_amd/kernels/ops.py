@@ -83,6 +83,15 @@ def _gpu(*tensors: Optional[torch.Tensor]) -> None:
             _need(t.is_contiguous(), "kernel operands must be contiguous")
 
 
+def _gpu_rows(*tensors: Optional[torch.Tensor]) -> None:
+    """Rows that may be columns of wider rows: 2-d, neighbouring columns side by side."""
+    for t in tensors:
+        if t is not None:
+            _need(t.is_cuda, "kernel operands must be on the GPU (there is no CPU path)")
+            _need(t.dim() == 2 and (t.shape[1] == 1 or t.stride(1) == 1) and t.stride(0) >= t.shape[1],
+                  "rows of a kernel operand must have their columns side by side")
+
+
 def _i32(t: Optional[torch.Tensor], n: Optional[int] = None) -> None:
     if t is not None:
         _need(t.dtype == torch.int32, "index tensors must be int32")
@@ -111,6 +120,28 @@ def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float = 1.0, copies:
     out = torch.empty((T, E), dtype=torch.float32, device=table.device)
     _check(_lib().illm_embed_scaled(_p(tokens), _p(table), _code(table), _p(out), T, E, V,
                                     ctypes.c_float(scale), _stream()), "embed")
+    return out
+
+
+def embed_norm(tokens: torch.Tensor, table: torch.Tensor, weight: torch.Tensor, eps: float,
+               scale: float = 1.0) -> torch.Tensor:
+    """float32 [T, E]: the rows of `table` at `tokens` times `scale`, under the RMS norm of `weight`, `eps`."""
+    _gpu(tokens, table, weight)
+    _i32(tokens)
+    T, (V, E) = tokens.numel(), table.shape
+    _need(weight.shape == (E,), "embed_norm: weight [E]")
+    out = torch.empty((T, E), dtype=torch.float32, device=table.device)
+    _check(_lib().illm_embed_norm(_p(tokens), _p(table), _code(table), _p(weight), _code(weight), _p(out), None, T, E,
+                                  V, ctypes.c_float(scale), ctypes.c_float(eps), _stream()), "embed_norm")
+    return out
+
+
+def copy_rows(x: torch.Tensor) -> torch.Tensor:
+    """A copy of float32 rows by a kernel of the library (also under graph capture)."""
+    _gpu(x)
+    _need(x.dtype == torch.float32, "copy_rows: float32")
+    out = torch.empty_like(x)
+    _check(_lib().illm_copy_rows(_p(x), _p(out), ctypes.c_size_t(x.numel()), _stream()), "copy_rows")
     return out
 
 
@@ -178,6 +209,22 @@ class ScaledSum:
                                            ctypes.c_float(self.sb), _p(out),
                                            ctypes.c_size_t(a.numel()), _stream()), "sum_rows_scaled")
         return out
+
+
+class NormedPair:
+    """scale (rms(a) wa + rms(b) wb), not yet formed: two mixers' outputs for the same rows, each under an
+    RMS norm of its own.  A block that forms it in a kernel of its own takes the pieces (`PostNormed`), any
+    other asks for `tensor()` (float32)."""
+
+    def __init__(self, a: torch.Tensor, wa: torch.Tensor, b: torch.Tensor, wb: torch.Tensor, eps: float,
+                 scale: float = 0.5):
+        _need(a.shape == b.shape and wa.dtype == wb.dtype, "NormedPair: outputs of one shape, weights of one dtype")
+        self.a, self.wa, self.b, self.wb, self.eps, self.scale = a, wa, b, wb, float(eps), float(scale)
+        self.shape = a.shape
+
+    def tensor(self) -> torch.Tensor:
+        return sum_rows(rms_rows_gain(self.a, self.wa, self.eps, self.scale),
+                        rms_rows_gain(self.b, self.wb, self.eps, self.scale))
 
 
 def relu_squared(x: torch.Tensor) -> torch.Tensor:
@@ -1380,20 +1427,24 @@ MOE_PLAIN_ACTIVATIONS = ("relu_squared",)            # of experts without a gate
 
 
 def moe_route(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, score: str = "softmax",
-              scale: float = 1.0):
+              scale: float = 1.0, groups=None):
     """(idx int32 [T, top], weight float32 [T, top]): per row of the router's float32 outputs z
     the `top` largest score(z) + correction, and `scale` times their scores (`score`: "softmax" over
-    all outputs, or "sigmoid" of each)."""
+    all outputs, or "sigmoid" of each).  `groups` = (count, keep): the outputs are `count` equal groups of
+    neighbours, and only those of the `keep` groups with the largest sums of their two largest choice scores
+    can be chosen."""
     _need(score in MOE_SCORES, f"moe_route: score {score!r}; known: {sorted(MOE_SCORES)}")
     _gpu(z, correction)
     _need(z.dtype == torch.float32 and z.dim() == 2, "moe_route: float32 [T, outputs]")
     T, NE = z.shape
     _need(correction is None or correction.shape == (NE,), "moe_route: correction [outputs]")
+    count, keep = groups or (0, 0)
     idx = torch.empty((T, top), dtype=torch.int32, device=z.device)
     wt = torch.empty((T, top), dtype=torch.float32, device=z.device)
     _check(_lib().illm_moe_route(_p(z), _p(correction),
                                  _code(correction) if correction is not None else 0, T, NE, top,
-                                 _p(idx), _p(wt), MOE_SCORES[score], ctypes.c_float(scale), _stream()), "moe_route")
+                                 _p(idx), _p(wt), MOE_SCORES[score], ctypes.c_float(scale), int(count), int(keep),
+                                 _stream()), "moe_route")
     return idx, wt
 
 
@@ -1425,14 +1476,14 @@ def _moe_group(idx: torch.Tensor, n_exp: int, dtype: torch.dtype, E: int, F: int
 
 def moe_plan(h: torch.Tensor, w_router: torch.Tensor, correction: Optional[torch.Tensor], top: int,
              w_gate_up: Optional[torch.Tensor], score: str = "softmax", scale: float = 1.0,
-             gated: bool = True):
+             gated: bool = True, groups=None):
     """A routed layer's plan for the rows h: (idx, weight, grouped).  idx, weight [T, top] as
     `moe_route` gives them for the router's float32 outputs h . w_router^T; grouped: the pairs
     grouped by expert for `moe_experts` (None without stacked experts).  `gated` False: the stacked
     experts have an up matrix [F, E] alone."""
     E = h.shape[1]
     n_exp = w_gate_up.shape[0] if w_gate_up is not None else 0
-    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score, scale)
+    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score, scale, groups)
     grouped = (_moe_group(idx, n_exp, h.dtype, E, w_gate_up.shape[1] // (2 if gated else 1))
                if n_exp else None)
     return idx, wt, grouped
@@ -1543,6 +1594,12 @@ def _cap_extras_ok(q, slopes, gate, gate_off, nh, dv, what, gate_heads=False):
           f"{what}: gate rows of the queries' dtype with {nh * dv} columns from {gate_off}")
 
 
+def _sink_ok(sink, nh, what):
+    if sink is not None:
+        _gpu(sink)
+        _need(sink.dtype == torch.float32 and sink.shape == (nh,), f"{what}: sink float32 [{nh}]")
+
+
 def _lse_ok(lse, rows, nh, what):
     if lse is not None:
         _gpu(lse)
@@ -1591,7 +1648,8 @@ def attn_cap_rows(q: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Ten
                   window: int, slopes: Optional[torch.Tensor] = None, chunk: int = 0,
                   gate: Optional[torch.Tensor] = None, gate_off: int = 0,
                   gate_heads: bool = False, lse: Optional[torch.Tensor] = None, keep: int = 0,
-                  kept: int = 0, own=None) -> torch.Tensor:
+                  kept: int = 0, own=None, own_values: Optional[torch.Tensor] = None,
+                  sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal attention of a step's packed rows over the paged cache (which holds the step's own
     keys and values by now): row r of sequence b stands at position seq_start[b] + r; scores
     cap tanh(q . k scale / cap) (cap 0: none); queries and keys of width dk, values of dv.
@@ -1601,11 +1659,18 @@ def attn_cap_rows(q: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Ten
     max + log(sum) of every row's and head's softmax.  `keep` (with a window): the sequence's first
     `keep` tokens are seen beside the window; `kept`: pages that stay ahead of the line's ring.
     `own` = (k_off, v_off): keys and values are read from those columns of q's own rows and not from
-    the cache (steps whose sequences all start).  Returns [T, nh dv]."""
+    the cache (steps whose sequences all start); with `own_values` [T, nkv dv] the values are its rows.
+    `sink` float32 [nh]: exp(sink[h]) stands in the softmax's denominator too.  Returns [T, nh dv]."""
     _need(0 <= keep and (keep == 0 or (window > 0 and chunk == 0)), "attn_cap_rows: kept tokens go with a window, without chunks")
     own_stride, own_k, own_v = (q.shape[1], int(own[0]), int(own[1])) if own is not None else (0, 0, 0)
-    _need(own is None or (own_k + nkv * dk <= own_stride and own_v + nkv * dv <= own_stride),
+    values, own_v_stride = q, own_stride
+    if own is not None and own_values is not None:
+        _gpu(own_values)
+        values, own_v, own_v_stride = own_values, 0, own_values.shape[1]
+        _need(values.dtype == q.dtype and values.shape == (q.shape[0], nkv * dv), "attn_cap_rows: own values [T, nkv dv]")
+    _need(own is None or (own_k + nkv * dk <= own_stride and own_v + nkv * dv <= own_v_stride),
           "attn_cap_rows: own keys and values lie within the rows")
+    _sink_ok(sink, nh, "attn_cap_rows")
     _cap_extras_ok(q, slopes, gate, gate_off, nh, dv, "attn_cap_rows", gate_heads)
     _lse_ok(lse, q.shape[0], nh, "attn_cap_rows")
     _gpu(q, cu_seqlens, seq_slot, seq_start, kcache, vcache, page_table)
@@ -1614,11 +1679,11 @@ def attn_cap_rows(q: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Ten
     out = torch.empty((q.shape[0], nh * dv), dtype=q.dtype, device=q.device)
     _check(_lib().illm_attn_cap_rows(
         _p(q), q.shape[1], _p(out), _code(q), _p(cu_seqlens), _p(seq_slot), _p(seq_start),
-        _p(q if own is not None else kcache), _p(q if own is not None else vcache), _p(page_table),
+        _p(q if own is not None else kcache), _p(values if own is not None else vcache), _p(page_table),
         page_table.shape[1], page_size, ring, n_seqs, max_rows, nh, nkv,
         dk, dv, ctypes.c_float(scale), ctypes.c_float(cap), window, _p(slopes), int(chunk), _p(gate),
         gate.shape[1] if gate is not None else 0, gate_off, 1 if gate_heads else 0, _p(lse), int(keep),
-        int(kept), own_stride, own_k, own_v, _stream()),
+        int(kept), own_stride, own_k, own_v_stride, own_v, _p(sink), _stream()),
         f"attn_cap_rows (sizes {dk}, {dv})")
     return out
 
@@ -1629,12 +1694,13 @@ def attn_cap_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
                     cap: float, window: int, nsplit: int, slopes: Optional[torch.Tensor] = None,
                     chunk: int = 0, gate: Optional[torch.Tensor] = None, gate_off: int = 0,
                     gate_heads: bool = False, lse: Optional[torch.Tensor] = None, keep: int = 0,
-                    kept: int = 0) -> torch.Tensor:
+                    kept: int = 0, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The same attention for one new token per sequence: row b of q against the seq_len[b] keys
     (the new one included) of its slot, the keys cut into `nsplit` ranges.  Returns [B, nh dv]."""
     _need(0 <= keep and (keep == 0 or (window > 0 and chunk == 0)), "attn_cap_decode: kept tokens go with a window, without chunks")
     _cap_extras_ok(q, slopes, gate, gate_off, nh, dv, "attn_cap_decode", gate_heads)
     _lse_ok(lse, q.shape[0], nh, "attn_cap_decode")
+    _sink_ok(sink, nh, "attn_cap_decode")
     _need(lse is None or nsplit >= 2, "attn_cap_decode: lse comes from the merge of two or more ranges")
     _gpu(q, kcache, vcache, page_table, seq_slot, seq_len)
     B = q.shape[0]
@@ -1647,7 +1713,7 @@ def attn_cap_decode(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
         page_table.shape[1], page_size, ring, _p(seq_slot), _p(seq_len), _p(partial), nsplit, B, nh,
         nkv, dk, dv, ctypes.c_float(scale), ctypes.c_float(cap), window, _p(slopes), int(chunk),
         _p(gate), gate.shape[1] if gate is not None else 0, gate_off, 1 if gate_heads else 0, _p(lse),
-        int(keep), int(kept), _stream()), f"attn_cap_decode (sizes {dk}, {dv})")
+        int(keep), int(kept), _p(sink), _stream()), f"attn_cap_decode (sizes {dk}, {dv})")
     return out
 
 
@@ -1707,12 +1773,13 @@ def delta_conv_tail(P: torch.Tensor, tail: torch.Tensor, cu_seqlens: torch.Tenso
 
 
 def delta_scan(qn, kn, vv, beta, dec, state: torch.Tensor, cu_seqlens: torch.Tensor,
-               seq_slot: torch.Tensor, n_seqs: int, max_rows: int, correct: bool = True,
+               seq_slot: torch.Tensor, n_seqs: int, max_rows: int, correct=True,
                removal: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The recurrence S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q over every
     sequence's rows in order, from `state` float32 [slots, H, dk, dv] and back into it.  With
     `correct` False the plain gated rule, u = beta v: S <- diag(g) S + k (beta v)^T; with `removal`
-    float32 [T, H, dk] too, S_new = diag(g) S - removal (u^T S) + k v^T with u = beta k.
+    float32 [T, H, dk] too, S_new = diag(g) S - removal (u^T S) + k v^T with u = beta k.  `correct` "bonus":
+    o = S^T q + beta v from the state before the token, then S <- diag(g) S + k v^T.
     `max_rows`: the most rows a sequence brings (long sequences are laid out for their chain of
     tokens, short steps for the state's bytes).  Returns o float32 [T, H, dv]."""
     _gpu(qn, kn, vv, beta, dec, state, cu_seqlens, seq_slot)
@@ -1723,12 +1790,12 @@ def delta_scan(qn, kn, vv, beta, dec, state: torch.Tensor, cu_seqlens: torch.Ten
     _need(kn.shape == qn.shape and beta.shape == (T, H) and dec.shape[:2] == (T, H)
           and dec.shape[2] in (1, dk) and state.shape[1:] == (H, dk, dv), "delta_scan: shapes")
     _gpu(removal)
-    _need(removal is None or (not correct and G == H and removal.dtype == torch.float32
+    _need(removal is None or (correct is False and G == H and removal.dtype == torch.float32
                               and removal.shape == (T, H, dk)), "delta_scan: removal float32 [T, H, dk], without `correct`")
     o = torch.empty((T, H, dv), dtype=torch.float32, device=qn.device)
     _check(_lib().illm_gated_scan(_p(qn), _p(kn), _p(vv), _p(beta), _p(dec), dec.shape[2], _p(state),
                                   _p(cu_seqlens), _p(seq_slot), _p(o), n_seqs, max_rows, G, H, dk, dv,
-                                  1 if correct else 0, _p(removal), _stream()),
+                                  2 if correct == "bonus" else 1 if correct else 0, _p(removal), _stream()),
            "delta_scan")
     return o
 
@@ -1915,18 +1982,42 @@ class PostNormed:
     layer norm with `weight` and, if given, `bias`.  A norm that adds it in its own kernel
     (`post_add_rmsnorm`, `post_add_norm`) takes the pieces, any other asks for `tensor()` (float32)."""
 
-    def __init__(self, a: torch.Tensor, weight: torch.Tensor, eps: float, gain: float, kind: str = "rms",
-                 bias: Optional[torch.Tensor] = None):
+    def __init__(self, a, weight: torch.Tensor, eps: float, gain: float, kind: str = "rms",
+                 bias: Optional[torch.Tensor] = None, plus: Optional[torch.Tensor] = None):
         _need(kind in ("rms", "layer") and (bias is None or kind == "layer"), f"PostNormed: kind {kind!r}")
-        self.a, self.weight, self.eps, self.gain = a, weight, float(eps), float(gain)
-        self.kind, self.bias = kind, bias
+        # `a` may be a `NormedPair` (kind "rms"); `plus`: float32 rows to be added to the stream as well
+        self.pair = a if isinstance(a, NormedPair) else None
+        _need(self.pair is None or kind == "rms", "PostNormed: a pair goes with an RMS norm")
+        self.a, self.weight, self.eps, self.gain = a.a if self.pair is not None else a, weight, float(eps), float(gain)
+        self.kind, self.bias, self.plus = kind, bias, plus
+
+    @property
+    def plain(self) -> bool:
+        """One output under its norm and nothing else."""
+        return self.pair is None and self.plus is None
 
     def tensor(self) -> torch.Tensor:
         if self.kind == "rms":
-            return rms_rows_gain(self.a, self.weight, self.eps, self.gain)
-        out = torch.zeros(self.a.shape, dtype=torch.float32, device=self.a.device)
-        post_add_norm(out, self, None, None, None, 0.0, None)
-        return out
+            out = rms_rows_gain(self.pair.tensor() if self.pair is not None else self.a, self.weight, self.eps, self.gain)
+        else:
+            out = torch.zeros(self.a.shape, dtype=torch.float32, device=self.a.device)
+            post_add_norm(out, PostNormed(self.a, self.weight, self.eps, self.gain, self.kind, self.bias), None, None, None,
+                          0.0, None)
+        return out if self.plus is None else sum_rows(out, self.plus)
+
+
+def plus_rows(pending, rows: torch.Tensor):
+    """What a block left to be added to the residual stream, with float32 `rows` to be added as well."""
+    if pending is None or isinstance(pending, NormedRows):      # (prepared rows: their sum is in the stream already)
+        return rows
+    if isinstance(pending, PostNormed):
+        return PostNormed(pending.pair or pending.a, pending.weight, pending.eps, pending.gain, pending.kind, pending.bias,
+                          rows if pending.plus is None else sum_rows(pending.plus, rows))
+    if isinstance(pending, tuple):
+        pending = sum_rows(*pending)
+    _need(isinstance(pending, torch.Tensor) and pending.shape == rows.shape,
+          f"rows cannot be added to what a block left as {type(pending).__name__}")
+    return sum_rows(pending, rows)
 
 
 NORM_KINDS = {None: 0, "rms": 1, "layer": 2}
@@ -1949,6 +2040,8 @@ def post_add_norm(x: torch.Tensor, post, kind: Optional[str], weight: Optional[t
     _need(E <= POST_NORM_MAX_WIDTH or E % 4 == 0 and E <= 8192, f"post_add_norm: width {E} is beyond the kernel's {POST_NORM_MAX_WIDTH}")
     for t in (weight, bias):
         _need(t is None or (t.shape == (E,) and t.dtype == weight.dtype), "post_add_norm: weight and bias [E] of one dtype")
+    if isinstance(post, PostNormed) and not post.plain:
+        post = post.tensor()
     a = pw = pb = None
     post_kind, post_eps, gain = None, 0.0, 1.0
     if isinstance(post, PostNormed):
@@ -1975,15 +2068,24 @@ POST_ADD_MAX_WIDTH = 16384
 
 
 def post_add_rmsnorm(x: torch.Tensor, post: Optional[PostNormed], weight: torch.Tensor, eps: float,
-                     out_dtype: torch.dtype, row_idx: Optional[torch.Tensor] = None, conv=None) -> torch.Tensor:
+                     out_dtype: torch.dtype, row_idx: Optional[torch.Tensor] = None, conv=None, shift=None) -> torch.Tensor:
     """One pass between two sublayers: x += `post` (its norm formed here; None: nothing), then the
     RMS norm of x under `weight` in `out_dtype`, then, with `conv` = (weight float32 [E, taps], tail
     [slots, taps - 1, E], row_slot), the normed row plus its short convolution over time, the tail
-    moved on (for steps of one row a sequence).  With `row_idx` only those rows, and x stays."""
+    moved on (for steps of one row a sequence).  With `row_idx` only those rows, and x stays.  `post` may be a
+    `NormedPair` under its norm and have rows to be added as well (`plus`).  With `shift` = (mu float32 [S, E],
+    tail [slots, 1, E], row_slot), for steps of one row a sequence, the result is [S, T, E]: the normed row h
+    mixed with the tail's row, h + (tail - h) mu[s], and the tail takes h."""
     _gpu(x, weight, row_idx)
     _i32(row_idx)
     _need(x.dtype == torch.float32 and x.dim() == 2, "post_add_rmsnorm: x must be float32 [T, E]")
     T, E = x.shape
+    if shift is not None or (post is not None and not post.plain):
+        if conv is not None:                     # (no kernel does both: the stream moves on first)
+            post_add_norm(x, post.tensor(), None, None, None, 0.0, None)
+            post = None
+        else:
+            return _post_mix_norm(x, post, weight, eps, out_dtype, row_idx, shift)
     _need(weight.shape == (E,) and E <= POST_ADD_MAX_WIDTH, f"post_add_rmsnorm: weight [{E}], width up to {POST_ADD_MAX_WIDTH}")
     a = pw = None
     if post is not None:
@@ -2010,6 +2112,44 @@ def post_add_rmsnorm(x: torch.Tensor, post: Optional[PostNormed], weight: torch.
     return out
 
 
+def post_mix_fits(E: int) -> bool:
+    """Widths of the pass with two outputs side by side, added rows or a token shift."""
+    return E <= 6144 or (E % 4 == 0 and E <= 8192)
+
+
+def _post_mix_norm(x, post, weight, eps, out_dtype, row_idx, shift) -> torch.Tensor:
+    T, E = x.shape
+    _need(weight.shape == (E,) and post_mix_fits(E), f"post_mix_norm: weight [{E}]; width {E} is beyond the kernel")
+    a = b = aw = bw = pw = plus = mu = tail = slots = None
+    pair_eps = pair_scale = 0.0
+    if post is not None:
+        _need(post.kind == "rms", "post_mix_norm: the sublayer's own norm is an RMS norm")
+        a, pw, plus = post.a, post.weight, post.plus
+        if post.pair is not None:
+            q = post.pair
+            b, aw, bw, pair_eps, pair_scale = q.b, q.wa, q.wb, q.eps, q.scale
+            _need(b.shape == x.shape and aw.shape == (E,) and bw.shape == (E,), "post_mix_norm: the pair has x's shape")
+        _need(a.shape == x.shape and pw.shape == (E,) and (plus is None or (plus.shape == x.shape and plus.dtype == torch.float32)),
+              "post_mix_norm: what is added has x's shape")
+    S = 0
+    if shift is not None:
+        mu, tail, slots = shift
+        _i32(slots, T)
+        S = mu.shape[0]
+        _need(row_idx is None and mu.dtype == torch.float32 and mu.shape == (S, E) and tail.dim() == 3
+              and tail.shape[1:] == (1, E), "post_mix_norm: mu float32 [S, E], tail [slots, 1, E]")
+    _gpu(a, b, aw, bw, pw, plus, mu, tail, slots)
+    rows = T if row_idx is None else row_idx.numel()
+    out = torch.empty((S, rows, E) if S else (rows, E), dtype=out_dtype, device=x.device)
+    code = lambda t: _code(t) if t is not None else 0
+    _check(_lib().illm_post_mix_norm(
+        _p(x), _p(a), code(a), _p(b), code(b), _p(aw), _p(bw), code(aw), ctypes.c_float(pair_eps),
+        ctypes.c_float(pair_scale), _p(pw), code(pw), ctypes.c_float(post.eps if post is not None else 0.0),
+        ctypes.c_float(post.gain if post is not None else 0.0), _p(plus), _p(weight), _code(weight), ctypes.c_float(eps),
+        _p(out), _code(out), _p(mu), S, _p(tail), code(tail), _p(slots), _p(row_idx), rows, E, _stream()), "post_mix_norm")
+    return out
+
+
 SWISH_ALPHA = 1.702
 
 
@@ -2033,7 +2173,8 @@ def qk_rotate_store(rows: torch.Tensor, k_off: int, v_off: int, cos_sin: Optiona
                     ring: int, nh: int, nkv: int, dk: int, dv: int,
                     q_scale: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None,
                     q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None,
-                    slot_len: Optional[torch.Tensor] = None, kept: int = 0) -> None:
+                    slot_len: Optional[torch.Tensor] = None, kept: int = 0, values_from_keys: bool = False,
+                    values_out: Optional[torch.Tensor] = None) -> None:
     """In place on packed rows [q (nh dk) | .. k at k_off (nkv dk) | v at v_off (nkv dv)], in float32:
     the first `rot` dims of every q and k head turned by the row's position (cos_sin float32
     [positions, rot / 2, 2]; pairing 0: i with i + rot / 2, 1: 2i with 2i + 1), then with `unit_norm`
@@ -2043,7 +2184,13 @@ def qk_rotate_store(rows: torch.Tensor, k_off: int, v_off: int, cos_sin: Optiona
     of queries alone).  Before all that `bias` float32 [q | k | v] is added and every q and k head is
     RMS-normed (`eps`) under `q_weight`, `k_weight` [dk].  `kept`: pages that stay ahead of the cache
     line's ring; `slot_len` (the slots' lengths after the step): rows that a later row of the step
-    overwrites in the ring are not stored."""
+    overwrites in the ring are not stored.  `values_from_keys` (dv = dk): the rows have no value columns; a
+    value head is its key head as projected, ahead of norm and rotation, and `values_out` [T, nkv dv] (None:
+    not) takes the values."""
+    _need(not values_from_keys or (dk == dv and bias is None), "qk_rotate_store: values that are the keys have their width and no biases")
+    _gpu(values_out)
+    _need(values_out is None or (values_from_keys and values_out.dtype == rows.dtype
+                                 and values_out.shape == (rows.shape[0], nkv * dv)), "qk_rotate_store: values_out [T, nkv dv]")
     _gpu(rows, cos_sin, row_pos, row_slot, kcache, vcache, page_table, q_scale, bias, q_weight, k_weight, slot_len)
     _i32(slot_len)
     _need(bias is None or (bias.dtype == torch.float32 and bias.shape == (nh * dk + nkv * (dk + dv),)
@@ -2070,7 +2217,7 @@ def qk_rotate_store(rows: torch.Tensor, k_off: int, v_off: int, cos_sin: Optiona
         _p(q_scale), _p(row_pos), _p(row_slot), _p(kcache), _p(vcache), _p(page_table),
         page_table.shape[1] if page_table is not None else 0, page_size, ring, T, nh, nkv, dk, dv, _p(bias),
         _p(q_weight), _p(k_weight), _code(q_weight) if q_weight is not None else 0, _p(slot_len), int(kept),
-        _stream()), "qk_rotate_store")
+        1 if values_from_keys else 0, _p(values_out), _stream()), "qk_rotate_store")
 
 
 def pool_store(row_pos: torch.Tensor, row_slot: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
@@ -2384,20 +2531,241 @@ def removal_step(U: torch.Tensor, r_off: int, k_off: int, v_off: int, a_off: int
     return o
 
 
-def group_norm_gate(o: torch.Tensor, groups: int, weight: torch.Tensor, Z: torch.Tensor, z_off: int, gate: str,
+def group_norm_gate(o: torch.Tensor, groups: int, weight: Optional[torch.Tensor], Z: torch.Tensor, z_off: int, gate: str,
                     eps: float, out_dtype: torch.dtype) -> torch.Tensor:
     """[T, width] rows o (float32 [T, ..], width numbers each) RMS-normed in `groups` equal parts of the
-    row, times weight [width], times act(Z[:, z_off ..]), act "silu" or "sigmoid"."""
-    _gpu(o, weight, Z)
+    row, times weight [width] (None: no weight), times act(Z[:, z_off ..]), act "silu" or "sigmoid"."""
+    _gpu(o, weight)
+    _gpu_rows(Z)
     T = o.shape[0]
-    width = weight.numel()
+    width = weight.numel() if weight is not None else o[0].numel() if T else Z.shape[1] - z_off
     _need(o.dtype == torch.float32 and o.numel() == T * width and width % groups == 0 and gate in DELTA_GATES
-          and Z.dim() == 2 and Z.shape[0] == T and z_off + width <= Z.shape[1], "group_norm_gate: shapes or gate")
+          and Z.shape[0] == T and z_off + width <= Z.shape[1], "group_norm_gate: shapes or gate")
     out = torch.empty((T, width), dtype=out_dtype, device=o.device)
-    _check(_lib().illm_group_norm_gate(_p(o), _p(weight), _code(weight), _p(Z), _code(Z), Z.shape[1], z_off,
-                                       DELTA_GATES[gate], _p(out), _code(out), T, width, int(groups),
+    _check(_lib().illm_group_norm_gate(_p(o), _p(weight), _code(weight) if weight is not None else 0, _p(Z), _code(Z),
+                                       Z.stride(0), z_off, DELTA_GATES[gate], _p(out), _code(out), T, width, int(groups),
                                        ctypes.c_float(eps), _stream()), "group_norm_gate")
     return out
+
+
+# ------------------------------------------------------------------ retention
+def _rot_ok(cos_sin: Optional[torch.Tensor], rot: int, dk: int, what: str) -> None:
+    _gpu(cos_sin)
+    _need(0 <= rot <= dk and rot % 2 == 0 and (rot == 0 or (cos_sin is not None and cos_sin.dtype == torch.float32
+                                                              and cos_sin.dim() == 3 and cos_sin.shape[1:] == (rot // 2, 2))),
+          f"{what}: cos_sin float32 [positions, rot / 2, 2] with rot even and at most the key size")
+
+
+def retention_prepare(U: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor,
+                      cos_sin: Optional[torch.Tensor], rot: int, k_scale: float, row_pos: torch.Tensor, H: int, dk: int,
+                      dv: int, scan: bool = True):
+    """Retention's q and k as float32: U's columns turned by the row's position (pairs i, i + rot / 2), k times
+    `k_scale`.  Returns (q [T, H, dk], k) or, with `scan`, all inputs of the plain gated rule (`delta_scan`):
+    (q, k, v [T, H, dv], weight 1 [T, H], the heads' fixed decays [T, H, 1])."""
+    _gpu(U, decay, row_pos)
+    _columns_ok(U, "retention_prepare", (q_off, H * dk), (k_off, H * dk), (v_off, H * dv))
+    _rot_ok(cos_sin, rot, dk, "retention_prepare")
+    _need(decay.dtype == torch.float32 and decay.shape == (H,), "retention_prepare: decay float32 [H]")
+    T = U.shape[0]
+    _i32(row_pos, T)
+    new = lambda *shape: torch.empty(shape, dtype=torch.float32, device=U.device)
+    qn, kn = new(T, H, dk), new(T, H, dk)
+    vv, beta, dec = (new(T, H, dv), new(T, H), new(T, H, 1)) if scan else (None, None, None)
+    _check(_lib().illm_retention_prepare(
+        _p(U), _code(U), U.shape[1], q_off, k_off, v_off, _p(decay), _p(cos_sin), cos_sin.shape[0] if rot else 0, rot,
+        ctypes.c_float(k_scale), _p(row_pos), _p(qn), _p(kn), _p(vv), _p(beta), _p(dec), T, H, dk, dv, _stream()),
+        "retention_prepare")
+    return (qn, kn, vv, beta, dec) if scan else (qn, kn)
+
+
+def retention_step(U: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor,
+                   cos_sin: Optional[torch.Tensor], rot: int, k_scale: float, row_pos: torch.Tensor, state: torch.Tensor,
+                   row_slot: torch.Tensor, H: int, dk: int, dv: int) -> torch.Tensor:
+    """One row a sequence: rotation, S <- decay S + k v^T, o = S^T q in one launch.  Returns o float32
+    [rows, H, dv]."""
+    _gpu(U, decay, state, row_slot, row_pos)
+    _columns_ok(U, "retention_step", (q_off, H * dk), (k_off, H * dk), (v_off, H * dv))
+    _rot_ok(cos_sin, rot, dk, "retention_step")
+    _decay_ok(decay, state, H, dk, dv, "retention_step")
+    B = U.shape[0]
+    _i32(row_slot, B); _i32(row_pos, B)
+    o = torch.empty((B, H, dv), dtype=torch.float32, device=U.device)
+    _check(_lib().illm_retention_step(
+        _p(U), _code(U), U.shape[1], q_off, k_off, v_off, _p(decay), _p(cos_sin), cos_sin.shape[0] if rot else 0, rot,
+        ctypes.c_float(k_scale), _p(row_pos), _p(state), _p(row_slot), _p(o), B, H, dk, dv, _stream()), "retention_step")
+    return o
+
+
+def retention_chunks_fits(U: torch.Tensor, v_off: int, dk: int, dv: int) -> bool:
+    return dk <= 128 and dv <= 128 and all(n % 4 == 0 for n in (dk, dv, v_off, U.shape[1]))
+
+
+def retention_chunks(qn: torch.Tensor, kn: torch.Tensor, U: torch.Tensor, v_off: int, decay: torch.Tensor,
+                     state: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Tensor, n_seqs: int,
+                     max_rows: int, H: int, dk: int, dv: int) -> torch.Tensor:
+    """The recurrence over every sequence's rows, chunk by chunk in parallel as `lightning_chunks`, from
+    `retention_prepare`'s q and k and U's value columns.  Returns o float32 [T, H, dv]."""
+    _gpu(qn, kn, U, decay, state, cu_seqlens, seq_slot)
+    _i32(cu_seqlens, n_seqs + 1); _i32(seq_slot, n_seqs)
+    T = U.shape[0]
+    _columns_ok(U, "retention_chunks", (v_off, H * dv))
+    _decay_ok(decay, state, H, dk, dv, "retention_chunks")
+    _need(all(t.dtype == torch.float32 and t.shape == (T, H, dk) for t in (qn, kn))
+          and retention_chunks_fits(U, v_off, dk, dv), "retention_chunks: sizes not taken")
+    places = T // _lib().illm_lightning_chunk() + n_seqs + 1
+    part = torch.empty((places, H, dk, dv), dtype=torch.float32, device=U.device)
+    o = torch.empty((T, H, dv), dtype=torch.float32, device=U.device)
+    _check(_lib().illm_retention_chunks(_p(qn), _p(kn), _p(U), _code(U), U.shape[1], v_off, _p(decay), _p(state), _p(part),
+                                        _p(cu_seqlens), _p(seq_slot), _p(o), n_seqs, int(max_rows), H, dk, dv,
+                                        _stream()), "retention_chunks")
+    return o
+
+
+# ------------------------------------------------------------------ time mixing with a token shift
+class TokenMixes:
+    """Rows mixed with the row of the token before, one plane a mix: `planes` [S, T, E]."""
+
+    def __init__(self, planes: torch.Tensor):
+        self.planes = planes
+
+
+def token_mix(h: torch.Tensor, mu: torch.Tensor, tail: torch.Tensor, row_slot: torch.Tensor,
+              update_tail: bool) -> torch.Tensor:
+    """[S, T, E] of h's dtype: h + (h_before - h) mu[s] for every mix (mu float32 [S, E]); the row before a step's
+    first row of a sequence is tail [slots, 1, E], which `update_tail` (one row a sequence) moves on."""
+    _gpu(h, mu, tail, row_slot)
+    T, E = h.shape
+    _i32(row_slot, T)
+    _need(mu.dtype == torch.float32 and mu.dim() == 2 and mu.shape[1] == E and tail.dim() == 3
+          and tail.shape[1:] == (1, E) and tail.dtype == h.dtype, "token_mix: mu float32 [S, E], tail [slots, 1, E]")
+    out = torch.empty((mu.shape[0], T, E), dtype=h.dtype, device=h.device)
+    _check(_lib().illm_token_mix(_p(h), _code(h), _p(mu), mu.shape[0], _p(tail), _p(row_slot), _p(out), _code(out), T, E,
+                                 1 if update_tail else 0, _stream()), "token_mix")
+    return out
+
+
+MAX_PLANES = 8           # planes of rows a product with parts takes
+PARTS_MAX_ROWS = 128     # rows up to which such a product is one launch (or two)
+
+
+def _planes_product(planes: torch.Tensor, w, ends, few: bool) -> torch.Tensor:
+    S, M, K = planes.shape
+    N = ends[-1]
+    y = torch.empty((M, N), dtype=planes.dtype, device=planes.device)
+    arr = (ctypes.c_int * len(ends))(*ends)
+    if few:
+        plain, wt = _w(w)
+        _check(_lib().illm_gemm_skinny_planes(_p(planes), _p(plain), wt, _p(y), _code(y), M, N, K, len(ends), arr,
+                                              _stream()), "linear_parts")
+    else:
+        _check(_lib().illm_gemm_rows_planes(_p(planes), _p(w.tiled), _p(y), _code(y), M, N, K, len(ends), arr,
+                                            _stream()), "linear_parts")
+    return y
+
+
+def linear_parts(planes: torch.Tensor, w, ends):
+    """Products of one stacked matrix w [N, K] whose parts read rows of their own: part p, w's rows ends[p - 1] ..
+    ends[p] - 1, times planes[p] of [S, M, K].  Returns one [M, part] tensor a part (columns of wider rows where one
+    launch made several).  Few bfloat16 rows: one launch; up to 128 rows from the decode copy: one, or two
+    where the last part is no multiple of the blocks; else one product a part."""
+    ends = [int(e) for e in ends]
+    S, M, K = planes.shape
+    _need(planes.dim() == 3 and S == len(ends) and w.shape[1] == K and w.shape[0] == ends[-1], "linear_parts: shapes")
+    _gpu(planes)
+    starts = [0] + ends[:-1]
+    columns = lambda y, n: [y[:, a:b] for a, b in zip(starts[:n], ends[:n])]
+    bf16 = planes.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and 1 <= M and S <= MAX_PLANES
+    if bf16 and M <= SKINNY_BEST_ROWS and K % 8 == 0 and all(e % 16 == 0 for e in ends[:-1]):
+        return columns(_planes_product(planes, w, ends, True), S)
+    if (bf16 and M <= PARTS_MAX_ROWS and isinstance(w, Weight) and w.tiled is not None and w.mode == "plain" and K % 64 == 0
+            and all(e % 32 == 0 for e in ends[:-1])):
+        return columns(_planes_product(planes, w, ends, False), S)
+    plain = plain_weight(w)
+    return [linear(planes[p], plain[a:b]) for p, (a, b) in enumerate(zip(starts, ends))]
+
+
+def tanh_rows(x: torch.Tensor) -> torch.Tensor:
+    """float32 tanh(x) of rows that may be columns of wider rows."""
+    _gpu_rows(x)
+    T, n = x.shape
+    out = torch.empty((T, n), dtype=torch.float32, device=x.device)
+    _check(_lib().illm_tanh_columns(_p(x), _code(x), x.stride(0), 0, _p(out), T, n, _stream()), "tanh_rows")
+    return out
+
+
+def _time_mix_ok(r, k, v, w0, bonus, state, H, d, what):
+    _gpu_rows(r, k, v)
+    _gpu(w0, bonus, state)
+    _need(all(t.shape == (r.shape[0], H * d) and t.dtype == r.dtype and t.stride(0) == r.stride(0) for t in (r, k, v)),
+          f"{what}: r, k, v [T, H d] of one dtype and row stride")
+    _need(all(t.dtype == torch.float32 and t.shape == (H * d,) for t in (w0, bonus)), f"{what}: w0, bonus float32 [H d]")
+    _need(state is None or (state.dtype == torch.float32 and state.dim() == 4 and state.shape[1:] == (H, d, d)),
+          f"{what}: state float32 [slots, H, d, d]")
+
+
+TIME_MIX_STEP_MAX_RANK = 512
+
+
+def time_mix_step(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, low: torch.Tensor, w2: torch.Tensor,
+                  w0: torch.Tensor, bonus: torch.Tensor, state: torch.Tensor, row_slot: torch.Tensor, H: int,
+                  d: int) -> torch.Tensor:
+    """One row a sequence: decay = exp(-exp(w2 tanh(low) + w0)), o = (S + diag(bonus) k v^T)^T r, S <- diag(decay) S
+    + k v^T in one launch.  r, k, v [B, H d], low [B, rank] (columns of wider rows, perhaps), w2 [H d, rank] of
+    their dtype.  Returns o float32 [B, H, d]."""
+    _time_mix_ok(r, k, v, w0, bonus, state, H, d, "time_mix_step")
+    _gpu_rows(low)
+    _gpu(w2, row_slot)
+    B, rank = low.shape
+    _i32(row_slot, B)
+    _need(w2.shape == (H * d, rank) and w2.dtype == r.dtype and low.dtype == r.dtype and low.shape[0] == r.shape[0]
+          and 0 < rank <= TIME_MIX_STEP_MAX_RANK, "time_mix_step: low [B, rank], w2 [H d, rank] of one dtype")
+    o = torch.empty((B, H, d), dtype=torch.float32, device=r.device)
+    _check(_lib().illm_time_mix_step(_p(r), _p(k), _p(v), _code(r), r.stride(0), _p(low), low.stride(0), rank, _p(w2),
+                                     _p(w0), _p(bonus), _p(state), _p(row_slot), _p(o), B, H, d, _stream()),
+           "time_mix_step")
+    return o
+
+
+def time_mix_prepare(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, Z: torch.Tensor, w0: torch.Tensor,
+                     bonus: torch.Tensor, H: int, d: int):
+    """Float32 inputs of `delta_scan` with `correct` "bonus" from r, k, v [T, H d] and the decays' float32
+    pre-activations Z [T, H d]: (r [T, H, d], k, v, beta = sum bonus r k [T, H], decay = exp(-exp(Z + w0)))."""
+    _time_mix_ok(r, k, v, w0, bonus, None, H, d, "time_mix_prepare")
+    _gpu(Z)
+    T = r.shape[0]
+    _need(Z.dtype == torch.float32 and Z.shape == (T, H * d), "time_mix_prepare: Z float32 [T, H d]")
+    new = lambda *shape: torch.empty(shape, dtype=torch.float32, device=r.device)
+    qn, kn, vv, beta, dec = new(T, H, d), new(T, H, d), new(T, H, d), new(T, H), new(T, H, d)
+    _check(_lib().illm_time_mix_prepare(_p(r), _p(k), _p(v), _code(r), r.stride(0), _p(Z), _p(w0), _p(bonus), _p(qn),
+                                        _p(kn), _p(vv), _p(beta), _p(dec), T, H, d, _stream()), "time_mix_prepare")
+    return qn, kn, vv, beta, dec
+
+
+TIME_MIX_CHUNKS_FROM = 32      # rows a sequence from which the chunks run in parallel
+
+
+def time_mix_chunks_fits(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, d: int) -> bool:
+    return (d <= 128 and d % 4 == 0 and r.stride(0) % 4 == 0
+            and all(t.data_ptr() % (4 * t.element_size()) == 0 for t in (r, k, v)))
+
+
+def time_mix_chunks(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, Z: torch.Tensor, w0: torch.Tensor,
+                    bonus: torch.Tensor, state: torch.Tensor, cu_seqlens: torch.Tensor, seq_slot: torch.Tensor,
+                    n_seqs: int, max_rows: int, H: int, d: int) -> torch.Tensor:
+    """`time_mix_prepare` and the scan for many rows a sequence, chunk by chunk in parallel (csrc/time_mix.hip): a
+    row's sums run in another order than token by token.  Returns o float32 [T, H, d]."""
+    _time_mix_ok(r, k, v, w0, bonus, state, H, d, "time_mix_chunks")
+    _gpu(Z, cu_seqlens, seq_slot)
+    _i32(cu_seqlens, n_seqs + 1); _i32(seq_slot, n_seqs)
+    T = r.shape[0]
+    _need(Z.dtype == torch.float32 and Z.shape == (T, H * d) and time_mix_chunks_fits(r, k, v, d), "time_mix_chunks: sizes not taken")
+    places = T // _lib().illm_time_mix_chunk() + n_seqs + 1
+    new = lambda *shape: torch.empty(shape, dtype=torch.float32, device=r.device)
+    sums, part, whole, o = new(T, H * d), new(places, H, d, d), new(places, H, d), new(T, H, d)
+    _check(_lib().illm_time_mix_chunks(_p(r), _p(k), _p(v), _code(r), r.stride(0), _p(Z), _p(w0), _p(bonus), _p(state),
+                                       _p(sums), _p(part), _p(whole), _p(cu_seqlens), _p(seq_slot), _p(o), n_seqs,
+                                       int(max_rows), H, d, _stream()), "time_mix_chunks")
+    return o
 
 
 # ------------------------------------------------------------------ sampling

@@ -1,3 +1,3 @@
-from . import dotorax, febivik, kukupel, llama, rabapel, sabipel  # registers Dotorax, Febivik, Kukupel, LlamaForCausalLM, Rabapel and Sabipel
+from . import dotorax, febivik, kukupel, llama, rabapel, sabipel, vupolix  # registers the architectures
 
-__all__ = ["dotorax", "febivik", "kukupel", "llama", "rabapel", "sabipel"]
+__all__ = ["dotorax", "febivik", "kukupel", "llama", "rabapel", "sabipel", "vupolix"]

@@ -260,6 +260,10 @@ class GatedAttention(Mixer):
     * `bias`: stored biases of the q, k and v projections;
     * `qk_norm` "head_weighted": every q and k head passes an RMS norm over its dims (`eps`) with a
       plain weight [key_dim] that the heads share, before the rotation;
+    * `values` "keys": no value projection; a value head is its key head as projected, before norm and
+      rotation (value_dim = key_dim);
+    * `sink`: a stored number a head whose exponential stands in the softmax's denominator, without a key
+      or a value;
     * `own_kv` False: the layer has no key and value projections and reads the cache line of an
       earlier layer of the step (the schedule names it with `writes_cache` False).
 
@@ -277,8 +281,14 @@ class GatedAttention(Mixer):
                  window: Optional[int] = None, chunk: int = 0, slope_power: float = 0.0,
                  qk_norm=False, eps: float = 1e-6, value_mix: Optional[str] = None,
                  gate=False, head_scale: bool = False, pool: int = 0, own_kv: bool = True, keep_first: int = 0,
-                 bias: bool = False, tensors=None):
+                 bias: bool = False, values: str = "projected", sink: bool = False, tensors=None):
         super().__init__(tensors)
+        if values not in ("projected", "keys") or (values == "keys" and (
+                key_dim != value_dim or bias or value_mix or pool or not own_kv or qk_norm is True)):
+            raise ValueError("gated attention: values that are the keys have the keys' width and go with neither biases, "
+                             "mixed values, pooled blocks, another layer's keys nor a norm over all heads")
+        if sink and pool:
+            raise ValueError("gated attention: a sink goes without pooled blocks")
         if qk_norm not in (False, True, "head", "head_weighted") or gate not in (False, True, "head"):
             raise ValueError(f"gated attention: qk_norm {qk_norm!r} or gate {gate!r}: False, True or 'head' "
                              "(qk_norm also 'head_weighted')")
@@ -312,17 +322,22 @@ class GatedAttention(Mixer):
         self.qk_norm, self.eps, self.value_mix, self.gate = qk_norm, float(eps), value_mix, gate
         self.has_head_scale, self.pool, self.own_kv = bool(head_scale), int(pool or 0), bool(own_kv)
         self.keep_first, self.has_bias = int(keep_first or 0), bool(bias)
+        self.values_are_keys, self.has_sink, self.sink = values == "keys", bool(sink), None
         self.gate_width = self.nh * (1 if gate == "head" else self.dv)
         self.k_off = self.nh * self.dk
         self.v_off = self.k_off + (self.nkv * self.dk if self.own_kv else 0)
-        self.g_off = self.v_off + (self.nkv * self.dv if self.own_kv else 0)
+        self.g_off = self.v_off + (self.nkv * self.dv if self.own_kv and not self.values_are_keys else 0)
         self.slopes = self.lam = self.q_norm = self.k_norm = self.head_scale = self.bias = None
 
     def shapes(self) -> Dict[str, TensorWant]:
         keep = dict(keep_stored=True)
         out = {"q": TensorWant((self.nh * self.dk, self.E)), "o": TensorWant((self.E, self.nh * self.dv))}
         if self.own_kv:
-            out.update(k=TensorWant((self.nkv * self.dk, self.E)), v=TensorWant((self.nkv * self.dv, self.E)))
+            out["k"] = TensorWant((self.nkv * self.dk, self.E))
+            if not self.values_are_keys:
+                out["v"] = TensorWant((self.nkv * self.dv, self.E))
+        if self.has_sink:
+            out["sink"] = TensorWant((self.nh,), **keep)
         if self.has_head_scale:
             out["head_scale"] = TensorWant((self.nh,), init="ones_normal", **keep)
         if self.qk_norm is True:
@@ -353,7 +368,8 @@ class GatedAttention(Mixer):
 
     def load(self, tensors) -> None:
         take = lambda n: self._take(tensors, n)
-        rows = [take(n) for n in (("q", "k", "v") if self.own_kv else ("q",))] + ([take("g")] if self.gate else [])
+        names = ("q",) if not self.own_kv else ("q", "k") if self.values_are_keys else ("q", "k", "v")
+        rows = [take(n) for n in names] + ([take("g")] if self.gate else [])
         self.w_in = ops.decode_weight(_fuse(rows), "plain", self.decode_copies)     # [q | k | v | g]
         self.w_o = ops.decode_weight(take("o").contiguous(), "plain", self.decode_copies)
         dev = take("q").device
@@ -361,6 +377,8 @@ class GatedAttention(Mixer):
             self.bias = torch.cat([take(n).to(torch.float32) for n in ("q_bias", "k_bias", "v_bias")]).contiguous()
         if self.qk_norm in (True, "head_weighted"):
             self.q_norm, self.k_norm = take("q_norm").contiguous(), take("k_norm").contiguous()
+        if self.has_sink:
+            self.sink = take("sink").to(torch.float32).contiguous()
         if self.has_head_scale:
             self.head_scale = take("head_scale").to(torch.float32).contiguous()
         if self.value_mix == "mixed":
@@ -382,7 +400,10 @@ class GatedAttention(Mixer):
         rows = ops.linear(h, self.w_in)
         store = writes_cache
         weighted = self.qk_norm == "head_weighted"
-        if position is not None or self.qk_norm == "head" or weighted or self.has_bias:
+        own = (self.k_off, self.v_off) if ctx.prefill and group.ring and not ctx.continues else None
+        own_values = (torch.empty((rows.shape[0], nkv * dv), dtype=rows.dtype, device=rows.device)
+                      if own and self.values_are_keys else None)
+        if position is not None or self.qk_norm == "head" or weighted or self.has_bias or self.values_are_keys:
             # biases, norms a head, rotation and the store in one pass over the rows
             table = position.table(ctx.device) if position is not None else None
             ops.qk_rotate_store(rows, self.k_off, self.v_off, table,
@@ -394,7 +415,7 @@ class GatedAttention(Mixer):
                                 bias=self.bias, q_weight=self.q_norm if weighted else None,
                                 k_weight=self.k_norm if weighted else None,
                                 slot_len=ctx.overwritten_lengths if group.ring else None,
-                                kept=group.kept_pages)
+                                kept=group.kept_pages, values_from_keys=self.values_are_keys, values_out=own_values)
         else:
             if group.ring:
                 raise ValueError("gated attention: a window whose line is a ring of pages needs the store that "
@@ -428,8 +449,8 @@ class GatedAttention(Mixer):
             o = ops.attn_cap_rows(rows, ctx.cu_seqlens, ctx.seq_slot, ctx.seq_start, kc, vc, group.table,
                                   group.page_size, group.ring, ctx.n_seqs, ctx.max_rows, nh, nkv, dk, dv,
                                   self.scale, self.softcap, window, self.slopes, self.chunk, gate, self.g_off,
-                                  by_head, lse, keep=self.keep_first, kept=group.kept_pages,
-                                  own=(self.k_off, self.v_off) if group.ring and not ctx.continues else None)
+                                  by_head, lse, keep=self.keep_first, kept=group.kept_pages, own=own,
+                                  own_values=own_values, sink=self.sink)
             if lse is not None:
                 ops.attn_pooled_rows(rows, ctx.cu_seqlens, ctx.seq_slot, ctx.seq_start, kc, vc, kp, vp,
                                      group.table, group.page_size, ctx.n_seqs, ctx.max_rows, nh, nkv, dk, dv,
@@ -448,7 +469,7 @@ class GatedAttention(Mixer):
             o = ops.attn_cap_decode(rows, kc, vc, group.table, group.page_size, group.ring, ctx.seq_slot,
                                     ctx.seq_len, nh, nkv, dk, dv, self.scale, self.softcap, window,
                                     nsplit, self.slopes, self.chunk, gate, self.g_off, by_head, lse,
-                                    keep=self.keep_first, kept=group.kept_pages)
+                                    keep=self.keep_first, kept=group.kept_pages, sink=self.sink)
             if lse is not None:
                 ops.attn_pooled_decode(rows, kc, vc, kp, vp, group.table, group.page_size, ctx.seq_slot,
                                        ctx.seq_len, nh, nkv, dk, dv, self.scale, None, window, self.pool,

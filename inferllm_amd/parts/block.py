@@ -120,6 +120,8 @@ class SandwichBlock(Block):
         self.has_ff = feed_forward_norm is not None
         self.post = [None, None]
         self.conv = [None, None]
+        if hasattr(mixer, "takes_normed_pairs") and ops.post_mix_fits(self.size):
+            mixer.takes_normed_pairs = True      # the pass behind the mixer forms its two outputs' norms
 
     def _sublayers(self):
         return (1, 2) if self.has_ff else (1,)
@@ -159,9 +161,10 @@ class SandwichBlock(Block):
             ops.short_conv_tail(h, 0, tail, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs, self.taps)
         return out
 
-    def _enter(self, norm, q: int, x, pending, ctx: StepContext):
+    def _enter(self, norm, q: int, x, pending, ctx: StepContext, line=None):
         """Sublayer q's input: `pending` added to x, the norm, the convolution.  A plain RMS norm
-        and a step of single tokens make that one kernel."""
+        and a step of single tokens make that one kernel; a mixer that reads mixes with the token before
+        gets them from the same kernel then."""
         if isinstance(pending, ops.NormedRows):
             pending = None                       # its sum is in x already
         params = norm.rms_params()
@@ -170,6 +173,10 @@ class SandwichBlock(Block):
                 and self.size <= ops.POST_ADD_MAX_WIDTH):
             return ops.post_add_rmsnorm(x, pending, params[0], params[1], ctx.act_dtype,
                                         conv=(self.conv[q - 1], self._tail(q, ctx), ctx.row_slot))
+        if (q == 1 and params is not None and plain and not ctx.prefill and not self.taps
+                and getattr(self.mixer, "takes_token_mixes", False) and ops.post_mix_fits(self.size)):
+            return ops.TokenMixes(ops.post_add_rmsnorm(x, pending, params[0], params[1], ctx.act_dtype,
+                                                       shift=self.mixer.shift(ctx, line)))
         if isinstance(pending, ops.PostNormed) and not getattr(norm, "adds_post_normed", False):
             pending = pending.tensor()
         return self._read(norm.forward(x, pending, ctx), q, ctx)
@@ -181,7 +188,7 @@ class SandwichBlock(Block):
         return post if next_norm is not None and getattr(next_norm, "adds_post_normed", False) else post.tensor()
 
     def forward(self, x, pending, ctx: StepContext, line, writes_cache, next_norm=None):
-        h = self._enter(self.mixer_norm, 1, x, pending, ctx)
+        h = self._enter(self.mixer_norm, 1, x, pending, ctx, line)
         a = self.mixer.forward(h, ctx, line, writes_cache, self.position)
         if not self.has_ff:
             return self._leave(a, 1, next_norm)

@@ -15,24 +15,35 @@ from .base import Embedding, Head, StepContext, register_part
 class TokenEmbedding(Embedding):
     """Row copy (src/kern/naive/naive.cpp:43-54); rows become float32 and are multiplied by
     `scale` (1: the reference's plain copy).  `streams` > 0: a model with several residual
-    streams; the rows come out as [rows, streams, hidden], every stream the embedded row."""
+    streams; the rows come out as [rows, streams, hidden], every stream the embedded row.
+    `norm_eps` > 0: the scaled row passes an RMS norm (tensor `norm`)."""
 
     graph_safe_prompts = True
 
     def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, streams: int = 0,
-                 tensors=None):
+                 norm_eps: float = 0.0, tensors=None):
         super().__init__(tensors)
         self.V, self.E = int(vocab_size), int(hidden_size)
-        self.scale, self.streams = float(scale), int(streams)
+        self.scale, self.streams, self.norm_eps = float(scale), int(streams), float(norm_eps)
+        if self.streams and self.norm_eps:
+            raise ValueError("token_embedding: a norm goes with one residual stream")
         self.weight: Optional[torch.Tensor] = None
+        self.norm: Optional[torch.Tensor] = None
 
     def shapes(self) -> Dict[str, TensorWant]:
-        return {"weight": TensorWant((self.V, self.E))}
+        out = {"weight": TensorWant((self.V, self.E))}
+        if self.norm_eps:
+            out["norm"] = TensorWant((self.E,), init="ones_normal", keep_stored=True)
+        return out
 
     def load(self, tensors) -> None:
         self.weight = self._take(tensors, "weight").contiguous()
+        if self.norm_eps:
+            self.norm = self._take(tensors, "norm").contiguous()
 
     def forward(self, ctx: StepContext):
+        if self.norm_eps:
+            return ops.embed_norm(ctx.tokens, self.weight, self.norm, self.norm_eps, self.scale)
         if self.streams:
             return ops.embed(ctx.tokens, self.weight, self.scale, self.streams)
         return ops.embed(ctx.tokens, self.weight, self.scale)

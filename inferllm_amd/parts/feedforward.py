@@ -162,7 +162,8 @@ class RoutedExperts(FeedForward):
     weight multiplies what the expert reads, out = sum over chosen e of expert_e(s_e h).
     `activation` "relu_squared": experts (and the shared one) without a gate, expert(h) =
     W_down max(W_up h, 0)^2, and no ".gate" tensors.  `router_scale`: the weights are that times the
-    chosen scores.
+    chosen scores.  `groups` = (count, keep): the outputs are `count` equal groups of neighbours, and only
+    those of the `keep` groups with the largest sums of their two largest choice scores can be chosen.
     Tensor parameters: "router", "correction", "e<i>.gate" / ".up" / ".down", "shared.gate" /
     ".up" / ".down", "shared.sg".  The result is float32.
     """
@@ -172,7 +173,8 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int,
                  num_identity: int = 0, correction: bool = True, shared_size: int = 0,
                  shared_gate: bool = True, score: str = "softmax", activation: str = "silu",
-                 limit: float = 0.0, weight_on: str = "output", router_scale: float = 1.0, tensors=None):
+                 limit: float = 0.0, weight_on: str = "output", router_scale: float = 1.0, groups=None,
+                 tensors=None):
         super().__init__(tensors)
         if score not in ops.MOE_SCORES or activation not in ops.MOE_ACTIVATIONS:
             raise ValueError(f"routed experts: score {score!r} or activation {activation!r} is unknown; "
@@ -192,6 +194,11 @@ class RoutedExperts(FeedForward):
         n_all = self.n_real + self.n_id
         if self.n_real < 0 or self.n_id < 0 or n_all <= 0 or not 0 < self.top <= n_all:
             raise ValueError(f"routed experts: {self.top} of {self.n_real} + {self.n_id} cannot be chosen")
+        self.groups = (int(groups[0]), int(groups[1])) if groups else None
+        if self.groups:
+            count, keep = self.groups
+            if count <= 0 or n_all % count or not 0 < keep <= count or self.top > keep * (n_all // count):
+                raise ValueError(f"routed experts: {self.top} of {n_all} cannot be chosen from {keep} of {count} groups")
         if n_all > 512:
             raise ValueError("routed experts: more than 512 router outputs are beyond the kernels")
         if self.n_real and self.F <= 0:
@@ -237,7 +244,7 @@ class RoutedExperts(FeedForward):
 
     def forward(self, h, ctx: StepContext):
         idx, weight, grouped = ops.moe_plan(h, self.w_router, self.correction, self.top,
-                                            self.w_gate_up, self.score, self.router_scale, self.gated)
+                                            self.w_gate_up, self.score, self.router_scale, self.gated, self.groups)
         on_input = self.weight_on == "input"
         y = (ops.moe_experts(h, idx, self.w_gate_up, self.w_down, grouped, self.activation, self.limit,
                              weight if on_input else None) if self.n_real else None)

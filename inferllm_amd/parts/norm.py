@@ -17,7 +17,8 @@ class RMSNorm(Norm):
     src/kern/naive/naive.cpp:186-207 and src/core/op.cpp:37-47; eps is a parameter
     (the reference fixes 1e-6 / 1e-5 at src/graph/llama_like.cpp:78 and src/core/graph.h:163).
     `weight_offset` c: the stored tensor lies around zero and the gain is c + stored (formed once,
-    in float32, as the tensor is taken).
+    in float32, as the tensor is taken).  `scale`: the gain is that times it (the last norm of a model whose
+    logits are multiplied by a constant).
     """
 
     graph_safe_prompts = True
@@ -27,9 +28,9 @@ class RMSNorm(Norm):
     # added as x + (first + second) in the norm's own kernel
     adds_pairs = True
 
-    def __init__(self, size: int, eps: float, weight_offset: float = 0.0, tensors=None):
+    def __init__(self, size: int, eps: float, weight_offset: float = 0.0, scale: float = 1.0, tensors=None):
         super().__init__(tensors)
-        self.size, self.eps, self.weight_offset = int(size), float(eps), float(weight_offset)
+        self.size, self.eps, self.weight_offset, self.scale = int(size), float(eps), float(weight_offset), float(scale)
         self.weight: Optional[torch.Tensor] = None
 
     def shapes(self) -> Dict[str, TensorWant]:
@@ -38,8 +39,8 @@ class RMSNorm(Norm):
 
     def load(self, tensors) -> None:
         self.weight = self._take(tensors, "weight").contiguous()
-        if self.weight_offset:
-            self.weight = (self.weight.to(torch.float32) + self.weight_offset).contiguous()
+        if self.weight_offset or self.scale != 1.0:
+            self.weight = ((self.weight.to(torch.float32) + self.weight_offset) * self.scale).contiguous()
 
     def rms_params(self):
         return self.weight, self.eps
@@ -52,7 +53,7 @@ class RMSNorm(Norm):
         if isinstance(delta, ops.PostNormed):
             if delta.kind != "rms":
                 return ops.post_add_norm(x, delta, "rms", self.weight, None, self.eps, ctx.act_dtype, row_idx)
-            if self.size <= ops.POST_ADD_MAX_WIDTH:
+            if self.size <= ops.POST_ADD_MAX_WIDTH and (delta.plain or ops.post_mix_fits(self.size)):
                 return ops.post_add_rmsnorm(x, delta, self.weight, self.eps, ctx.act_dtype, row_idx)
             delta = delta.tensor()
         return ops.add_rmsnorm(x, delta, self.weight, self.eps, ctx.act_dtype, row_idx)

@@ -1,8 +1,9 @@
 """Mixers that keep a matrix of state per head and update it by the plain gated rule
 S <- g S + k (w v)^T, o = S^T q: a state-space mixer with a scalar decay a head, and a matrix
 memory with exponential gates; gated linear attention, which is that rule with a decay per key
-channel; lightning attention, with one fixed decay a head; the delta rule with a removal vector of
-its own; and a gated linear recurrent unit, whose state is one number a channel."""
+channel; lightning attention and retention, with one fixed decay a head; the delta rule with a removal
+vector of its own; time mixing with a token shift and a bonus for the current token; and a gated linear
+recurrent unit, whose state is one number a channel."""
 from __future__ import annotations
 
 import math
@@ -299,6 +300,169 @@ class LightningAttention(Mixer):
             o = ops.delta_scan(qn, kn, vv, weight, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
                                ctx.max_rows, correct=False)
         y = ops.group_norm_gate(o, 1, self.norm_w, U, self.g_off, "sigmoid", self.eps, ctx.act_dtype)
+        return ops.linear(y, self.w_o)
+
+
+@register_part("mixer", "retention")
+class Retention(Mixer):
+    """Per head a matrix of state S [key_dim, value_dim] with one fixed decay:
+
+        q = rot(W_q h),  k = rot(W_k h) key_dim^-1/2,  v = W_v h       rot: the layer's rotary encoding, if any
+        S <- decay_h S + k v^T;   o = S^T q
+        out = W_o (o / rms(o) * silu(W_g h))
+
+    rms over each head's outputs (`eps`), without a weight.  Kept per sequence: S (float32).  A step
+    goes on from whatever the slot holds: single tokens in one launch, many rows a sequence in chunks.
+    Rotation and recurrence are float32; the projections take the engine's dtype.
+    """
+
+    graph_safe_prompts = True
+    takes_continuations = True
+
+    def __init__(self, hidden_size: int, num_heads: int, key_dim: int, value_dim: int, decay: Sequence[float],
+                 eps: float, tensors=None):
+        super().__init__(tensors)
+        if key_dim > 256:
+            raise ValueError(f"retention: a key size of {key_dim} is beyond the kernels' limit of 256")
+        if len(decay) != int(num_heads) or any(not 0.0 <= float(g) <= 1.0 for g in decay):
+            raise ValueError(f"retention: one decay in [0, 1] for each of {num_heads} heads, got {decay!r}")
+        self.E, self.H, self.dk, self.dv = int(hidden_size), int(num_heads), int(key_dim), int(value_dim)
+        self.eps, self.decay_values, self.decay = float(eps), [float(g) for g in decay], None
+        self.k_scale = 1.0 / math.sqrt(self.dk)
+
+    def shapes(self) -> Dict[str, TensorWant]:
+        E, H, dk, dv = self.E, self.H, self.dk, self.dv
+        return {"q": TensorWant((H * dk, E)), "k": TensorWant((H * dk, E)), "v": TensorWant((H * dv, E)),
+                "g": TensorWant((H * dv, E)), "o": TensorWant((E, H * dv))}
+
+    def state_spec(self):
+        return {"S": StateSpec((self.H, self.dk, self.dv), torch.float32)}
+
+    def load(self, tensors) -> None:
+        take = lambda n: self._take(tensors, n)
+        H, dk, dv = self.H, self.dk, self.dv
+        # one product for everything that reads h: [q | k | v | g]
+        self.w_in = ops.decode_weight(_fuse([take(n) for n in ("q", "k", "v", "g")]), "plain", self.decode_copies)
+        self.k_off, self.v_off = H * dk, 2 * H * dk
+        self.g_off = self.v_off + H * dv
+        self.decay = torch.tensor(self.decay_values, dtype=torch.float32, device=take("q").device)
+        self.w_o = ops.decode_weight(take("o").contiguous(), "plain", self.decode_copies)
+
+    def tunables(self):
+        return (("plain", self.w_o, {}),)
+
+    def forward(self, h, ctx: StepContext, line, writes_cache, position):
+        H, dk, dv = self.H, self.dk, self.dv
+        table, rot = (None, 0)
+        if position is not None:
+            if position.pairing != "half":
+                raise ValueError("retention: the rotation pairs i with i + rotary_dim / 2")
+            table, rot = position.table(ctx.device), position.rotary_dim
+        U = ops.linear(h, self.w_in)
+        S = ctx.cache.state_line(line)["S"]
+        cols = (0, self.k_off, self.v_off)
+        if not ctx.prefill:
+            o = ops.retention_step(U, *cols, self.decay, table, rot, self.k_scale, ctx.row_pos, S, ctx.row_slot, H, dk, dv)
+        elif ctx.max_rows >= ops.LIGHTNING_CHUNKS_FROM and ops.retention_chunks_fits(U, self.v_off, dk, dv):
+            qn, kn = ops.retention_prepare(U, *cols, self.decay, table, rot, self.k_scale, ctx.row_pos, H, dk, dv, scan=False)
+            o = ops.retention_chunks(qn, kn, U, self.v_off, self.decay, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
+                                     ctx.max_rows, H, dk, dv)
+        else:
+            qn, kn, vv, weight, dec = ops.retention_prepare(U, *cols, self.decay, table, rot, self.k_scale, ctx.row_pos,
+                                                            H, dk, dv)
+            o = ops.delta_scan(qn, kn, vv, weight, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs, ctx.max_rows,
+                               correct=False)
+        y = ops.group_norm_gate(o, H, None, U, self.g_off, "silu", self.eps, ctx.act_dtype)
+        return ops.linear(y, self.w_o)
+
+
+@register_part("mixer", "time_mix")
+class TimeMix(Mixer):
+    """Recurrent time mixing with a token shift (an RWKV-style layer).  Each of five projections reads a mix of
+    its own of the token's row and the one before it (zeros before the sequence):
+
+        in_s = h + (h_before - h) mu_s                       s of r, k, v, g, w
+        r = W_r in_r,  k = W_k in_k,  v = W_v in_v,  w = exp(-exp(W_w2 tanh(W_w1 in_w) + w0))   one a head and channel
+        o = (S + diag(u) k v^T)^T r;   S <- diag(w) S + k v^T           the bonus u counts for the current token alone
+        out = W_o (o / rms(o) * norm * silu(W_g in_g))
+
+    rms over each head's outputs (`eps`), `norm` of all heads' width.  Kept per sequence: S [dim, dim] a head
+    (float32) and the last row h.  A step goes on from whatever the slot holds: single tokens in one launch, many
+    rows a sequence in chunks.  Decays, bonus and the state are float32; the mixes and projections take the
+    engine's dtype.  A block that mixes single tokens in its own pass (`takes_token_mixes`, `shift`) hands
+    `forward` the mixes as `ops.TokenMixes`.
+    """
+
+    graph_safe_prompts = True
+    takes_continuations = True
+    takes_token_mixes = True
+    MIXES = ("r", "k", "v", "g", "w")
+
+    def __init__(self, hidden_size: int, num_heads: int, dim: int, decay_rank: int, eps: float, tensors=None):
+        super().__init__(tensors)
+        if dim > 256:
+            raise ValueError(f"time mixing: a head size of {dim} is beyond the kernels' limit of 256")
+        if int(decay_rank) <= 0:
+            raise ValueError("time mixing: the decays' rank must be positive")
+        self.E, self.H, self.d, self.rank, self.eps = int(hidden_size), int(num_heads), int(dim), int(decay_rank), float(eps)
+
+    def shapes(self) -> Dict[str, TensorWant]:
+        E, n, R = self.E, self.H * self.d, self.rank
+        keep = dict(keep_stored=True)
+        return {**{f"mu_{s}": TensorWant((E,), **keep) for s in self.MIXES},
+                "r": TensorWant((n, E)), "k": TensorWant((n, E)), "v": TensorWant((n, E)), "g": TensorWant((n, E)),
+                "w1": TensorWant((R, E)), "w2": TensorWant((n, R)), "w0": TensorWant((n,), **keep),
+                "u": TensorWant((self.H, self.d), **keep), "norm": TensorWant((n,), init="ones_normal", **keep),
+                "o": TensorWant((E, n))}
+
+    def state_spec(self):
+        return {"S": StateSpec((self.H, self.d, self.d), torch.float32), "tail": StateSpec((1, self.E), None)}
+
+    def load(self, tensors) -> None:
+        take = lambda n: self._take(tensors, n)
+        f32 = lambda n: take(n).to(torch.float32).contiguous()
+        n = self.H * self.d
+        self.mu = torch.stack([f32(f"mu_{s}") for s in self.MIXES]).contiguous()
+        # one stacked matrix; each part reads rows of its own: [r | k | v | g | w1]
+        self.w_in = ops.decode_weight(_fuse([take(t) for t in ("r", "k", "v", "g", "w1")]), "plain", self.decode_copies)
+        self.ends = (n, 2 * n, 3 * n, 4 * n, 4 * n + self.rank)
+        # (from the tanh on the decays' map is float32 arithmetic: single tokens read the stored rows, steps of
+        # several tokens a float32 copy)
+        self.w2_rows = take("w2").to(ops.plain_weight(self.w_in).dtype).contiguous()
+        self.w_w2 = self.w2_rows.to(torch.float32).contiguous()
+        self.w0, self.u, self.norm_w = f32("w0"), f32("u").reshape(-1).contiguous(), take("norm").contiguous()
+        self.w_o = ops.decode_weight(take("o").contiguous(), "plain", self.decode_copies)
+
+    def tunables(self):
+        return (("plain", self.w_o, {}),)
+
+    def shift(self, ctx: StepContext, line):
+        """(mu, tail, row_slot): what a pass that mixes single tokens needs (`ops.post_add_rmsnorm`)."""
+        return self.mu, ctx.cache.state_line(line)["tail"], ctx.row_slot
+
+    def forward(self, h, ctx: StepContext, line, writes_cache, position):
+        H, d = self.H, self.d
+        state = ctx.cache.state_line(line)
+        S = state["S"]
+        if isinstance(h, ops.TokenMixes):
+            planes = h.planes
+        else:
+            planes = ops.token_mix(h, self.mu, state["tail"], ctx.row_slot, update_tail=not ctx.prefill)
+            if ctx.prefill:
+                ops.short_conv_tail(h, 0, state["tail"], ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs, 2)
+        r, k, v, g, low = ops.linear_parts(planes, self.w_in, self.ends)
+        if not ctx.prefill and self.rank <= ops.TIME_MIX_STEP_MAX_RANK and self.w2_rows.dtype == r.dtype:
+            o = ops.time_mix_step(r, k, v, low, self.w2_rows, self.w0, self.u, S, ctx.row_slot, H, d)
+        else:
+            Z = ops.linear(ops.tanh_rows(low), self.w_w2)
+            if ctx.prefill and ctx.max_rows >= ops.TIME_MIX_CHUNKS_FROM and ops.time_mix_chunks_fits(r, k, v, d):
+                o = ops.time_mix_chunks(r, k, v, Z, self.w0, self.u, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
+                                        ctx.max_rows, H, d)
+            else:
+                rn, kn, vv, beta, dec = ops.time_mix_prepare(r, k, v, Z, self.w0, self.u, H, d)
+                o = ops.delta_scan(rn, kn, vv, beta, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
+                                   ctx.max_rows if ctx.prefill else 1, correct="bonus")
+        y = ops.group_norm_gate(o, H, self.norm_w, g, 0, "silu", self.eps, ctx.act_dtype)
         return ops.linear(y, self.w_o)
 
 
