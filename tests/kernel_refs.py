@@ -376,15 +376,27 @@ def few_outputs_f32(x, w):
     return (x.to(F64) @ w.to(F64).t()).to(torch.float32)
 
 
-def moe_route(z, correction, top, score="softmax", scale=1.0):
+def _best_groups(choice, groups):
+    """The choice scores with those outside the best groups (by the sum of their two largest) at -inf."""
+    count, keep = groups
+    by_group = choice.view(choice.shape[0], count, -1)
+    score = torch.topk(by_group, min(2, by_group.shape[2]), dim=2).values.sum(2)
+    best = torch.topk(score, keep, dim=1).indices
+    allowed = torch.zeros_like(score, dtype=torch.bool).scatter_(1, best, True)
+    return by_group.masked_fill(~allowed[:, :, None], float("-inf")).reshape(choice.shape)
+
+
+def moe_route(z, correction, top, score="softmax", scale=1.0, groups=None):
     s = torch.softmax(z.to(F64), dim=-1) if score == "softmax" else torch.sigmoid(z.to(F64))
     pick = s + correction.to(F64) if correction is not None else s
+    if groups:
+        pick = _best_groups(pick, groups)
     idx = torch.topk(pick, top, dim=-1).indices
     return idx.to(torch.int32), (scale * torch.gather(s, 1, idx)).to(torch.float32)
 
 
-def moe_plan(h, w_router, correction, top, w_gate_up, score="softmax", scale=1.0, gated=True):
-    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score, scale)
+def moe_plan(h, w_router, correction, top, w_gate_up, score="softmax", scale=1.0, gated=True, groups=None):
+    idx, wt = moe_route(few_outputs_f32(h, w_router), correction, top, score, scale, groups)
     return idx, wt, None
 
 
@@ -455,9 +467,9 @@ def kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table,
         vcache[page, :, at, :] = rows[r, v_off:v_off + nkv * dv].view(nkv, dv)
 
 
-def _attend_capped(q, k, v, scale, cap, slopes=None, lse=None):
+def _attend_capped(q, k, v, scale, cap, slopes=None, lse=None, sink=None):
     """q [nh, dk], k [L, nkv, dk], v [L, nkv, dv]: every key visible, the last one the query's own.
-    `lse` [nh] takes log(sum(exp(score))) of every head."""
+    `lse` [nh] takes log(sum(exp(score))) of every head; `sink` [nh]: one more score, without a value."""
     nh, per, L = q.shape[0], q.shape[0] // k.shape[1], k.shape[0]
     out = torch.zeros(nh, v.shape[2], dtype=F64)
     for h in range(nh):
@@ -466,7 +478,9 @@ def _attend_capped(q, k, v, scale, cap, slopes=None, lse=None):
             s = cap * torch.tanh(s / cap)
         if slopes is not None:
             s = s - slopes[h].to(F64) * torch.arange(L - 1, -1, -1, dtype=F64)
-        out[h] = torch.softmax(s, dim=0) @ v[:, h // per, :].to(F64)
+        if sink is not None:
+            s = torch.cat([s, sink[h:h + 1].to(F64)])
+        out[h] = torch.softmax(s, dim=0)[:L] @ v[:, h // per, :].to(F64)
         if lse is not None:
             lse[h] = torch.logsumexp(s, dim=0).to(lse.dtype)
     return out
@@ -510,7 +524,7 @@ def _cached(kcache, vcache, page_table, slot, first, total, page_size, ring, kee
 
 def attn_cap_rows(q, cu_seqlens, seq_slot, seq_start, kcache, vcache, page_table, page_size, ring,
                   n_seqs, max_rows, nh, nkv, dk, dv, scale, cap, window, slopes=None, chunk=0, gate=None,
-                  gate_off=0, gate_heads=False, lse=None, keep=0, kept=0, own=None):
+                  gate_off=0, gate_heads=False, lse=None, keep=0, kept=0, own=None, own_values=None, sink=None):
     out = torch.zeros(q.shape[0], nh * dv, dtype=q.dtype)
     for b in range(n_seqs):
         s0, s1 = int(cu_seqlens[b]), int(cu_seqlens[b + 1])
@@ -522,23 +536,23 @@ def attn_cap_rows(q, cu_seqlens, seq_slot, seq_start, kcache, vcache, page_table
             else:
                 seen = [s0 + j for j in list(range(min(keep, first))) + list(range(first, pos + 1))]
                 k = q[seen, own[0]:own[0] + nkv * dk].view(-1, nkv, dk)
-                v = q[seen, own[1]:own[1] + nkv * dv].view(-1, nkv, dv)
+                v = (q[seen, own[1]:own[1] + nkv * dv] if own_values is None else own_values[seen]).view(-1, nkv, dv)
             row = _attend_capped(q[s0 + a, :nh * dk].view(nh, dk), k, v, scale, cap, slopes,
-                                 lse[s0 + a] if lse is not None else None).reshape(-1)
+                                 lse[s0 + a] if lse is not None else None, sink).reshape(-1)
             out[s0 + a] = _gated(row, gate, s0 + a, gate_off, nh if gate_heads else 0).to(q.dtype)
     return out
 
 
 def attn_cap_decode(q, kcache, vcache, page_table, page_size, ring, seq_slot, seq_len, nh, nkv, dk, dv,
                     scale, cap, window, nsplit, slopes=None, chunk=0, gate=None, gate_off=0, gate_heads=False,
-                    lse=None, keep=0, kept=0):
+                    lse=None, keep=0, kept=0, sink=None):
     out = torch.zeros(q.shape[0], nh * dv, dtype=q.dtype)
     for b in range(q.shape[0]):
         n = int(seq_len[b])
         first = _first_seen(n - 1, window, chunk)
         k, v = _cached(kcache, vcache, page_table, int(seq_slot[b]), first, n, page_size, ring, keep, kept)
         row = _attend_capped(q[b, :nh * dk].view(nh, dk), k, v, scale, cap, slopes,
-                             lse[b] if lse is not None else None).reshape(-1)
+                             lse[b] if lse is not None else None, sink).reshape(-1)
         out[b] = _gated(row, gate, b, gate_off, nh if gate_heads else 0).to(q.dtype)
     return out
 
@@ -596,6 +610,11 @@ def delta_scan(qn, kn, vv, beta, dec, state, cu_seqlens, seq_slot, n_seqs, max_r
             for h in range(H):
                 g = h // (H // G)
                 S = state[slot, h].to(F64) * dec[r, h].to(F64).expand(dk)[:, None]
+                if correct == "bonus":                  # o from the state before the token
+                    o[r, h] = (state[slot, h].to(F64).t() @ qn[r, g].to(F64)
+                               + beta[r, h].to(F64) * vv[r, h].to(F64)).to(torch.float32)
+                    state[slot, h] = (S + torch.outer(kn[r, g].to(F64), vv[r, h].to(F64))).to(torch.float32)
+                    continue
                 if removal is not None:
                     unit = beta[r, h].to(F64) * kn[r, g].to(F64)
                     S = (S - torch.outer(removal[r, h].to(F64), unit @ state[slot, h].to(F64))
@@ -771,9 +790,23 @@ def rms_rows_gain(a, weight, eps, gain):
     return (gain * (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * weight.to(F64))).to(torch.float32)
 
 
-def post_add_rmsnorm(x, post, weight, eps, out_dtype, row_idx=None, conv=None):
-    delta = rms_rows_gain(post.a, post.weight, post.eps, post.gain) if post is not None else None
+def _left_to_add(post):
+    """What a `PostNormed` stands for, float64."""
+    unit = lambda v, w, e: v.to(F64) / torch.sqrt((v.to(F64) ** 2).mean(-1, keepdim=True) + e) * w.to(F64)
+    y = post.a.to(F64)
+    if post.pair is not None:
+        q = post.pair
+        y = q.scale * (unit(q.a, q.wa, q.eps) + unit(q.b, q.wb, q.eps))
+    y = post.gain * (unit(y, post.weight, post.eps) if post.kind == "rms"
+                     else _norm_rows(y, post.kind, post.weight, post.bias, post.eps))
+    return y if post.plus is None else y + post.plus.to(F64)
+
+
+def post_add_rmsnorm(x, post, weight, eps, out_dtype, row_idx=None, conv=None, shift=None):
+    delta = _left_to_add(post).to(torch.float32) if post is not None else None
     h = add_rmsnorm(x, delta, weight, eps, out_dtype, row_idx)
+    if shift is not None:
+        return token_mix(h, *shift, update_tail=True)
     if conv is None:
         return h
     cw, tail, slots = conv
@@ -790,7 +823,10 @@ def clamped_swish_mul(gate_up, limit):
 # ---------------------------------------------------------------- attention over a window and pooled blocks
 def qk_rotate_store(rows, k_off, v_off, cos_sin, rot, pairing, unit_norm, eps, row_pos, row_slot, kcache,
                     vcache, page_table, page_size, ring, nh, nkv, dk, dv, q_scale=None, bias=None, q_weight=None,
-                    k_weight=None, slot_len=None, kept=0):
+                    k_weight=None, slot_len=None, kept=0, values_from_keys=False, values_out=None):
+    values = rows[:, k_off:k_off + nkv * dk].clone() if values_from_keys else None
+    if values_out is not None:
+        values_out.copy_(values)
     half = rot // 2
     for r in range(rows.shape[0]):
         if bias is not None:
@@ -816,6 +852,8 @@ def qk_rotate_store(rows, k_off, v_off, cos_sin, rot, pairing, unit_norm, eps, r
                 x = x * q_scale.to(F64)[:, None]
             rows[r, off:off + heads * dk] = x.reshape(-1).to(rows.dtype)
     if kcache is not None:
+        if values_from_keys:
+            rows, v_off = torch.cat([rows, values], dim=1), rows.shape[1]
         kv_store2(rows, k_off, v_off, row_pos, row_slot, kcache, vcache, page_table, page_size, ring, nkv, dk, dv,
                   kept, slot_len)
 
@@ -922,7 +960,7 @@ def _norm_rows(v, kind, weight, bias, eps):
 def post_add_norm(x, post, kind, weight, bias, eps, out_dtype, row_idx=None):
     v = x.to(F64)
     if post is not None and hasattr(post, "kind"):
-        v = v + post.gain * _norm_rows(post.a.to(F64), post.kind, post.weight, post.bias, post.eps)
+        v = v + _left_to_add(post)
     elif post is not None:
         v = v + post.to(F64)
     if row_idx is None:
@@ -993,11 +1031,103 @@ def removal_step(U, r_off, k_off, v_off, a_off, a_bias, w1_off, w2, w0, rate, st
 
 
 def group_norm_gate(o, groups, weight, Z, z_off, gate, eps, out_dtype):
-    T, width = o.shape[0], weight.numel()
+    T = o.shape[0]
     x = o.to(F64).reshape(T, groups, -1)
-    x = (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)).reshape(T, width) * weight.to(F64)
+    x = (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)).reshape(T, -1)
+    width = x.shape[1]
+    x = x if weight is None else x * weight.to(F64)
     z = Z[:, z_off:z_off + width].to(F64)
     return (x * (torch.sigmoid(z) if gate == "sigmoid" else _silu(z))).to(out_dtype)
+
+
+# ---------------------------------------------------------------- retention, time mixing, an embedding under a norm
+def embed_norm(tokens, table, weight, eps, scale=1.0):
+    v = table[tokens.long()].to(F64) * scale
+    return (v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * weight.to(F64)).to(torch.float32)
+
+
+def copy_rows(x):
+    return x.clone()
+
+
+def normed_pair_tensor(self):
+    return sum_rows(rms_rows_gain(self.a, self.wa, self.eps, self.scale), rms_rows_gain(self.b, self.wb, self.eps, self.scale))
+
+
+def _turned(x, cos_sin, rot, row_pos):
+    """x float64 [T, H, d]: the first `rot` dims turned by the rows' positions, i with i + rot / 2."""
+    if not rot:
+        return x
+    half = rot // 2
+    c, s = (cos_sin[row_pos.long()][:, None, :, j].to(F64) for j in (0, 1))
+    out = x.clone()
+    u, v = x[..., :half], x[..., half:rot]
+    out[..., :half], out[..., half:rot] = u * c - v * s, v * c + u * s
+    return out
+
+
+def retention_prepare(U, q_off, k_off, v_off, decay, cos_sin, rot, k_scale, row_pos, H, dk, dv, scan=True):
+    T = U.shape[0]
+    cols = lambda off, d: U[:, off:off + H * d].to(F64).reshape(T, H, d)
+    q = _turned(cols(q_off, dk), cos_sin, rot, row_pos)
+    k = _turned(cols(k_off, dk), cos_sin, rot, row_pos) * k_scale
+    out = (q, k) if not scan else (q, k, cols(v_off, dv), torch.ones(T, H), decay.expand(T, H).reshape(T, H, 1))
+    return tuple(t.to(torch.float32).contiguous() for t in out)
+
+
+def retention_chunks(qn, kn, U, v_off, decay, state, cu_seqlens, seq_slot, n_seqs, max_rows, H, dk, dv):
+    T = U.shape[0]
+    v = U[:, v_off:v_off + H * dv].reshape(T, H, dv).to(torch.float32)
+    dec = decay.expand(T, H).reshape(T, H, 1)
+    return delta_scan(qn, kn, v, torch.ones(T, H), dec, state, cu_seqlens, seq_slot, n_seqs, max_rows, correct=False)
+
+
+def retention_step(U, q_off, k_off, v_off, decay, cos_sin, rot, k_scale, row_pos, state, row_slot, H, dk, dv):
+    B = U.shape[0]
+    ins = retention_prepare(U, q_off, k_off, v_off, decay, cos_sin, rot, k_scale, row_pos, H, dk, dv)
+    return delta_scan(*ins, state, torch.arange(B + 1), row_slot, B, 1, correct=False)
+
+
+def token_mix(h, mu, tail, row_slot, update_tail):
+    out = torch.zeros((mu.shape[0],) + tuple(h.shape), dtype=h.dtype)
+    for r in range(h.shape[0]):
+        slot = int(row_slot[r])
+        before = h[r - 1] if r > 0 and int(row_slot[r - 1]) == slot else tail[slot, 0]
+        x, step = h[r].to(F64), before.to(F64) - h[r].to(F64)
+        for s in range(mu.shape[0]):
+            out[s, r] = (x + step * mu[s].to(F64)).to(h.dtype)
+    if update_tail:
+        for r in range(h.shape[0]):
+            tail[int(row_slot[r]), 0] = h[r]
+    return out
+
+
+def linear_parts(planes, w, ends):
+    starts = [0] + list(ends[:-1])
+    return [linear(planes[p], w[a:b]) for p, (a, b) in enumerate(zip(starts, ends))]
+
+
+def tanh_rows(x):
+    return torch.tanh(x.to(F64)).to(torch.float32)
+
+
+def time_mix_prepare(r, k, v, Z, w0, bonus, H, d):
+    T = r.shape[0]
+    rr, kk, vv = (t.to(F64).reshape(T, H, d) for t in (r, k, v))
+    dec = torch.exp(-torch.exp(Z.to(F64) + w0.to(F64))).view(T, H, d)
+    beta = (rr * kk * bonus.to(F64).view(H, d)).sum(-1)
+    return tuple(t.to(torch.float32).contiguous() for t in (rr, kk, vv, beta, dec))
+
+
+def time_mix_chunks(r, k, v, Z, w0, bonus, state, cu_seqlens, seq_slot, n_seqs, max_rows, H, d):
+    ins = time_mix_prepare(r, k, v, Z, w0, bonus, H, d)
+    return delta_scan(*ins, state, cu_seqlens, seq_slot, n_seqs, max_rows, correct="bonus")
+
+
+def time_mix_step(r, k, v, low, w2, w0, bonus, state, row_slot, H, d):
+    B = r.shape[0]
+    Z = torch.tanh(low.to(F64)) @ w2.to(F64).t()
+    return time_mix_chunks(r, k, v, Z, w0, bonus, state, torch.arange(B + 1), row_slot, B, 1, H, d)
 
 
 def patch(monkeypatch):
@@ -1016,6 +1146,9 @@ def patch(monkeypatch):
                  "short_conv", "short_conv_tail", "rms_rows_gain", "post_add_rmsnorm", "gate_up_act", "clamped_swish_mul", "qk_rotate_store",
                  "pool_store", "attn_pooled_rows", "attn_pooled_decode", "gla_prepare", "lru_gates", "lru_scan",
                  "post_add_norm", "xielu", "lightning_prepare", "lightning_chunks", "lightning_step", "tanh_columns",
-                 "removal_prepare", "removal_chunks", "removal_step", "group_norm_gate"):
+                 "removal_prepare", "removal_chunks", "removal_step", "group_norm_gate", "embed_norm", "copy_rows",
+                 "retention_prepare", "retention_chunks", "retention_step", "token_mix", "linear_parts", "tanh_rows",
+                 "time_mix_prepare", "time_mix_chunks", "time_mix_step"):
         monkeypatch.setattr(ops, name, globals()[name])
     monkeypatch.setattr(ops.ScaledSum, "tensor", scaled_sum_tensor)
+    monkeypatch.setattr(ops.NormedPair, "tensor", normed_pair_tensor)
