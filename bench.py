@@ -22,7 +22,7 @@ of MI355X (HBM 8 TB/s, dense bf16 MFMA 2.5 PFLOP/s, float32 157.3 TFLOP/s).
 The run fails (non-zero) if any timed run produced a non-finite logit or the same
 greedy token everywhere.
 
-`--design rabapel`, `kukupel`, `sabipel`, `dotorax` and `febivik` are other workloads with a line of their own (the
+`--design rabapel`, `kukupel`, `sabipel`, `dotorax`, `febivik` and `vupolix` are other workloads with a line of their own (the
 default's stays as it is):
 Rabapel (latent attention, layers that alternate a dense and a routed feed-forward) at two
 sizes beside LLaMA at the same width, heads and layer count: prefill of 2,048 tokens and decoding
@@ -32,7 +32,9 @@ layers with dense feed-forwards) beside Kukupel, and Dotorax (rotated attention 
 gated linear attention, a window with pooled blocks beside a recurrent unit, gated feed-forwards,
 sublayers between two norms behind a short convolution) beside Sabipel, and Febivik (lightning
 attention, a delta rule with a removal vector, a window that keeps the first tokens, squared-ReLU
-experts, norms behind the sublayers) beside Kukupel.
+experts, norms behind the sublayers) beside Kukupel, and Vupolix (time mixing with a token shift,
+windowed attention with a sink over its own keys beside retention, gated experts chosen within groups,
+sublayers between two norms) beside Febivik.
 """
 import argparse
 import json
@@ -716,35 +718,32 @@ def febivik_counts(cfg, esz):
     return step_bytes, flops
 
 
-def febivik_main(args) -> int:
-    """Febivik at two sizes beside Kukupel, the library's closest design (a delta rule, attention and
-    routed feed-forwards), at the same width, heads, experts and number of layers (four): tokens/s of
-    these four-layer models, with the fraction of the matrix peak for prompts and of the HBM peak for
-    decode steps."""
+SIZES = {"2048": dict(width=2048, heads=16, kv_heads=4, experts=64, expert_ff=1408, top=6),
+         "4096": dict(width=4096, heads=32, kv_heads=8, experts=32, expert_ff=2048, top=4)}
+
+
+def two_designs(args, metric, designs) -> int:
+    """A line of four-layer models at two sizes: tokens/s with the fraction of the matrix peak for prompts and of
+    the HBM peak for decode steps.  designs: (name, configuration of a size, its counts, what is done to its engine)."""
     import torch
     from inferllm_amd import Engine
     layers = args.layers or 4
     esz = 2 if args.dtype == "bfloat16" else 4
-    sizes = {"2048": dict(width=2048, heads=16, kv_heads=4, experts=64, expert_ff=1408, top=6),
-             "4096": dict(width=4096, heads=32, kv_heads=8, experts=32, expert_ff=2048, top=4)}
     few = min(args.steps, 128)
-    out = {"metric": "Febivik beside Kukupel at equal width, heads, experts and layers: prefill tok/s at 2,048 tokens, decode tok/s at batch 1/8/64",
-           "unit": "tokens/s", "n_gpus": 1, "steps": few, "warmup": 4, "dtype": "bf16" if esz == 2 else "fp32",
+    out = {"metric": metric, "unit": "tokens/s", "n_gpus": 1, "steps": few, "warmup": 4,
+           "dtype": "bf16" if esz == 2 else "fp32",
            "data": "synthetic: seeded random weights, uniform random token ids", "layers": layers, "sizes": {}}
-    for name, sz in sizes.items():
+    for name, sz in SIZES.items():
         if args.size and args.size != name:
             continue
         row = {}
-        fcfg, kcfg = febivik_config(layers=layers, **sz), kukupel_config(layers=layers, **sz)
-        for design, cfg, counts in (("febivik", fcfg, febivik_counts), ("kukupel", kcfg, kukupel_counts)):
+        for design, config, counts, prepare in designs:
             if args.only and args.only != design:
                 continue
+            cfg = config(layers=layers, **sz)
             eng = Engine.from_random(cfg, seed=0, dtype=args.dtype, device="cuda:0", max_batch=64,
                                      max_seq_len=4096, max_tokens=64 * 1024)
-            if design == "febivik":
-                # embedded rows of unit size, as every sublayer's norm leaves what it adds: next to that,
-                # rows of N(0, 0.02) would not tell one token from another
-                eng.model.embedding.weight.mul_(50.0)
+            prepare(eng)
             b = Bench.around(eng, cfg["vocab"], layers, args.dtype, *counts(cfg, esz))
             torch.cuda.synchronize()
             r = {"prefill_2048": b.prefill_run(2048, reps=4)}
@@ -758,6 +757,91 @@ def febivik_main(args) -> int:
         out["sizes"][name] = row
     print(json.dumps(out), flush=True)
     return 0
+
+
+def larger_embedding(eng) -> None:
+    """Embedded rows of unit size, as every norm behind a sublayer leaves what it adds: next to that, rows of
+    N(0, 0.02) would not tell one token from another."""
+    eng.model.embedding.weight.mul_(50.0)
+
+
+def febivik_main(args) -> int:
+    """Febivik at two sizes beside Kukupel, its closest design (a delta rule, attention and routed
+    feed-forwards), at the same width, heads, experts and number of layers."""
+    return two_designs(args, "Febivik beside Kukupel at equal width, heads, experts and layers: prefill tok/s at 2,048 tokens, decode tok/s at batch 1/8/64",
+                       (("febivik", febivik_config, febivik_counts, larger_embedding),
+                        ("kukupel", kukupel_config, kukupel_counts, lambda eng: None)))
+
+
+# ---------------------------------------------------------------- Vupolix beside Febivik
+def vupolix_config(width, heads, kv_heads, layers, experts, expert_ff, top, window=1024, vocab=32000):
+    """Layers in the order wkv, parallel, wkv, parallel: time-mixing heads of 128 (decays' rank 64); attention heads
+    of 128 dims, half of each rotated, over a window, beside retention heads of 128 x 128; routed feed-forwards (8
+    groups of experts of which 4 are kept) beside a shared expert of twice an expert's size.  No layer is repeated (a
+    repeated layer costs what another one of its kind does)."""
+    wkv = {"heads": heads, "dim": 128, "rank": 64}
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": window},
+            "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 1024, "fast": 32.0, "slow": 1.0}}}
+    right = {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** -(5 + 5 * h / heads) for h in range(heads)],
+             "rot": {"base": 10000.0, "dims": 128}}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff},
+           "router": {"experts": experts, "top": top, "groups": {"count": 8, "keep": 4}}, "shared": {"ff": 2 * expert_ff}}
+    kinds = (("wkv", wkv, moe), ("parallel", {"left": left, "right": right}, moe))
+    return {"architecture": "Vupolix", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": 8192,
+            "residual_mult": 0.7, "logit_scale": 2.0,
+            "layers": [dict(zip(("type", "mixer", "mlp"), json.loads(json.dumps(kinds[i % 2])))) for i in range(layers)]}
+
+
+def vupolix_counts(cfg, esz):
+    """(step_bytes(batch, mean_ctx), flops(tokens, lens)) of a Vupolix configuration, counted as Febivik's: values
+    that are keys are stored, so read, for themselves; gated experts have three matrices."""
+    E, V = cfg["width"], cfg["vocab"]
+
+    def mixer_parts(layer):
+        """(weights, float32 state, state products a token, cache columns a token, score columns a pair, keys seen at most)"""
+        m = layer["mixer"]
+        if layer["type"] == "wkv":
+            n = m["heads"] * m["dim"]
+            return 5 * E * n + m["rank"] * (E + n), n * m["dim"], 2 * n * m["dim"], 0, 0, 0
+        q, r = m["left"], m["right"]
+        H, G, d = q["heads"], q["kv_heads"], q["dim"]
+        h, dk, dv = r["heads"], r["dim"], r["vdim"]
+        weights = E * (H * d + G * d + H) + H * d * E + E * h * (2 * dk + 3 * dv)
+        return weights, h * dk * dv, 2 * h * dk * dv, 2 * G * d, 2 * H * d, (q.get("mask") or {}).get("size", 0)
+
+    def ff_parts(mlp, batch):
+        """(weights read by `batch` tokens together, multiply-adds a token, router entries)"""
+        r, ff, sh = mlp["router"], mlp["expert"]["ff"], (mlp.get("shared") or {}).get("ff", 0)
+        used = r["experts"] * (1.0 - (1.0 - r["top"] / r["experts"]) ** batch)
+        return 3 * E * (used * ff + sh), 3 * E * (r["top"] * ff + sh) + E * r["experts"], E * r["experts"]
+
+    seen = lambda n, most: min(n, most) if most else n
+
+    def step_bytes(batch, mean_ctx):
+        total = V * E * esz
+        for layer in cfg["layers"]:
+            w, state, _, kv_row, _, most = mixer_parts(layer)
+            f, _, router = ff_parts(layer["mlp"], batch)
+            total += (w + f + batch * seen(mean_ctx, most) * kv_row) * esz + router * 4 + batch * state * 4 * 2
+        return total
+
+    def flops(tokens, lens):
+        total = 2.0 * len(lens) * V * E
+        for layer in cfg["layers"]:
+            w, _, products, _, qk, most = mixer_parts(layer)
+            pairs = sum(sum(seen(p + 1, most) for p in range(n)) for n in lens) if qk else 0
+            total += 2.0 * tokens * (w + ff_parts(layer["mlp"], 1)[1] + products) + 2.0 * qk * pairs
+        return total
+
+    return step_bytes, flops
+
+
+def vupolix_main(args) -> int:
+    """Vupolix at two sizes beside Febivik, the library's closest design (a fixed decay a head, a recurrence with decays
+    from a low-rank map, a window, experts beside a shared one), at the same width, heads, experts and number of layers."""
+    return two_designs(args, "Vupolix beside Febivik at equal width, heads, experts and layers: prefill tok/s at 2,048 tokens, decode tok/s at batch 1/8/64",
+                       (("vupolix", vupolix_config, vupolix_counts, lambda eng: None),
+                        ("febivik", febivik_config, febivik_counts, larger_embedding)))
 
 
 def main() -> int:
@@ -777,15 +861,17 @@ def main() -> int:
     ap.add_argument("--no-70b", action="store_true",
                     help="leave the LLaMA-2-70B shape out of `points` (138 GB of weights: half a minute)")
     ap.add_argument("--with-70b", action="store_true", help="(the default now; kept for old command lines)")
-    ap.add_argument("--design", default="llama", choices=["llama", "rabapel", "kukupel", "sabipel", "dotorax", "febivik"],
+    ap.add_argument("--design", default="llama", choices=["llama", "rabapel", "kukupel", "sabipel", "dotorax", "febivik",
+                                                              "vupolix"],
                     help="rabapel: that design at two sizes beside LLaMA at equal size (a line of its own); "
                          "kukupel: that design at two sizes beside Rabapel at equal size (likewise); "
                          "sabipel: that design at two sizes beside Kukupel at equal size (likewise); "
                          "dotorax: that design at two sizes beside Sabipel at equal size (likewise); "
-                         "febivik: that design at two sizes beside Kukupel at equal size (likewise)")
+                         "febivik: that design at two sizes beside Kukupel at equal size (likewise); "
+                         "vupolix: that design at two sizes beside Febivik at equal size (likewise)")
     ap.add_argument("--size", default="", help="with another --design than llama: only this width (2048 or 4096)")
-    ap.add_argument("--only", default="", help="with --design kukupel, sabipel, dotorax or febivik: only this one of the two designs")
-    ap.add_argument("--batches", default="", help="with --design febivik: decode batches in place of 1,8,64")
+    ap.add_argument("--only", default="", help="with --design kukupel, sabipel, dotorax, febivik or vupolix: only this one of the two designs")
+    ap.add_argument("--batches", default="", help="with --design febivik or vupolix: decode batches in place of 1,8,64")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU only (this library has no multi-GPU path); --gpus must be 1")
@@ -801,6 +887,8 @@ def main() -> int:
         return dotorax_main(args)
     if args.design == "febivik":
         return febivik_main(args)
+    if args.design == "vupolix":
+        return vupolix_main(args)
 
     shape_name, shape_cfg = SHAPES[args.shape]
     ctx_len = shape_cfg["max_position_embeddings"]
