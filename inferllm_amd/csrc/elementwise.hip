@@ -38,7 +38,9 @@ extern "C" int illm_embed(const int32_t* tokens, const void* table, int table_dt
 }
 
 // The token's row under an RMS norm: out = v / sqrt(mean(v^2) + eps) * w with v = table[id] * scale.  `copy`
-// (null: none) takes the rows a second time.  grid (rows); 256 threads.
+// (null: none) takes the rows a second time.  grid (rows); 256 threads, NV groups of 4 columns a thread, the row
+// and the weights asked for together; NV 0: any width.
+template <int NV>
 __global__ void __launch_bounds__(256)
 embed_norm_kernel(const int32_t* __restrict__ tokens, const void* __restrict__ table, int table_dt,
                   const void* __restrict__ w, int w_dt, float* __restrict__ out, float* __restrict__ copy, int E,
@@ -47,6 +49,34 @@ embed_norm_kernel(const int32_t* __restrict__ tokens, const void* __restrict__ t
     const int t = blockIdx.x;
     int id = tokens[t];
     id = id < 0 ? 0 : (id >= V ? V - 1 : id);
+    if (NV > 0) {
+        const size_t n4 = E / 4, src = (size_t)id * n4, dst = (size_t)t * n4;
+        float4 v[NV ? NV : 1], g[NV ? NV : 1];
+        float ss = 0.f;
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const size_t i = threadIdx.x + 256 * k;
+            v[k] = i < n4 ? ld_f4(table, table_dt, src + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+            g[k] = i < n4 ? ld_f4(w, w_dt, i) : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            v[k].x *= scale; v[k].y *= scale; v[k].z *= scale; v[k].w *= scale;
+            ss += (v[k].x * v[k].x + v[k].y * v[k].y) + (v[k].z * v[k].z + v[k].w * v[k].w);
+        }
+        ss = block_sum(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)E + eps);
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const size_t i = threadIdx.x + 256 * k;
+            if (i >= n4) continue;
+            const float4 y = make_float4(v[k].x * inv * g[k].x, v[k].y * inv * g[k].y, v[k].z * inv * g[k].z,
+                                         v[k].w * inv * g[k].w);
+            ((float4*)out)[dst + i] = y;
+            if (copy) ((float4*)copy)[dst + i] = y;
+        }
+        return;
+    }
     const size_t src = (size_t)id * E, dst = (size_t)t * E;
     float ss = 0.f;
     for (int i = threadIdx.x; i < E; i += 256) {
@@ -66,8 +96,15 @@ extern "C" int illm_embed_norm(const int32_t* tokens, const void* table, int tab
                                float* out, float* copy, int T, int E, int V, float scale, float eps, void* stream) {
     if (T < 0 || E <= 0 || V <= 0 || !illm_dtype_ok(table_dt) || !illm_dtype_ok(w_dt)) return ILLM_ERR_ARG;
     if (T == 0) return ILLM_OK;
-    hipLaunchKernelGGL(embed_norm_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, tokens, table, table_dt, w, w_dt,
-                       out, copy, E, V, scale, eps);
+#define GO(NV_)                                                                                            \
+    hipLaunchKernelGGL(embed_norm_kernel<NV_>, dim3(T), dim3(256), 0, (hipStream_t)stream, tokens, table, table_dt, w, \
+                       w_dt, out, copy, E, V, scale, eps)
+    if (E % 4 || E > 8192) GO(0);
+    else if (E <= 1024) GO(1);
+    else if (E <= 2048) GO(2);
+    else if (E <= 4096) GO(4);
+    else GO(8);
+#undef GO
     return illm_launch_status();
 }
 

@@ -72,7 +72,30 @@ retention_prepare_kernel(const void* __restrict__ U, int dt, int u_stride, int q
     const size_t t = blockIdx.x, u0 = t * u_stride;
     const float* cs = rot > 0 ? cos_sin + (size_t)row_pos[t] * rot : nullptr;
     const int half = rot / 2;
-    for (int e = threadIdx.x; e < H * dk; e += 256) {
+    const bool quads = dk % 4 == 0 && half % 4 == 0 && u_stride % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0;
+    // four neighbouring pairs (or dims beyond the rotation) of a head at a time
+    for (int e4 = threadIdx.x; quads && e4 < H * dk / 4; e4 += 256) {
+        const int e = 4 * e4, i = e % dk;
+        if (i >= half && i < rot) continue;              // (the partners, brought along by the first of a pair)
+        const size_t at = t * H * dk + e;
+        float4 q = ld_f4(U, dt, (u0 + q_off + e) / 4), k = ld_f4(U, dt, (u0 + k_off + e) / 4);
+        if (i < rot) {
+            const float4 q2 = ld_f4(U, dt, (u0 + q_off + e + half) / 4), k2 = ld_f4(U, dt, (u0 + k_off + e + half) / 4);
+            const float4 c0 = *(const float4*)(cs + 2 * i), c1 = *(const float4*)(cs + 2 * i + 4);   // c s c s
+            *(float4*)(qn + at + half) = make_float4(q2.x * c0.x + q.x * c0.y, q2.y * c0.z + q.y * c0.w,
+                                                     q2.z * c1.x + q.z * c1.y, q2.w * c1.z + q.w * c1.w);
+            *(float4*)(kn + at + half) =
+                make_float4((k2.x * c0.x + k.x * c0.y) * k_scale, (k2.y * c0.z + k.y * c0.w) * k_scale,
+                            (k2.z * c1.x + k.z * c1.y) * k_scale, (k2.w * c1.z + k.w * c1.w) * k_scale);
+            q = make_float4(q.x * c0.x - q2.x * c0.y, q.y * c0.z - q2.y * c0.w, q.z * c1.x - q2.z * c1.y,
+                            q.w * c1.z - q2.w * c1.w);
+            k = make_float4(k.x * c0.x - k2.x * c0.y, k.y * c0.z - k2.y * c0.w, k.z * c1.x - k2.z * c1.y,
+                            k.w * c1.z - k2.w * c1.w);
+        }
+        *(float4*)(qn + at) = q;
+        *(float4*)(kn + at) = make_float4(k.x * k_scale, k.y * k_scale, k.z * k_scale, k.w * k_scale);
+    }
+    for (int e = threadIdx.x; !quads && e < H * dk; e += 256) {
         const int i = e % dk;
         float q = ld_f(U, dt, u0 + q_off + e), k = ld_f(U, dt, u0 + k_off + e);
         if (i < rot) {

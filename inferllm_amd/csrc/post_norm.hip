@@ -199,6 +199,8 @@ __device__ __forceinline__ float2 block_sum2(float u, float v, float* red) {
 }
 __device__ __forceinline__ float sum_sq(const float4 v) { return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w); }
 
+#define POST_MIX_AHEAD 5   // mixes whose weights are asked for with the row (rows of up to 2,048 columns)
+
 template <int NV, bool PAIR, bool SHIFT>
 __global__ void __launch_bounds__(256)
 post_mix_norm_kernel(PostMix m) {
@@ -213,6 +215,8 @@ post_mix_norm_kernel(PostMix m) {
         const float4 zero4 = make_float4(0.f, 0.f, 0.f, 0.f);
         float4 x[NV ? NV : 1], a[NV ? NV : 1], b[NV && PAIR ? NV : 1], aw[NV && PAIR ? NV : 1], bw[NV && PAIR ? NV : 1];
         float4 pw[NV ? NV : 1], w[NV ? NV : 1], pl[NV ? NV : 1], old[NV && SHIFT ? NV : 1];
+        constexpr bool AHEAD = SHIFT && NV > 0 && NV <= 2;
+        float4 mu[AHEAD ? NV : 1][AHEAD ? POST_MIX_AHEAD : 1];
 #pragma unroll
         for (int k = 0; k < NV; ++k) {
             const int i = threadIdx.x + 256 * k;
@@ -227,6 +231,11 @@ post_mix_norm_kernel(PostMix m) {
             pw[k] = (m.a && in) ? ld_f4(m.pw, m.pw_dt, i) : zero4;
             pl[k] = (m.plus && in) ? ((const float4*)m.plus)[ib + i] : zero4;
             w[k] = in ? ld_f4(m.w, m.w_dt, i) : zero4;
+            if (AHEAD) {
+#pragma unroll
+                for (int s = 0; s < POST_MIX_AHEAD; ++s)
+                    if (s < m.S) mu[k][s] = in ? ((const float4*)m.mu)[(size_t)s * n4 + i] : zero4;
+            }
             if (SHIFT) old[k] = in ? ld_f4(m.tail, m.tail_dt, (size_t)slot * n4 + i) : zero4;
         }
         if (m.a) {
@@ -282,11 +291,16 @@ post_mix_norm_kernel(PostMix m) {
                 h.z = bf16_to_f32(f32_to_bf16(h.z)); h.w = bf16_to_f32(f32_to_bf16(h.w));
             }
             const float4 d = make_float4(old[k].x - h.x, old[k].y - h.y, old[k].z - h.z, old[k].w - h.w);
-            for (int s = 0; s < m.S; ++s) {
-                const float4 u = ((const float4*)m.mu)[(size_t)s * n4 + i];
+            auto mix = [&](int s, const float4 u) __attribute__((always_inline)) {
                 st_f4(m.out, m.out_dt, ((size_t)s * m.rows) * n4 + ob + i,
                       make_float4(fmaf(d.x, u.x, h.x), fmaf(d.y, u.y, h.y), fmaf(d.z, u.z, h.z), fmaf(d.w, u.w, h.w)));
+            };
+            if (AHEAD) {
+#pragma unroll
+                for (int s = 0; s < POST_MIX_AHEAD; ++s)
+                    if (s < m.S) mix(s, mu[k][s]);
             }
+            for (int s = AHEAD ? POST_MIX_AHEAD : 0; s < m.S; ++s) mix(s, ((const float4*)m.mu)[(size_t)s * n4 + i]);
             st_f4(m.tail, m.tail_dt, (size_t)slot * n4 + i, h);
         }
         return;

@@ -275,6 +275,7 @@ class GatedAttention(Mixer):
 
     graph_safe_prompts = True
     takes_continuations = True
+    takes_projected = True            # (its own products at column 0)
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, key_dim: int,
                  value_dim: int, softmax_scale: Optional[float] = None, softcap: float = 0.0,
@@ -390,14 +391,16 @@ class GatedAttention(Mixer):
     def tunables(self):
         return (("plain", self.w_o, {}),)
 
-    def forward(self, h, ctx: StepContext, line, writes_cache, position):
+    def forward(self, h, ctx: StepContext, line, writes_cache, position, projected=None):
         nh, nkv, dk, dv = self.nh, self.nkv, self.dk, self.dv
         kc, vc, group = ctx.cache.kv_line(line)
         window = self.window or 0
         if writes_cache != self.own_kv:
             raise ValueError("gated attention: a layer with key and value projections stores them, and "
                              "one without reads a line that an earlier layer of the step stored")
-        rows = ops.linear(h, self.w_in)
+        if projected is not None and projected[1] != 0:
+            raise ValueError("gated attention: its queries begin the projected rows")
+        rows = projected[0] if projected is not None else ops.linear(h, self.w_in)
         store = writes_cache
         weighted = self.qk_norm == "head_weighted"
         own = (self.k_off, self.v_off) if ctx.prefill and group.ring and not ctx.continues else None

@@ -127,6 +127,11 @@ class Mixer(Part):
     # token; the step function refuses anything else and names the mixer.
     takes_continuations = False
 
+    # True: the mixer reads its input through one stacked matrix `w_in` alone, and `forward` also takes
+    # `projected` = (U, column): the rows' products with that matrix, made by whoever stacked it with others
+    # (`side_by_side`), from that column of U on.
+    takes_projected = False
+
     def kv_spec(self) -> Optional[KVSpec]:
         """Keys/values the mixer keeps per token, or None."""
         return None

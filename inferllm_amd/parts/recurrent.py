@@ -318,6 +318,7 @@ class Retention(Mixer):
 
     graph_safe_prompts = True
     takes_continuations = True
+    takes_projected = True
 
     def __init__(self, hidden_size: int, num_heads: int, key_dim: int, value_dim: int, decay: Sequence[float],
                  eps: float, tensors=None):
@@ -351,28 +352,28 @@ class Retention(Mixer):
     def tunables(self):
         return (("plain", self.w_o, {}),)
 
-    def forward(self, h, ctx: StepContext, line, writes_cache, position):
+    def forward(self, h, ctx: StepContext, line, writes_cache, position, projected=None):
         H, dk, dv = self.H, self.dk, self.dv
         table, rot = (None, 0)
         if position is not None:
             if position.pairing != "half":
                 raise ValueError("retention: the rotation pairs i with i + rotary_dim / 2")
             table, rot = position.table(ctx.device), position.rotary_dim
-        U = ops.linear(h, self.w_in)
+        U, at = projected if projected is not None else (ops.linear(h, self.w_in), 0)
         S = ctx.cache.state_line(line)["S"]
-        cols = (0, self.k_off, self.v_off)
+        cols = (at, at + self.k_off, at + self.v_off)
         if not ctx.prefill:
             o = ops.retention_step(U, *cols, self.decay, table, rot, self.k_scale, ctx.row_pos, S, ctx.row_slot, H, dk, dv)
-        elif ctx.max_rows >= ops.LIGHTNING_CHUNKS_FROM and ops.retention_chunks_fits(U, self.v_off, dk, dv):
+        elif ctx.max_rows >= ops.LIGHTNING_CHUNKS_FROM and ops.retention_chunks_fits(U, cols[2], dk, dv):
             qn, kn = ops.retention_prepare(U, *cols, self.decay, table, rot, self.k_scale, ctx.row_pos, H, dk, dv, scan=False)
-            o = ops.retention_chunks(qn, kn, U, self.v_off, self.decay, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
+            o = ops.retention_chunks(qn, kn, U, cols[2], self.decay, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs,
                                      ctx.max_rows, H, dk, dv)
         else:
             qn, kn, vv, weight, dec = ops.retention_prepare(U, *cols, self.decay, table, rot, self.k_scale, ctx.row_pos,
                                                             H, dk, dv)
             o = ops.delta_scan(qn, kn, vv, weight, dec, S, ctx.cu_seqlens, ctx.seq_slot, ctx.n_seqs, ctx.max_rows,
                                correct=False)
-        y = ops.group_norm_gate(o, H, None, U, self.g_off, "silu", self.eps, ctx.act_dtype)
+        y = ops.group_norm_gate(o, H, None, U, at + self.g_off, "silu", self.eps, ctx.act_dtype)
         return ops.linear(y, self.w_o)
 
 

@@ -3,6 +3,8 @@ from __future__ import annotations
 
 from typing import Dict
 
+import torch
+
 from ..kernels import ops
 from ..weights.loader import TensorWant
 from .base import Mixer, StepContext, build_part, register_part
@@ -21,6 +23,9 @@ class SideBySide(Mixer):
     `left_norm`, `right_norm`), and the two scales are one and the same.  A block that forms that in a kernel
     of its own sets `takes_normed_pairs` and gets the pieces as `ops.NormedPair`.
 
+    Mixers that both read their input through one stacked matrix (`Mixer.takes_projected`) get theirs stacked
+    into one: a single product makes the columns of both.
+
     `left_position`, `right_position`: `PartSpec`s of position encodings of the mixers' own, in place of the
     block's.
     """
@@ -38,7 +43,8 @@ class SideBySide(Mixer):
         if self.norm_size and self.left_scale != self.right_scale:
             raise ValueError("side_by_side: outputs with norms of their own have one scale")
         self.own_positions = [build_part("position", p) if p is not None else None for p in (left_position, right_position)]
-        self.norms = None
+        self.norms = self.w_in = None
+        self.right_column = 0
         if sum(m.kv_spec() is not None for m in both) > 1 or sum(m.state_spec() is not None for m in both) > 1:
             raise ValueError("side_by_side: a cache line holds one mixer's keys and values and one "
                              "mixer's state; these two both keep the same kind")
@@ -63,6 +69,14 @@ class SideBySide(Mixer):
         for m, own in zip((self.left, self.right), self.own_positions):
             m.decode_copies, m.position = self.decode_copies, own if own is not None else self.position
             m.load(tensors)
+        if self.left.takes_projected and self.right.takes_projected:
+            a, b = ops.plain_weight(self.left.w_in), ops.plain_weight(self.right.w_in)
+            if a.dtype == b.dtype:
+                # (rows of zeros up to a multiple of 8, so that the right mixer's columns are as aligned as alone)
+                pad = a.new_zeros((-a.shape[0] % 8, a.shape[1]))
+                self.right_column = a.shape[0] + pad.shape[0]
+                self.w_in = ops.decode_weight(torch.cat([a, pad, b], dim=0).contiguous(), "plain", self.decode_copies)
+                self.left.w_in = self.right.w_in = None
         if self.norm_size:
             self.norms = [self._take(tensors, n).contiguous() for n in ("left_norm", "right_norm")]
 
@@ -71,8 +85,12 @@ class SideBySide(Mixer):
 
     def forward(self, h, ctx: StepContext, line, writes_cache, position):
         of_left, of_right = (own if own is not None else position for own in self.own_positions)
-        a = self.left.forward(h, ctx, line, writes_cache, of_left)
-        b = self.right.forward(h, ctx, line, writes_cache, of_right)
+        of_both = ({}, {})
+        if self.w_in is not None:
+            U = ops.linear(h, self.w_in)
+            of_both = ({"projected": (U, 0)}, {"projected": (U, self.right_column)})
+        a = self.left.forward(h, ctx, line, writes_cache, of_left, **of_both[0])
+        b = self.right.forward(h, ctx, line, writes_cache, of_right, **of_both[1])
         if self.norm_size:
             pair = ops.NormedPair(a, self.norms[0], b, self.norms[1], self.norm_eps, self.left_scale)
             return pair if self.takes_normed_pairs else pair.tensor()
