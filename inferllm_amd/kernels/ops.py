@@ -2645,7 +2645,7 @@ def token_mix(h: torch.Tensor, mu: torch.Tensor, tail: torch.Tensor, row_slot: t
 
 
 MAX_PLANES = 8           # planes of rows a product with parts takes
-PARTS_MAX_ROWS = 128     # rows up to which such a product is one launch (or two)
+PARTS_MAX_ROWS = 128     # rows up to which such a product is one launch
 
 
 def _planes_product(planes: torch.Tensor, w, ends, few: bool) -> torch.Tensor:
@@ -2666,8 +2666,8 @@ def _planes_product(planes: torch.Tensor, w, ends, few: bool) -> torch.Tensor:
 def linear_parts(planes: torch.Tensor, w, ends):
     """Products of one stacked matrix w [N, K] whose parts read rows of their own: part p, w's rows ends[p - 1] ..
     ends[p] - 1, times planes[p] of [S, M, K].  Returns one [M, part] tensor a part (columns of wider rows where one
-    launch made several).  Few bfloat16 rows: one launch; up to 128 rows from the decode copy: one, or two
-    where the last part is no multiple of the blocks; else one product a part."""
+    launch made several).  One launch for few bfloat16 rows (parts but the last in steps of 16) and from the
+    decode copy for up to 128 (in steps of 32); else one product a part."""
     ends = [int(e) for e in ends]
     S, M, K = planes.shape
     _need(planes.dim() == 3 and S == len(ends) and w.shape[1] == K and w.shape[0] == ends[-1], "linear_parts: shapes")
